@@ -27,7 +27,10 @@ DEBUG_ONLY = ["debug.hip", "bb_engine.hip", "bb_all.hip"]
 EXTRA = {"debug.hip": ["-mllvm", "-amdgpu-kernarg-preload-count=16"]}
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function",
-         "-fno-gpu-rdc"]
+         "-fno-gpu-rdc",
+         # no packed fp32 (v_pk_fma / mul / add_f32): hipcc forms them from ordinary float code, and some of their operand forms have returned
+         # wrong values beside another wave's MFMAs (tests/test_build_rules.py)
+         "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 def _headers() -> list[str]:
@@ -68,6 +71,10 @@ def _build_one(lib: str, sources: list[str], objdir: str, extra: list[str], forc
     hdrs = _headers()
     os.makedirs(objdir, exist_ok=True)
     sources = [s for s in sources if os.path.exists(os.path.join(CSRC, s))]
+    # objects of other flags are stale whatever their age
+    flag_file, flags = os.path.join(objdir, "flags"), repr((HIPCC, FLAGS, extra, sorted(EXTRA.items())))
+    if not os.path.exists(flag_file) or open(flag_file).read() != flags:
+        force = True
     jobs = []
     for s in sources:
         src = os.path.join(CSRC, s)
@@ -76,6 +83,8 @@ def _build_one(lib: str, sources: list[str], objdir: str, extra: list[str], forc
             jobs.append([HIPCC, *FLAGS, *extra, *EXTRA.get(s, []), "-c", src, "-o", obj])
     with ThreadPoolExecutor(max_workers=4) as ex:
         list(ex.map(lambda c: _run(c, verbose), jobs))
+    with open(flag_file, "w") as f:
+        f.write(flags)
     objs = [os.path.join(objdir, s.replace(".hip", ".o")) for s in sources]
     stamp = lib + ".digest"
     old = open(stamp).read().strip() if os.path.exists(stamp) else ""

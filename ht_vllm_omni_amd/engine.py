@@ -279,8 +279,7 @@ class TalkerEngine:
                     lw["moe_shared_gate_f"] = frag_shuffle(g16)
             if d.moe_experts > 0:
                 # the batched hipBLASLt prefill (prefill_gemm="blas", kept for A/B) wants [E, K, N] operands stored that way:
-                # torch.bmm on the transposed VIEW of [E, N, K] faults on this ROCm build at the talker's shapes
-                # (scripts/diag_bmm.py); they replace the row-major expert copies, which nothing else reads
+                # torch.bmm on the transposed VIEW of [E, N, K] faults on this ROCm build at the talker's shapes; they replace the row-major expert copies, which nothing else reads
                 for n in ("moe_gate_up", "moe_down"):
                     rm = lw.pop(n)
                     if self.prefill_gemm in ("blas", "both"):
