@@ -1,4 +1,4 @@
-"""ctypes binding of libomni_talker.so (the C-ABI of include/omni_talker.h).
+"""ctypes binding of libomni_talker.so (the C-ABI of include/omni_talker.h) and libomni_decoder.so (include/omni_decoder.h).
 
 The product path has NO fallback: if the HIP library is missing or an entry point fails,
 this module raises.  `import torch` happens first so the library resolves libamdhip64.so.7
@@ -45,10 +45,36 @@ class TileGemm(C.Structure):
     _fields_ = [("x", vp), ("x_rows", i64), ("ldx", i32), ("seg_len", i32), ("seg_rows", i32), ("row_off", i32),
                 ("w", vp), ("bias", vp), ("scale", vp), ("act", i32), ("resid", vp), ("ldr", i32), ("out_f32", vp), ("ldf", i32), ("out", vp), ("ldo", i32),
                 ("out2", vp), ("ldo2", i32), ("snake_alpha", vp), ("snake_inv_beta", vp), ("M", i32), ("N", i32), ("K", i32), ("tile_hint", i32),
-                ("groups", i32), ("x_group_rows", i64), ("w_group_elems", i64), ("out_group_rows", i64), ("group_rows", vp)]
+                ("groups", i32), ("x_group_rows", i64), ("w_group_elems", i64), ("out_group_rows", i64), ("group_rows", vp),
+                ("act_p", f32), ("act_n", f32), ("x_group_cols", i64), ("out_group_cols", i64)]
 
 
-TILE_ACT_NONE, TILE_ACT_GELU, TILE_ACT_SILU_MUL_GU8 = 0, 1, 2
+TILE_ACT_NONE, TILE_ACT_GELU, TILE_ACT_SILU_MUL_GU8, TILE_ACT_XIELU = 0, 1, 2, 3
+
+
+class StreamRows(C.Structure):
+    """omni_stream_rows (include/omni_decoder.h)."""
+    _fields_ = [("ids", vp), ("table", vp), ("vocab", i32), ("x_in", vp), ("y", vp), ("gain", f32), ("eps", f32), ("mu", vp), ("state", vp),
+                ("state_slot", vp), ("row_of_tok", vp), ("positions", vp), ("use_final", i32), ("final_gain", f32), ("sel", vp), ("x_out", vp),
+                ("h_out", vp), ("frag", i32), ("rows", i32), ("width", i32), ("wp", i32), ("elem", i32)]
+
+
+class LatentWrite(C.Structure):
+    """omni_latent_write."""
+    _fields_ = [("proj", vp), ("ld", i32), ("q_rank", i32), ("qp", i32), ("kv_rank", i32), ("rp", i32), ("heads", i32), ("qw", vp), ("kw", vp),
+                ("eps", f32), ("cq", vp), ("frag", i32), ("cache", vp), ("gate", vp), ("block_table", vp), ("bt_stride", i32), ("block_size", i32),
+                ("row_of_tok", vp), ("positions", vp), ("num_live", vp), ("x", vp), ("wp", i32), ("state", vp), ("state_slot", vp), ("T", i32),
+                ("elem", i32)]
+
+
+class LatentAttn(C.Structure):
+    """omni_latent_attn."""
+    _fields_ = [("q", vp), ("cache", vp), ("gate", vp), ("out", vp), ("block_table", vp), ("bt_stride", i32), ("block_size", i32),
+                ("row_of_tok", vp), ("positions", vp), ("tiles", vp), ("n_tiles", i32), ("T", i32), ("n_decode", i32), ("heads", i32), ("rp", i32),
+                ("scale", f32), ("max_keys", i32), ("workspace", vp), ("workspace_bytes", i64), ("elem", i32)]
+
+
+LATENT_TILE = 128           # OMNI_LATENT_TILE
 
 
 class ResUnit(C.Structure):
@@ -163,12 +189,28 @@ SIGNATURES = {
     "omni_talker_code_predictor": (i32, [vp, vp, vp, vp, vp, vp, i32, i32, f32, i32, f32, u32, vp, vp]),
 }
 
+# what libomni_decoder.so exports: its own entries and the shared ones (same sources as the talker's)
+DECODER_SIGNATURES = {
+    **{n: SIGNATURES[n] for n in ("omni_last_error", "omni_abi_version", "omni_gemm_bf16_ex", "omni_gemm_tile", "omni_sample", "omni_sample_rows")},
+    "omni_stream_rows_run": (i32, [C.POINTER(StreamRows), vp]),
+    "omni_latent_write_run": (i32, [C.POINTER(LatentWrite), vp]),
+    "omni_latent_attn_run": (i32, [C.POINTER(LatentAttn), vp]),
+    "omni_latent_attn_workspace_bytes": (i64, [i32, i32, i32]),
+    "omni_latent_attn_mfma": (i32, [i32]),
+    "omni_head_gemm": (i32, [vp, vp, vp, i32, i32, i32, i32, i32, vp]),
+    "omni_gemm_f32": (i32, [vp, i32, i64, vp, i64, vp, i32, i64, i32, i32, i32, i32, i32, f32, f32, vp]),
+    "omni_gemm_xielu": (i32, [vp, i32, vp, vp, i32, i32, i32, f32, f32, i32, vp]),
+    "omni_sample_step": (i32, [vp, i32, i32, i32, C.POINTER(RowSampling), vp, vp, vp, vp, vp, vp, vp]),
+}
+
 _lib = None
+_decoder = None
 _product = None
+DECODER_LIB_PATH = os.path.join(HERE, "libomni_decoder.so")
 DEBUG_LIB_PATH = os.path.join(HERE, "libomni_talker_debug.so")
 
 
-def _open(path: str, debug: bool) -> C.CDLL:
+def _open(path: str, debug: bool, signatures: dict | None = None, sources: list[str] | None = None) -> C.CDLL:
     if not os.path.exists(path):
         raise OmniError(
             f"{path} is missing: build it with `python -m ht_vllm_omni_amd.build` "
@@ -179,11 +221,11 @@ def _open(path: str, debug: bool) -> C.CDLL:
     if os.path.isdir(csrc) and os.environ.get("OMNI_SKIP_STALE_CHECK") != "1":
         from .build import sources_digest
         have = open(stamp).read().strip() if os.path.exists(stamp) else "<no stamp>"
-        if have != sources_digest(debug):
+        if have != sources_digest(debug, sources):
             raise OmniError(f"{path} is stale: built from other sources than {csrc} (digest {have[:12]}); "
                             "rebuild with `python -m ht_vllm_omni_amd.build`")
     lib = C.CDLL(path)
-    for name, (res, args) in SIGNATURES.items():
+    for name, (res, args) in (signatures or SIGNATURES).items():
         try:
             fn = getattr(lib, name)
         except AttributeError as e:
@@ -203,6 +245,15 @@ def load() -> C.CDLL:
     return _lib
 
 
+def load_decoder() -> C.CDLL:
+    """dlopen libomni_decoder.so (the language-model engine's library); raises OmniError when absent or stale."""
+    global _decoder
+    if _decoder is None:
+        from .build import DECODER_SOURCES
+        _decoder = _open(DECODER_LIB_PATH, False, DECODER_SIGNATURES, DECODER_SOURCES)
+    return _decoder
+
+
 class debug_library:
     """Context manager for the tile-sweep / A-B tests: engines and ops created inside run on libomni_talker_debug.so
     (same sources, run-time policy knobs); the product library is restored on exit."""
@@ -218,9 +269,9 @@ class debug_library:
         _lib = _product
 
 
-def check(rc: int, what: str = "") -> None:
+def check(rc: int, what: str = "", lib: C.CDLL | None = None) -> None:
     if rc != 0:
-        msg = load().omni_last_error().decode(errors="replace")
+        msg = (lib or load()).omni_last_error().decode(errors="replace")
         raise OmniError(f"{what or 'omni call'} failed (rc={rc}): {msg}")
 
 

@@ -1,10 +1,12 @@
 """Build the HIP libraries in-tree with hipcc for gfx950 (cross-compiles without a GPU).
 
   libomni_talker.so        the product: HIP kernels + the C-ABI of include/omni_talker.h, policy knobs compiled in
-  libomni_talker_debug.so  the same sources with -DOMNI_DEBUG_HOOKS (run-time policy knobs, omni_debug_* setters) plus
+  libomni_decoder.so       the kernels of the decoder-only language models (include/omni_decoder.h): its own few sources plus the GEMMs and the
+                           sampler both libraries link
+  libomni_talker_debug.so  the talker's sources with -DOMNI_DEBUG_HOOKS (run-time policy knobs, omni_debug_* setters) plus
                            csrc/debug.hip (launch / memory-system probes): scripts/ and the tile-sweep tests only
 
-Both are git-ignored but travel with the repo snapshot.  `sources_digest()` is stamped into a side file next to each
+All are git-ignored but travel with the repo snapshot.  `sources_digest()` is stamped into a side file next to each
 library so that _lib.load() can refuse a library that is older than csrc/.
 """
 from __future__ import annotations
@@ -18,9 +20,11 @@ from concurrent.futures import ThreadPoolExecutor
 HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 LIB = os.path.join(HERE, "libomni_talker.so")
+LIB_DECODER = os.path.join(HERE, "libomni_decoder.so")
 LIB_DEBUG = os.path.join(HERE, "libomni_talker_debug.so")
-SOURCES = ["capi.hip", "gemm.hip", "gemm_prefill.hip", "norm.hip", "rope_kv.hip", "paged_attn.hip", "prefill_attn.hip", "moe.hip",
+SOURCES = ["errors.hip", "capi.hip", "gemm.hip", "gemm_prefill.hip", "norm.hip", "rope_kv.hip", "paged_attn.hip", "prefill_attn.hip", "moe.hip",
            "sampler.hip", "cp_chain.hip", "bb_chain.hip", "moe_chain.hip", "allreduce.hip", "codec.hip", "conv_unit.hip"]
+DECODER_SOURCES = ["errors.hip", "gemm.hip", "gemm_prefill.hip", "sampler.hip", "decoder_rows.hip", "head_gemm.hip", "latent_attn.hip"]
 # debug library only: the probes, and the losing A/B arms of the backbone chain (rounds 3 and 4; no product knob reaches them)
 DEBUG_ONLY = ["debug.hip", "bb_engine.hip", "bb_all.hip"]
 # per-file extra flags
@@ -40,10 +44,10 @@ def _headers() -> list[str]:
     return hdrs
 
 
-def sources_digest(debug: bool = False) -> str:
+def sources_digest(debug: bool = False, sources: list[str] | None = None) -> str:
     """sha256 over every file the library is built from (+ the flags): what _lib.load() compares the stamp with."""
     h = hashlib.sha256()
-    names = [s for s in SOURCES + (DEBUG_ONLY if debug else []) if os.path.exists(os.path.join(CSRC, s))]
+    names = [s for s in (sources or SOURCES + (DEBUG_ONLY if debug else [])) if os.path.exists(os.path.join(CSRC, s))]
     for f in [os.path.join(CSRC, s) for s in names] + _headers():
         h.update(os.path.basename(f).encode())
         h.update(open(f, "rb").read())
@@ -97,10 +101,35 @@ def _build_one(lib: str, sources: list[str], objdir: str, extra: list[str], forc
 
 def build(force: bool = False, verbose: bool = False, debug: bool = True) -> str:
     lib = _build_one(LIB, SOURCES, os.path.join(HERE, "build"), [], force, verbose, sources_digest(False))
+    build_decoder(force, verbose, shared_fresh=True)
     if debug:
         _build_one(LIB_DEBUG, SOURCES + DEBUG_ONLY, os.path.join(HERE, "build", "debug"), ["-DOMNI_DEBUG_HOOKS"], force, verbose,
                    sources_digest(True))
     return lib
+
+
+def build_decoder(force: bool = False, verbose: bool = False, shared_fresh: bool = False) -> str:
+    """The language-model library alone (what a process that serves no talker needs).  shared_fresh: the objects it shares with the talker's
+    library were just compiled."""
+    if force and shared_fresh:
+        for s in DECODER_SOURCES:
+            obj = os.path.join(HERE, "build", s.replace(".hip", ".o"))
+            if s not in SOURCES and os.path.exists(obj):
+                os.remove(obj)
+        force = False
+    return _build_one(LIB_DECODER, DECODER_SOURCES, os.path.join(HERE, "build"), [], force, verbose, sources_digest(sources=DECODER_SOURCES))
+
+
+def ensure_decoder() -> str:
+    """libomni_decoder.so of the sources that are here: compiled when absent or older (one process at a time)."""
+    import fcntl
+    os.makedirs(os.path.join(HERE, "build"), exist_ok=True)
+    with open(os.path.join(HERE, "build", "decoder.lock"), "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        stamp = LIB_DECODER + ".digest"
+        if not (os.path.exists(LIB_DECODER) and os.path.exists(stamp) and open(stamp).read().strip() == sources_digest(sources=DECODER_SOURCES)):
+            build_decoder()
+    return LIB_DECODER
 
 
 if __name__ == "__main__":

@@ -134,6 +134,26 @@ def load_talker_checkpoint(path: str, dtype: torch.dtype = BF16) -> tuple[dict, 
     return map_hf_talker_weights(iter_safetensors(path), dtype)
 
 
+def load_decoder_checkpoint(path: str, dims) -> dict[str, torch.Tensor]:
+    """A decoder-only model's tensors under their checkpoint names (decoder_config.tensor_shapes), every name and shape checked: a tensor that
+    is missing, of another shape, or that no layer of the config owns is an error."""
+    from .decoder_config import tensor_shapes
+    want = tensor_shapes(dims)
+    w: dict[str, torch.Tensor] = {}
+    unknown = []
+    for name, t in iter_safetensors(path):
+        if name not in want:
+            unknown.append(name)
+        elif tuple(t.shape) != want[name]:
+            raise ValueError(f"{name}: checkpoint shape {tuple(t.shape)} != {want[name]} from the config")
+        else:
+            w[name] = t
+    missing = sorted(set(want) - set(w))
+    if unknown or missing:
+        raise KeyError(f"checkpoint and config differ: unknown {sorted(unknown)}, missing {missing}")
+    return w
+
+
 def check_against_dims(w: dict, d: TalkerDims) -> None:
     """Shapes of a loaded checkpoint vs the dimensions the engine will be built with (raises ValueError)."""
     want = {"embed": (d.vocab, d.hidden), "norm": (d.hidden,), "lm_head": (d.vocab, d.hidden), "cp.norm": (d.cp_hidden,),

@@ -10,17 +10,6 @@
 #include "common.cuh"
 #include "kernels.h"
 
-// ------------------------------------------------------------------ error plumbing
-static thread_local char g_err[512] = "";
-void omni_set_error(const char* fmt, ...) {
-    va_list ap;
-    va_start(ap, fmt);
-    vsnprintf(g_err, sizeof(g_err), fmt, ap);
-    va_end(ap);
-}
-extern "C" const char* omni_last_error(void) { return g_err; }
-extern "C" int omni_abi_version(void) { return 5; }
-
 #define TRY(expr)                    \
     do {                             \
         int rc__ = (expr);           \

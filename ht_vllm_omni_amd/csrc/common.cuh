@@ -154,6 +154,11 @@ __device__ __forceinline__ void wave_argmax(float& v, int& idx) {
 __device__ __forceinline__ float wave_sum(float v) { return xor32_sum(xor16_sum(row16_sum(v))); }
 __device__ __forceinline__ float wave_max(float v) { return xor32_max(xor16_max(row16_max(v))); }
 
+// ---- xIELU: a quadratic branch above zero, an exponential one below, both with slope 1/2 at zero; ap, an are the two positive coefficients
+__device__ __forceinline__ float xielu(float z, float ap, float an) {
+    return fmaf(0.5f, z, z > 0.f ? ap * z * z : an * (expm1f(fminf(z, 0.f)) - z));
+}
+
 // ---- OCP e4m3fn <-> f32 (saturating, round-nearest-even: clamp then hardware cvt)
 #define OMNI_FP8_MAX 448.0f
 __device__ __forceinline__ uint32_t pack_fp8x4(float a, float b, float c, float d) {

@@ -1,0 +1,253 @@
+// Row-wise kernels of the decoder-only language models (include/omni_decoder.h): everything between two matrix products of a layer.
+// The residual stream is fp32; norms, gates and the token-shift state are fp32; only matrix operands are rounded (once) to bf16.
+#include "common.cuh"
+#include "../../include/omni_decoder.h"
+
+#define DR_THREADS 256
+#define DR_WAVES (DR_THREADS / 64)
+
+// ---- element type of matrix operands: 4 consecutive values
+template <typename E>
+__device__ __forceinline__ void ld4(const E* p, float (&v)[4]);
+template <>
+__device__ __forceinline__ void ld4<float>(const float* p, float (&v)[4]) {
+    const float4 a = *reinterpret_cast<const float4*>(p);
+    v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
+}
+template <>
+__device__ __forceinline__ void ld4<uint16_t>(const uint16_t* p, float (&v)[4]) {
+    const uint2 a = *reinterpret_cast<const uint2*>(p);
+    v[0] = bf_lo(a.x); v[1] = bf_hi(a.x); v[2] = bf_lo(a.y); v[3] = bf_hi(a.y);
+}
+template <typename E>
+__device__ __forceinline__ void st4(E* p, const float (&v)[4]);
+template <>
+__device__ __forceinline__ void st4<float>(float* p, const float (&v)[4]) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
+template <>
+__device__ __forceinline__ void st4<uint16_t>(uint16_t* p, const float (&v)[4]) {
+    *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf2(v[0], v[1]), pack_bf2(v[2], v[3]));
+}
+
+// sum over the workgroup, result in every thread; `buf` alternates between calls so that one barrier per sum is enough
+struct BlockSum {
+    float* lds;      // [2][DR_WAVES]
+    int flip;
+    __device__ __forceinline__ float operator()(float v) {
+        v = wave_sum(v);
+        float* b = lds + flip * DR_WAVES;
+        flip ^= 1;
+        if ((threadIdx.x & 63) == 0) b[threadIdx.x >> 6] = v;
+        __syncthreads();
+        float t = 0.f;
+#pragma unroll
+        for (int w = 0; w < DR_WAVES; ++w) t += b[w];
+        return t;
+    }
+};
+
+// A workgroup walks `strip` consecutive tokens so that the token shift finds the previous token's NEW stream row in registers; only the
+// strip's first token rebuilds its predecessor (or reads it from the sequence's state, or takes zeros).
+template <typename E, int MAXC, bool SHIFT>
+__global__ __launch_bounds__(DR_THREADS) void stream_rows_kernel(const omni_stream_rows a, int strip) {
+    __shared__ float red[2 * DR_WAVES];
+    BlockSum bsum{red, 0};
+    const int wp = a.wp;
+    const E* table = reinterpret_cast<const E*>(a.table);
+    const E* mu = reinterpret_cast<const E*>(a.mu);
+    E* h_out = reinterpret_cast<E*>(a.h_out);
+    auto load_new = [&](int t, float (&v)[MAXC][4]) {      // the stream row of token t behind the sublayer that just ran
+        if (a.ids) {
+            const int id = a.ids[t];
+            const bool ok = id >= 0 && id < a.vocab;
+#pragma unroll
+            for (int c = 0; c < MAXC; ++c) {
+                const int k = (c * DR_THREADS + threadIdx.x) * 4;
+                v[c][0] = v[c][1] = v[c][2] = v[c][3] = 0.f;
+                if (ok && k < wp) ld4<E>(table + (size_t)id * wp + k, v[c]);
+            }
+            return;
+        }
+        float y[MAXC][4], ss = 0.f;
+#pragma unroll
+        for (int c = 0; c < MAXC; ++c) {
+            const int k = (c * DR_THREADS + threadIdx.x) * 4;
+            v[c][0] = v[c][1] = v[c][2] = v[c][3] = 0.f;
+            y[c][0] = y[c][1] = y[c][2] = y[c][3] = 0.f;
+            if (k < wp) {
+                ld4<float>(a.x_in + (size_t)t * wp + k, v[c]);
+                if (a.y) ld4<float>(a.y + (size_t)t * wp + k, y[c]);
+            }
+        }
+        if (!a.y) return;
+#pragma unroll
+        for (int c = 0; c < MAXC; ++c) ss += sq4_sum(y[c][0], y[c][1], y[c][2], y[c][3]);
+        ss = bsum(ss);
+        const float r = a.gain / sqrtf(ss / (float)a.width + a.eps);
+#pragma unroll
+        for (int c = 0; c < MAXC; ++c)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[c][e] = fmaf(y[c][e], r, v[c][e]);
+    };
+    const int i0 = blockIdx.x * strip, i1 = min(i0 + strip, a.rows);
+    float cur[MAXC][4], prev[MAXC][4];
+    for (int i = i0; i < i1; ++i) {
+        const int t = a.sel ? a.sel[i] : i;
+        if (SHIFT) {
+            const int row = a.row_of_tok[t];
+            const bool first = t == 0 || a.row_of_tok[t - 1] != row;
+            if (first) {
+                const bool zero = a.positions[t] == 0;
+                const float* st = a.state + (size_t)a.state_slot[row] * wp;
+#pragma unroll
+                for (int c = 0; c < MAXC; ++c) {
+                    const int k = (c * DR_THREADS + threadIdx.x) * 4;
+                    prev[c][0] = prev[c][1] = prev[c][2] = prev[c][3] = 0.f;
+                    if (!zero && k < wp) ld4<float>(st + k, prev[c]);
+                }
+            } else if (i == i0) {
+                load_new(t - 1, prev);
+            } else {
+#pragma unroll
+                for (int c = 0; c < MAXC; ++c)
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) prev[c][e] = cur[c][e];
+            }
+        }
+        load_new(t, cur);
+        float rf = 0.f;
+        if (!SHIFT && a.use_final) {
+            float ss = 0.f;
+#pragma unroll
+            for (int c = 0; c < MAXC; ++c) ss += sq4_sum(cur[c][0], cur[c][1], cur[c][2], cur[c][3]);
+            rf = a.final_gain / sqrtf(bsum(ss) / (float)a.width + a.eps);
+        }
+#pragma unroll
+        for (int c = 0; c < MAXC; ++c) {
+            const int k = (c * DR_THREADS + threadIdx.x) * 4;
+            if (k >= wp) continue;
+            if (a.x_out) st4<float>(a.x_out + (size_t)t * wp + k, cur[c]);
+            if (!h_out) continue;
+            float h[4];
+            if (SHIFT) {
+                float m[4];
+                ld4<E>(mu + k, m);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) h[e] = fmaf(prev[c][e] - cur[c][e], m[e], cur[c][e]);
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) h[e] = a.use_final ? cur[c][e] * rf : cur[c][e];
+            }
+            st4<E>(h_out + (a.frag ? frag_off(i, k, wp) : (size_t)i * wp + k), h);
+        }
+    }
+}
+
+template <typename E, int MAXC>
+static void stream_rows_launch(const omni_stream_rows& a, int strip, hipStream_t st) {
+    const dim3 grid((a.rows + strip - 1) / strip), block(DR_THREADS);
+    if (a.mu) hipLaunchKernelGGL((stream_rows_kernel<E, MAXC, true>), grid, block, 0, st, a, strip);
+    else hipLaunchKernelGGL((stream_rows_kernel<E, MAXC, false>), grid, block, 0, st, a, strip);
+}
+
+template <typename E>
+static int stream_rows_pick(const omni_stream_rows& a, int strip, hipStream_t st) {
+    const int chunks = (a.wp / 4 + DR_THREADS - 1) / DR_THREADS;
+    if (chunks <= 1) stream_rows_launch<E, 1>(a, strip, st);
+    else if (chunks <= 2) stream_rows_launch<E, 2>(a, strip, st);
+    else if (chunks <= 4) stream_rows_launch<E, 4>(a, strip, st);
+    else stream_rows_launch<E, 8>(a, strip, st);
+    OMNI_CHECK_LAUNCH("omni_stream_rows");
+    return OMNI_OK;
+}
+
+extern "C" int omni_stream_rows_run(const omni_stream_rows* p, void* stream) {
+    OMNI_CHECK_ARG(p && (p->ids ? p->table != nullptr : p->x_in != nullptr) && (p->x_out || p->h_out), "omni_stream_rows: null pointer");
+    const omni_stream_rows& a = *p;
+    OMNI_CHECK_ARG(a.width > 0 && a.wp >= a.width && a.wp % 32 == 0 && a.wp <= DR_THREADS * 4 * 8, "omni_stream_rows: width=%d wp=%d (multiple of 32, <= 8192)", a.width, a.wp);
+    OMNI_CHECK_ARG(a.elem == 0 || a.elem == 1, "omni_stream_rows: elem=%d", a.elem);
+    OMNI_CHECK_ARG(!a.frag || a.elem == 0, "omni_stream_rows: fragment-major output is bf16");
+    OMNI_CHECK_ARG(!a.mu || (a.state && a.state_slot && a.row_of_tok && a.positions && !a.sel && !a.use_final), "omni_stream_rows: token shift needs state, rows and positions, and no selection");
+    OMNI_CHECK_ARG(!a.sel || !a.x_out, "omni_stream_rows: a selection writes h only");
+    // (a strip's first token and the shift read rows of x_in that another workgroup may already have rewritten: never in place)
+    OMNI_CHECK_ARG(a.x_out == nullptr || a.x_out != a.x_in, "omni_stream_rows: x_out must not be x_in");
+    if (a.rows <= 0) return OMNI_OK;
+    const int strip = a.mu && a.rows > 1024 ? 4 : 1;
+    return a.elem ? stream_rows_pick<float>(a, strip, (hipStream_t)stream) : stream_rows_pick<uint16_t>(a, strip, (hipStream_t)stream);
+}
+
+// ---- latents: norms, cache write, gates, token-shift state.  One workgroup per token.
+template <typename E>
+__global__ __launch_bounds__(DR_THREADS) void latent_write_kernel(const omni_latent_write a) {
+    __shared__ float red[2][DR_WAVES];
+    const int t = blockIdx.x;
+    const int row = a.row_of_tok[t], pos = a.positions[t];
+    const float* yq = a.proj + (size_t)t * a.ld;
+    const float* yk = yq + a.qp;
+    float sq = 0.f, sk = 0.f;
+    for (int k = threadIdx.x * 4; k < a.qp; k += DR_THREADS * 4) {       // padded columns hold zeros
+        float v[4];
+        ld4<float>(yq + k, v);
+        sq += sq4_sum(v[0], v[1], v[2], v[3]);
+    }
+    for (int k = threadIdx.x * 4; k < a.rp; k += DR_THREADS * 4) {
+        float v[4];
+        ld4<float>(yk + k, v);
+        sk += sq4_sum(v[0], v[1], v[2], v[3]);
+    }
+    sq = wave_sum(sq);
+    sk = wave_sum(sk);
+    if ((threadIdx.x & 63) == 0) { red[0][threadIdx.x >> 6] = sq; red[1][threadIdx.x >> 6] = sk; }
+    __syncthreads();
+    sq = sk = 0.f;
+#pragma unroll
+    for (int w = 0; w < DR_WAVES; ++w) { sq += red[0][w]; sk += red[1][w]; }
+    const float rq = 1.0f / sqrtf(sq / (float)a.q_rank + a.eps), rk = 1.0f / sqrtf(sk / (float)a.kv_rank + a.eps);
+    E* cq = reinterpret_cast<E*>(a.cq);
+    const E* qw = reinterpret_cast<const E*>(a.qw);
+    for (int k = threadIdx.x * 4; k < a.qp; k += DR_THREADS * 4) {
+        float v[4], w[4];
+        ld4<float>(yq + k, v);
+        ld4<E>(qw + k, w);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = v[e] * rq * w[e];
+        st4<E>(cq + (a.frag ? frag_off(t, k, a.qp) : (size_t)t * a.qp + k), v);
+    }
+    if (a.gate)
+        for (int h = threadIdx.x; h < a.heads; h += DR_THREADS) a.gate[(size_t)t * a.heads + h] = 1.0f / (1.0f + expf(-yk[a.rp + h]));
+    if (a.num_live && row >= *a.num_live) return;
+    const int blk = a.block_table[(size_t)row * a.bt_stride + pos / a.block_size];
+    E* dst = reinterpret_cast<E*>(a.cache) + ((size_t)blk * a.block_size + pos % a.block_size) * a.rp;
+    const E* kw = reinterpret_cast<const E*>(a.kw);
+    for (int k = threadIdx.x * 4; k < a.rp; k += DR_THREADS * 4) {
+        float v[4], w[4];
+        ld4<float>(yk + k, v);
+        ld4<E>(kw + k, w);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = v[e] * rk * w[e];
+        st4<E>(dst + k, v);
+    }
+    if (a.state && (t == a.T - 1 || a.row_of_tok[t + 1] != row)) {
+        float* s = a.state + (size_t)a.state_slot[row] * a.wp;
+        for (int k = threadIdx.x * 4; k < a.wp; k += DR_THREADS * 4) {
+            float v[4];
+            ld4<float>(a.x + (size_t)t * a.wp + k, v);
+            st4<float>(s + k, v);
+        }
+    }
+}
+
+extern "C" int omni_latent_write_run(const omni_latent_write* p, void* stream) {
+    OMNI_CHECK_ARG(p && p->proj && p->qw && p->kw && p->cq && p->cache && p->block_table && p->row_of_tok && p->positions, "omni_latent_write: null pointer");
+    const omni_latent_write& a = *p;
+    OMNI_CHECK_ARG(a.q_rank > 0 && a.kv_rank > 0 && a.qp >= a.q_rank && a.rp >= a.kv_rank && a.qp % 32 == 0 && a.rp % 32 == 0 && a.ld % 4 == 0 &&
+                   a.ld >= a.qp + a.rp + (a.gate ? a.heads : 0), "omni_latent_write: q %d / %d, kv %d / %d, ld %d", a.q_rank, a.qp, a.kv_rank, a.rp, a.ld);
+    OMNI_CHECK_ARG(a.block_size > 0 && a.bt_stride > 0 && a.heads > 0, "omni_latent_write: block_size=%d bt_stride=%d", a.block_size, a.bt_stride);
+    OMNI_CHECK_ARG(!a.state || (a.x && a.state_slot && a.wp % 4 == 0), "omni_latent_write: state needs the stream rows and slots");
+    OMNI_CHECK_ARG(a.elem == 1 || a.elem == 0, "omni_latent_write: elem=%d", a.elem);
+    OMNI_CHECK_ARG(!a.frag || a.elem == 0, "omni_latent_write: fragment-major output is bf16");
+    if (a.T <= 0) return OMNI_OK;
+    if (a.elem) hipLaunchKernelGGL(latent_write_kernel<float>, dim3(a.T), dim3(DR_THREADS), 0, (hipStream_t)stream, a);
+    else hipLaunchKernelGGL(latent_write_kernel<uint16_t>, dim3(a.T), dim3(DR_THREADS), 0, (hipStream_t)stream, a);
+    OMNI_CHECK_LAUNCH("omni_latent_write");
+    return OMNI_OK;
+}

@@ -51,6 +51,8 @@ struct TileArgs {
     // tiles past it leave at once, rows past it read as zero and are not stored
     long long gx_rows, gw_elems, gout_rows;
     const int32_t* group_rows;
+    float act_p, act_n;              // OMNI_TILE_ACT_XIELU
+    long long gx_cols, gout_cols;    // grouped launch: column offset of a group in x and in the outputs (per-head products of one token array)
 };
 
 __device__ __forceinline__ f32x4 tg_mfma(u32x4 a, u32x4 b, f32x4 c) {
@@ -60,7 +62,7 @@ __device__ __forceinline__ f32x4 tg_mfma(u32x4 a, u32x4 b, f32x4 c) {
 __device__ __forceinline__ float tg_gelu(float v) { return 0.5f * v * (1.0f + erff(v * 0.70710678118654752f)); }
 
 __device__ __forceinline__ bool tile_plain(const TileArgs& a) {
-    return !a.bias && !a.scale && a.act != OMNI_TILE_ACT_GELU && !a.resid && !a.out_f32 && !a.out2 && a.out;
+    return !a.bias && !a.scale && a.act != OMNI_TILE_ACT_GELU && a.act != OMNI_TILE_ACT_XIELU && !a.resid && !a.out_f32 && !a.out2 && a.out;
 }
 
 // Epilogue of a tile kernel: `acc[j][i]` = this wave's WN n-tiles x WM m-tiles (D[n][m] fragments), first row mw0, first column nw0; `lds` is dead.
@@ -90,7 +92,7 @@ __device__ __forceinline__ void tile_epilogue(const TileArgs& a, f32x4 (&acc)[WN
             if (a.scale) sq[j] = *reinterpret_cast<const f32x4*>(a.scale + n);
         }
     }
-    const bool gelu = !PLAIN && a.act == OMNI_TILE_ACT_GELU;
+    const bool gelu = !PLAIN && a.act == OMNI_TILE_ACT_GELU, xie = !PLAIN && a.act == OMNI_TILE_ACT_XIELU;
     auto write_image = [&](const int pass) {
         if (PLAIN) {
 #pragma unroll
@@ -101,6 +103,14 @@ __device__ __forceinline__ void tile_epilogue(const TileArgs& a, f32x4 (&acc)[WN
                 f32x4 v;
 #pragma unroll
                 for (int e = 0; e < 4; ++e) v[e] = tg_gelu(acc[j][pass][e] + bq[j][e]) * sq[j][e];
+                *reinterpret_cast<f32x4*>(img + c * IPITCH + (j * 16 + 4 * q) * 4) = v;
+            }
+        } else if (xie) {
+#pragma unroll
+            for (int j = 0; j < WN; ++j) {
+                f32x4 v;
+#pragma unroll
+                for (int e = 0; e < 4; ++e) v[e] = xielu(acc[j][pass][e] + bq[j][e], a.act_p, a.act_n) * sq[j][e];
                 *reinterpret_cast<f32x4*>(img + c * IPITCH + (j * 16 + 4 * q) * 4) = v;
             }
         } else {
@@ -229,7 +239,7 @@ template <int WAVES_N, int WN, int WM, bool GU8>
 __global__ __launch_bounds__(TG_THREADS) void gemm_tile_kernel(const TileArgs a_in) {
     using G = TileGeom<WAVES_N, WN, WM>;
     TileArgs a = a_in;
-    long long x_lo = 0, x_hi = a.x_rows;                                      // rows of x this launch may read
+    long long x_lo = 0, x_hi = a.x_rows, x_skip = 0;                          // rows of x this launch may read; elements ahead of the group's first column
     if (gridDim.y > 1 || a.group_rows) {
         const int grp = blockIdx.y;
         if (a.group_rows) a.M = min(a.M, a.group_rows[grp]);
@@ -241,6 +251,11 @@ __global__ __launch_bounds__(TG_THREADS) void gemm_tile_kernel(const TileArgs a_
         if (a.out2) a.out2 += orow * a.ldo2;
         if (a.out_f32) a.out_f32 += orow * a.ldf;
         if (a.resid) a.resid += orow * a.ldr;
+        x_skip = grp * a.gx_cols;
+        a.x += x_skip;
+        const size_t ocol = (size_t)grp * a.gout_cols;
+        if (a.out) a.out += ocol;
+        if (a.out_f32) a.out_f32 += ocol;
     }
     constexpr int NTILES = G::NTILES, SLICE = G::SLICE, NLW = G::NLW, NLX = G::NLX, NBUF = G::NBUF;
     constexpr int INFLIGHT = NBUF - 2;                                        // slices still landing when slice t + 1 is awaited
@@ -273,7 +288,7 @@ __global__ __launch_bounds__(TG_THREADS) void gemm_tile_kernel(const TileArgs a_
     const int nsteps = a.K >> 5;                                              // 32-deep slices
 
     const __amdgpu_buffer_rsrc_t rw = __builtin_amdgcn_make_buffer_rsrc((void*)a.W, 0, (int)((size_t)a.N * a.K * 2), 0x00020000);
-    const __amdgpu_buffer_rsrc_t rx = __builtin_amdgcn_make_buffer_rsrc((void*)a.x, 0, (int)(a.x_rows * a.ldx * 2), 0x00020000);
+    const __amdgpu_buffer_rsrc_t rx = __builtin_amdgcn_make_buffer_rsrc((void*)a.x, 0, (int)((a.x_rows * a.ldx - x_skip) * 2), 0x00020000);
 
     // ---- staging.  Slice image: W tile f at f KB, x tile g at (NTILES + g) KB.  Wave w issues W tiles w + 8 i (i < NLW; a wave
     // without an i-th tile loads zeros into a spare KB so that every wave has the same count in flight) and x tiles w + 8 i.
@@ -641,7 +656,7 @@ extern "C" int omni_gemm_tile(const omni_tile_gemm* g, void* stream) {
     OMNI_CHECK_ARG(g->x_rows > 0 && g->x_rows * (int64_t)g->ldx * 2 < (int64_t)TG_OOB, "omni_gemm_tile: x of %lld rows x %d exceeds the 2 GB descriptor", (long long)g->x_rows, g->ldx);
     OMNI_CHECK_ARG((int64_t)g->N * g->K * 2 < (int64_t)TG_OOB, "omni_gemm_tile: W exceeds the 2 GB descriptor");
     const bool gu8 = g->act == OMNI_TILE_ACT_SILU_MUL_GU8;
-    OMNI_CHECK_ARG(g->act == OMNI_TILE_ACT_NONE || g->act == OMNI_TILE_ACT_GELU || gu8, "omni_gemm_tile: act=%d", g->act);
+    OMNI_CHECK_ARG(g->act == OMNI_TILE_ACT_NONE || g->act == OMNI_TILE_ACT_GELU || g->act == OMNI_TILE_ACT_XIELU || gu8, "omni_gemm_tile: act=%d", g->act);
     OMNI_CHECK_ARG(g->tile_hint >= 0 && g->tile_hint <= 7, "omni_gemm_tile: tile_hint=%d", g->tile_hint);
     OMNI_CHECK_ARG(g->tile_hint < 3 || g->N % 256 == 0, "omni_gemm_tile: tile_hint=%d needs N %% 256 == 0", g->tile_hint);
     OMNI_CHECK_ARG(!gu8 || (g->out && !g->resid && !g->out2 && !g->out_f32), "omni_gemm_tile: SiLU-mul takes out only");
@@ -666,6 +681,15 @@ extern "C" int omni_gemm_tile(const omni_tile_gemm* g, void* stream) {
     OMNI_CHECK_ARG(groups == 1 || (int64_t)groups * g->w_group_elems * 2 + (int64_t)g->N * g->K * 2 < ((int64_t)1 << 40), "omni_gemm_tile: W groups");
     a.gx_rows = groups > 1 ? g->x_group_rows : 0; a.gw_elems = groups > 1 ? g->w_group_elems : 0; a.gout_rows = groups > 1 ? g->out_group_rows : 0;
     a.group_rows = g->group_rows;
+    a.act_p = g->act_p; a.act_n = g->act_n;
+    // groups as column ranges of one token array: group g reads x columns [g * x_group_cols, + K) and writes columns [g * out_group_cols, + N)
+    OMNI_CHECK_ARG(groups == 1 || (g->x_group_cols >= 0 && g->out_group_cols >= 0 && g->x_group_cols % 8 == 0 && g->out_group_cols % 8 == 0 &&
+                                   (groups - 1) * g->x_group_cols + seg_len <= g->ldx &&
+                                   (!g->out || (groups - 1) * g->out_group_cols + nout <= g->ldo) &&
+                                   (!g->out_f32 || (groups - 1) * g->out_group_cols + nout <= g->ldf) &&
+                                   (g->out_group_cols == 0 || (!g->out2 && !g->resid))),
+                   "omni_gemm_tile: group columns leave the rows of x / out");
+    a.gx_cols = groups > 1 ? g->x_group_cols : 0; a.gout_cols = groups > 1 ? g->out_group_cols : 0;
     hipStream_t st = (hipStream_t)stream;
     const int N = g->N;
     // <waves along n, n tiles per wave, m tiles per wave>: 256 x 256 | 192 x 256 | 128 x 512 | 96 x 512 output tiles, and 128 x 64

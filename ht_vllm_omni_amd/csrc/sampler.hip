@@ -239,3 +239,11 @@ extern "C" int omni_sample_rows(const float* logits, int ld, int B, int V, const
     return k_sample(logits, ld, B, V, 1, 1.0f, 0, 1.0f, 1.0f, seen, 0, steps, step_mul, step_add, inc_steps, out_ids, 1, stream,
                     nullptr, nullptr, rows, nullptr);
 }
+
+// (declared in omni_decoder.h) the decode step of a language model: per-row parameters, live rows only, ids replaced and counters advanced in place
+extern "C" int omni_sample_step(const float* logits, int ld, int B, int V, const omni_row_sampling* rows, uint8_t* seen, int32_t* steps,
+                                int32_t* ids, int32_t* positions, int32_t* seq_lens, const int32_t* num_live, void* stream) {
+    OMNI_CHECK_ARG(rows && rows->greedy && rows->temperature && rows->top_k && rows->top_p && rows->rep_penalty && rows->seed,
+                   "omni_sample_step: every per-row array is required");
+    return k_sample(logits, ld, B, V, 1, 1.0f, 0, 1.0f, 1.0f, seen, 0, steps, 1, 0, 1, ids, 1, stream, positions, seq_lens, rows, num_live);
+}

@@ -293,7 +293,8 @@ def rope_table(max_pos: int, head_dim: int, theta: float) -> torch.Tensor:
 
 def gemm_tile(x: torch.Tensor, w_frag: torch.Tensor, *, M: int | None = None, bias=None, scale=None, act: int = L.TILE_ACT_NONE,
               resid=None, out=None, out_f32=None, out2=None, snake=None, taps: int = 1, dilation: int = 1,
-              row_off: int | None = None, want: str = "b", tile_hint: int = 0, groups: int = 1, group_rows=None):
+              row_off: int | None = None, want: str = "b", tile_hint: int = 0, groups: int = 1, group_rows=None,
+              act_params: tuple[float, float] = (0.0, 0.0), group_cols: bool = False, lib=None):
     """omni_gemm_tile: y[M, N] = act(A . W^T + bias) * scale (+ resid) on the matrix cores, A = x for taps == 1, else the
     causal conv window A[m] = [x[m + row_off], x[m + row_off + dilation], ...] (taps rows of x.shape[1] channels; row_off
     defaults to -(taps - 1) * dilation; rows outside x read as zero).  x bf16 [rows, C] (row stride = x.stride(0)); w_frag bf16
@@ -302,10 +303,16 @@ def gemm_tile(x: torch.Tensor, w_frag: torch.Tensor, *, M: int | None = None, bi
     given buffers (out_f32 / out / out2) are used, missing ones allocated.  Returns them in the order of `want` (a single
     tensor when one is wanted).
     groups > 1: the batched form -- x [groups * cap, C] (cap rows per group), w_frag [groups, N, K] (each matrix fragment-major),
-    outputs [groups * cap, N]; group_rows int32 [groups] (device) = live rows per group (the rest is neither computed nor written)."""
+    outputs [groups * cap, N]; group_rows int32 [groups] (device) = live rows per group (the rest is neither computed nor written).
+    group_cols: the groups are column ranges instead -- x [rows, groups * K], output [rows, groups * N] (one product per head).
+    act_params: the two coefficients of TILE_ACT_XIELU.  lib: the library to launch from (default: the talker's)."""
     assert x.dtype == BF16 and w_frag.dtype == BF16 and x.dim() == 2 and x.stride(1) == 1
     rows, Cin = x.shape
-    if groups > 1:
+    if group_cols:
+        assert w_frag.dim() == 3 and w_frag.shape[0] == groups and w_frag.is_contiguous() and taps == 1 and Cin % groups == 0 and group_rows is None
+        N, K = w_frag.shape[1:]
+        Cin //= groups
+    elif groups > 1:
         assert w_frag.dim() == 3 and w_frag.shape[0] == groups and w_frag.is_contiguous() and taps == 1 and rows % groups == 0
         N, K = w_frag.shape[1:]
         cap = rows // groups
@@ -314,8 +321,9 @@ def gemm_tile(x: torch.Tensor, w_frag: torch.Tensor, *, M: int | None = None, bi
     assert K == taps * Cin, (K, taps, Cin)
     M = rows if M is None else M
     gu8 = act == L.TILE_ACT_SILU_MUL_GU8
-    nout = N // 2 if gu8 else N
+    nout = (N // 2 if gu8 else N) * (groups if group_cols else 1)
     g = L.TileGemm()
+    g.act_p, g.act_n = act_params
     g.x, g.x_rows, g.ldx = x.data_ptr(), rows, x.stride(0)
     g.seg_len, g.seg_rows = Cin, dilation
     g.row_off = (-(taps - 1) * dilation if row_off is None else row_off) if taps > 1 or row_off is not None else 0
@@ -341,11 +349,14 @@ def gemm_tile(x: torch.Tensor, w_frag: torch.Tensor, *, M: int | None = None, bi
         else:
             raise ValueError(want)
     g.M, g.N, g.K, g.tile_hint = M, N, K, tile_hint
-    if groups > 1:
+    if group_cols and groups > 1:
+        g.groups, g.w_group_elems, g.x_group_cols, g.out_group_cols = groups, N * K, K, N
+    elif groups > 1:
         assert M == rows, "a grouped launch covers every group's cap rows"
         g.M, g.groups, g.x_group_rows, g.w_group_elems, g.out_group_rows = cap, groups, cap, N * K, cap
         if group_rows is not None:
             assert group_rows.dtype == torch.int32 and group_rows.numel() == groups and group_rows.is_contiguous()
             g.group_rows = group_rows.data_ptr()
-    L.check(L.load().omni_gemm_tile(C.byref(g), L.current_stream()), "omni_gemm_tile")
+    lib = lib or L.load()
+    L.check(lib.omni_gemm_tile(C.byref(g), L.current_stream()), "omni_gemm_tile", lib)
     return res[0] if len(res) == 1 else tuple(res)

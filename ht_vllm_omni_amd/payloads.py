@@ -44,6 +44,7 @@ class OmniNewRequestData:
     prompt_embeds: torch.Tensor | None = None
     external_req_id: str | None = None
     additional_information: Any = None      # AdditionalInformationPayload (the reference's wire type) or a plain dict
+    open_prompt: bool = False               # more prompt tokens follow in later steps (OmniCachedRequestData.new_token_ids): nothing is sampled
 
 
 @dataclass
@@ -65,6 +66,8 @@ class OmniSchedulerOutput:
     preempted_req_ids: set[str] = field(default_factory=set)
     # omni: {req_id: {"seq_len": int, "block_ids": [...], "custom_metadata": {...}?}}  (output.py:73-77)
     finished_requests_needing_kv_transfer: dict[str, dict] = field(default_factory=dict)
+    # language models: the tokens of this step whose logits are asked for, {req_id: places among the request's scheduled tokens}
+    logits_at: dict[str, list[int]] = field(default_factory=dict)
 
 
 @dataclass
@@ -95,6 +98,7 @@ class OmniModelRunnerOutput:
     cudagraph_stats: Any = None
     multimodal_outputs: dict[str, torch.Tensor] | None = None
     kv_extracted_req_ids: list[str] | None = None
+    token_logits: dict[str, torch.Tensor] | None = None      # fp32 [places, vocab] per request of OmniSchedulerOutput.logits_at
 
 
 EMPTY_MODEL_RUNNER_OUTPUT = OmniModelRunnerOutput(req_ids=[], req_id_to_index={}, sampled_token_ids=[])

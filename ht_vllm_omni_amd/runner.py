@@ -169,6 +169,8 @@ _ROW_BUFFERS = ("input_ids", "positions", "seq_lens", "block_table", "last_hidde
 
 
 class MI355XARModelRunner:
+    row_buffers = _ROW_BUFFERS          # the engine's per-row buffers that move with a batch row
+
     def __init__(self, engine, *, kv_transfer: OmniKVTransferManager | None = None, use_graphs: bool = True,
                  engine_output_type: str = "latent", prompt_builder=None, async_scheduling: bool = False):
         self.engine = engine
@@ -235,7 +237,7 @@ class MI355XARModelRunner:
             return
         self._tt_flush()
         idx = self._h2d("perm", np.asarray(perm, np.int64), torch.int64)
-        for name in _ROW_BUFFERS + ("rope_delta",):
+        for name in self.row_buffers + ("rope_delta",):
             buf = getattr(self.engine, name, None)
             if buf is None:
                 continue
@@ -288,13 +290,14 @@ class MI355XARModelRunner:
             r = self.rows.index(rid)
             last = len(self.rows) - 1
             if r != last:
-                for name in _ROW_BUFFERS:
+                for name in self.row_buffers:
                     buf = getattr(e, name)
                     buf[r] = buf[last]
                 self.rows[r] = self.rows[last]
             self.rows.pop()
             self._reset_row(last)
             del self.requests[rid]
+            self._left_batch(rid)
             if rid not in self.preempted:
                 self.model_intermediate_buffer.pop(rid, None)                # gpu_model_runner.py:259
         # new requests (a preempted request re-enters here with fresh blocks and num_computed_tokens = 0)
@@ -302,71 +305,9 @@ class MI355XARModelRunner:
             if len(self.rows) >= self.max_num_seqs:
                 raise RuntimeError(f"batch overflow: max_num_seqs={self.max_num_seqs}")
             if nr.req_id in self.preempted:
-                self._resume(nr.req_id, list(nr.block_ids[0]), int(nr.num_computed_tokens))
+                self._resume(nr.req_id, list(nr.block_ids[0]), int(nr.num_computed_tokens), nr)
                 continue
-            info = decode_additional_information(nr.additional_information)
-            pe = nr.prompt_embeds if nr.prompt_embeds is not None else info.get("talker_prompt_embeds")
-            tail = info.get("tailing_text_hidden")
-            pad = info.get("tts_pad_embed")
-            if pe is None and info.get("thinker_prefill_embeddings") is not None:
-                if self.prompt_builder is None:
-                    raise ValueError(f"request {nr.req_id}: thinker outputs given but the runner has no prompt_builder")
-                prompt, upd = self.prompt_builder.from_info(info)     # qwen3_omni.py:678-809
-                pe, tail, pad = prompt.embeds, upd.get("trailing_text_hidden"), prompt.tts_pad
-                info.update(upd)      # (merged into model_intermediate_buffer below, once the request is admitted)
-            elif pe is None and getattr(self.prompt_builder, "from_info", None) is not None and (info.get("text") or info.get("input_ids") is not None):
-                # Qwen3-TTS request (text / task_type / speaker / voice_clone_prompt): _build_prompt_embeds on the device
-                # (prompt_builder_tts.TTSTalkerPromptBuilder = qwen3_tts_talker.py:1211-1567)
-                tp = self.prompt_builder.from_info(info)
-                pe, tail, pad = tp.embeds, tp.trailing_text_hidden, tp.tts_pad
-                if tp.ref_code is not None:
-                    info.update({"ref_code": tp.ref_code, "ref_code_len": tp.ref_code_len})
-            if pe is None or pe.ndim != 2 or pe.shape[1] != self.d.hidden:
-                raise ValueError(f"request {nr.req_id}: missing talker_prompt_embeds [T,{self.d.hidden}]")
-            dev = e.input_ids.device
-            if pad is None:
-                raise ValueError(f"request {nr.req_id}: missing tts_pad_embed (prefill must initialise it)")
-            row_sampling = self._row_sampling(nr.req_id, nr.sampling_params or self.default_sampling)   # validated BEFORE any state changes
-            st = RequestState(req_id=nr.req_id, prompt_embeds=pe.to(BF16).cpu().contiguous(),
-                              block_ids=list(nr.block_ids[0]), sampling=nr.sampling_params or self.default_sampling,
-                              num_computed=int(nr.num_computed_tokens),
-                              tail=None if tail is None else self._up(tail, BF16).reshape(-1, self.d.hidden),
-                              tts_pad=self._up(pad, BF16).reshape(-1), info=info)
-            mp = getattr(nr, "mrope_positions", None)
-            mp = info.get("mrope_positions") if mp is None else mp
-            if mp is not None:
-                mp = torch.as_tensor(mp, dtype=torch.int64).reshape(3, -1)
-                md = getattr(nr, "mrope_position_delta", None)
-                md = info.get("mrope_position_delta", 0) if md is None else md
-                md = int(md.item() if isinstance(md, torch.Tensor) else md)
-                if mp.shape[1] != st.prompt_len:
-                    raise ValueError(f"request {nr.req_id}: mrope_positions cover {mp.shape[1]} tokens, the prompt has {st.prompt_len}")
-                # every rotary id of the request's life must be a row of the cos / sin table (max_model_len rows): the prompt's
-                # ids as given (video temporal ids run ahead of the token count), then index + delta up to the last token it may
-                # emit (an id outside the table read device memory out of bounds)
-                rows = int(getattr(e, "rope_rows", 0) or self.d.max_model_len)
-                # last sequence index the request can reach: the scheduler stops it at max_model_len whatever max_tokens says
-                # (max_tokens None / 0 = vLLM's "no cap": the bound is then max_model_len itself)
-                mt = int(getattr(st.sampling, "max_tokens", 0) or 0)
-                end = (min(st.prompt_len + mt, int(self.d.max_model_len)) if mt > 0 else int(self.d.max_model_len)) - 1
-                lo = min([st.prompt_len + md, end + md] + ([int(mp.min())] if mp.numel() else []))
-                hi = max([st.prompt_len + md, end + md] + ([int(mp.max())] if mp.numel() else []))
-                if lo < 0 or hi >= rows:
-                    raise ValueError(f"request {nr.req_id}: M-RoPE ids {lo}..{hi} (prompt ids, then index + delta {md} up to sequence index {end}) "
-                                     f"leave the rotary table [0, {rows})")
-                if getattr(e, "rope_delta", None) is None and not (torch.equal(mp[0], mp[1]) and torch.equal(mp[0], mp[2]) and md == 0
-                                                                   and torch.equal(mp[0], torch.arange(mp.shape[1]))):
-                    raise ValueError(f"request {nr.req_id}: M-RoPE ids with differing rows, but the model has no mrope_section")
-                if getattr(e, "rope_delta", None) is not None:
-                    st.mrope_positions, st.mrope_delta = mp, md
-            self.requests[nr.req_id] = st
-            # per-request model state the stage hooks read and extend (gpu_model_runner.py:60,371,935): same dict as st.info
-            self.model_intermediate_buffer[nr.req_id] = st.info
-            r = len(self.rows)
-            self.rows.append(nr.req_id)
-            self._reset_row(r)
-            e.set_row_sampling(r, **row_sampling)
-            e.block_table[r, :len(st.block_ids)] = self._up(st.block_ids, torch.int32)
+            self._admit(nr)
         # cached requests: new blocks (block_table.append_row, gpu_model_runner.py:489); vLLM's own scheduler brings a
         # preempted request back HERE, flagged resumed_from_preemption, with its complete new block list (:470-489)
         c = so.scheduled_cached_reqs
@@ -378,6 +319,8 @@ class MI355XARModelRunner:
                 self._resume(rid, list(nb[0]) if nb else [], int(c.num_computed_tokens[i]) if i < len(c.num_computed_tokens) else 0)
                 continue
             st = self.requests[rid]
+            if i < len(c.new_token_ids) and c.new_token_ids[i]:
+                self._fed(st, c.new_token_ids[i])
             nb = c.new_block_ids[i] if i < len(c.new_block_ids) else None
             if nb:
                 new = list(nb[0])
@@ -391,6 +334,81 @@ class MI355XARModelRunner:
             # until the step in flight had drained: profiles/r05_pinned_read_probe.txt)
             t = self._h2d("bt_upd", np.asarray([upd_at, upd_val], np.int64), torch.int64)
             e.block_table.view(-1).index_put_((t[0],), t[1].to(torch.int32))
+
+    def _fed(self, st, token_ids: list[int]) -> None:
+        """Hook: more prompt tokens of a request whose prompt is open."""
+        raise ValueError(f"request {st.req_id}: prompts arrive whole on this path")
+
+    def _left_batch(self, rid: str) -> None:
+        """Hook: a request gave its row up (finished or preempted)."""
+
+    def _admit(self, nr) -> None:
+        """A new request into the next free row: its prompt (embeddings, or what the prompt builder makes of the request), sampling parameters
+        and blocks."""
+        e = self.engine
+        info = decode_additional_information(nr.additional_information)
+        pe = nr.prompt_embeds if nr.prompt_embeds is not None else info.get("talker_prompt_embeds")
+        tail = info.get("tailing_text_hidden")
+        pad = info.get("tts_pad_embed")
+        if pe is None and info.get("thinker_prefill_embeddings") is not None:
+            if self.prompt_builder is None:
+                raise ValueError(f"request {nr.req_id}: thinker outputs given but the runner has no prompt_builder")
+            prompt, upd = self.prompt_builder.from_info(info)     # qwen3_omni.py:678-809
+            pe, tail, pad = prompt.embeds, upd.get("trailing_text_hidden"), prompt.tts_pad
+            info.update(upd)      # (merged into model_intermediate_buffer below, once the request is admitted)
+        elif pe is None and getattr(self.prompt_builder, "from_info", None) is not None and (info.get("text") or info.get("input_ids") is not None):
+            # Qwen3-TTS request (text / task_type / speaker / voice_clone_prompt): _build_prompt_embeds on the device
+            # (prompt_builder_tts.TTSTalkerPromptBuilder = qwen3_tts_talker.py:1211-1567)
+            tp = self.prompt_builder.from_info(info)
+            pe, tail, pad = tp.embeds, tp.trailing_text_hidden, tp.tts_pad
+            if tp.ref_code is not None:
+                info.update({"ref_code": tp.ref_code, "ref_code_len": tp.ref_code_len})
+        if pe is None or pe.ndim != 2 or pe.shape[1] != self.d.hidden:
+            raise ValueError(f"request {nr.req_id}: missing talker_prompt_embeds [T,{self.d.hidden}]")
+        dev = e.input_ids.device
+        if pad is None:
+            raise ValueError(f"request {nr.req_id}: missing tts_pad_embed (prefill must initialise it)")
+        row_sampling = self._row_sampling(nr.req_id, nr.sampling_params or self.default_sampling)   # validated BEFORE any state changes
+        st = RequestState(req_id=nr.req_id, prompt_embeds=pe.to(BF16).cpu().contiguous(),
+                          block_ids=list(nr.block_ids[0]), sampling=nr.sampling_params or self.default_sampling,
+                          num_computed=int(nr.num_computed_tokens),
+                          tail=None if tail is None else self._up(tail, BF16).reshape(-1, self.d.hidden),
+                          tts_pad=self._up(pad, BF16).reshape(-1), info=info)
+        mp = getattr(nr, "mrope_positions", None)
+        mp = info.get("mrope_positions") if mp is None else mp
+        if mp is not None:
+            mp = torch.as_tensor(mp, dtype=torch.int64).reshape(3, -1)
+            md = getattr(nr, "mrope_position_delta", None)
+            md = info.get("mrope_position_delta", 0) if md is None else md
+            md = int(md.item() if isinstance(md, torch.Tensor) else md)
+            if mp.shape[1] != st.prompt_len:
+                raise ValueError(f"request {nr.req_id}: mrope_positions cover {mp.shape[1]} tokens, the prompt has {st.prompt_len}")
+            # every rotary id of the request's life must be a row of the cos / sin table (max_model_len rows): the prompt's
+            # ids as given (video temporal ids run ahead of the token count), then index + delta up to the last token it may
+            # emit (ADVICE r3: an id outside the table read device memory out of bounds)
+            rows = int(getattr(e, "rope_rows", 0) or self.d.max_model_len)
+            # last sequence index the request can reach: the scheduler stops it at max_model_len whatever max_tokens says
+            # (max_tokens None / 0 = vLLM's "no cap": the bound is then max_model_len itself -- ADVICE r4)
+            mt = int(getattr(st.sampling, "max_tokens", 0) or 0)
+            end = (min(st.prompt_len + mt, int(self.d.max_model_len)) if mt > 0 else int(self.d.max_model_len)) - 1
+            lo = min([st.prompt_len + md, end + md] + ([int(mp.min())] if mp.numel() else []))
+            hi = max([st.prompt_len + md, end + md] + ([int(mp.max())] if mp.numel() else []))
+            if lo < 0 or hi >= rows:
+                raise ValueError(f"request {nr.req_id}: M-RoPE ids {lo}..{hi} (prompt ids, then index + delta {md} up to sequence index {end}) "
+                                 f"leave the rotary table [0, {rows})")
+            if getattr(e, "rope_delta", None) is None and not (torch.equal(mp[0], mp[1]) and torch.equal(mp[0], mp[2]) and md == 0
+                                                               and torch.equal(mp[0], torch.arange(mp.shape[1]))):
+                raise ValueError(f"request {nr.req_id}: M-RoPE ids with differing rows, but the model has no mrope_section")
+            if getattr(e, "rope_delta", None) is not None:
+                st.mrope_positions, st.mrope_delta = mp, md
+        self.requests[nr.req_id] = st
+        # per-request model state the stage hooks read and extend (gpu_model_runner.py:60,371,935): same dict as st.info
+        self.model_intermediate_buffer[nr.req_id] = st.info
+        r = len(self.rows)
+        self.rows.append(nr.req_id)
+        self._reset_row(r)
+        e.set_row_sampling(r, **row_sampling)
+        e.block_table[r, :len(st.block_ids)] = self._up(st.block_ids, torch.int32)
 
     def _update_intermediate_buffer(self, req_id: str, upd: dict) -> None:
         """Merge a per-request update into ``model_intermediate_buffer`` (V/worker/gpu_model_runner.py:1330-1353, known answers
@@ -450,7 +468,7 @@ class MI355XARModelRunner:
         text = torch.stack([st.tail[j] if j < nt else st.tts_pad for j in range(J)])
         return (acc.to(BF16).float() + text.float()).to(BF16)
 
-    def _resume(self, rid: str, block_ids: list[int], num_computed: int) -> None:
+    def _resume(self, rid: str, block_ids: list[int], num_computed: int, nr=None) -> None:
         """A preempted request comes back: new blocks, KV gone.  Its prefill now covers the prompt AND the inputs of the
         L - 1 decode steps behind its L emitted tokens; when that completes nothing is sampled -- the row continues as a
         decode row with input_ids = its last token, h = the hidden state of the last recomputed position, and its

@@ -1,4 +1,4 @@
-"""Minimal KV block pool with the allocation order the path depends on.
+"""Minimal KV block pool with the allocation order the path depends on, and the state slots of sequences in the batch.
 
 The reference delegates block allocation to vLLM's ``KVCacheManager`` / ``BlockPool`` (third
 party, SURVEY Appendix A "Block allocation order"): free list = queue initialised in id order;
@@ -46,6 +46,27 @@ class BlockPool:
 
     def block_ids(self, req_id: str) -> list[int]:
         return list(self.owned.get(req_id, []))
+
+
+class SlotPool:
+    """State slots of the sequences in the batch (recurrent or shifted state: a fixed size per sequence, whatever its length).  Slot 0 belongs
+    to no sequence -- padded batch rows point at it, as their block tables point at the null block.  A slot's old contents are never read: a
+    sequence's first token starts from zeros by its position."""
+
+    def __init__(self, num_slots: int):
+        self.free = deque(range(1, num_slots + 1))
+        self.owned: dict[str, int] = {}
+
+    def acquire(self, req_id: str) -> int:
+        if not self.free:
+            raise MemoryError("no state slot free")
+        self.owned[req_id] = s = self.free.popleft()
+        return s
+
+    def release(self, req_id: str) -> None:
+        s = self.owned.pop(req_id, None)
+        if s is not None:
+            self.free.append(s)
 
 
 def slot_of(block_ids, pos: int, block_size: int) -> int:

@@ -71,6 +71,10 @@ class Request:
     # async scheduling (vLLM Request.num_output_placeholders): tokens this request has been scheduled to sample whose ids the
     # scheduler has not seen yet -- the step that samples them is still in flight while the next one is scheduled
     num_output_placeholders: int = 0
+    # a prompt that arrives in pieces (``MI355XARScheduler.feed``): nothing is sampled for it
+    open_prompt: bool = False
+    fed: list[int] = field(default_factory=list)             # pieces the runner has not been given yet
+    logits_at: set[int] = field(default_factory=set)         # sequence positions whose logits are asked for
 
     def __post_init__(self):
         if self.external_req_id is None:
@@ -131,11 +135,24 @@ class MI355XARScheduler:
     def add_request(self, request: Request) -> None:
         if request.request_id in self.requests:
             raise ValueError(f"duplicate request id {request.request_id}")
-        if request.num_prompt_tokens <= 0 or request.num_prompt_tokens >= self.max_model_len:
+        if request.num_prompt_tokens <= 0 or request.num_prompt_tokens >= self.max_model_len + request.open_prompt:
             raise ValueError(f"request {request.request_id}: prompt of {request.num_prompt_tokens} tokens outside (0, max_model_len)")
         self.requests[request.request_id] = request
         request.status = RequestStatus.WAITING
         self.waiting.append(request)
+
+    def feed(self, request_id: str, token_ids: list[int], logits_at=()) -> None:
+        """More prompt tokens for a request whose prompt is open (it keeps its blocks and its state between the pieces); logits_at: places
+        among these tokens whose logits its steps return."""
+        req = self.requests[request_id]
+        if not req.open_prompt:
+            raise ValueError(f"request {request_id}: its prompt is closed")
+        if req.num_prompt_tokens + len(token_ids) > self.max_model_len:
+            raise ValueError(f"request {request_id}: {req.num_prompt_tokens} + {len(token_ids)} tokens pass max_model_len")
+        req.logits_at.update(req.num_prompt_tokens + int(k) for k in logits_at)
+        req.prompt_token_ids.extend(int(t) for t in token_ids)
+        req.fed.extend(int(t) for t in token_ids)
+        req.num_prompt_tokens += len(token_ids)
 
     def abort_request(self, request_id: str) -> None:
         req = self.requests.get(request_id)
@@ -204,7 +221,8 @@ class MI355XARScheduler:
                 continue                            # (id test: `req not in self.running` compared whole dataclasses, 0.6 ms / step at 64)
             cached.req_ids.append(req.request_id)
             cached.resumed_from_preemption.append(False)
-            cached.new_token_ids.append([])
+            cached.new_token_ids.append(req.fed)
+            req.fed = []
             cached.new_block_ids.append((new_blocks,) if new_blocks else None)
             cached.num_computed_tokens.append(req.num_computed_tokens)
             num_sched[req.request_id] = n
@@ -232,8 +250,10 @@ class MI355XARScheduler:
             resumed = req.status == RequestStatus.PREEMPTED
             req.status = RequestStatus.RUNNING
             self.running.append(req)
+            req.fed = []
             new_reqs.append(OmniNewRequestData(
-                req_id=req.request_id, external_req_id=req.external_req_id, prompt_token_ids=req.prompt_token_ids,
+                req_id=req.request_id, external_req_id=req.external_req_id, open_prompt=req.open_prompt,
+                prompt_token_ids=None if req.prompt_token_ids is None else list(req.prompt_token_ids),
                 sampling_params=req.sampling_params, block_ids=(self.pool.block_ids(req.request_id),),
                 num_computed_tokens=req.num_computed_tokens, prompt_embeds=req.prompt_embeds,
                 additional_information=req.additional_information))
@@ -241,15 +261,20 @@ class MI355XARScheduler:
             num_sched[req.request_id] = n
             budget -= n
         # vLLM advances num_computed_tokens at schedule time (_update_after_schedule)
+        logits_at: dict[str, list[int]] = {}
         for rid, n in num_sched.items():
             req = self.requests[rid]
+            if req.logits_at:
+                at = sorted(p for p in req.logits_at if req.num_computed_tokens <= p < req.num_computed_tokens + n)
+                if at:
+                    logits_at[rid] = [p - req.num_computed_tokens for p in at]
             req.num_computed_tokens += n
-            if self.async_scheduling and req.num_computed_tokens == req.num_tokens + req.num_output_placeholders:
+            if self.async_scheduling and not req.open_prompt and req.num_computed_tokens == req.num_tokens + req.num_output_placeholders:
                 req.num_output_placeholders += 1         # this step samples a token for it (AsyncScheduler._update_after_schedule)
         out = OmniSchedulerOutput(
             scheduled_new_reqs=new_reqs, scheduled_cached_reqs=cached, num_scheduled_tokens=num_sched,
             total_num_scheduled_tokens=sum(num_sched.values()), finished_req_ids=self.finished_req_ids,
-            preempted_req_ids=set(self._preempted),
+            preempted_req_ids=set(self._preempted), logits_at=logits_at,
             finished_requests_needing_kv_transfer=self.get_finished_requests_needing_kv_transfer())
         self.finished_req_ids = set()
         return out

@@ -105,6 +105,38 @@ def peak_predictor_heads(d: TalkerDims, w: dict[str, torch.Tensor], gamma: float
     return out
 
 
+def make_decoder_weights(d, seed: int = 1234, device: str = "cpu") -> dict[str, torch.Tensor]:
+    """Random weights of a decoder-only model (decoder_config.DecoderDims) under its checkpoint's names: every product keeps its input's scale."""
+    from .decoder_config import tensor_shapes
+    g = torch.Generator(device=device).manual_seed(seed)
+    w: dict[str, torch.Tensor] = {}
+    for name, shape in tensor_shapes(d).items():
+        leaf = name.rsplit(".", 1)[-1]
+        if leaf in ("norm", "norm1", "norm2"):
+            t = 1.0 + 0.1 * torch.randn(shape, generator=g, device=device)
+        elif leaf == "shift":
+            t = torch.rand(shape, generator=g, device=device)
+        elif leaf == "act":
+            t = torch.randn(shape, generator=g, device=device)
+        elif leaf == "embed":
+            t = torch.randn(shape, generator=g, device=device)
+        else:
+            t = torch.randn(shape, generator=g, device=device) / shape[-1] ** 0.5
+        w[name] = t.to(torch.bfloat16)
+    return w
+
+
+def decoder_weight_bytes(d) -> int:
+    """Matrix bytes a decode step of a decoder-only model streams (bf16): every layer RUN once -- borrowed weights are read again -- and the head."""
+    from .decoder_config import tensor_shapes
+    n = d.vocab * d.hidden
+    shapes = tensor_shapes(d)
+    for i in range(d.num_layers):
+        p = f"l{d.owner(i)}."
+        n += sum(s[0] * s[1] for k, s in shapes.items() if k.startswith(p) and len(s) == 2)
+    return 2 * n
+
+
 def weight_bytes(d: TalkerDims) -> dict[str, int]:
     """Algorithmic weight bytes read once per talker step."""
     if d.moe_experts > 0:      # every expert counted once (T * k = 512 assignments over 128 experts hit ~98 % of them) + shared + router

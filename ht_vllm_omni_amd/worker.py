@@ -20,52 +20,54 @@ from typing import Any
 
 import torch
 
+from . import models
 from .config import TalkerDims, get_dims
 from .connectors import OmniConnectorFactory, OmniKVTransferManager
-from .weights import make_weights, weight_bytes
+from .decoder_config import DecoderDims
 
 logger = logging.getLogger("ht_vllm_omni_amd.worker")
 
 
-def make_config(model: str | TalkerDims = "tts-1.7b", *, kv_cache_dtype: str = "fp8", block_size: int = 16,
+def make_config(model: str | TalkerDims | DecoderDims = "tts-1.7b", *, kv_cache_dtype: str | None = None, block_size: int = 16,
                 max_num_seqs: int = 64, tensor_parallel_size: int = 1, gpu_memory_utilization: float = 0.9,
                 num_gpu_blocks_override: int | None = None, weights: dict | None = None, seed: int = 1234,
                 connector: str | None = None, enforce_eager: bool = False, default_sampling_params=None,
                 prompt_builder: dict | None = None, model_path: str | None = None, calculate_kv_scales: bool = False,
-                async_scheduling: bool = False) -> SimpleNamespace:
+                async_scheduling: bool = False, dtype: str = "bfloat16", max_model_len: int = 4096) -> SimpleNamespace:
+    """kv_cache_dtype None: the model family's default (models.ModelEntry).  dtype: "float32" runs a decoder-only model in 32-bit throughout."""
     if model_path and isinstance(model, str) and model == "tts-1.7b" and os.path.exists(os.path.join(model_path, "config.json")):
-        from .checkpoint import dims_from_hf_config
-        model = dims_from_hf_config(os.path.join(model_path, "config.json"))          # dimensions come from the checkpoint
+        model = models.dims_of_model_dir(model_path, max_model_len)          # family and dimensions come from the checkpoint
+    if kv_cache_dtype is None:
+        kv_cache_dtype = (models.entry_for_dims(model) if not isinstance(model, str) else models.entry_for_dims_type(TalkerDims)).kv_cache_dtype
     return SimpleNamespace(model=model, kv_cache_dtype=kv_cache_dtype, block_size=block_size, max_num_seqs=max_num_seqs,
                            tensor_parallel_size=tensor_parallel_size, gpu_memory_utilization=gpu_memory_utilization,
                            num_gpu_blocks_override=num_gpu_blocks_override, weights=weights, seed=seed, connector=connector,
                            enforce_eager=enforce_eager, default_sampling_params=default_sampling_params,
                            prompt_builder=prompt_builder, model_path=model_path, calculate_kv_scales=calculate_kv_scales,
-                           async_scheduling=bool(async_scheduling))
+                           async_scheduling=bool(async_scheduling), dtype=dtype)
 
 
 _PRESET_HINTS = (("omni", "omni-talker"), ("1.7b", "tts-1.7b"), ("0.6b", "tts-0.6b"))
 
 
-def _dims_from_model_config(mc) -> str | TalkerDims:
-    """What the talker stage is, from ``model_config``: a TalkerDims, a preset name, a checkpoint directory (its config.json
+def _dims_from_model_config(mc) -> str | TalkerDims | DecoderDims:
+    """What the stage serves, from ``model_config``: a dimensions object, a preset name, a checkpoint directory (its config.json
     decides, as in the reference: configuration_qwen3_tts.py), an ``hf_config`` carrying ``talker_config``, else the size
     tag in the model id ("Qwen/Qwen3-TTS-1.7B-Base")."""
     from .config import PRESETS
     model = getattr(mc, "model", None)
-    if isinstance(model, TalkerDims):
+    if isinstance(model, (TalkerDims, DecoderDims)):
         return model
     if isinstance(model, str) and model in PRESETS:
         return model
     if isinstance(model, str) and os.path.exists(os.path.join(model, "config.json")):
-        from .checkpoint import dims_from_hf_config
-        return dims_from_hf_config(os.path.join(model, "config.json"), max_model_len=int(getattr(mc, "max_model_len", 4096) or 4096))
+        return models.dims_of_model_dir(model, int(getattr(mc, "max_model_len", 4096) or 4096))
     hf = getattr(mc, "hf_config", None)
     if hf is not None:
         as_dict = hf if isinstance(hf, dict) else (hf.to_dict() if hasattr(hf, "to_dict") else None)
-        if as_dict and ("talker_config" in as_dict or "code_predictor_config" in as_dict):
-            from .checkpoint import dims_from_hf_config
-            return dims_from_hf_config(as_dict, max_model_len=int(getattr(mc, "max_model_len", 4096) or 4096))
+        entry = models.entry_for_config(as_dict) if as_dict else None
+        if entry is not None:
+            return entry.parse(as_dict, int(getattr(mc, "max_model_len", 4096) or 4096))
     low = str(model).lower()
     for tag, preset in _PRESET_HINTS:
         if tag in low:
@@ -97,8 +99,9 @@ def config_from_vllm(vllm_config) -> SimpleNamespace:
     from . import _lib as L
     if cache_dtype not in L.KV_CODES:
         raise ValueError(f"MI355XARWorker: cache_config.cache_dtype={cache_dtype!r} is not one of {sorted(L.KV_CODES)}")
+    dtype = str(getattr(mc, "dtype", "bfloat16") or "bfloat16").replace("torch.", "")
     return SimpleNamespace(
-        model=model, kv_cache_dtype=cache_dtype, block_size=int(getattr(cc, "block_size", 16) or 16),
+        dtype="float32" if dtype == "float32" else "bfloat16", model=model, kv_cache_dtype=cache_dtype, block_size=int(getattr(cc, "block_size", 16) or 16),
         max_num_seqs=int(getattr(sc, "max_num_seqs", 64) or 64),
         tensor_parallel_size=int(getattr(pc, "tensor_parallel_size", 1) or 1),
         gpu_memory_utilization=float(getattr(cc, "gpu_memory_utilization", 0.9) or 0.9),
@@ -137,7 +140,8 @@ class MI355XARWorker:
         self.distributed_init_method = distributed_init_method
         self.is_driver_worker = is_driver_worker
         self.tp_size = int(getattr(vllm_config, "tensor_parallel_size", 1))
-        self.dims: TalkerDims = vllm_config.model if isinstance(vllm_config.model, TalkerDims) else get_dims(vllm_config.model)
+        self.dims = get_dims(vllm_config.model) if isinstance(vllm_config.model, str) else vllm_config.model
+        self.entry = models.entry_for_dims(self.dims)         # the model family: its loader, cache spec, engine and runner
         self.device: torch.device | None = None
         self.model_runner = None
         self.engine = None
@@ -167,10 +171,8 @@ class MI355XARWorker:
         w = getattr(self.vllm_config, "weights", None)
         path = getattr(self.vllm_config, "model_path", None)
         if w is None and path:
-            from .checkpoint import check_against_dims, load_talker_checkpoint
-            w, self.checkpoint_extras = load_talker_checkpoint(path)
-            check_against_dims(w, self.dims)
-        self._weights = w if w is not None else make_weights(self.dims, seed=getattr(self.vllm_config, "seed", 1234))
+            w, self.checkpoint_extras = self.entry.load(path, self.dims)
+        self._weights = w if w is not None else self.entry.random(self.dims, getattr(self.vllm_config, "seed", 1234))
 
     # ---- memory (base.py:78-156): bytes available for the KV cache after weights and step scratch -- MEASURED, per process
     def determine_available_memory(self) -> int:
@@ -216,19 +218,16 @@ class MI355XARWorker:
 
     # ---- KV cache spec (vLLM Worker.get_kv_cache_spec -> {layer name: KVCacheSpec}; the executor sizes the cache from the
     # specs' page sizes and hands the result back as a KVCacheConfig, V/worker/base.py:78-156, gpu_ar_model_runner.py:118-124)
-    def get_kv_cache_spec(self) -> dict[str, "AttentionSpec"]:
-        d, cfg = self.dims, self.vllm_config
-        store = {"bf16": torch.bfloat16, "auto": torch.bfloat16, "fp16": torch.float16, "float16": torch.float16, "half": torch.float16,
-                 "fp8": torch.uint8, "fp8_e4m3": torch.uint8, "int8": torch.int8}[cfg.kv_cache_dtype]
-        hkv = max(d.kv_heads // self.tp_size, 1)
-        spec = AttentionSpec(block_size=int(cfg.block_size), num_kv_heads=hkv, head_size=d.head_dim, dtype=store,
-                             scale_bytes_per_token=2 * hkv * 4 if cfg.kv_cache_dtype == "int8" else 0)
-        return {f"model.layers.{l}.self_attn.attn": spec for l in range(d.layers)}
+    def get_kv_cache_spec(self) -> dict[str, Any]:
+        return self.entry.cache_spec(self.dims, self.vllm_config, self.tp_size)
 
     def kv_bytes_per_block(self) -> int:
         return sum(s.page_size_bytes for s in self.get_kv_cache_spec().values())
 
     def _build_engine(self, num_blocks: int) -> None:
+        self.engine = self.entry.build_engine(self, int(num_blocks))
+
+    def _build_talker_engine(self, num_blocks: int):
         from .engine import TalkerEngine
         cfg = self.vllm_config
         # tensor-parallel ranks: the all-reduce of the step is a kernel of the step (peer-mapped buffers over hipIpc, fused with
@@ -239,20 +238,20 @@ class MI355XARWorker:
             from .tp_comm import setup_peer_allreduce
             self.peer_allreduce = setup_peer_allreduce(self.dims.hidden, min(cfg.max_num_seqs, 64), self.rank, self.tp_size,
                                                        log=logger.info)
-        self.engine = TalkerEngine(self.dims, self._weights, kv_dtype=cfg.kv_cache_dtype, num_blocks=int(num_blocks),
-                                   block_size=cfg.block_size, max_batch=cfg.max_num_seqs, device=str(self.device),
-                                   tp_rank=self.rank, tp_size=self.tp_size, peer_allreduce=self.peer_allreduce,
-                                   calculate_kv_scales=bool(getattr(cfg, "calculate_kv_scales", False)))
+        engine = TalkerEngine(self.dims, self._weights, kv_dtype=cfg.kv_cache_dtype, num_blocks=int(num_blocks),
+                              block_size=cfg.block_size, max_batch=cfg.max_num_seqs, device=str(self.device),
+                              tp_rank=self.rank, tp_size=self.tp_size, peer_allreduce=self.peer_allreduce,
+                              calculate_kv_scales=bool(getattr(cfg, "calculate_kv_scales", False)))
         # ... and the all-reduce INSIDE the backbone's persistent launches only after four scratch steps both ways agreed on every rank
         self.tp_backbone_chain = False
         if self.peer_allreduce is not None:
             from .tp_comm import check_backbone_chain
-            self.tp_backbone_chain = check_backbone_chain(self.engine, log=logger.info)
+            self.tp_backbone_chain = check_backbone_chain(engine, log=logger.info)
         self._embed_table = self._weights["embed"]
         self._weights = None
+        return engine
 
     def initialize_from_config(self, kv_cache_config: Any = None) -> None:
-        from .runner import MI355XARModelRunner
         cfg = self.vllm_config
         # a KVCacheConfig-shaped object: .num_blocks, or .kv_cache_tensors = [{size, shared_by: [layer names]}] (one per layer in
         # vLLM's default layout): the smallest tensor bounds the block count
@@ -272,6 +271,11 @@ class MI355XARWorker:
             self.engine.resize_kv_cache(int(nb))
         else:
             self._build_engine(int(nb))
+        self.model_runner = self.entry.build_runner(self)
+
+    def _build_talker_runner(self):
+        from .runner import MI355XARModelRunner
+        cfg = self.vllm_config
         embed_table = self._embed_table
         conn = OmniConnectorFactory.create_connector(cfg.connector) if getattr(cfg, "connector", None) else None
         # Qwen3-Omni talker: config.prompt_builder = {"weights": {text, hidden, codec_embed}, "ids": OmniPromptIds | dict}
@@ -282,9 +286,8 @@ class MI355XARWorker:
             pw = dict(pb_cfg["weights"])
             pw.setdefault("codec_embed", embed_table)        # talker.embed_input_ids = the talker's own codec table
             builder = OmniTalkerPromptBuilder(pw, ids, self.device)
-        self.model_runner = MI355XARModelRunner(self.engine, kv_transfer=OmniKVTransferManager(conn),
-                                                use_graphs=not getattr(cfg, "enforce_eager", False), prompt_builder=builder,
-                                                async_scheduling=bool(getattr(cfg, "async_scheduling", False)))
+        return MI355XARModelRunner(self.engine, kv_transfer=OmniKVTransferManager(conn), use_graphs=not getattr(cfg, "enforce_eager", False),
+                                   prompt_builder=builder, async_scheduling=bool(getattr(cfg, "async_scheduling", False)))
 
     def compile_or_warm_up_model(self) -> None:
         # sampling parameters are per-request device rows read inside the captured step (a request without any gets the

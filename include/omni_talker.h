@@ -52,9 +52,11 @@ extern "C" {
 #define OMNI_EPI_SILU_MUL_GU8 5 /* as SILU_MUL for a fragment-major W whose rows were interleaved first: rows 16t..16t+7 =
                                  * gate[8t..8t+7], rows 16t+8..16t+15 = up[8t..8t+7] -- one 16-row MFMA tile then yields 8
                                  * finished act columns, so any number of tiles per workgroup divides the chip evenly */
+#define OMNI_EPI_XIELU 6       /* omni_gemm_xielu only (omni_decoder.h): out bf16 = xielu(acc) */
 
 const char* omni_last_error(void);
-int omni_abi_version(void);   /* 5 (round 6: omni_ar_peers.tile_flags, omni_talker_set_chains modes 2 / 3, a zero-filled attention workspace) */
+int omni_abi_version(void);   /* 6: omni_tile_gemm column groups and the xIELU activation (5: omni_ar_peers.tile_flags, omni_talker_set_chains
+                                 modes 2 / 3, a zero-filled attention workspace) */
 
 /* ------------------------------------------------------------------ per-op entry points */
 
@@ -147,7 +149,7 @@ int omni_moe_experts_resid(const void* x, const int32_t* topk_idx, const void* t
  *            K = k * C_in, seg_len = C_in, seg_rows = d, row_off = -(k - 1) * d.
  *   w        bf16 [N, K] fragment-major (OMNI_LAYOUT_W_FRAG); N % 16 == 0, K % 32 == 0, seg_len % 32 == 0.
  *   bias / scale  fp32 [N] or NULL.  y = act(acc + bias) * scale (+ resid), all fp32.
- *   act      OMNI_TILE_ACT_NONE | _GELU (erf) | _SILU_MUL_GU8 (w rows interleaved as OMNI_EPI_SILU_MUL_GU8; out is [M, N / 2],
+ *   act      OMNI_TILE_ACT_NONE | _GELU (erf) | _XIELU (act_p, act_n) | _SILU_MUL_GU8 (w rows interleaved as OMNI_EPI_SILU_MUL_GU8; out is [M, N / 2],
  *            = bf16(bf16(SiLU(bf16 gate)) * bf16 up), omni_silu_mul's rounding points; no other output).
  *   resid    fp32 [M, ldr] or NULL (may alias out_f32: the residual stream updated in place).
  *   out_f32  fp32 [M, ldf] or NULL: y.   out  bf16 [M, ldo] or NULL: bf16(y).
@@ -156,6 +158,7 @@ int omni_moe_experts_resid(const void* x, const int32_t* topk_idx, const void* t
 #define OMNI_TILE_ACT_NONE 0
 #define OMNI_TILE_ACT_GELU 1
 #define OMNI_TILE_ACT_SILU_MUL_GU8 2
+#define OMNI_TILE_ACT_XIELU 3
 typedef struct omni_tile_gemm {
     const void* x; int64_t x_rows; int ldx;
     int seg_len, seg_rows, row_off;
@@ -175,6 +178,9 @@ typedef struct omni_tile_gemm {
      * V/model_executor/models/qwen3_omni/qwen3_moe.py:8,152-161).  group_rows (device int32 [groups], or NULL = M each) is the
      * live row count per group: rows past it read as zero and are not written, whole tiles past it are skipped. */
     int groups; int64_t x_group_rows, w_group_elems, out_group_rows; const int32_t* group_rows;
+    float act_p, act_n;                          /* OMNI_TILE_ACT_XIELU: coefficients of the two branches */
+    int64_t x_group_cols, out_group_cols;        /* groups > 1: column offset of group g in x / out / out_f32 (elements): per-head products of
+                                                    one [tokens, heads * K] array with x_group_rows = out_group_rows = 0 */
 } omni_tile_gemm;
 int omni_gemm_tile(const omni_tile_gemm* g, void* stream);
 
