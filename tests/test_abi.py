@@ -51,6 +51,25 @@ def test_struct_layout_matches_c(tmp_path):
     assert got[7] == _lib.ArPeers.tile_flags.offset
 
 
+def test_decoder_library_symbols_and_struct_layouts(tmp_path):
+    """include/omni_decoder.h: every function it declares is exported by libomni_decoder.so and bound; the ctypes structs have the C layout."""
+    from ht_vllm_omni_amd import _lib
+    hdr = os.path.join(ROOT, "include", "omni_decoder.h")
+    names = set(re.findall(r"\b(omni_[a-z0-9_]+)\s*\(", re.sub(r"/\*.*?\*/", "", open(hdr).read(), flags=re.S)))
+    assert len(names) >= 9
+    lib = _lib.load_decoder()
+    for n in names | {"omni_gemm_tile", "omni_sample_rows", "omni_last_error"}:
+        assert hasattr(lib, n) and n in _lib.DECODER_SIGNATURES, n
+    pairs = [("omni_stream_rows", _lib.StreamRows), ("omni_latent_write", _lib.LatentWrite), ("omni_latent_attn", _lib.LatentAttn), ("omni_tile_gemm", _lib.TileGemm)]
+    exprs = [f"sizeof({c})" for c, _ in pairs] + [f"offsetof({c},{f[0]})" for c, t in pairs for f in t._fields_]
+    want = [C.sizeof(t) for _, t in pairs] + [getattr(t, f[0]).offset for _, t in pairs for f in t._fields_]
+    src = tmp_path / "sz.c"
+    src.write_text('#include <stdio.h>\n#include <stddef.h>\n#include "%s"\nint main(){%s return 0;}\n' % (hdr, "".join(f'printf("%zu\\n",{e});' for e in exprs)))
+    exe = tmp_path / "sz"
+    subprocess.check_call(["gcc", str(src), "-o", str(exe)])
+    assert [int(x) for x in subprocess.check_output([str(exe)]).split()] == want
+
+
 def test_argument_errors_do_not_abort():
     """Bad arguments come back as error codes + message (host-side checks run before any launch)."""
     from ht_vllm_omni_amd import _lib
