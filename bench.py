@@ -13,6 +13,10 @@ N > 1 without WORLD_SIZE in the environment: this process (which has made no GPU
 the child's code; under torchrun (WORLD_SIZE set) each rank runs the tensor-parallel step over RCCL (strong scaling).
 The timed window is centred on the BASELINE context (mean ctx 352) whatever --steps is: untimed decode steps advance
 the batch there first, over KV the steps themselves wrote.  Prints ONE JSON line on rank 0.
+
+  python bench.py --decoder [2048|1024|all]
+Another measurement, of its own: prefill and decode throughput of the decoder-only design (Zefedra-shaped layers, random weights) beside the
+talker's backbone at equal width, depth and matrix bytes.  The default workload is not run.
 """
 from __future__ import annotations
 
@@ -246,6 +250,110 @@ def copy_probe_gbs():
     return 2 * n * 10 / (e0.elapsed_time(e1) * 1e-3) / 1e9
 
 
+# Zefedra-shaped models beside the talker backbone of the same width and depth; q / kv ranks and ff chosen for equal matrix bytes per layer
+DECODER_SIZES = {
+    "2048": dict(talker="tts-1.7b", width=2048, heads=16, dim=128, vdim=128, kv_rank=512, q_rank=1536, ff=9216),
+    "1024": dict(talker="tts-0.6b", width=1024, heads=16, dim=128, vdim=128, kv_rank=256, q_rank=768, ff=4608),
+}
+
+
+def graph_ms(fn, n=24, warm=3):
+    """ms per replay of fn() captured as one hipGraph."""
+    fn()
+    torch.cuda.synchronize()
+    g = torch.cuda.CUDAGraph()
+    with torch.cuda.graph(g):
+        fn()
+    return eager_ms(g.replay, n, warm)
+
+
+def eager_ms(fn, n=5, warm=2):
+    for _ in range(warm):
+        fn()
+    e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+    torch.cuda.synchronize()
+    e0.record()
+    for _ in range(n):
+        fn()
+    e1.record()
+    torch.cuda.synchronize()
+    return e0.elapsed_time(e1) / n
+
+
+def decoder_bench(args):
+    """Decode (a captured step, rows x context) and prefill (one forward over whole prompts) of both models of a size, on one GPU."""
+    from ht_vllm_omni_amd.config import get_dims
+    from ht_vllm_omni_amd.decoder_config import DecoderDims, DenseMLPSpec, LatentAttentionSpec, LayerSpec
+    from ht_vllm_omni_amd.decoder_engine import DecoderEngine
+    from ht_vllm_omni_amd.engine import TalkerEngine
+    from ht_vllm_omni_amd.weights import make_decoder_weights, make_weights, weight_bytes
+    decode_points = [(64, 352), (64, 2048), (8, 2048), (1, 2048)]
+    prefill_points = [(16, 128), (1, 2048), (4, 2048), (1, 8192)]
+    maxlen, block = 8448, 16
+    res = {}
+    for size in (DECODER_SIZES if args.decoder == "all" else (args.decoder,)):
+        z, td = DECODER_SIZES[size], get_dims(DECODER_SIZES[size]["talker"]).with_(max_model_len=maxlen)
+        mix = [LatentAttentionSpec(heads=z["heads"], dim=z["dim"], vdim=z["vdim"], q_rank=z["q_rank"], kv_rank=z["kv_rank"], scale=z["dim"] ** -0.5, out_gate=bool(i % 2))
+               for i in range(td.layers)]
+        dd = DecoderDims("zefedra", z["width"], td.vocab, tuple(LayerSpec(m, DenseMLPSpec(z["ff"])) for m in mix), 1e-6, maxlen)
+        out = {"config": {"zefedra": {k: v for k, v in z.items() if k != "talker"}, "layers": td.layers, "vocab": td.vocab, "talker": z["talker"],
+                          "talker_kv": "bf16", "zefedra_cache": "bf16 latents"}}
+        nblk = 64 * ((2048 + 32) // block) + 2
+        for kind in ("zefedra", "talker"):
+            if kind == "zefedra":
+                eng = DecoderEngine(dd, make_decoder_weights(dd, device="cuda"), num_blocks=nblk, block_size=block, max_batch=64)
+            else:
+                eng = TalkerEngine(td, make_weights(td, seed=1, device="cuda"), kv_dtype="bf16", num_blocks=nblk, block_size=block, max_batch=64, allow_eos=False)
+                eng.set_sampling(greedy=1, cp_greedy=1)
+            bt = torch.zeros(64, eng.bt_stride, dtype=torch.int32)
+            r = {"decode": {}, "prefill": {}}
+            for rows, ctx in decode_points:
+                need = ctx // block + 1
+                for i in range(rows):
+                    bt[i, :need] = torch.arange(1 + i * need, 1 + (i + 1) * need)
+                eng.block_table.copy_(bt)
+                eng.positions.fill_(ctx - 1)
+                eng.seq_lens.fill_(ctx)
+                eng.num_live.fill_(rows)
+                if kind == "zefedra":
+                    ms = graph_ms(lambda: eng.decode_step(rows, advance=False))
+                    by = eng.step_bytes([ctx] * rows)["total"]
+                else:
+                    ms = graph_ms(lambda: eng.backbone_step(rows))
+                    b = eng.step_bytes([ctx] * rows)
+                    by = b["total"] - b["code_predictor"]
+                r["decode"][f"{rows}x{ctx}"] = {"ms": round(ms, 4), "tokens_per_s": round(rows / ms * 1e3, 1), "gb": round(by / 1e9, 3), "hbm_frac": round(by / ms / 1e6 / HBM_PEAK_GBS, 4)}
+                log(size, kind, "decode", rows, ctx, r["decode"][f"{rows}x{ctx}"])
+            for seqs, n in prefill_points:
+                need = (n + block - 1) // block
+                for i in range(seqs):
+                    bt[i, :need] = torch.arange(1 + i * need, 1 + (i + 1) * need)
+                eng.block_table.copy_(bt)
+                T = seqs * n
+                row, pos = torch.arange(seqs).repeat_interleave(n).to(torch.int32), torch.arange(n).repeat(seqs).to(torch.int32)
+                if kind == "zefedra":
+                    b = eng.make_batch(torch.randint(0, dd.vocab, (T,), dtype=torch.int32), row, pos, [n] * seqs)
+                    last = (torch.arange(1, seqs + 1) * n - 1).to(torch.int32).cuda()
+                    ms = eager_ms(lambda: eng.forward(b, sel=last))
+                    per_tok = sum(2 * t.numel() for l in eng.layer_w.values() for t in (l.down.t, l.uq.t, l.uk.t, l.uv.t, l.o.t, l.up.t, l.dn.t))
+                    attn = sum(4 * m.heads * m.kv_rank for m in mix)
+                else:
+                    x = torch.randn(T, td.hidden, device="cuda").to(torch.bfloat16)
+                    slots = (bt[row.long(), pos.long() // block] * block + pos % block).to(torch.int64).cuda()
+                    pd, rd = pos.cuda(), row.cuda()
+                    ms = eager_ms(lambda: eng.prefill_wide(x, pd, rd, slots))
+                    per_tok = weight_bytes(td)["backbone"]
+                    attn = td.layers * 4 * td.q_heads * td.head_dim
+                fl = T * per_tok + seqs * n * (n + 1) // 2 * attn
+                r["prefill"][f"{seqs}x{n}"] = {"ms": round(ms, 3), "tokens_per_s": round(T / ms * 1e3, 1), "tflop": round(fl / 1e12, 3), "tflops": round(fl / ms / 1e9, 1)}
+                log(size, kind, "prefill", seqs, n, r["prefill"][f"{seqs}x{n}"])
+            out[kind] = r
+            del eng
+            torch.cuda.empty_cache()
+        res[size] = out
+    return {"metric": "decoder-only design beside the talker backbone", "unit": "ms / tokens per s", "n_gpus": 1, "dtype": "bf16", "data": "synthetic", "sizes": res}
+
+
 def main():
     # the ONE JSON line owns stdout: native libraries (the RCCL version banner, hipBLASLt notices) write to fd 1 too, so
     # fd 1 is pointed at stderr for the whole run and the JSON goes to the saved descriptor
@@ -288,8 +396,16 @@ def main():
     ap.add_argument("--ctx-extra", type=int, default=0, help="long-context points: start decoding this many positions later")
     ap.add_argument("--target-ctx", type=int, default=352, help="mean context of the timed window (W3: 96 + 256); untimed decode "
                     "steps advance the batch until the window is centred there (0: time from wherever warm-up ends)")
+    ap.add_argument("--decoder", nargs="?", const="all", choices=("all", *DECODER_SIZES), default=None, help="measure the decoder-only design beside the talker "
+                    "backbone instead (prefill and decode throughput at widths 2048 / 1024)")
     ap.add_argument("--master-port", type=int, default=0, help="N > 1 self-launch: rendezvous port (0: pick a free one)")
     args = ap.parse_args()
+
+    if args.decoder:
+        out = decoder_bench(args)
+        sys.stdout.flush()
+        os.write(json_fd, (json.dumps(out) + "\n").encode())
+        return
 
     if args.gpus > 1 and "WORLD_SIZE" not in os.environ:
         # One process per GPU: start the ranks as CHILDREN of this process, which has not touched the GPU (no exec after

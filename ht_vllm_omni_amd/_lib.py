@@ -54,14 +54,14 @@ TILE_ACT_NONE, TILE_ACT_GELU, TILE_ACT_SILU_MUL_GU8, TILE_ACT_XIELU = 0, 1, 2, 3
 
 class StreamRows(C.Structure):
     """omni_stream_rows (include/omni_decoder.h)."""
-    _fields_ = [("ids", vp), ("table", vp), ("vocab", i32), ("x_in", vp), ("y", vp), ("gain", f32), ("eps", f32), ("mu", vp), ("state", vp),
+    _fields_ = [("ids", vp), ("table", vp), ("vocab", i32), ("x_in", vp), ("y", vp), ("y_slabs", i32), ("y_stride", i64), ("gain", f32), ("eps", f32), ("mu", vp), ("state", vp),
                 ("state_slot", vp), ("row_of_tok", vp), ("positions", vp), ("use_final", i32), ("final_gain", f32), ("sel", vp), ("x_out", vp),
                 ("h_out", vp), ("frag", i32), ("rows", i32), ("width", i32), ("wp", i32), ("elem", i32)]
 
 
 class LatentWrite(C.Structure):
     """omni_latent_write."""
-    _fields_ = [("proj", vp), ("ld", i32), ("q_rank", i32), ("qp", i32), ("kv_rank", i32), ("rp", i32), ("heads", i32), ("qw", vp), ("kw", vp),
+    _fields_ = [("proj", vp), ("slabs", i32), ("slab_stride", i64), ("ld", i32), ("q_rank", i32), ("qp", i32), ("kv_rank", i32), ("rp", i32), ("heads", i32), ("qw", vp), ("kw", vp),
                 ("eps", f32), ("cq", vp), ("frag", i32), ("cache", vp), ("gate", vp), ("block_table", vp), ("bt_stride", i32), ("block_size", i32),
                 ("row_of_tok", vp), ("positions", vp), ("num_live", vp), ("x", vp), ("wp", i32), ("state", vp), ("state_slot", vp), ("T", i32),
                 ("elem", i32)]
@@ -75,6 +75,8 @@ class LatentAttn(C.Structure):
 
 
 LATENT_TILE = 128           # OMNI_LATENT_TILE
+STREAM_F32, STREAM_BF16, STREAM_XIELU = 0, 1, 2      # omni_gemm_stream kinds
+STREAM_MAX_SPLITS = 8
 
 
 class ResUnit(C.Structure):
@@ -191,7 +193,7 @@ SIGNATURES = {
 
 # what libomni_decoder.so exports: its own entries and the shared ones (same sources as the talker's)
 DECODER_SIGNATURES = {
-    **{n: SIGNATURES[n] for n in ("omni_last_error", "omni_abi_version", "omni_gemm_bf16_ex", "omni_gemm_tile", "omni_sample", "omni_sample_rows")},
+    **{n: SIGNATURES[n] for n in ("omni_last_error", "omni_abi_version", "omni_gemm_tile", "omni_sample", "omni_sample_rows")},
     "omni_stream_rows_run": (i32, [C.POINTER(StreamRows), vp]),
     "omni_latent_write_run": (i32, [C.POINTER(LatentWrite), vp]),
     "omni_latent_attn_run": (i32, [C.POINTER(LatentAttn), vp]),
@@ -199,7 +201,8 @@ DECODER_SIGNATURES = {
     "omni_latent_attn_mfma": (i32, [i32]),
     "omni_head_gemm": (i32, [vp, vp, vp, i32, i32, i32, i32, i32, vp]),
     "omni_gemm_f32": (i32, [vp, i32, i64, vp, i64, vp, i32, i64, i32, i32, i32, i32, i32, f32, f32, vp]),
-    "omni_gemm_xielu": (i32, [vp, i32, vp, vp, i32, i32, i32, f32, f32, i32, vp]),
+    "omni_gemm_stream": (i32, [vp, vp, vp, i32, i32, i32, i32, i32, f32, f32, i32, vp]),
+    "omni_gemm_stream_splits": (i32, [i32, i32, i32]),
     "omni_sample_step": (i32, [vp, i32, i32, i32, C.POINTER(RowSampling), vp, vp, vp, vp, vp, vp, vp]),
 }
 

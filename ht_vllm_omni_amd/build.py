@@ -1,8 +1,8 @@
 """Build the HIP libraries in-tree with hipcc for gfx950 (cross-compiles without a GPU).
 
   libomni_talker.so        the product: HIP kernels + the C-ABI of include/omni_talker.h, policy knobs compiled in
-  libomni_decoder.so       the kernels of the decoder-only language models (include/omni_decoder.h): its own few sources plus the GEMMs and the
-                           sampler both libraries link
+  libomni_decoder.so       the kernels of the decoder-only language models (include/omni_decoder.h): its own few sources plus the large-M GEMM and
+                           the sampler both libraries link
   libomni_talker_debug.so  the talker's sources with -DOMNI_DEBUG_HOOKS (run-time policy knobs, omni_debug_* setters) plus
                            csrc/debug.hip (launch / memory-system probes): scripts/ and the tile-sweep tests only
 
@@ -24,7 +24,7 @@ LIB_DECODER = os.path.join(HERE, "libomni_decoder.so")
 LIB_DEBUG = os.path.join(HERE, "libomni_talker_debug.so")
 SOURCES = ["errors.hip", "capi.hip", "gemm.hip", "gemm_prefill.hip", "norm.hip", "rope_kv.hip", "paged_attn.hip", "prefill_attn.hip", "moe.hip",
            "sampler.hip", "cp_chain.hip", "bb_chain.hip", "moe_chain.hip", "allreduce.hip", "codec.hip", "conv_unit.hip"]
-DECODER_SOURCES = ["errors.hip", "gemm.hip", "gemm_prefill.hip", "sampler.hip", "decoder_rows.hip", "head_gemm.hip", "latent_attn.hip"]
+DECODER_SOURCES = ["errors.hip", "gemm_prefill.hip", "sampler.hip", "decoder_rows.hip", "gemm_stream.hip", "head_gemm.hip", "latent_attn.hip"]
 # debug library only: the probes, and the losing A/B arms of the backbone chain (rounds 3 and 4; no product knob reaches them)
 DEBUG_ONLY = ["debug.hip", "bb_engine.hip", "bb_all.hip"]
 # per-file extra flags

@@ -75,7 +75,15 @@ __global__ __launch_bounds__(DR_THREADS) void stream_rows_kernel(const omni_stre
             y[c][0] = y[c][1] = y[c][2] = y[c][3] = 0.f;
             if (k < wp) {
                 ld4<float>(a.x_in + (size_t)t * wp + k, v[c]);
-                if (a.y) ld4<float>(a.y + (size_t)t * wp + k, y[c]);
+                if (a.y) {
+                    ld4<float>(a.y + (size_t)t * wp + k, y[c]);
+                    for (int s = 1; s < a.y_slabs; ++s) {          // partial sums of the product, in slab order
+                        float z[4];
+                        ld4<float>(a.y + (size_t)s * a.y_stride + (size_t)t * wp + k, z);
+#pragma unroll
+                        for (int e = 0; e < 4; ++e) y[c][e] += z[e];
+                    }
+                }
             }
         }
         if (!a.y) return;
@@ -178,21 +186,29 @@ extern "C" int omni_stream_rows_run(const omni_stream_rows* p, void* stream) {
 // ---- latents: norms, cache write, gates, token-shift state.  One workgroup per token.
 template <typename E>
 __global__ __launch_bounds__(DR_THREADS) void latent_write_kernel(const omni_latent_write a) {
+    extern __shared__ __attribute__((aligned(16))) float sp[];     // the token's projections, partial sums added up
     __shared__ float red[2][DR_WAVES];
     const int t = blockIdx.x;
     const int row = a.row_of_tok[t], pos = a.positions[t];
-    const float* yq = a.proj + (size_t)t * a.ld;
-    const float* yk = yq + a.qp;
+    const bool live = !a.num_live || row < *a.num_live;
+    const int blk = a.block_table[(size_t)row * a.bt_stride + pos / a.block_size];
+    const bool last = a.state && (t == a.T - 1 || a.row_of_tok[t + 1] != row);
+    const int slot = a.state ? a.state_slot[row] : 0;
+    const float* y = a.proj + (size_t)t * a.ld;
     float sq = 0.f, sk = 0.f;
-    for (int k = threadIdx.x * 4; k < a.qp; k += DR_THREADS * 4) {       // padded columns hold zeros
+    for (int k = threadIdx.x * 4; k < a.ld; k += DR_THREADS * 4) {
         float v[4];
-        ld4<float>(yq + k, v);
-        sq += sq4_sum(v[0], v[1], v[2], v[3]);
-    }
-    for (int k = threadIdx.x * 4; k < a.rp; k += DR_THREADS * 4) {
-        float v[4];
-        ld4<float>(yk + k, v);
-        sk += sq4_sum(v[0], v[1], v[2], v[3]);
+        ld4<float>(y + k, v);
+        for (int s = 1; s < a.slabs; ++s) {
+            float z[4];
+            ld4<float>(y + (size_t)s * a.slab_stride + k, z);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] += z[e];
+        }
+        st4<float>(sp + k, v);
+        const float ss = sq4_sum(v[0], v[1], v[2], v[3]);          // (padded columns hold zeros; qp and rp are multiples of 4)
+        if (k < a.qp) sq += ss;
+        else if (k < a.qp + a.rp) sk += ss;
     }
     sq = wave_sum(sq);
     sk = wave_sum(sk);
@@ -206,34 +222,31 @@ __global__ __launch_bounds__(DR_THREADS) void latent_write_kernel(const omni_lat
     const E* qw = reinterpret_cast<const E*>(a.qw);
     for (int k = threadIdx.x * 4; k < a.qp; k += DR_THREADS * 4) {
         float v[4], w[4];
-        ld4<float>(yq + k, v);
+        ld4<float>(sp + k, v);
         ld4<E>(qw + k, w);
 #pragma unroll
         for (int e = 0; e < 4; ++e) v[e] = v[e] * rq * w[e];
         st4<E>(cq + (a.frag ? frag_off(t, k, a.qp) : (size_t)t * a.qp + k), v);
     }
     if (a.gate)
-        for (int h = threadIdx.x; h < a.heads; h += DR_THREADS) a.gate[(size_t)t * a.heads + h] = 1.0f / (1.0f + expf(-yk[a.rp + h]));
-    if (a.num_live && row >= *a.num_live) return;
-    const int blk = a.block_table[(size_t)row * a.bt_stride + pos / a.block_size];
+        for (int h = threadIdx.x; h < a.heads; h += DR_THREADS) a.gate[(size_t)t * a.heads + h] = 1.0f / (1.0f + expf(-sp[a.qp + a.rp + h]));
+    if (!live) return;
     E* dst = reinterpret_cast<E*>(a.cache) + ((size_t)blk * a.block_size + pos % a.block_size) * a.rp;
     const E* kw = reinterpret_cast<const E*>(a.kw);
     for (int k = threadIdx.x * 4; k < a.rp; k += DR_THREADS * 4) {
         float v[4], w[4];
-        ld4<float>(yk + k, v);
+        ld4<float>(sp + a.qp + k, v);
         ld4<E>(kw + k, w);
 #pragma unroll
         for (int e = 0; e < 4; ++e) v[e] = v[e] * rk * w[e];
         st4<E>(dst + k, v);
     }
-    if (a.state && (t == a.T - 1 || a.row_of_tok[t + 1] != row)) {
-        float* s = a.state + (size_t)a.state_slot[row] * a.wp;
+    if (last)
         for (int k = threadIdx.x * 4; k < a.wp; k += DR_THREADS * 4) {
             float v[4];
             ld4<float>(a.x + (size_t)t * a.wp + k, v);
-            st4<float>(s + k, v);
+            st4<float>(a.state + (size_t)slot * a.wp + k, v);
         }
-    }
 }
 
 extern "C" int omni_latent_write_run(const omni_latent_write* p, void* stream) {
@@ -245,9 +258,11 @@ extern "C" int omni_latent_write_run(const omni_latent_write* p, void* stream) {
     OMNI_CHECK_ARG(!a.state || (a.x && a.state_slot && a.wp % 4 == 0), "omni_latent_write: state needs the stream rows and slots");
     OMNI_CHECK_ARG(a.elem == 1 || a.elem == 0, "omni_latent_write: elem=%d", a.elem);
     OMNI_CHECK_ARG(!a.frag || a.elem == 0, "omni_latent_write: fragment-major output is bf16");
+    OMNI_CHECK_ARG(a.ld <= 15 * 1024, "omni_latent_write: ld=%d (<= 15360: a token's projections are staged in LDS)", a.ld);
     if (a.T <= 0) return OMNI_OK;
-    if (a.elem) hipLaunchKernelGGL(latent_write_kernel<float>, dim3(a.T), dim3(DR_THREADS), 0, (hipStream_t)stream, a);
-    else hipLaunchKernelGGL(latent_write_kernel<uint16_t>, dim3(a.T), dim3(DR_THREADS), 0, (hipStream_t)stream, a);
+    const size_t lds = (size_t)a.ld * sizeof(float);
+    if (a.elem) hipLaunchKernelGGL(latent_write_kernel<float>, dim3(a.T), dim3(DR_THREADS), lds, (hipStream_t)stream, a);
+    else hipLaunchKernelGGL(latent_write_kernel<uint16_t>, dim3(a.T), dim3(DR_THREADS), lds, (hipStream_t)stream, a);
     OMNI_CHECK_LAUNCH("omni_latent_write");
     return OMNI_OK;
 }

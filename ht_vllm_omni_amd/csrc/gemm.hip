@@ -44,7 +44,6 @@ struct GemmArgs {
     float mask_fill;           // logit written where mask[n] == 0 (-inf; the Omni talker writes -1e9)
     int counted;               // use the counted (unpredicated, 2-deep) schedule when K % 512 == 0
     const int32_t* num_live;   // PRO_XNORM normed_out: rows >= *num_live are not written (NULL: all M rows)
-    float act_p, act_n;        // EPI_XIELU: the activation's two coefficients (common.cuh xielu)
     int dbg_stage;             // debug library only: leave the kernel after stage N (launch-cost attribution), 0 = run all
 };
 
@@ -377,11 +376,7 @@ __global__ __launch_bounds__(GEMM_THREADS) void gemm_skinny_kernel(const GemmArg
                 float ss = sq4_sum(rv[0], rv[1], rv[2], rv[3]);
                 ss = xor32_sum(xor16_sum(ss));       // the 4 lanes (l & 15) + 16 * {0..3} hold the 16 columns of row m
                 if (l < 16) a.part_out[blockIdx.x * a.pstride + m] = ss;   // slabs [n group][pstride rows]
-            } else if (EPI == OMNI_EPI_BF16 || EPI == OMNI_EPI_XIELU) {
-                if (EPI == OMNI_EPI_XIELU) {
-#pragma unroll
-                    for (int g = 0; g < 4; ++g) v[g] = xielu(v[g], a.act_p, a.act_n);
-                }
+            } else if (EPI == OMNI_EPI_BF16) {
                 *reinterpret_cast<uint2*>(reinterpret_cast<uint16_t*>(a.out) + (a.oshuf ? frag_off(m, n, N) : (size_t)m * N + n)) =
                     make_uint2(pack_bf2(v[0], v[1]), pack_bf2(v[2], v[3]));
             } else {
@@ -511,9 +506,6 @@ static int dispatch_epi(const GemmArgs& a, int epilogue, hipStream_t st) {
         case OMNI_EPI_F32_BF16RND:
             if constexpr (PRO != 3) return dispatch_tile<PRO, OMNI_EPI_F32_BF16RND>(a, st);
             break;
-        case OMNI_EPI_XIELU:
-            if constexpr (PRO == 0) return dispatch_tile<0, OMNI_EPI_XIELU>(a, st);
-            break;
         case OMNI_EPI_RESID:
             if constexpr (PRO == 0) return dispatch_tile<0, OMNI_EPI_RESID>(a, st);
             break;
@@ -544,26 +536,6 @@ int k_gemm_bf16_ex(const void* x, int ldx, const void* w, const void* bias, void
     OMNI_CHECK_ARG(x, "omni_gemm_bf16: null x");
     OMNI_CHECK_ARG(a.xshuf || (ldx >= K && ldx % 8 == 0), "omni_gemm_bf16: ldx=%d (need >= K, multiple of 8)", ldx);
     return dispatch_epi<0>(a, epilogue, (hipStream_t)stream);
-}
-
-// out bf16 = xielu(x . W^T); the ff1 GEMM of a dense feed-forward with that activation
-extern "C" int omni_gemm_xielu(const void* x, int ldx, const void* w, void* out, int M, int N, int K, float act_p, float act_n, int layout,
-                               void* stream) {
-    GemmArgs a{};
-    a.mask_fill = -INFINITY;
-    a.pstride = 64;
-    a.counted = g_gemm_counted;
-    a.wshuf = (layout & OMNI_LAYOUT_W_FRAG) != 0;
-    a.xshuf = (layout & OMNI_LAYOUT_X_FRAG) != 0;
-    a.oshuf = (layout & OMNI_LAYOUT_OUT_FRAG) != 0;
-    a.x = (const uint16_t*)x; a.ldx = ldx; a.W = (const uint16_t*)w; a.out = out;
-    a.M = M; a.N = N; a.K = K; a.act_p = act_p; a.act_n = act_n;
-    const int rc = check_common(a);
-    if (rc != OMNI_OK) return rc;
-    OMNI_CHECK_ARG(x, "omni_gemm_xielu: null x");
-    OMNI_CHECK_ARG(!a.oshuf || N % 32 == 0, "omni_gemm_xielu: fragment-major output needs N %% 32 == 0");
-    OMNI_CHECK_ARG(a.xshuf || (ldx >= K && ldx % 8 == 0), "omni_gemm_xielu: ldx=%d (need >= K, multiple of 8)", ldx);
-    return dispatch_epi<0>(a, OMNI_EPI_XIELU, (hipStream_t)stream);
 }
 
 extern "C" int omni_gemm_bf16_ex(const void* x, int ldx, const void* w, const void* bias, void* out, int M, int N,

@@ -1,0 +1,145 @@
+// Weight-streaming GEMM of the language models' decode step: out[M <= 64, N] = x[M, K] . W[N, K]^T, both operands fragment-major
+// (common.cuh frag_off), every W byte read once.
+//
+// A workgroup owns NT 16-column tiles for all rows and 1 / S of K (grid.y = S); its 8 waves take the k-steps round-robin, P steps of W and x in
+// flight each, and combine through LDS in a fixed order.  What bounds the op at 64 rows is not only W: every workgroup reads all of
+// x for its K range, 64 rows against its 16 NT columns of W, so wide tiles with K split over workgroups move the fewest bytes through L2.  The
+// S partial sums leave as fp32 slabs [S][M][N]; the row kernels that consume them (decoder_rows.hip) add them up in slab order.
+//   out kinds: fp32 slabs (S >= 1) | bf16 row- or fragment-major | the same through xIELU (common.cuh)
+#include "common.cuh"
+#include "gemm_frag.cuh"
+#include "../../include/omni_decoder.h"
+
+#define GS_WAVES 8
+#define GS_THREADS (GS_WAVES * 64)
+enum { GS_F32 = 0, GS_BF16 = 1, GS_XIELU = 2 };
+
+struct StreamArgs {
+    const uint16_t* x; const uint16_t* W; void* out;
+    int M, N, nsteps, split_steps, oshuf;
+    float ap, an;
+};
+
+template <int MT, int NT, int KIND>
+__global__ __launch_bounds__(GS_THREADS) void gemm_stream_kernel(const StreamArgs a) {
+    constexpr int P = MT * NT >= 8 ? 3 : 4;
+    extern __shared__ __attribute__((aligned(16))) f32x4 part[];      // [wave][NT * MT][lane]
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int k0 = blockIdx.y * a.split_steps, nk = min(a.split_steps, a.nsteps - k0);
+    const uint16_t* wp[NT];
+    const uint16_t* xp[MT];
+#pragma unroll
+    for (int j = 0; j < NT; ++j) wp[j] = a.W + ((size_t)(blockIdx.x * NT + j) * a.nsteps + k0 + wave) * 512 + lane * 8;
+#pragma unroll
+    for (int i = 0; i < MT; ++i) xp[i] = a.x + ((size_t)min(i, ((a.M + 15) >> 4) - 1) * a.nsteps + k0 + wave) * 512 + lane * 8;      // row tiles past M: re-read, discarded
+    f32x4 acc[NT][MT];
+#pragma unroll
+    for (int j = 0; j < NT; ++j)
+#pragma unroll
+        for (int i = 0; i < MT; ++i) acc[j][i] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    const int mine = nk > wave ? (nk - wave + GS_WAVES - 1) / GS_WAVES : 0;
+    u32x4 W[P][NT], X[P][MT];
+    auto load = [&](int d, int s) {
+#pragma unroll
+        for (int j = 0; j < NT; ++j) W[d][j] = ld16_nt(wp[j] + (size_t)s * (GS_WAVES * 512));
+#pragma unroll
+        for (int i = 0; i < MT; ++i) X[d][i] = ld16(xp[i] + (size_t)s * (GS_WAVES * 512));
+    };
+    auto mul = [&](int d) {
+#pragma unroll
+        for (int j = 0; j < NT; ++j)
+#pragma unroll
+            for (int i = 0; i < MT; ++i) acc[j][i] = mfma16(W[d][j], X[d][i], acc[j][i]);
+    };
+    int s = 0;
+    if (mine >= P) {                       // whole groups of P steps: no predicated load, each product waits for its own operands only
+#pragma unroll
+        for (int d = 0; d < P; ++d) load(d, d);
+        for (; s + 2 * P <= mine; s += P) {
+#pragma unroll
+            for (int d = 0; d < P; ++d) {
+                mul(d);
+                load(d, s + P + d);
+            }
+        }
+#pragma unroll
+        for (int d = 0; d < P; ++d) mul(d);
+        s += P;
+    }
+    if (s < mine) {                        // fewer than P steps left
+#pragma unroll
+        for (int d = 0; d < P - 1; ++d)
+            if (s + d < mine) load(d, s + d);
+#pragma unroll
+        for (int d = 0; d < P - 1; ++d)
+            if (s + d < mine) mul(d);
+    }
+#pragma unroll
+    for (int j = 0; j < NT; ++j)
+#pragma unroll
+        for (int i = 0; i < MT; ++i) part[(wave * (NT * MT) + j * MT + i) * 64 + lane] = acc[j][i];
+    __syncthreads();
+    for (int it = threadIdx.x; it < NT * MT * 64; it += GS_THREADS) {
+        const int l = it & 63, f = it >> 6, j = f / MT, i = f - j * MT;
+        const int m = i * 16 + (l & 15), n = (blockIdx.x * NT + j) * 16 + 4 * (l >> 4);
+        if (m >= a.M) continue;
+        f32x4 v = part[f * 64 + l];
+#pragma unroll
+        for (int w = 1; w < GS_WAVES; ++w) v += part[(w * (NT * MT) + f) * 64 + l];
+        if (KIND == GS_F32) {
+            *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(a.out) + ((size_t)blockIdx.y * a.M + m) * a.N + n) = v;
+        } else {
+            if (KIND == GS_XIELU) {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) v[e] = xielu(v[e], a.ap, a.an);
+            }
+            uint16_t* d = reinterpret_cast<uint16_t*>(a.out) + (a.oshuf ? frag_off(m, n, a.N) : (size_t)m * a.N + n);
+            *reinterpret_cast<uint2*>(d) = make_uint2(pack_bf2(v[0], v[1]), pack_bf2(v[2], v[3]));
+        }
+    }
+}
+
+// columns per workgroup and K splits: wide tiles at many rows (x is most of the traffic there), then enough splits for about 1.5 workgroups per CU,
+// each wave keeping at least two steps
+static void gs_policy(int M, int N, int nsteps, bool slabs, int* nt, int* splits) {
+    const int tiles = N / 16;
+    *nt = (M > 16 && tiles % 2 == 0 && tiles >= (slabs ? 64 : 512)) ? 2 : 1;
+    *splits = 1;
+    if (!slabs) return;
+    const int groups = tiles / *nt;
+    int s = (384 + groups - 1) / groups, most = nsteps / (2 * GS_WAVES);
+    if (s > most) s = most;
+    if (s > OMNI_STREAM_MAX_SPLITS) s = OMNI_STREAM_MAX_SPLITS;
+    *splits = s < 1 ? 1 : s;
+}
+
+template <int MT, int NT, int KIND>
+static int gs_launch(const StreamArgs& a, int splits, hipStream_t st) {
+    constexpr int LDS = GS_WAVES * NT * MT * 1024;
+    hipLaunchKernelGGL((gemm_stream_kernel<MT, NT, KIND>), dim3(a.N / (16 * NT), splits), dim3(GS_THREADS), LDS, st, a);
+    OMNI_CHECK_LAUNCH("omni_gemm_stream");
+    return OMNI_OK;
+}
+
+extern "C" int omni_gemm_stream_splits(int M, int N, int K) {
+    int nt, s;
+    gs_policy(M, N, K / 32, true, &nt, &s);
+    return s;
+}
+
+extern "C" int omni_gemm_stream(const void* x, const void* w, void* out, int M, int N, int K, int kind, int one, float act_p, float act_n, int out_frag, void* stream) {
+    OMNI_CHECK_ARG(x && w && out, "omni_gemm_stream: null pointer");
+    OMNI_CHECK_ARG(M >= 1 && M <= 64 && N > 0 && N % 16 == 0 && K > 0 && K % 32 == 0, "omni_gemm_stream: M=%d (<= 64) N=%d (%% 16) K=%d (%% 32)", M, N, K);
+    OMNI_CHECK_ARG(kind >= GS_F32 && kind <= GS_XIELU && (!out_frag || (kind != GS_F32 && N % 32 == 0)), "omni_gemm_stream: kind=%d out_frag=%d", kind, out_frag);
+    StreamArgs a{(const uint16_t*)x, (const uint16_t*)w, out, M, N, K / 32, 0, out_frag, act_p, act_n};
+    int nt, splits;
+    gs_policy(M, N, a.nsteps, kind == GS_F32 && !one, &nt, &splits);
+    a.split_steps = (a.nsteps + splits - 1) / splits;
+    const int mt = M > 32 ? 4 : (M > 16 ? 2 : 1);
+    hipStream_t st = (hipStream_t)stream;
+#define GS(MT_, NT_, K_) if (mt == MT_ && nt == NT_ && kind == K_) return gs_launch<MT_, NT_, K_>(a, splits, st);
+#define GS_ALL(K_) GS(1, 1, K_) GS(2, 1, K_) GS(4, 1, K_) GS(2, 2, K_) GS(4, 2, K_)
+    GS_ALL(GS_F32) GS_ALL(GS_BF16) GS_ALL(GS_XIELU)
+    omni_set_error("omni_gemm_stream: no tile for M=%d N=%d", M, N);
+    return OMNI_EINVAL;
+}

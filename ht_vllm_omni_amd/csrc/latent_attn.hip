@@ -9,8 +9,9 @@
 //                                row-major tile (a 16-lane group reads 4 rows x 32 B and gets them transposed)
 // Scores, softmax statistics and weights are fp32; the weights enter the second product as three bf16 terms whose sum is the fp32 value.
 //
-//   latent_decode_kernel   one token: up to 16 heads fill the 16 query rows; every wave walks its own 32-key tiles (private LDS image, no
-//                          barrier in the loop, the next tile travels in registers), waves and KV splits merge at the end
+//   latent_decode_kernel   one token: up to 16 heads fill the 16 query rows.  Four waves take one 16-key tile each for the scores, agree on the
+//                          row maxima, and share the second product by output columns: no sums to merge across waves at the end.  The
+//                          next tiles travel in registers meanwhile.  KV splits leave records a small kernel merges
 //   latent_prefill_kernel  tiles of up to 128 query rows of one sequence; PW waves share each 32-key tile (double-buffered, one barrier per
 //                          tile), MT 16-row groups per wave
 //   latent_plain_kernel    any width, bf16 or fp32: one wave per query row on the vector units (the 32-bit mode)
@@ -35,6 +36,9 @@ struct LatentArgs {
     float* partial; int nsplit;
 };
 
+// KV splits a row of `ntiles` 16-key tiles uses, of the nsplit the launch offers: fewer than six tiles are not worth a split of their own
+__device__ __forceinline__ int la_row_splits(int ntiles, int nsplit) { return min(nsplit, (ntiles + 5) / 6); }
+
 template <int RS>
 struct LatentGeom {
     static constexpr int ROWB = RS * 64;              // bytes of a cache row
@@ -43,45 +47,50 @@ struct LatentGeom {
     static constexpr int TILE = LA_KEYS * PITCH;
 };
 
-// scores of one 16-row group against the 32-key tile at `img` -> online softmax update -> weights as three bf16 terms
+// scores of one 16-row group against the 32-key tile at `img` (four independent MFMA chains)
 template <int RS>
 __device__ __forceinline__ void la_scores(const unsigned char* img, const u32x4 (&Q)[RS], int c, int qk, f32x4 (&S)[2]) {
     constexpr int PITCH = LatentGeom<RS>::PITCH;
+    f32x4 T[2];
 #pragma unroll
-    for (int kt = 0; kt < 2; ++kt) {
-        S[kt] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int kt = 0; kt < 2; ++kt) S[kt] = T[kt] = (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int s = 0; s < RS; ++s) {
+    for (int s = 0; s < RS; ++s) {
+#pragma unroll
+        for (int kt = 0; kt < 2; ++kt) {
             const u32x4 A = *reinterpret_cast<const u32x4*>(img + (16 * kt + c) * PITCH + (32 * s + 8 * qk) * 2);
-            S[kt] = mfma16(A, Q[s], S[kt]);
+            if (s & 1) T[kt] = mfma16(A, Q[s], T[kt]);
+            else S[kt] = mfma16(A, Q[s], S[kt]);
         }
     }
+#pragma unroll
+    for (int kt = 0; kt < 2; ++kt) S[kt] += T[kt];
 }
 
-struct LaWeights { u32x4 hi, mid, lo; };
-// nlive: keys of the tile this row sees (<= 0: none)
-__device__ __forceinline__ LaWeights la_softmax(const f32x4 (&S)[2], float qs, int nlive, int qk, float& m, float& l, float& alpha) {
-    float sv[8], mx = LA_SENT;
-    bool ok[8];
+// this lane's 8 scores of row c in exponent units; returns the row's maximum over the tile.  nlive: keys of the tile the row sees (<= 0: none)
+__device__ __forceinline__ float la_row_max(const f32x4 (&S)[2], float qs, int nlive, int qk, float (&sv)[8]) {
+    float mx = LA_SENT;
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
         const int kidx = (j < 4) ? 4 * qk + j : 16 + 4 * qk + (j - 4);
         sv[j] = S[j >> 2][j & 3] * qs;
-        ok[j] = kidx < nlive;
-        if (ok[j]) mx = fmaxf(mx, sv[j]);
+        if (kidx < nlive) mx = fmaxf(mx, sv[j]);
     }
-    mx = xor32_max(xor16_max(mx));
-    const float mn = fmaxf(m, mx);
-    alpha = exp2f(m - mn);                   // both the sentinel: 1, harmless (l = 0, O = 0)
-    float p[8], rs = 0.f;
+    return xor32_max(xor16_max(mx));
+}
+
+struct LaWeights { u32x4 hi, mid, lo; };
+// weights exp2(sv - m) of the visible keys as three bf16 terms; rs = their sum over the tile
+__device__ __forceinline__ LaWeights la_weights(const float (&sv)[8], int nlive, int qk, float m, float& rs) {
+    float p[8];
+    rs = 0.f;
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
-        p[j] = ok[j] ? exp2f(sv[j] - mn) : 0.f;
+        const int kidx = (j < 4) ? 4 * qk + j : 16 + 4 * qk + (j - 4);
+        p[j] = kidx < nlive ? exp2f(sv[j] - m) : 0.f;
         rs += p[j];
     }
     rs = xor32_sum(xor16_sum(rs));
-    l = l * alpha + rs;
-    m = mn;
     LaWeights w;
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
@@ -107,114 +116,173 @@ __device__ __forceinline__ u32x4 la_transposed(const unsigned char* img, int dt,
 }
 
 template <int RS>
-__global__ __launch_bounds__(64 * LA_DEC_WAVES, 1) void latent_decode_kernel(const LatentArgs a) {
+__global__ __launch_bounds__(64 * LA_DEC_WAVES, 2) void latent_decode_kernel(const LatentArgs a) {
     using G = LatentGeom<RS>;
-    constexpr int LOADS = LA_KEYS * G::CH / 64;       // 16-byte loads per lane and tile
-    extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
+    constexpr int HALF = 16 * G::PITCH;               // one wave's 16-key image; two waves' images are one 32-key tile of the second product
+    constexpr int DPW = (2 * RS + LA_DEC_WAVES - 1) / LA_DEC_WAVES;      // output column tiles of a wave: wave, wave + 4, ...
+    extern __shared__ __attribute__((aligned(16))) unsigned char lds[];  // [wave] images | [pair][term][lane] weights
     __shared__ float sm[LA_DEC_WAVES][16], sl[LA_DEC_WAVES][16];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int c = lane & 15, qk = lane >> 4;
     const int t = blockIdx.y, split = blockIdx.z;
     const int head = blockIdx.x * 16 + c, hc = min(head, a.heads - 1);
-    const int rp = RS * 32;
-    unsigned char* img = lds + wave * G::TILE;
-    u32x4 Q[RS];
-#pragma unroll
-    for (int s = 0; s < RS; ++s) Q[s] = ld16(a.q + ((size_t)t * a.heads + hc) * rp + 32 * s + 8 * qk);
+    constexpr int rp = RS * 32;
+    unsigned char* img = lds + wave * HALF;
+    u32x4* pw = reinterpret_cast<u32x4*>(lds + LA_DEC_WAVES * HALF);
     const int len = a.positions[t] + 1;
     const int32_t* bt = a.block_table + (size_t)a.row_of_tok[t] * a.bt_stride;
-    const int ntiles = (len + LA_KEYS - 1) / LA_KEYS, step = a.nsplit * LA_DEC_WAVES;
-    f32x4 O[2 * RS];
+    const int ntiles = (len + 15) / 16;
+    const int nsplit = la_row_splits(ntiles, a.nsplit);
+    if (split >= nsplit) return;
+    const int t0 = (int)((long long)ntiles * split / nsplit), t1 = (int)((long long)ntiles * (split + 1) / nsplit);
+    const int end = min(len, t1 * 16);                // keys of this split
+    u32x4 st[RS];                                     // the wave's next tile on its way to LDS (16 rows = RS 16-byte loads per lane)
+    auto block_of = [&](int tile) { return bt[min(tile * 16 + c, len - 1) >> a.bs_shift]; };
+    auto fetch = [&](int tile, int blk) {
+        const int key = min(tile * 16 + c, len - 1);  // keys past the end: a valid row, masked below
+        const int slot = (blk << a.bs_shift) + (key & a.bs_mask);
 #pragma unroll
-    for (int d = 0; d < 2 * RS; ++d) O[d] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    float m = LA_SENT, l = 0.f;
-    u32x4 st[LOADS];
-    auto fetch = [&](int tile) {
-        const int key = min(tile * LA_KEYS + (lane & 31), len - 1);          // tail keys: a valid row, masked below
-        const int slot = (bt[key >> a.bs_shift] << a.bs_shift) + (key & a.bs_mask);
-#pragma unroll
-        for (int j = 0; j < LOADS; ++j) {
+        for (int j = 0; j < RS; ++j) {
             const int i = lane + 64 * j;
             const int kk = i / G::CH, ch = i - kk * G::CH;
             const int row = G::CH % 64 == 0 ? __builtin_amdgcn_readlane(slot, j / (G::CH / 64 > 0 ? G::CH / 64 : 1)) : __shfl(slot, kk, 64);
-            st[j] = ld16(a.cache + (size_t)row * rp + ch * 8);
+            st[j] = ld16_nt(a.cache + (size_t)row * rp + ch * 8);
         }
     };
-    int tile = split * LA_DEC_WAVES + wave;
-    if (tile < ntiles) fetch(tile);
-    for (; tile < ntiles; tile += step) {
+    int blk = 0;                                      // block ids are looked up a round ahead of the rows
+    if (t0 < t1) {
+        blk = block_of(t0 + wave);
+        fetch(t0 + wave, blk);
+        blk = block_of(t0 + wave + LA_DEC_WAVES);
+    }
+    u32x4 Q[RS];
 #pragma unroll
-        for (int j = 0; j < LOADS; ++j) {
+    for (int s = 0; s < RS; ++s) Q[s] = ld16(a.q + ((size_t)t * a.heads + hc) * rp + 32 * s + 8 * qk);
+    f32x4 O[DPW];
+#pragma unroll
+    for (int i = 0; i < DPW; ++i) O[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    float m = LA_SENT, l = 0.f;                       // m: common to the waves; l: this wave's keys
+    for (int base = t0; base < t1; base += LA_DEC_WAVES) {
+        const int key0 = (base + wave) * 16 + 4 * qk; // the lane's keys: key0 .. key0 + 3
+#pragma unroll
+        for (int j = 0; j < RS; ++j) {
             const int i = lane + 64 * j;
             const int kk = i / G::CH, ch = i - kk * G::CH;
             *reinterpret_cast<u32x4*>(img + kk * G::PITCH + ch * 16) = st[j];
         }
-        if (tile + step < ntiles) fetch(tile + step);
-        __builtin_amdgcn_wave_barrier();
-        f32x4 S[2];
-        la_scores<RS>(img, Q, c, qk, S);
-        float alpha;
-        const LaWeights w = la_softmax(S, a.qs, len - tile * LA_KEYS, qk, m, l, alpha);
-        if (__any(alpha != 1.0f)) {
-#pragma unroll
-            for (int d = 0; d < 2 * RS; ++d) O[d] *= alpha;
-        }
-#pragma unroll
-        for (int d = 0; d < 2 * RS; ++d) {
-            const u32x4 VT = la_transposed<RS>(img, d, c, qk);
-            O[d] = mfma16(VT, w.hi, mfma16(VT, w.mid, mfma16(VT, w.lo, O[d])));
+        if (base + LA_DEC_WAVES < t1) {
+            fetch(base + wave + LA_DEC_WAVES, blk);
+            blk = block_of(base + wave + 2 * LA_DEC_WAVES);
         }
         __builtin_amdgcn_wave_barrier();
+        f32x4 S4[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) S4[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
+        constexpr int AB = RS < 8 ? RS : 8;           // operand reads in flight
+#pragma unroll
+        for (int s0 = 0; s0 < RS; s0 += AB) {
+            u32x4 A[AB];
+#pragma unroll
+            for (int s = 0; s < AB; ++s)
+                if (s0 + s < RS) A[s] = *reinterpret_cast<const u32x4*>(img + c * G::PITCH + (32 * (s0 + s) + 8 * qk) * 2);
+#pragma unroll
+            for (int s = 0; s < AB; ++s)
+                if (s0 + s < RS) S4[s & 3] = mfma16(A[s], Q[s0 + s], S4[s & 3]);
+        }
+        const f32x4 S = (S4[0] + S4[1]) + (S4[2] + S4[3]);
+        float sv[4], mx = LA_SENT;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            sv[j] = S[j] * a.qs;
+            if (key0 + j < end) mx = fmaxf(mx, sv[j]);
+        }
+        mx = xor32_max(xor16_max(mx));
+        if (qk == 0) sm[wave][c] = mx;
+        __syncthreads();                              // maxima and images of this round
+        float mn = m;
+#pragma unroll
+        for (int w = 0; w < LA_DEC_WAVES; ++w) mn = fmaxf(mn, sm[w][c]);
+        const float alpha = exp2f(m - mn);            // both the sentinel: 1, harmless (l = 0, O = 0)
+        m = mn;
+        float p[4], rs = 0.f;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            p[j] = key0 + j < end ? exp2f(sv[j] - m) : 0.f;
+            rs += p[j];
+        }
+        l = l * alpha + xor32_sum(xor16_sum(rs));
+        u32x2 w3[3];                                  // three bf16 terms whose sum is the fp32 weight
+#pragma unroll
+        for (int e = 0; e < 2; ++e) {
+            const float x = p[2 * e], y = p[2 * e + 1];
+            const float xr = x - bfround(x), yr = y - bfround(y);
+            const float xm = bfround(xr), ym = bfround(yr);
+            w3[0][e] = pack_bf2(x, y);
+            w3[1][e] = pack_bf2(xm, ym);
+            w3[2][e] = pack_bf2(xr - xm, yr - ym);
+        }
+#pragma unroll
+        for (int i = 0; i < 3; ++i) reinterpret_cast<u32x2*>(pw + ((wave >> 1) * 3 + i) * 64 + lane)[wave & 1] = w3[i];
+#pragma unroll
+        for (int i = 0; i < DPW; ++i) O[i] *= alpha;
+        __syncthreads();                              // weights of this round
+#pragma unroll
+        for (int u = 0; u < LA_DEC_WAVES / 2; ++u) {
+            if (base + 2 * u >= t1) break;            // (uniform; an image past t1 inside a pair holds valid rows with zero weights)
+            u32x4 W[3], VT[DPW];
+#pragma unroll
+            for (int i = 0; i < 3; ++i) W[i] = pw[(u * 3 + i) * 64 + lane];
+#pragma unroll
+            for (int i = 0; i < DPW; ++i) VT[i] = la_transposed<RS>(lds + u * 2 * HALF, min(wave + LA_DEC_WAVES * i, 2 * RS - 1), c, qk);
+#pragma unroll
+            for (int k = 2; k >= 0; --k)
+#pragma unroll
+                for (int i = 0; i < DPW; ++i) O[i] = mfma16(VT[i], W[k], O[i]);
+        }
+        if (base + LA_DEC_WAVES < t1) __syncthreads();      // the images are rewritten by the next round
     }
-    // ---- the four waves' partial results
-    if (qk == 0) { sm[wave][c] = m; sl[wave][c] = l; }
-    __syncthreads();                                   // (also: every wave is done with its tile image)
-    float M = LA_SENT, L = 0.f;
-#pragma unroll
-    for (int w = 0; w < LA_DEC_WAVES; ++w) M = fmaxf(M, sm[w][c]);
-#pragma unroll
-    for (int w = 0; w < LA_DEC_WAVES; ++w) L += sl[w][c] * exp2f(sm[w][c] - M);
-    const float f = exp2f(m - M);
-    f32x4* ex = reinterpret_cast<f32x4*>(lds);         // [wave][d tile][lane]
-#pragma unroll
-    for (int d = 0; d < 2 * RS; ++d) ex[(wave * 2 * RS + d) * 64 + lane] = O[d] * f;
+    if (qk == 0) sl[wave][c] = l;
     __syncthreads();
+    float L = 0.f;
+#pragma unroll
+    for (int w = 0; w < LA_DEC_WAVES; ++w) L += sl[w][c];
     if (head >= a.heads) return;
     const size_t rh = (size_t)t * a.heads + head;
-    float* rec = a.nsplit > 1 ? a.partial + (rh * a.nsplit + split) * (rp + 4) : nullptr;
-    if (rec && wave == 0 && qk == 0) { rec[0] = M; rec[1] = L; }
+    float* rec = nsplit > 1 ? a.partial + (rh * a.nsplit + split) * (rp + 4) : nullptr;
+    if (rec && wave == 0 && qk == 0) { rec[0] = m; rec[1] = L; }
     const float inv = (L > 0.f ? 1.0f / L : 0.f) * (a.gate ? a.gate[rh] : 1.0f);
-    for (int d = wave; d < 2 * RS; d += LA_DEC_WAVES) {
-        f32x4 v = ex[d * 64 + lane];
 #pragma unroll
-        for (int w = 1; w < LA_DEC_WAVES; ++w) v += ex[(w * 2 * RS + d) * 64 + lane];
+    for (int i = 0; i < DPW; ++i) {
+        const int d = wave + LA_DEC_WAVES * i;
+        if (d >= 2 * RS) continue;
         if (rec) {
-            *reinterpret_cast<f32x4*>(rec + 4 + 16 * d + 4 * qk) = v;
+            *reinterpret_cast<f32x4*>(rec + 4 + 16 * d + 4 * qk) = O[i];
         } else {
-            v *= inv;
+            const f32x4 v = O[i] * inv;
             *reinterpret_cast<uint2*>(a.out + rh * rp + 16 * d + 4 * qk) = make_uint2(pack_bf2(v[0], v[1]), pack_bf2(v[2], v[3]));
         }
     }
 }
 
-// KV splits of one (token, head)
-__global__ __launch_bounds__(64) void latent_merge_kernel(const float* __restrict__ partial, const float* __restrict__ gate, uint16_t* __restrict__ out,
-                                                          int nsplit, int rp) {
+// KV splits of one (token, head): lane s holds split s's weight, every thread 4 columns
+__global__ __launch_bounds__(128) void latent_merge_kernel(const float* __restrict__ partial, const float* __restrict__ gate, uint16_t* __restrict__ out,
+                                                           const int32_t* __restrict__ positions, int heads, int max_split, int rp) {
     const size_t rh = blockIdx.x;
-    const float* base = partial + rh * nsplit * (rp + 4);
-    float M = LA_SENT, L = 0.f;
-    for (int s = 0; s < nsplit; ++s) M = fmaxf(M, base[(size_t)s * (rp + 4)]);
-    for (int s = 0; s < nsplit; ++s) L += base[(size_t)s * (rp + 4) + 1] * exp2f(base[(size_t)s * (rp + 4)] - M);
-    const float inv = (L > 0.f ? 1.0f / L : 0.f) * (gate ? gate[rh] : 1.0f);
-    for (int k = threadIdx.x * 4; k < rp; k += 256) {
-        f32x4 v = (f32x4){0.f, 0.f, 0.f, 0.f};
-        for (int s = 0; s < nsplit; ++s) {
-            const float* rec = base + (size_t)s * (rp + 4);
-            v += *reinterpret_cast<const f32x4*>(rec + 4 + k) * exp2f(rec[0] - M);
-        }
-        v *= inv;
-        *reinterpret_cast<uint2*>(out + rh * rp + k) = make_uint2(pack_bf2(v[0], v[1]), pack_bf2(v[2], v[3]));
-    }
+    const int nsplit = la_row_splits((positions[rh / heads] + 16) / 16, max_split);
+    if (nsplit == 1) return;                           // the decode kernel wrote the row
+    const float* base = partial + rh * max_split * (rp + 4);
+    const int lane = threadIdx.x & 63, k = threadIdx.x * 4;
+    const float2 ml = lane < nsplit ? *reinterpret_cast<const float2*>(base + (size_t)lane * (rp + 4)) : make_float2(LA_SENT, 0.f);
+    const float M = wave_max(ml.x);
+    const float w = lane < nsplit ? exp2f(ml.x - M) : 0.f;
+    const float L = wave_sum(ml.y * w);
+    if (k >= rp) return;
+    f32x4 v = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int s = 0; s < nsplit; ++s)
+        v += *reinterpret_cast<const f32x4*>(base + (size_t)s * (rp + 4) + 4 + k) * __int_as_float(__builtin_amdgcn_readlane(__float_as_int(w), s));
+    v *= (L > 0.f ? 1.0f / L : 0.f) * (gate ? gate[rh] : 1.0f);
+    *reinterpret_cast<uint2*>(out + rh * rp + k) = make_uint2(pack_bf2(v[0], v[1]), pack_bf2(v[2], v[3]));
 }
 
 template <int RS, int PW, int MT>
@@ -279,18 +347,31 @@ __global__ __launch_bounds__(64 * PW, PW / 4) void latent_prefill_kernel(const L
         for (int i = 0; i < MT; ++i) {
             f32x4 S[2];
             la_scores<RS>(img, Q[i], c, qk, S);
-            float alpha;
-            w[i] = la_softmax(S, a.qs, see[i] - k0, qk, m[i], l[i], alpha);
+            float sv[8], rs;
+            const float mn = fmaxf(m[i], la_row_max(S, a.qs, see[i] - k0, qk, sv));
+            const float alpha = exp2f(m[i] - mn);       // both the sentinel: 1, harmless (l = 0, O = 0)
+            m[i] = mn;
+            w[i] = la_weights(sv, see[i] - k0, qk, mn, rs);
+            l[i] = l[i] * alpha + rs;
             if (__any(alpha != 1.0f)) {
 #pragma unroll
                 for (int d = 0; d < 2 * RS; ++d) O[i][d] *= alpha;
             }
         }
 #pragma unroll
-        for (int d = 0; d < 2 * RS; ++d) {
-            const u32x4 VT = la_transposed<RS>(img, d, c, qk);
+        for (int d0 = 0; d0 < 2 * RS; d0 += 2) {        // pairs of column tiles: independent chains between dependent MFMAs
+            u32x4 VT[2];
 #pragma unroll
-            for (int i = 0; i < MT; ++i) O[i][d] = mfma16(VT, w[i].hi, mfma16(VT, w[i].mid, mfma16(VT, w[i].lo, O[i][d])));
+            for (int d = 0; d < 2; ++d) VT[d] = la_transposed<RS>(img, d0 + d, c, qk);
+#pragma unroll
+            for (int i = 0; i < MT; ++i) {
+#pragma unroll
+                for (int d = 0; d < 2; ++d) O[i][d0 + d] = mfma16(VT[d], w[i].lo, O[i][d0 + d]);
+#pragma unroll
+                for (int d = 0; d < 2; ++d) O[i][d0 + d] = mfma16(VT[d], w[i].mid, O[i][d0 + d]);
+#pragma unroll
+                for (int d = 0; d < 2; ++d) O[i][d0 + d] = mfma16(VT[d], w[i].hi, O[i][d0 + d]);
+            }
         }
     }
 #pragma unroll
@@ -367,8 +448,8 @@ __global__ __launch_bounds__(64) void latent_plain_kernel(const E* __restrict__ 
 // ---- host side
 static int la_splits(int n_decode, int heads, int max_keys) {
     const int wgs = n_decode * ((heads + 15) / 16);
-    int ns = 256 / (wgs > 0 ? wgs : 1);
-    const int cap = (max_keys + 127) / 128;             // at least one tile per wave and split
+    int ns = 512 / (wgs > 0 ? wgs : 1);                 // two workgroups per CU
+    const int cap = (max_keys + 63) / 64;               // at least one tile per wave and split
     if (ns > cap) ns = cap;
     if (ns > LA_MAX_SPLIT) ns = LA_MAX_SPLIT;
     return ns < 1 ? 1 : ns;
@@ -388,7 +469,7 @@ extern "C" int omni_latent_attn_mfma(int rp) {
 
 template <typename K>
 static int la_lds(K kernel, int bytes) {
-    if (bytes <= 64 * 1024) return OMNI_OK;
+    if (bytes <= 60 * 1024) return OMNI_OK;         // (static shared memory comes on top)
     const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
     if (e != hipSuccess) { omni_set_error("omni_latent_attn: LDS attribute: %s", hipGetErrorString(e)); return OMNI_EHIP; }
     return OMNI_OK;
@@ -398,14 +479,14 @@ template <int RS>
 static int la_run(const omni_latent_attn& p, LatentArgs a, hipStream_t st) {
     using G = LatentGeom<RS>;
     if (p.n_decode > 0) {
-        constexpr int LDS = LA_DEC_WAVES * G::TILE;
+        constexpr int LDS = LA_DEC_WAVES * 16 * G::PITCH + LA_DEC_WAVES / 2 * 3 * 1024;
         static const int rc = la_lds(latent_decode_kernel<RS>, LDS);
         if (rc != OMNI_OK) return rc;
         a.nsplit = p.workspace ? la_splits(p.n_decode, p.heads, p.max_keys) : 1;
         hipLaunchKernelGGL(latent_decode_kernel<RS>, dim3((p.heads + 15) / 16, p.n_decode, a.nsplit), dim3(64 * LA_DEC_WAVES), LDS, st, a);
         OMNI_CHECK_LAUNCH("omni_latent_attn(decode)");
         if (a.nsplit > 1) {
-            hipLaunchKernelGGL(latent_merge_kernel, dim3(p.n_decode * p.heads), dim3(64), 0, st, (const float*)a.partial, a.gate, a.out, a.nsplit, p.rp);
+            hipLaunchKernelGGL(latent_merge_kernel, dim3(p.n_decode * p.heads), dim3(p.rp > 256 ? 128 : 64), 0, st, (const float*)a.partial, a.gate, a.out, a.positions, p.heads, a.nsplit, p.rp);
             OMNI_CHECK_LAUNCH("omni_latent_attn(merge)");
         }
     }

@@ -11,7 +11,7 @@ One forward serves every step: a batch is T tokens, sequence after sequence, the
   stream_rows    x += g * y / rms(y) -> bf16 x;  GEMM with xIELU in its epilogue;  GEMM -> y (fp32)
 
 The residual stream, norms, gates, scores and state are fp32; matrix operands are bf16 (``dtype="bfloat16"``) or everything is fp32
-(``dtype="float32"``).  GEMMs of up to 64 tokens stream fragment-major weights (omni_gemm_bf16_ex), larger ones run omni_gemm_tile on the
+(``dtype="float32"``).  GEMMs of up to 64 tokens stream fragment-major weights (omni_gemm_stream), larger ones run omni_gemm_tile on the
 SAME bytes.  Every width is padded to a multiple of 32 with zero weights at load, so no size is special.
 """
 from __future__ import annotations
@@ -121,8 +121,10 @@ class _Scratch:
         W = eng.width
         z = lambda n, dt: torch.zeros(n, dtype=dt, device=dev)  # noqa: E731
         self.x = (z(rows * W, torch.float32), z(rows * W, torch.float32))
-        self.y, self.h = z(rows * W, torch.float32), z(r16 * W, E)
-        self.proj = z(rows * max(l.down.N for l in ls), torch.float32)
+        # products that leave as partial sums (omni_gemm_stream): as many slabs as up to SKINNY rows may take
+        slabs = lambda n: max(rows, min(rows, SKINNY) * L.STREAM_MAX_SPLITS) * n  # noqa: E731
+        self.y, self.h = z(slabs(W), torch.float32), z(r16 * W, E)
+        self.proj = z(slabs(max(l.down.N for l in ls)), torch.float32)
         self.cq = z(r16 * max(l.qp for l in ls), E)
         self.q = z(rows * max(h * l.dp for h, l in zip(hs, ls)), E)
         self.ql = z(rows * max(h * l.rp for h, l in zip(hs, ls)), E)
@@ -255,24 +257,23 @@ class DecoderEngine:
             getattr(self, "row_" + k)[row] = v
 
     # ------------------------------------------------------------------ products
-    def _mm(self, x: torch.Tensor, w: _Matrix, out: torch.Tensor, T: int, *, f32_out: bool = False, act=None, out_frag: bool = False) -> None:
-        """out [T, N] = (xIELU of) x . w^T.  x: fragment-major when T <= SKINNY and bf16 (its producer wrote it so), else row-major."""
+    def _mm(self, x: torch.Tensor, w: _Matrix, out: torch.Tensor, T: int, *, f32_out: bool = False, one: bool = False, act=None, out_frag: bool = False) -> int:
+        """out [T, N] = (xIELU of) x . w^T.  x: fragment-major when T <= SKINNY and bf16 (its producer wrote it so), else row-major.  Returns how
+        many partial sums [T, N] an fp32 output consists of (its consumer adds them up; one: a single one)."""
         st, lib = L.current_stream(), self.lib
+        a, b = act or (0.0, 0.0)
         if self.elem.code == 1:
-            a, b = act or (0.0, 0.0)
             L.check(lib.omni_gemm_f32(x.data_ptr(), w.K, 0, w.t.data_ptr(), 0, out.data_ptr(), w.N, 0, T, w.N, w.K, 1, int(act is not None), a, b, st),
                     "omni_gemm_f32", lib)
         elif T <= SKINNY:
-            layout = L.LAYOUT_W_FRAG | L.LAYOUT_X_FRAG | (L.LAYOUT_OUT_FRAG if out_frag else 0)
-            if act is not None:
-                L.check(lib.omni_gemm_xielu(x.data_ptr(), w.K, w.t.data_ptr(), out.data_ptr(), T, w.N, w.K, act[0], act[1], layout, st), "omni_gemm_xielu", lib)
-            else:
-                L.check(lib.omni_gemm_bf16_ex(x.data_ptr(), w.K, w.t.data_ptr(), None, out.data_ptr(), T, w.N, w.K, L.EPI_F32 if f32_out else L.EPI_BF16,
-                                              None, layout, st), "omni_gemm_bf16_ex", lib)
+            kind = L.STREAM_F32 if f32_out else (L.STREAM_BF16 if act is None else L.STREAM_XIELU)
+            L.check(lib.omni_gemm_stream(x.data_ptr(), w.t.data_ptr(), out.data_ptr(), T, w.N, w.K, kind, int(one), a, b, int(out_frag), st), "omni_gemm_stream", lib)
+            return lib.omni_gemm_stream_splits(T, w.N, w.K) if f32_out and not one else 1
         else:
             o = out[:T * w.N].view(T, w.N)
-            ops.gemm_tile(x[:T * w.K].view(T, w.K), w.t, act=L.TILE_ACT_NONE if act is None else L.TILE_ACT_XIELU, act_params=act or (0.0, 0.0),
+            ops.gemm_tile(x[:T * w.K].view(T, w.K), w.t, act=L.TILE_ACT_NONE if act is None else L.TILE_ACT_XIELU, act_params=(a, b),
                           want="f" if f32_out else "b", lib=lib, **({"out_f32": o} if f32_out else {"out": o}))
+        return 1
 
     def _heads_mm(self, x: torch.Tensor, w: _Matrix, out: torch.Tensor, T: int, heads: int, out_frag: bool = False) -> None:
         """out[t, h] = x[t, h] . w[h]^T."""
@@ -318,13 +319,13 @@ class DecoderEngine:
             self._any = _Scratch(self, max(T, 256) if T <= 256 else (T + 1023) // 1024 * 1024)
         return self._any
 
-    def _mixer(self, b: Batch, i: int, s: _Scratch, x: torch.Tensor, frag: bool) -> None:
-        """s.h -> s.y"""
+    def _mixer(self, b: Batch, i: int, s: _Scratch, x: torch.Tensor, frag: bool) -> int:
+        """s.h -> s.y (returns its partial sums)"""
         m, w, lib, st = self.d.layers[i].mixer, self.layer_w[self.d.owner(i)], self.lib, L.current_stream()
         T, H = b.T, m.heads
-        self._mm(s.h, w.down, s.proj, T, f32_out=True)
+        slabs = self._mm(s.h, w.down, s.proj, T, f32_out=True)
         gate = s.gate if m.out_gate else None
-        a = L.LatentWrite(proj=s.proj.data_ptr(), ld=w.down.N, q_rank=m.q_rank, qp=w.qp, kv_rank=m.kv_rank, rp=w.rp, heads=H, qw=w.qw.data_ptr(),
+        a = L.LatentWrite(proj=s.proj.data_ptr(), slabs=slabs, slab_stride=T * w.down.N, ld=w.down.N, q_rank=m.q_rank, qp=w.qp, kv_rank=m.kv_rank, rp=w.rp, heads=H, qw=w.qw.data_ptr(),
                           kw=w.kw.data_ptr(), eps=self.d.eps, cq=s.cq.data_ptr(), frag=int(frag), cache=self.kv_caches[i].data_ptr(), gate=L.ptr(gate),
                           block_table=self.block_table.data_ptr(), bt_stride=self.bt_stride, block_size=self.block_size, row_of_tok=b.row_of_tok.data_ptr(),
                           positions=b.positions.data_ptr(), num_live=L.ptr(b.num_live), x=x.data_ptr(), wp=self.width, state=self.state[i].data_ptr(),
@@ -339,7 +340,7 @@ class DecoderEngine:
                          max_keys=b.max_keys, workspace=self.attn_ws.data_ptr(), workspace_bytes=self.attn_ws.numel() * 4, elem=self.elem.code)
         L.check(lib.omni_latent_attn_run(C.byref(a), st), "omni_latent_attn", lib)
         self._heads_mm(s.ol, w.uv, s.v, T, H, out_frag=frag)
-        self._mm(s.v, w.o, s.y, T, f32_out=True)
+        return self._mm(s.v, w.o, s.y, T, f32_out=True)
 
     def forward(self, b: Batch, *, sel: torch.Tensor | None = None, logits: torch.Tensor | None = None, scratch: _Scratch | None = None,
                 trail: list | None = None) -> torch.Tensor | None:
@@ -354,19 +355,18 @@ class DecoderEngine:
         self._rows(ids=b.ids, table=self.embed, vocab=d.vocab, mu=lw(0).mu, state=self.state[0], x_out=s.x[k], h_out=s.h, frag=int(frag), **where)
         for i in range(d.num_layers):
             w = lw(i)
-            self._mixer(b, i, s, s.x[k], frag)
-            gain = w.gain1
+            ny, gain = self._mixer(b, i, s, s.x[k], frag), w.gain1
             if d.layers[i].mlp is not None:
-                self._rows(x_in=s.x[k], y=s.y, gain=gain, x_out=s.x[k ^ 1], h_out=s.h, frag=int(frag), rows=T)
+                self._rows(x_in=s.x[k], y=s.y, y_slabs=ny, y_stride=T * self.width, gain=gain, x_out=s.x[k ^ 1], h_out=s.h, frag=int(frag), rows=T)
                 k ^= 1
                 self._mm(s.h, w.up, s.act, T, act=w.act, out_frag=frag)
-                self._mm(s.act, w.dn, s.y, T, f32_out=True)
-                gain = w.gain2
+                ny, gain = self._mm(s.act, w.dn, s.y, T, f32_out=True), w.gain2
+            add = dict(x_in=s.x[k], y=s.y, y_slabs=ny, y_stride=T * self.width, gain=gain)
             if trail is not None:
-                self._rows(x_in=s.x[k], y=s.y, gain=gain, x_out=s.x[k ^ 1], rows=T)
+                self._rows(**add, x_out=s.x[k ^ 1], rows=T)
                 trail.append(s.x[k ^ 1][:T * self.width].view(T, self.width)[:, :d.hidden].clone())
             if i + 1 < d.num_layers:
-                self._rows(x_in=s.x[k], y=s.y, gain=gain, mu=lw(i + 1).mu, state=self.state[i + 1], x_out=s.x[k ^ 1], h_out=s.h, frag=int(frag), **where)
+                self._rows(**add, mu=lw(i + 1).mu, state=self.state[i + 1], x_out=s.x[k ^ 1], h_out=s.h, frag=int(frag), **where)
                 k ^= 1
         n = T if sel is None else sel.numel()
         if n == 0:
@@ -374,10 +374,10 @@ class DecoderEngine:
         if n > s.rows:
             raise L.OmniError(f"logits of {n} rows from a batch of {T} tokens")
         nfrag = self.elem.code == 0 and n <= SKINNY
-        self._rows(x_in=s.x[k], y=s.y, gain=gain, use_final=1, final_gain=self.final_gain, sel=sel, h_out=s.hn, frag=int(nfrag), rows=n)
+        self._rows(**add, use_final=1, final_gain=self.final_gain, sel=sel, h_out=s.hn, frag=int(nfrag), rows=n)
         if logits is None:
             logits = torch.empty(n, self.head.N, dtype=torch.float32, device=self.device)
-        self._mm(s.hn, self.head, logits.view(-1), n, f32_out=True)
+        self._mm(s.hn, self.head, logits.view(-1), n, f32_out=True, one=True)
         return logits
 
     def sample_rows_in_place(self, B: int, num_live: torch.Tensor) -> None:

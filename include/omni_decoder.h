@@ -2,7 +2,7 @@
  * paged cache of latents, token shift with per-sequence state, output norms, dense feed-forwards).  Every entry launches on `stream`,
  * allocates nothing, synchronises nothing (capturable) and returns OMNI_OK or an error with omni_last_error().
  *
- * The library also exports omni_gemm_bf16_ex, omni_gemm_tile, omni_sample_rows (omni_talker.h): same sources, linked without the talker.
+ * The library also exports omni_gemm_tile and omni_sample / omni_sample_rows (omni_talker.h): same sources, linked without the talker.
  *
  * Conventions.  `elem`: 0 = bfloat16 (matrix operands, cache and activations bf16; sums, norms, scores, state fp32), 1 = fp32 throughout.
  * The residual stream x is fp32 [T, width] in both.  A batch is T tokens, sequence after sequence: row_of_tok[t] names the token's batch row
@@ -23,7 +23,7 @@ extern "C" {
  * h_out (optional) in `elem`, row-major [*, wp] or fragment-major (frag, bf16).  sel (optional): output i is token sel[i] (no mu, no x_out). */
 typedef struct omni_stream_rows {
     const int32_t* ids; const void* table; int vocab;
-    const float* x_in; const float* y; float gain, eps;
+    const float* x_in; const float* y; int y_slabs; int64_t y_stride; float gain, eps;     /* y = sum of y_slabs arrays y_stride elements apart (0, 1: one) */
     const void* mu; const float* state; const int32_t* state_slot; const int32_t* row_of_tok; const int32_t* positions;
     int use_final; float final_gain; const int32_t* sel;
     float* x_out; void* h_out; int frag;
@@ -33,14 +33,14 @@ typedef struct omni_stream_rows {
 } omni_stream_rows;
 int omni_stream_rows_run(const omni_stream_rows* a, void* stream);
 
-/* Behind the joint down-projection proj fp32 [T, ld] = [q latent (q_rank, padded to qp) | kv latent (kv_rank, padded to rp) | gate logits]:
+/* Behind the joint down-projection proj fp32 [T, ld] (the sum of `slabs` such arrays) = [q latent (q_rank, padded to qp) | kv latent (kv_rank, padded to rp) | gate logits]:
  *   cq[t]  = RMSnorm(q part) * qw        elem [T, qp], row-major or fragment-major
  *   cache slot of (row, position)  = RMSnorm(kv part) * kw      elem [blocks, block_size, rp]
  *   gate[t, h] = sigmoid(gate logits)    fp32 [T, heads]        (gate != NULL)
  *   state[state_slot[row]] = x[t] for the last token of each sequence of the batch     (state != NULL)
  * rows >= *num_live (optional) leave cache and state alone.                                                                          */
 typedef struct omni_latent_write {
-    const float* proj; int ld, q_rank, qp, kv_rank, rp, heads;
+    const float* proj; int slabs; int64_t slab_stride; int ld, q_rank, qp, kv_rank, rp, heads;
     const void* qw; const void* kw; float eps;
     void* cq; int frag; void* cache; float* gate;
     const int32_t* block_table; int bt_stride, block_size;
@@ -58,8 +58,12 @@ int omni_head_gemm(const void* x, const void* w, void* out, int T, int heads, in
 int omni_gemm_f32(const float* x, int ldx, int64_t xb, const float* w, int64_t wb, float* out, int ldo, int64_t ob, int M, int N, int K,
                   int batch, int act, float act_p, float act_n, void* stream);
 
-/* bf16 out = xIELU(x . w^T) on the weight-streaming kernel (M <= 64), layouts as omni_gemm_bf16_ex */
-int omni_gemm_xielu(const void* x, int ldx, const void* w, void* out, int M, int N, int K, float act_p, float act_n, int layout, void* stream);
+/* Weight-streaming GEMM of up to 64 rows: x and w fragment-major bf16 (x [M, K] in whole 16-row tiles).
+ *   kind 0: out fp32 [S][M, N], S = omni_gemm_stream_splits(M, N, K) partial sums over K (their sum is the product); `one`: S = 1
+ *   kind 1: out bf16 [M, N], kind 2: bf16 xIELU(product); row-major or fragment-major (out_frag)                                      */
+#define OMNI_STREAM_MAX_SPLITS 8
+int omni_gemm_stream(const void* x, const void* w, void* out, int M, int N, int K, int kind, int one, float act_p, float act_n, int out_frag, void* stream);
+int omni_gemm_stream_splits(int M, int N, int K);
 
 /* Causal attention over a paged cache of latents shared by all heads (keys and values are the same rp-wide rows):
  *   out[t, h] = gate[t, h] * sum_j softmax_j(scale * q[t, h] . c_j) c_j,   j <= positions[t],   q / out elem [T, heads, rp].

@@ -52,7 +52,6 @@ extern "C" {
 #define OMNI_EPI_SILU_MUL_GU8 5 /* as SILU_MUL for a fragment-major W whose rows were interleaved first: rows 16t..16t+7 =
                                  * gate[8t..8t+7], rows 16t+8..16t+15 = up[8t..8t+7] -- one 16-row MFMA tile then yields 8
                                  * finished act columns, so any number of tiles per workgroup divides the chip evenly */
-#define OMNI_EPI_XIELU 6       /* omni_gemm_xielu only (omni_decoder.h): out bf16 = xielu(acc) */
 
 const char* omni_last_error(void);
 int omni_abi_version(void);   /* 6: omni_tile_gemm column groups and the xIELU activation (5: omni_ar_peers.tile_flags, omni_talker_set_chains
