@@ -76,7 +76,7 @@ class LatentAttn(C.Structure):
 
 LATENT_TILE = 128           # OMNI_LATENT_TILE
 STREAM_F32, STREAM_BF16, STREAM_XIELU = 0, 1, 2      # omni_gemm_stream kinds
-STREAM_MAX_SPLITS = 8
+STREAM_MAX_SPLITS = 4
 
 
 class ResUnit(C.Structure):

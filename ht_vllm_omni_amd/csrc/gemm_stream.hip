@@ -22,7 +22,7 @@ struct StreamArgs {
 
 template <int MT, int NT, int KIND>
 __global__ __launch_bounds__(GS_THREADS) void gemm_stream_kernel(const StreamArgs a) {
-    constexpr int P = MT * NT >= 8 ? 3 : 4;
+    constexpr int P = 2;                               // (4 measured the same or slower at 1 .. 64 rows)
     extern __shared__ __attribute__((aligned(16))) f32x4 part[];      // [wave][NT * MT][lane]
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int k0 = blockIdx.y * a.split_steps, nk = min(a.split_steps, a.nsteps - k0);
@@ -99,23 +99,30 @@ __global__ __launch_bounds__(GS_THREADS) void gemm_stream_kernel(const StreamArg
     }
 }
 
-// columns per workgroup and K splits: wide tiles at many rows (x is most of the traffic there), then enough splits for about 1.5 workgroups per CU,
-// each wave keeping at least two steps
+// Columns per workgroup and K splits.  A workgroup's registers and LDS leave room for one per CU at 64 rows, so a grid runs in rounds of 256; a
+// workgroup's time goes with the operand tiles it reads (NT of W and MT of x per k-step) plus its epilogue, a split also costs its consumer.
+// Measured at 64 rows: 9216 x 2048 by 3 (192 workgroups) 12.1 us, by 2 (288: two rounds) 15.0; 2048 x 9216 by 2 in 4 splits (256) 11.4, in 6 13.3.
 static void gs_policy(int M, int N, int nsteps, bool slabs, int* nt, int* splits) {
-    const int tiles = N / 16;
-    *nt = (M > 16 && tiles % 2 == 0 && tiles >= (slabs ? 64 : 512)) ? 2 : 1;
-    *splits = 1;
-    if (!slabs) return;
-    const int groups = tiles / *nt;
-    int s = (384 + groups - 1) / groups, most = nsteps / (2 * GS_WAVES);
-    if (s > most) s = most;
-    if (s > OMNI_STREAM_MAX_SPLITS) s = OMNI_STREAM_MAX_SPLITS;
-    *splits = s < 1 ? 1 : s;
+    const int tiles = N / 16, mt = M > 32 ? 4 : (M > 16 ? 2 : 1);
+    long best = -1;
+    for (int n = 1; n <= 4; ++n) {
+        if (tiles % n) continue;
+        for (int s = 1; s <= (slabs ? OMNI_STREAM_MAX_SPLITS : 1); ++s) {
+            if (s > 1 && nsteps / s < 2 * GS_WAVES) break;
+            const long rounds = ((long)tiles / n * s + 255) / 256;
+            const long cost = rounds * ((n + mt) * ((nsteps + s - 1) / s) + 4 * n * mt) + 12 * s;
+            if (best < 0 || cost < best) { best = cost; *nt = n; *splits = s; }
+        }
+    }
 }
 
 template <int MT, int NT, int KIND>
 static int gs_launch(const StreamArgs& a, int splits, hipStream_t st) {
     constexpr int LDS = GS_WAVES * NT * MT * 1024;
+    if (LDS > 64 * 1024) {
+        static const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(gemm_stream_kernel<MT, NT, KIND>), hipFuncAttributeMaxDynamicSharedMemorySize, LDS);
+        if (e != hipSuccess) { omni_set_error("omni_gemm_stream: LDS attribute: %s", hipGetErrorString(e)); return OMNI_EHIP; }
+    }
     hipLaunchKernelGGL((gemm_stream_kernel<MT, NT, KIND>), dim3(a.N / (16 * NT), splits), dim3(GS_THREADS), LDS, st, a);
     OMNI_CHECK_LAUNCH("omni_gemm_stream");
     return OMNI_OK;
@@ -138,7 +145,8 @@ extern "C" int omni_gemm_stream(const void* x, const void* w, void* out, int M, 
     const int mt = M > 32 ? 4 : (M > 16 ? 2 : 1);
     hipStream_t st = (hipStream_t)stream;
 #define GS(MT_, NT_, K_) if (mt == MT_ && nt == NT_ && kind == K_) return gs_launch<MT_, NT_, K_>(a, splits, st);
-#define GS_ALL(K_) GS(1, 1, K_) GS(2, 1, K_) GS(4, 1, K_) GS(2, 2, K_) GS(4, 2, K_)
+#define GS_NT(NT_, K_) GS(1, NT_, K_) GS(2, NT_, K_) GS(4, NT_, K_)
+#define GS_ALL(K_) GS_NT(1, K_) GS_NT(2, K_) GS_NT(3, K_) GS_NT(4, K_)
     GS_ALL(GS_F32) GS_ALL(GS_BF16) GS_ALL(GS_XIELU)
     omni_set_error("omni_gemm_stream: no tile for M=%d N=%d", M, N);
     return OMNI_EINVAL;

@@ -61,7 +61,7 @@ int omni_gemm_f32(const float* x, int ldx, int64_t xb, const float* w, int64_t w
 /* Weight-streaming GEMM of up to 64 rows: x and w fragment-major bf16 (x [M, K] in whole 16-row tiles).
  *   kind 0: out fp32 [S][M, N], S = omni_gemm_stream_splits(M, N, K) partial sums over K (their sum is the product); `one`: S = 1
  *   kind 1: out bf16 [M, N], kind 2: bf16 xIELU(product); row-major or fragment-major (out_frag)                                      */
-#define OMNI_STREAM_MAX_SPLITS 8
+#define OMNI_STREAM_MAX_SPLITS 4
 int omni_gemm_stream(const void* x, const void* w, void* out, int M, int N, int K, int kind, int one, float act_p, float act_n, int out_frag, void* stream);
 int omni_gemm_stream_splits(int M, int N, int K);
 
