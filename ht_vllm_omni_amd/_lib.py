@@ -70,11 +70,10 @@ class LatentWrite(C.Structure):
 class LatentAttn(C.Structure):
     """omni_latent_attn."""
     _fields_ = [("q", vp), ("cache", vp), ("gate", vp), ("out", vp), ("block_table", vp), ("bt_stride", i32), ("block_size", i32),
-                ("row_of_tok", vp), ("positions", vp), ("tiles", vp), ("n_tiles", i32), ("T", i32), ("n_decode", i32), ("heads", i32), ("rp", i32),
+                ("row_of_tok", vp), ("positions", vp), ("tiles", vp), ("n_tiles", i32), ("tile_rows", i32), ("T", i32), ("n_decode", i32), ("heads", i32), ("rp", i32),
                 ("scale", f32), ("max_keys", i32), ("workspace", vp), ("workspace_bytes", i64), ("elem", i32)]
 
 
-LATENT_TILE = 128           # OMNI_LATENT_TILE
 STREAM_F32, STREAM_BF16, STREAM_XIELU = 0, 1, 2      # omni_gemm_stream kinds
 STREAM_MAX_SPLITS = 4
 

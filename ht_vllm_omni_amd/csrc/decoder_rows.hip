@@ -28,6 +28,20 @@ __device__ __forceinline__ void st4<uint16_t>(uint16_t* p, const float (&v)[4]) 
     *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf2(v[0], v[1]), pack_bf2(v[2], v[3]));
 }
 
+// 4 consecutive values of an array that arrives as `slabs` partial sums `stride` elements apart, added in slab order.  More than one: all
+// OMNI_STREAM_MAX_SPLITS loads leave at once (past the last slab: a repeated address, not added)
+__device__ __forceinline__ void ld4_slabs(const float* p, int slabs, int64_t stride, float (&v)[4]) {
+    ld4<float>(p, v);
+    if (slabs <= 1) return;
+    float z[OMNI_STREAM_MAX_SPLITS][4];
+#pragma unroll
+    for (int s = 1; s < OMNI_STREAM_MAX_SPLITS; ++s) ld4<float>(p + min(s, slabs - 1) * stride, z[s]);
+#pragma unroll
+    for (int s = 1; s < OMNI_STREAM_MAX_SPLITS; ++s)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] += s < slabs ? z[s][e] : 0.f;
+}
+
 // sum over the workgroup, result in every thread; `buf` alternates between calls so that one barrier per sum is enough
 struct BlockSum {
     float* lds;      // [2][DR_WAVES]
@@ -75,15 +89,7 @@ __global__ __launch_bounds__(DR_THREADS) void stream_rows_kernel(const omni_stre
             y[c][0] = y[c][1] = y[c][2] = y[c][3] = 0.f;
             if (k < wp) {
                 ld4<float>(a.x_in + (size_t)t * wp + k, v[c]);
-                if (a.y) {
-                    ld4<float>(a.y + (size_t)t * wp + k, y[c]);
-                    for (int s = 1; s < a.y_slabs; ++s) {          // partial sums of the product, in slab order
-                        float z[4];
-                        ld4<float>(a.y + (size_t)s * a.y_stride + (size_t)t * wp + k, z);
-#pragma unroll
-                        for (int e = 0; e < 4; ++e) y[c][e] += z[e];
-                    }
-                }
+                if (a.y) ld4_slabs(a.y + (size_t)t * wp + k, a.y_slabs, a.y_stride, y[c]);
             }
         }
         if (!a.y) return;
@@ -172,6 +178,7 @@ extern "C" int omni_stream_rows_run(const omni_stream_rows* p, void* stream) {
     OMNI_CHECK_ARG(p && (p->ids ? p->table != nullptr : p->x_in != nullptr) && (p->x_out || p->h_out), "omni_stream_rows: null pointer");
     const omni_stream_rows& a = *p;
     OMNI_CHECK_ARG(a.width > 0 && a.wp >= a.width && a.wp % 32 == 0 && a.wp <= DR_THREADS * 4 * 8, "omni_stream_rows: width=%d wp=%d (multiple of 32, <= 8192)", a.width, a.wp);
+    OMNI_CHECK_ARG(a.y_slabs <= OMNI_STREAM_MAX_SPLITS, "omni_stream_rows: y_slabs=%d", a.y_slabs);
     OMNI_CHECK_ARG(a.elem == 0 || a.elem == 1, "omni_stream_rows: elem=%d", a.elem);
     OMNI_CHECK_ARG(!a.frag || a.elem == 0, "omni_stream_rows: fragment-major output is bf16");
     OMNI_CHECK_ARG(!a.mu || (a.state && a.state_slot && a.row_of_tok && a.positions && !a.sel && !a.use_final), "omni_stream_rows: token shift needs state, rows and positions, and no selection");
@@ -198,13 +205,7 @@ __global__ __launch_bounds__(DR_THREADS) void latent_write_kernel(const omni_lat
     float sq = 0.f, sk = 0.f;
     for (int k = threadIdx.x * 4; k < a.ld; k += DR_THREADS * 4) {
         float v[4];
-        ld4<float>(y + k, v);
-        for (int s = 1; s < a.slabs; ++s) {
-            float z[4];
-            ld4<float>(y + (size_t)s * a.slab_stride + k, z);
-#pragma unroll
-            for (int e = 0; e < 4; ++e) v[e] += z[e];
-        }
+        ld4_slabs(y + k, a.slabs, a.slab_stride, v);
         st4<float>(sp + k, v);
         const float ss = sq4_sum(v[0], v[1], v[2], v[3]);          // (padded columns hold zeros; qp and rp are multiples of 4)
         if (k < a.qp) sq += ss;
@@ -258,6 +259,7 @@ extern "C" int omni_latent_write_run(const omni_latent_write* p, void* stream) {
     OMNI_CHECK_ARG(!a.state || (a.x && a.state_slot && a.wp % 4 == 0), "omni_latent_write: state needs the stream rows and slots");
     OMNI_CHECK_ARG(a.elem == 1 || a.elem == 0, "omni_latent_write: elem=%d", a.elem);
     OMNI_CHECK_ARG(!a.frag || a.elem == 0, "omni_latent_write: fragment-major output is bf16");
+    OMNI_CHECK_ARG(a.slabs <= OMNI_STREAM_MAX_SPLITS, "omni_latent_write: slabs=%d", a.slabs);
     OMNI_CHECK_ARG(a.ld <= 15 * 1024, "omni_latent_write: ld=%d (<= 15360: a token's projections are staged in LDS)", a.ld);
     if (a.T <= 0) return OMNI_OK;
     const size_t lds = (size_t)a.ld * sizeof(float);

@@ -12,8 +12,8 @@
 //   latent_decode_kernel   one token: up to 16 heads fill the 16 query rows.  Four waves take one 16-key tile each for the scores, agree on the
 //                          row maxima, and share the second product by output columns: no sums to merge across waves at the end.  The
 //                          next tiles travel in registers meanwhile.  KV splits leave records a small kernel merges
-//   latent_prefill_kernel  tiles of up to 128 query rows of one sequence; PW waves share each 32-key tile (double-buffered, one barrier per
-//                          tile), MT 16-row groups per wave
+//   latent_prefill_kernel  tiles of up to 64 or 128 query rows of one sequence, 16 per wave; the waves share each 32-key tile (double-buffered,
+//                          one barrier per tile)
 //   latent_plain_kernel    any width, bf16 or fp32: one wave per query row on the vector units (the 32-bit mode)
 #include "common.cuh"
 #include "gemm_frag.cuh"
@@ -285,37 +285,28 @@ __global__ __launch_bounds__(128) void latent_merge_kernel(const float* __restri
     *reinterpret_cast<uint2*>(out + rh * rp + k) = make_uint2(pack_bf2(v[0], v[1]), pack_bf2(v[2], v[3]));
 }
 
-template <int RS, int PW, int MT>
-__global__ __launch_bounds__(64 * PW, PW / 4) void latent_prefill_kernel(const LatentArgs a) {
+template <int RS, int PW>
+__global__ __launch_bounds__(64 * PW, 2) void latent_prefill_kernel(const LatentArgs a) {
     using G = LatentGeom<RS>;
-    static_assert(PW * MT * 16 == OMNI_LATENT_TILE, "a work item is one tile of query rows");
     constexpr int NT = 64 * PW, ITEMS = LA_KEYS * G::CH, LOADS = (ITEMS + NT - 1) / NT;
     extern __shared__ __attribute__((aligned(16))) unsigned char lds[];      // two tile images
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int c = lane & 15, qk = lane >> 4;
     const int row0 = a.tiles[2 * blockIdx.x], nrows = a.tiles[2 * blockIdx.x + 1];
-    const int rp = RS * 32;
+    constexpr int rp = RS * 32;
     const int32_t* bt = a.block_table + (size_t)a.row_of_tok[row0 / a.heads] * a.bt_stride;
-    u32x4 Q[MT][RS];
-    f32x4 O[MT][2 * RS];
-    float m[MT], l[MT];
-    int see[MT], wsee = 0;                              // keys a row sees; most keys any row of this wave sees
-    size_t frow[MT];
-#pragma unroll
-    for (int i = 0; i < MT; ++i) {
-        const int r = (wave * MT + i) * 16 + c;
-        frow[i] = (size_t)(row0 + min(r, nrows - 1));
-        see[i] = r < nrows ? a.positions[frow[i] / a.heads] + 1 : 0;
-        m[i] = LA_SENT;
-        l[i] = 0.f;
-#pragma unroll
-        for (int s = 0; s < RS; ++s) Q[i][s] = ld16(a.q + frow[i] * rp + 32 * s + 8 * qk);
-#pragma unroll
-        for (int d = 0; d < 2 * RS; ++d) O[i][d] = (f32x4){0.f, 0.f, 0.f, 0.f};
-        const int last = min((wave * MT + i) * 16 + 15, nrows - 1);
-        if ((wave * MT + i) * 16 < nrows) wsee = max(wsee, a.positions[(row0 + last) / a.heads] + 1);
-    }
+    const int r = wave * 16 + c;
+    const size_t frow = (size_t)(row0 + min(r, nrows - 1));
+    const int see = r < nrows ? a.positions[frow / a.heads] + 1 : 0;         // keys the row sees
+    const int wsee = wave * 16 < nrows ? a.positions[(row0 + min(wave * 16 + 15, nrows - 1)) / a.heads] + 1 : 0;      // most keys of the wave's rows
     const int nkeys = a.positions[(row0 + nrows - 1) / a.heads] + 1;
+    u32x4 Q[RS];
+    f32x4 O[2 * RS];
+#pragma unroll
+    for (int s = 0; s < RS; ++s) Q[s] = ld16(a.q + frow * rp + 32 * s + 8 * qk);
+#pragma unroll
+    for (int d = 0; d < 2 * RS; ++d) O[d] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    float m = LA_SENT, l = 0.f;
     u32x4 st[LOADS];
     auto fetch = [&](int k0) {
 #pragma unroll
@@ -342,21 +333,17 @@ __global__ __launch_bounds__(64 * PW, PW / 4) void latent_prefill_kernel(const L
         if (k0 + LA_KEYS < nkeys) fetch(k0 + LA_KEYS);
         __syncthreads();                                // image `buf` complete; image `buf ^ 1` is rewritten only behind the NEXT barrier's arrivals
         if (k0 >= wsee) continue;                       // (wave-uniform; the barriers above stay common)
-        LaWeights w[MT];
+        f32x4 S[2];
+        la_scores<RS>(img, Q, c, qk, S);
+        float sv[8], rs;
+        const float mn = fmaxf(m, la_row_max(S, a.qs, see - k0, qk, sv));
+        const float alpha = exp2f(m - mn);              // both the sentinel: 1, harmless (l = 0, O = 0)
+        m = mn;
+        const LaWeights w = la_weights(sv, see - k0, qk, mn, rs);
+        l = l * alpha + rs;
+        if (__any(alpha != 1.0f)) {
 #pragma unroll
-        for (int i = 0; i < MT; ++i) {
-            f32x4 S[2];
-            la_scores<RS>(img, Q[i], c, qk, S);
-            float sv[8], rs;
-            const float mn = fmaxf(m[i], la_row_max(S, a.qs, see[i] - k0, qk, sv));
-            const float alpha = exp2f(m[i] - mn);       // both the sentinel: 1, harmless (l = 0, O = 0)
-            m[i] = mn;
-            w[i] = la_weights(sv, see[i] - k0, qk, mn, rs);
-            l[i] = l[i] * alpha + rs;
-            if (__any(alpha != 1.0f)) {
-#pragma unroll
-                for (int d = 0; d < 2 * RS; ++d) O[i][d] *= alpha;
-            }
+            for (int d = 0; d < 2 * RS; ++d) O[d] *= alpha;
         }
 #pragma unroll
         for (int d0 = 0; d0 < 2 * RS; d0 += 2) {        // pairs of column tiles: independent chains between dependent MFMAs
@@ -364,25 +351,19 @@ __global__ __launch_bounds__(64 * PW, PW / 4) void latent_prefill_kernel(const L
 #pragma unroll
             for (int d = 0; d < 2; ++d) VT[d] = la_transposed<RS>(img, d0 + d, c, qk);
 #pragma unroll
-            for (int i = 0; i < MT; ++i) {
+            for (int d = 0; d < 2; ++d) O[d0 + d] = mfma16(VT[d], w.lo, O[d0 + d]);
 #pragma unroll
-                for (int d = 0; d < 2; ++d) O[i][d0 + d] = mfma16(VT[d], w[i].lo, O[i][d0 + d]);
+            for (int d = 0; d < 2; ++d) O[d0 + d] = mfma16(VT[d], w.mid, O[d0 + d]);
 #pragma unroll
-                for (int d = 0; d < 2; ++d) O[i][d0 + d] = mfma16(VT[d], w[i].mid, O[i][d0 + d]);
-#pragma unroll
-                for (int d = 0; d < 2; ++d) O[i][d0 + d] = mfma16(VT[d], w[i].hi, O[i][d0 + d]);
-            }
+            for (int d = 0; d < 2; ++d) O[d0 + d] = mfma16(VT[d], w.hi, O[d0 + d]);
         }
     }
+    if (see <= 0) return;
+    const float inv = 1.0f / l * (a.gate ? a.gate[frow] : 1.0f);
 #pragma unroll
-    for (int i = 0; i < MT; ++i) {
-        if (see[i] <= 0) continue;
-        const float inv = 1.0f / l[i] * (a.gate ? a.gate[frow[i]] : 1.0f);
-#pragma unroll
-        for (int d = 0; d < 2 * RS; ++d) {
-            const f32x4 v = O[i][d] * inv;
-            *reinterpret_cast<uint2*>(a.out + frow[i] * rp + 16 * d + 4 * qk) = make_uint2(pack_bf2(v[0], v[1]), pack_bf2(v[2], v[3]));
-        }
+    for (int d = 0; d < 2 * RS; ++d) {
+        const f32x4 v = O[d] * inv;
+        *reinterpret_cast<uint2*>(a.out + frow * rp + 16 * d + 4 * qk) = make_uint2(pack_bf2(v[0], v[1]), pack_bf2(v[2], v[3]));
     }
 }
 
@@ -491,10 +472,12 @@ static int la_run(const omni_latent_attn& p, LatentArgs a, hipStream_t st) {
         }
     }
     if (p.n_tiles > 0) {
-        constexpr int PW = 8, LDS = 2 * G::TILE;
-        static const int rc = la_lds(latent_prefill_kernel<RS, PW, 8 / PW>, LDS);
-        if (rc != OMNI_OK) return rc;
-        hipLaunchKernelGGL((latent_prefill_kernel<RS, PW, 8 / PW>), dim3(p.n_tiles), dim3(64 * PW), LDS, st, a);
+        constexpr int LDS = 2 * G::TILE;
+        static const int rc8 = la_lds(latent_prefill_kernel<RS, 8>, LDS), rc4 = la_lds(latent_prefill_kernel<RS, 4>, LDS);
+        if (rc8 != OMNI_OK) return rc8;
+        if (rc4 != OMNI_OK) return rc4;
+        if (p.tile_rows == 64) hipLaunchKernelGGL((latent_prefill_kernel<RS, 4>), dim3(p.n_tiles), dim3(256), LDS, st, a);
+        else hipLaunchKernelGGL((latent_prefill_kernel<RS, 8>), dim3(p.n_tiles), dim3(512), LDS, st, a);
         OMNI_CHECK_LAUNCH("omni_latent_attn(prefill)");
     }
     return OMNI_OK;
@@ -507,6 +490,7 @@ extern "C" int omni_latent_attn_run(const omni_latent_attn* pp, void* stream) {
     OMNI_CHECK_ARG(p.block_size > 0 && (p.block_size & (p.block_size - 1)) == 0 && p.bt_stride > 0, "omni_latent_attn: block_size=%d (a power of two)", p.block_size);
     OMNI_CHECK_ARG(p.n_decode >= 0 && p.n_decode <= p.T && p.n_decode <= 65535 && p.n_tiles >= 0 && (p.n_tiles == 0 || p.tiles) && (p.n_decode == p.T || p.n_tiles > 0 || p.elem == 1),
                    "omni_latent_attn: T=%d n_decode=%d n_tiles=%d", p.T, p.n_decode, p.n_tiles);
+    OMNI_CHECK_ARG(p.n_tiles == 0 || p.tile_rows == 64 || p.tile_rows == 128, "omni_latent_attn: tile_rows=%d (64 or 128)", p.tile_rows);
     OMNI_CHECK_ARG(!p.workspace || p.workspace_bytes >= omni_latent_attn_workspace_bytes(p.n_decode, p.heads, p.rp), "omni_latent_attn: workspace of %lld bytes", (long long)p.workspace_bytes);
     if (p.T <= 0) return OMNI_OK;
     hipStream_t st = (hipStream_t)stream;

@@ -148,14 +148,20 @@ class Batch:
     num_live: torch.Tensor | None = None
 
 
-def attention_tiles(seg_starts: list[int], seg_lens: list[int], heads: int) -> list[tuple[int, int]]:
-    """Work items of the prompt attention: runs of up to LATENT_TILE query rows (token-major, heads inside) of ONE sequence.  Longest first:
-    a later tile of a prompt sees more keys."""
+def attention_tile_rows(n_rows: int) -> int:
+    """Query rows per work item of the prompt attention: 128 share a key tile's staging; while that leaves fewer items than keep 256 CUs busy and
+    balanced (a late tile of a prompt sees many more keys than an early one), 64."""
+    return 128 if n_rows >= 128 * 768 else 64
+
+
+def attention_tiles(seg_starts: list[int], seg_lens: list[int], heads: int, tile_rows: int) -> list[tuple[int, int]]:
+    """Work items of the prompt attention: runs of up to `tile_rows` query rows (token-major, heads inside) of ONE sequence.  Longest first: a later
+    tile of a prompt sees more keys."""
     out = []
     for s, n in zip(seg_starts, seg_lens):
         lo, hi = s * heads, (s + n) * heads
-        out += [(f, min(L.LATENT_TILE, hi - f)) for f in range(lo, hi, L.LATENT_TILE)]
-    return out[::-1]
+        out += [(lo - f, f, min(tile_rows, hi - f)) for f in range(lo, hi, tile_rows)]
+    return [(f, n) for _, f, n in sorted(out)]
 
 
 class DecoderEngine:
@@ -302,7 +308,7 @@ class DecoderEngine:
             starts.append(o)
             o += n
         assert o == T, (o, T)
-        tl = {h: attention_tiles(starts, seg_lens, h) for h in heads}
+        tl = {h: attention_tiles(starts, seg_lens, h, attention_tile_rows((T - n_decode) * h)) for h in heads}
         flat = [torch.as_tensor(ids, dtype=torch.int32), torch.as_tensor(row_of_tok, dtype=torch.int32), torch.as_tensor(positions, dtype=torch.int32)]
         flat += [torch.tensor(tl[h], dtype=torch.int32).reshape(-1) for h in heads]
         buf = torch.cat(flat).pin_memory().to(self.device, non_blocking=True)
@@ -336,7 +342,7 @@ class DecoderEngine:
         tiles = b.tiles.get(H)
         a = L.LatentAttn(q=s.ql.data_ptr(), cache=self.kv_caches[i].data_ptr(), gate=L.ptr(gate), out=s.ol.data_ptr(), block_table=self.block_table.data_ptr(),
                          bt_stride=self.bt_stride, block_size=self.block_size, row_of_tok=b.row_of_tok.data_ptr(), positions=b.positions.data_ptr(),
-                         tiles=L.ptr(tiles), n_tiles=0 if tiles is None else tiles.numel() // 2, T=T, n_decode=b.n_decode, heads=H, rp=w.rp, scale=m.scale,
+                         tiles=L.ptr(tiles), n_tiles=0 if tiles is None else tiles.numel() // 2, tile_rows=attention_tile_rows((T - b.n_decode) * H), T=T, n_decode=b.n_decode, heads=H, rp=w.rp, scale=m.scale,
                          max_keys=b.max_keys, workspace=self.attn_ws.data_ptr(), workspace_bytes=self.attn_ws.numel() * 4, elem=self.elem.code)
         L.check(lib.omni_latent_attn_run(C.byref(a), st), "omni_latent_attn", lib)
         self._heads_mm(s.ol, w.uv, s.v, T, H, out_frag=frag)

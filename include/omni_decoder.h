@@ -68,13 +68,12 @@ int omni_gemm_stream_splits(int M, int N, int K);
 /* Causal attention over a paged cache of latents shared by all heads (keys and values are the same rp-wide rows):
  *   out[t, h] = gate[t, h] * sum_j softmax_j(scale * q[t, h] . c_j) c_j,   j <= positions[t],   q / out elem [T, heads, rp].
  * Tokens [0, n_decode) are single-token sequences (one work item per 16 heads and KV split; workspace for the splits); the others are
- * covered by `tiles` (int32 [n_tiles][2], device: first flat row t * heads + h and row count <= OMNI_LATENT_TILE, one sequence each).
+ * covered by `tiles` (int32 [n_tiles][2], device: first flat row t * heads + h and row count <= tile_rows, 64 or 128; one sequence each).
  * max_keys bounds positions[t] + 1 of the decode tokens (split choice only).                                                        */
-#define OMNI_LATENT_TILE 128
 typedef struct omni_latent_attn {
     const void* q; const void* cache; const float* gate; void* out;
     const int32_t* block_table; int bt_stride, block_size; const int32_t* row_of_tok; const int32_t* positions;
-    const int32_t* tiles; int n_tiles;
+    const int32_t* tiles; int n_tiles, tile_rows;
     int T, n_decode, heads, rp; float scale; int max_keys; float* workspace; int64_t workspace_bytes; int elem;
 } omni_latent_attn;
 int omni_latent_attn_run(const omni_latent_attn* a, void* stream);

@@ -124,11 +124,11 @@ def test_state_slots_are_unique_and_come_back():
 
 
 def test_attention_tiles_cover_every_row_once_and_never_straddle_sequences():
-    for heads in (1, 3, 16, 40, 200):
+    for heads, rows in ((1, 64), (3, 128), (16, 64), (40, 128), (200, 64)):
         starts, lens = [2, 9, 140], [7, 131, 2]
         seen = []
-        for f, n in attention_tiles(starts, lens, heads):
-            assert 1 <= n <= 128
+        for f, n in attention_tiles(starts, lens, heads, rows):
+            assert 1 <= n <= rows
             owner = [k for k, (s, c) in enumerate(zip(starts, lens)) if s * heads <= f and f + n <= (s + c) * heads]
             assert len(owner) == 1
             seen += range(f, f + n)

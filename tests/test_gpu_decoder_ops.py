@@ -271,7 +271,7 @@ class Seqs:
             out.append(D.causal_softmax_attention(qq, kv, kv, scale)[n - k:])
         return torch.cat(out) * self.gate[:, :, None]
 
-    def run(self, scale, split=True):
+    def run(self, scale, split=True, tile_rows=64):
         """Single-token sequences first, as the engine orders them."""
         order = sorted(range(len(self.lens)), key=lambda r: self.new[r] > 1)
         ones = sum(1 for n in self.new if n == 1)
@@ -286,13 +286,13 @@ class Seqs:
         for n in seg:
             starts.append(o)
             o += n
-        tiles = dev(torch.tensor(attention_tiles(starts, seg, self.heads), dtype=torch.int32)) if seg else None
+        tiles = dev(torch.tensor(attention_tiles(starts, seg, self.heads, tile_rows), dtype=torch.int32)) if seg else None
         out = torch.full_like(q, float("nan"))
         nb = L.load_decoder().omni_latent_attn_workspace_bytes(max(ones, 1), self.heads, self.rp)
         ws = torch.full((nb // 4,), float("nan"), device="cuda") if split else None
         keep = [dev(self.cache), dev(self.gate[perm]), dev(self.bt), dev(row), dev(pos)]
         run_struct("omni_latent_attn_run", L.LatentAttn(), q=q, cache=keep[0], gate=keep[1], out=out, block_table=keep[2], bt_stride=self.bt.shape[1], block_size=self.bs,
-                   row_of_tok=keep[3], positions=keep[4], tiles=tiles, n_tiles=0 if tiles is None else len(tiles), T=T, n_decode=ones, heads=self.heads, rp=self.rp, scale=scale,
+                   row_of_tok=keep[3], positions=keep[4], tiles=tiles, n_tiles=0 if tiles is None else len(tiles), tile_rows=tile_rows, T=T, n_decode=ones, heads=self.heads, rp=self.rp, scale=scale,
                    max_keys=max([self.lens[r] for r in order[:ones]] or [0]), workspace=ws, workspace_bytes=nb if split else 0, elem=self.elem)
         torch.cuda.synchronize()
         res = torch.empty_like(out, device="cpu")
@@ -308,7 +308,9 @@ ATTN_TOL = {0: 8e-3, 1: 1e-5}
 def test_latent_attention_over_mixed_batches(elem, rp, heads):
     """Decoded tokens (one key, page borders, hundreds of keys) beside prompts and portions that start in the middle of a page or a tile."""
     s = Seqs([1, 16, 17, 300, 5, 33, 130, 97], [1, 1, 1, 1, 5, 33, 2, 40], heads, rp, elem, seed=rp + heads)
-    close(s.run(0.4), s.reference(0.4), ATTN_TOL[elem])
+    ref = s.reference(0.4)
+    for rows in (64, 128):
+        close(s.run(0.4, tile_rows=rows), ref, ATTN_TOL[elem])
 
 
 @pytest.mark.parametrize("elem,rp,heads", [(0, 64, 4), (0, 512, 16), (1, 64, 2)])
