@@ -198,6 +198,7 @@ DECODER_SIGNATURES = {
     "omni_latent_attn_run": (i32, [C.POINTER(LatentAttn), vp]),
     "omni_latent_attn_workspace_bytes": (i64, [i32, i32, i32]),
     "omni_latent_attn_mfma": (i32, [i32]),
+    "omni_latent_attn_tile_rows": (i32, [i32]),
     "omni_head_gemm": (i32, [vp, vp, vp, i32, i32, i32, i32, i32, vp]),
     "omni_gemm_f32": (i32, [vp, i32, i64, vp, i64, vp, i32, i64, i32, i32, i32, i32, i32, f32, f32, vp]),
     "omni_gemm_stream": (i32, [vp, vp, vp, i32, i32, i32, i32, i32, f32, f32, i32, vp]),

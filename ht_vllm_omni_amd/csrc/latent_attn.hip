@@ -12,8 +12,8 @@
 //   latent_decode_kernel   one token: up to 16 heads fill the 16 query rows.  Four waves take one 16-key tile each for the scores, agree on the
 //                          row maxima, and share the second product by output columns: no sums to merge across waves at the end.  The
 //                          next tiles travel in registers meanwhile.  KV splits leave records a small kernel merges
-//   latent_prefill_kernel  tiles of up to 64 or 128 query rows of one sequence, 16 per wave; the waves share each 32-key tile (double-buffered,
-//                          one barrier per tile)
+//   latent_prefill_kernel  tiles of up to la_tile_rows() query rows of one sequence, 16 per wave; the waves share each 32-key tile
+//                          (double-buffered, one barrier per tile)
 //   latent_plain_kernel    any width, bf16 or fp32: one wave per query row on the vector units (the 32-bit mode)
 #include "common.cuh"
 #include "gemm_frag.cuh"
@@ -427,6 +427,11 @@ __global__ __launch_bounds__(64) void latent_plain_kernel(const E* __restrict__ 
 }
 
 // ---- host side
+// query rows per prompt work item.  Measured (16 heads, 1 x 2048 / 16 x 128 / 4 x 2048 tokens): width 512 by 128 rows 277 / 36 / 652 us, by 64 307 / 42 /
+// 750; width 256 by 128 rows 162 / 22 / 370, by 64 -- two workgroups fit a CU -- 129 / 18 / 340
+static constexpr int la_tile_rows(int rp) { return rp > 256 ? 128 : 64; }
+extern "C" int omni_latent_attn_tile_rows(int rp) { return la_tile_rows(rp); }
+
 static int la_splits(int n_decode, int heads, int max_keys) {
     const int wgs = n_decode * ((heads + 15) / 16);
     int ns = 512 / (wgs > 0 ? wgs : 1);                 // two workgroups per CU
@@ -472,12 +477,10 @@ static int la_run(const omni_latent_attn& p, LatentArgs a, hipStream_t st) {
         }
     }
     if (p.n_tiles > 0) {
-        constexpr int LDS = 2 * G::TILE;
-        static const int rc8 = la_lds(latent_prefill_kernel<RS, 8>, LDS), rc4 = la_lds(latent_prefill_kernel<RS, 4>, LDS);
-        if (rc8 != OMNI_OK) return rc8;
-        if (rc4 != OMNI_OK) return rc4;
-        if (p.tile_rows == 64) hipLaunchKernelGGL((latent_prefill_kernel<RS, 4>), dim3(p.n_tiles), dim3(256), LDS, st, a);
-        else hipLaunchKernelGGL((latent_prefill_kernel<RS, 8>), dim3(p.n_tiles), dim3(512), LDS, st, a);
+        constexpr int PW = la_tile_rows(RS * 32) / 16, LDS = 2 * G::TILE;
+        static const int rc = la_lds(latent_prefill_kernel<RS, PW>, LDS);
+        if (rc != OMNI_OK) return rc;
+        hipLaunchKernelGGL((latent_prefill_kernel<RS, PW>), dim3(p.n_tiles), dim3(64 * PW), LDS, st, a);
         OMNI_CHECK_LAUNCH("omni_latent_attn(prefill)");
     }
     return OMNI_OK;
@@ -490,7 +493,7 @@ extern "C" int omni_latent_attn_run(const omni_latent_attn* pp, void* stream) {
     OMNI_CHECK_ARG(p.block_size > 0 && (p.block_size & (p.block_size - 1)) == 0 && p.bt_stride > 0, "omni_latent_attn: block_size=%d (a power of two)", p.block_size);
     OMNI_CHECK_ARG(p.n_decode >= 0 && p.n_decode <= p.T && p.n_decode <= 65535 && p.n_tiles >= 0 && (p.n_tiles == 0 || p.tiles) && (p.n_decode == p.T || p.n_tiles > 0 || p.elem == 1),
                    "omni_latent_attn: T=%d n_decode=%d n_tiles=%d", p.T, p.n_decode, p.n_tiles);
-    OMNI_CHECK_ARG(p.n_tiles == 0 || p.tile_rows == 64 || p.tile_rows == 128, "omni_latent_attn: tile_rows=%d (64 or 128)", p.tile_rows);
+    OMNI_CHECK_ARG(p.n_tiles == 0 || p.tile_rows == la_tile_rows(p.rp), "omni_latent_attn: tile_rows=%d (omni_latent_attn_tile_rows(%d) = %d)", p.tile_rows, p.rp, la_tile_rows(p.rp));
     OMNI_CHECK_ARG(!p.workspace || p.workspace_bytes >= omni_latent_attn_workspace_bytes(p.n_decode, p.heads, p.rp), "omni_latent_attn: workspace of %lld bytes", (long long)p.workspace_bytes);
     if (p.T <= 0) return OMNI_OK;
     hipStream_t st = (hipStream_t)stream;

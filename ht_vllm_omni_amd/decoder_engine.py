@@ -137,21 +137,15 @@ class _Scratch:
 
 @dataclass
 class Batch:
-    """One forward's tokens (device tensors).  Tokens [0, n_decode) are single-token sequences; `tiles` covers the rest per head count."""
+    """One forward's tokens (device tensors).  Tokens [0, n_decode) are single-token sequences; `tiles` covers the rest per (head count, rows of a work item)."""
     T: int
     n_decode: int
     ids: torch.Tensor                   # int32 [T]
     row_of_tok: torch.Tensor            # int32 [T]
     positions: torch.Tensor             # int32 [T]
-    tiles: dict[int, torch.Tensor]      # heads -> int32 [n, 2]
+    tiles: dict[tuple, torch.Tensor]    # (heads, tile rows) -> int32 [2 n]
     max_keys: int                       # most keys a decode token sees
     num_live: torch.Tensor | None = None
-
-
-def attention_tile_rows(n_rows: int) -> int:
-    """Query rows per work item of the prompt attention: 128 share a key tile's staging; while that leaves fewer items than keep 256 CUs busy and
-    balanced (a late tile of a prompt sees many more keys than an early one), 64."""
-    return 128 if n_rows >= 128 * 768 else 64
 
 
 def attention_tiles(seg_starts: list[int], seg_lens: list[int], heads: int, tile_rows: int) -> list[tuple[int, int]]:
@@ -187,6 +181,8 @@ class DecoderEngine:
         self.head = _Matrix(pad2(weights["head"], r32(dims.vocab), self.width), self.elem, dev)
         self.final_gain = float(weights["final.norm"])
         self.layer_w = {i: _Layer(dims, i, weights, self.elem, dev) for i in range(dims.num_layers) if dims.owner(i) == i}
+        # per layer: heads and query rows per work item of its prompt attention
+        self.tile_kinds = [(s.mixer.heads, self.lib.omni_latent_attn_tile_rows(self.layer_w[dims.owner(i)].rp)) for i, s in enumerate(dims.layers)]
         self._alloc_kv(num_blocks)
         # ---- per-sequence state: what each layer's mixer read at the sequence's last token; slot 0 belongs to no sequence
         self.state_slots = max_batch + 1
@@ -302,20 +298,20 @@ class DecoderEngine:
     def make_batch(self, ids: torch.Tensor, row_of_tok, positions, seg_lens: list[int], *, n_decode: int = 0, max_keys: int = 0, ids_device=None) -> Batch:
         """A batch from host arrays: tokens [0, n_decode) single-token sequences, then segments of `seg_lens` tokens.  One upload."""
         T = len(row_of_tok)
-        heads = sorted({s.mixer.heads for s in self.d.layers}) if T > n_decode else []
+        kinds = sorted(set(self.tile_kinds)) if T > n_decode else []
         starts, o = [], n_decode
         for n in seg_lens:
             starts.append(o)
             o += n
         assert o == T, (o, T)
-        tl = {h: attention_tiles(starts, seg_lens, h, attention_tile_rows((T - n_decode) * h)) for h in heads}
+        tl = {k: attention_tiles(starts, seg_lens, *k) for k in kinds}
         flat = [torch.as_tensor(ids, dtype=torch.int32), torch.as_tensor(row_of_tok, dtype=torch.int32), torch.as_tensor(positions, dtype=torch.int32)]
-        flat += [torch.tensor(tl[h], dtype=torch.int32).reshape(-1) for h in heads]
+        flat += [torch.tensor(tl[k], dtype=torch.int32).reshape(-1) for k in kinds]
         buf = torch.cat(flat).pin_memory().to(self.device, non_blocking=True)
         tiles, o = {}, 3 * T
-        for h in heads:
-            n = 2 * len(tl[h])
-            tiles[h] = buf[o:o + n]
+        for k in kinds:
+            n = 2 * len(tl[k])
+            tiles[k] = buf[o:o + n]
             o += n
         return Batch(T, n_decode, buf[:T] if ids_device is None else ids_device, buf[T:2 * T], buf[2 * T:3 * T], tiles, max_keys)
 
@@ -339,10 +335,10 @@ class DecoderEngine:
         L.check(lib.omni_latent_write_run(C.byref(a), st), "omni_latent_write", lib)
         self._mm(s.cq, w.uq, s.q, T)
         self._heads_mm(s.q, w.uk, s.ql, T, H)
-        tiles = b.tiles.get(H)
+        tiles = b.tiles.get(self.tile_kinds[i])
         a = L.LatentAttn(q=s.ql.data_ptr(), cache=self.kv_caches[i].data_ptr(), gate=L.ptr(gate), out=s.ol.data_ptr(), block_table=self.block_table.data_ptr(),
                          bt_stride=self.bt_stride, block_size=self.block_size, row_of_tok=b.row_of_tok.data_ptr(), positions=b.positions.data_ptr(),
-                         tiles=L.ptr(tiles), n_tiles=0 if tiles is None else tiles.numel() // 2, tile_rows=attention_tile_rows((T - b.n_decode) * H), T=T, n_decode=b.n_decode, heads=H, rp=w.rp, scale=m.scale,
+                         tiles=L.ptr(tiles), n_tiles=0 if tiles is None else tiles.numel() // 2, tile_rows=self.tile_kinds[i][1], T=T, n_decode=b.n_decode, heads=H, rp=w.rp, scale=m.scale,
                          max_keys=b.max_keys, workspace=self.attn_ws.data_ptr(), workspace_bytes=self.attn_ws.numel() * 4, elem=self.elem.code)
         L.check(lib.omni_latent_attn_run(C.byref(a), st), "omni_latent_attn", lib)
         self._heads_mm(s.ol, w.uv, s.v, T, H, out_frag=frag)

@@ -68,7 +68,8 @@ int omni_gemm_stream_splits(int M, int N, int K);
 /* Causal attention over a paged cache of latents shared by all heads (keys and values are the same rp-wide rows):
  *   out[t, h] = gate[t, h] * sum_j softmax_j(scale * q[t, h] . c_j) c_j,   j <= positions[t],   q / out elem [T, heads, rp].
  * Tokens [0, n_decode) are single-token sequences (one work item per 16 heads and KV split; workspace for the splits); the others are
- * covered by `tiles` (int32 [n_tiles][2], device: first flat row t * heads + h and row count <= tile_rows, 64 or 128; one sequence each).
+ * covered by `tiles` (int32 [n_tiles][2], device: first flat row t * heads + h and row count <= tile_rows; one sequence each;
+ * tile_rows = omni_latent_attn_tile_rows(rp)).
  * max_keys bounds positions[t] + 1 of the decode tokens (split choice only).                                                        */
 typedef struct omni_latent_attn {
     const void* q; const void* cache; const float* gate; void* out;
@@ -78,6 +79,7 @@ typedef struct omni_latent_attn {
 } omni_latent_attn;
 int omni_latent_attn_run(const omni_latent_attn* a, void* stream);
 int64_t omni_latent_attn_workspace_bytes(int n_decode, int heads, int rp);
+int omni_latent_attn_tile_rows(int rp);
 /* 1 when the matrix-core kernels take this padded latent width (else the plain kernel runs it) */
 int omni_latent_attn_mfma(int rp);
 
