@@ -36,8 +36,8 @@ struct LatentArgs {
     float* partial; int nsplit;
 };
 
-// KV splits a row of `ntiles` 16-key tiles uses, of the nsplit the launch offers: fewer than six tiles are not worth a split of their own
-__device__ __forceinline__ int la_row_splits(int ntiles, int nsplit) { return min(nsplit, (ntiles + 5) / 6); }
+// KV splits a row of `ntiles` 16-key tiles uses, of the nsplit the launch offers: two rounds of the four waves each, or more
+__device__ __forceinline__ int la_row_splits(int ntiles, int nsplit) { return min(nsplit, (ntiles + 7) / 8); }
 
 template <int RS>
 struct LatentGeom {
