@@ -7,7 +7,7 @@
                            csrc/debug.hip (launch / memory-system probes): scripts/ and the tile-sweep tests only
 
 All are git-ignored but travel with the repo snapshot.  `sources_digest()` is stamped into a side file next to each
-library so that _lib.load() can refuse a library that is older than csrc/ (ADVICE r1).
+library so that _lib.load() can refuse a library that is older than csrc/.
 """
 from __future__ import annotations
 
@@ -25,7 +25,7 @@ LIB_DEBUG = os.path.join(HERE, "libomni_talker_debug.so")
 SOURCES = ["errors.hip", "capi.hip", "gemm.hip", "gemm_prefill.hip", "norm.hip", "rope_kv.hip", "paged_attn.hip", "prefill_attn.hip", "moe.hip",
            "sampler.hip", "cp_chain.hip", "bb_chain.hip", "moe_chain.hip", "allreduce.hip", "codec.hip", "conv_unit.hip"]
 DECODER_SOURCES = ["errors.hip", "gemm_prefill.hip", "sampler.hip", "decoder_rows.hip", "gemm_stream.hip", "head_gemm.hip", "latent_attn.hip"]
-# debug library only: the probes, and the losing A/B arms of the backbone chain (rounds 3 and 4; no product knob reaches them)
+# debug library only: the probes, and the losing A/B arms of the backbone chain (no product knob reaches them)
 DEBUG_ONLY = ["debug.hip", "bb_engine.hip", "bb_all.hip"]
 # per-file extra flags
 EXTRA = {"debug.hip": ["-mllvm", "-amdgpu-kernarg-preload-count=16"]}
