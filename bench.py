@@ -335,7 +335,7 @@ def decoder_bench(args):
                     b = eng.make_batch(torch.randint(0, dd.vocab, (T,), dtype=torch.int32), row, pos, [n] * seqs)
                     last = (torch.arange(1, seqs + 1) * n - 1).to(torch.int32).cuda()
                     ms = eager_ms(lambda: eng.forward(b, sel=last))
-                    per_tok = sum(2 * t.numel() for l in eng.layer_w.values() for t in (l.down.t, l.uq.t, l.uk.t, l.uv.t, l.o.t, l.up.t, l.dn.t))
+                    per_tok = sum(2 * m.t.numel() for l in eng.layer_w.values() for m in l.mats)
                     attn = sum(4 * m.heads * m.kv_rank for m in mix)
                 else:
                     x = torch.randn(T, td.hidden, device="cuda").to(torch.bfloat16)

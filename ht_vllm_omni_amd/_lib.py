@@ -46,17 +46,24 @@ class TileGemm(C.Structure):
                 ("w", vp), ("bias", vp), ("scale", vp), ("act", i32), ("resid", vp), ("ldr", i32), ("out_f32", vp), ("ldf", i32), ("out", vp), ("ldo", i32),
                 ("out2", vp), ("ldo2", i32), ("snake_alpha", vp), ("snake_inv_beta", vp), ("M", i32), ("N", i32), ("K", i32), ("tile_hint", i32),
                 ("groups", i32), ("x_group_rows", i64), ("w_group_elems", i64), ("out_group_rows", i64), ("group_rows", vp),
-                ("act_p", f32), ("act_n", f32), ("x_group_cols", i64), ("out_group_cols", i64)]
+                ("act_p", f32), ("act_n", f32), ("x_group_cols", i64), ("out_group_cols", i64),
+                ("act_cols", i32), ("mul_table", vp), ("mul_ids", vp), ("mul_rows", i32), ("mul_ld", i32)]
 
 
-TILE_ACT_NONE, TILE_ACT_GELU, TILE_ACT_SILU_MUL_GU8, TILE_ACT_XIELU = 0, 1, 2, 3
+TILE_ACT_NONE, TILE_ACT_GELU, TILE_ACT_SILU_MUL_GU8, TILE_ACT_XIELU, TILE_ACT_RELU2, TILE_ACT_SILU_SIGMOID, TILE_ACT_GELU_MUL = range(7)
+
+
+class RowTable(C.Structure):
+    """omni_row_table (include/omni_decoder.h): a table whose row ids[m] multiplies output row m of a product."""
+    _fields_ = [("table", vp), ("ids", vp), ("rows", i32), ("ld", i32)]
 
 
 class StreamRows(C.Structure):
     """omni_stream_rows (include/omni_decoder.h)."""
     _fields_ = [("ids", vp), ("table", vp), ("vocab", i32), ("x_in", vp), ("y", vp), ("y_slabs", i32), ("y_stride", i64), ("gain", f32), ("eps", f32), ("mu", vp), ("state", vp),
                 ("state_slot", vp), ("row_of_tok", vp), ("positions", vp), ("use_final", i32), ("final_gain", f32), ("sel", vp), ("x_out", vp),
-                ("h_out", vp), ("frag", i32), ("rows", i32), ("width", i32), ("wp", i32), ("elem", i32)]
+                ("h_out", vp), ("frag", i32), ("rows", i32), ("width", i32), ("wp", i32), ("elem", i32),
+                ("table_scale", f32), ("post", i32), ("alpha", f32), ("y_w", vp), ("final_w", vp)]
 
 
 class LatentWrite(C.Structure):
@@ -74,7 +81,36 @@ class LatentAttn(C.Structure):
                 ("scale", f32), ("max_keys", i32), ("workspace", vp), ("workspace_bytes", i64), ("elem", i32)]
 
 
-STREAM_F32, STREAM_BF16, STREAM_XIELU = 0, 1, 2      # omni_gemm_stream kinds
+class QkvWrite(C.Structure):
+    """omni_qkv_write."""
+    _fields_ = [("proj", vp), ("slabs", i32), ("slab_stride", i64), ("ld", i32), ("heads", i32), ("kv_heads", i32), ("dim", i32), ("dp", i32), ("vp", i32),
+                ("qw", vp), ("kw", vp), ("eps", f32), ("rot", vp), ("rot_dims", i32), ("rot_rows", i32), ("q", vp), ("kc", vp), ("vc", vp), ("gate", vp),
+                ("block_table", vp), ("bt_stride", i32), ("block_size", i32), ("row_of_tok", vp), ("positions", vp), ("num_live", vp), ("T", i32), ("elem", i32)]
+
+
+class GatedNorm(C.Structure):
+    """omni_gated_norm."""
+    _fields_ = [("o", vp), ("w", vp), ("gate", vp), ("slabs", i32), ("slab_stride", i64), ("ld", i32), ("n", i32), ("count", i32), ("eps", f32), ("out", vp),
+                ("frag", i32), ("T", i32), ("elem", i32)]
+
+
+class WindowAttn(C.Structure):
+    """omni_window_attn."""
+    _fields_ = [("q", vp), ("kc", vp), ("vc", vp), ("gate", vp), ("sink", vp), ("out", vp), ("frag", i32), ("block_table", vp), ("bt_stride", i32), ("block_size", i32),
+                ("row_of_tok", vp), ("positions", vp), ("tiles", vp), ("n_tiles", i32), ("tile_rows", i32), ("T", i32), ("n_decode", i32), ("heads", i32), ("kv_heads", i32),
+                ("dp", i32), ("vp", i32), ("scale", f32), ("window", i32), ("max_keys", i32), ("workspace", vp), ("workspace_bytes", i64), ("elem", i32)]
+
+
+class DecayRec(C.Structure):
+    """omni_decay_rec."""
+    _fields_ = [("proj", vp), ("slabs", i32), ("slab_stride", i64), ("ld", i32), ("heads", i32), ("dp", i32), ("vp", i32), ("decay", vp), ("log2_decay", vp),
+                ("state", vp), ("state_slot", vp), ("row_of_tok", vp), ("positions", vp), ("num_live", vp), ("n_decode", i32), ("runs", vp), ("n_runs", i32),
+                ("chunks", vp), ("n_chunks", i32), ("segs", vp), ("n_segs", i32), ("chunk_states", vp), ("out", vp)]
+
+
+STREAM_F32, STREAM_BF16, STREAM_XIELU, STREAM_RELU2 = 0, 1, 2, 3      # omni_gemm_stream kinds
+ACT_NONE, ACT_XIELU, ACT_RELU2, ACT_GELU_MUL = 0, 1, 2, 3            # OMNI_ACT_*
+REC_CHUNK, REC_MAX_DIM = 128, 256                                    # OMNI_REC_*
 STREAM_MAX_SPLITS = 4
 
 
@@ -203,6 +239,14 @@ DECODER_SIGNATURES = {
     "omni_gemm_f32": (i32, [vp, i32, i64, vp, i64, vp, i32, i64, i32, i32, i32, i32, i32, f32, f32, vp]),
     "omni_gemm_stream": (i32, [vp, vp, vp, i32, i32, i32, i32, i32, f32, f32, i32, vp]),
     "omni_gemm_stream_splits": (i32, [i32, i32, i32]),
+    "omni_gemm_stream_rows": (i32, [vp, vp, vp, i32, i32, i32, C.POINTER(RowTable), i32, vp]),
+    "omni_gemm_f32_rows": (i32, [vp, i32, vp, vp, i32, i32, i32, i32, C.POINTER(RowTable), vp]),
+    "omni_qkv_write_run": (i32, [C.POINTER(QkvWrite), vp]),
+    "omni_gated_norm_run": (i32, [C.POINTER(GatedNorm), vp]),
+    "omni_window_attn_run": (i32, [C.POINTER(WindowAttn), vp]),
+    "omni_window_attn_workspace_bytes": (i64, [i32, i32, i32]),
+    "omni_window_attn_tile_rows": (i32, [i32, i32]),
+    "omni_decay_rec_run": (i32, [C.POINTER(DecayRec), vp]),
     "omni_sample_step": (i32, [vp, i32, i32, i32, C.POINTER(RowSampling), vp, vp, vp, vp, vp, vp, vp]),
 }
 

@@ -24,7 +24,8 @@ LIB_DECODER = os.path.join(HERE, "libomni_decoder.so")
 LIB_DEBUG = os.path.join(HERE, "libomni_talker_debug.so")
 SOURCES = ["errors.hip", "capi.hip", "gemm.hip", "gemm_prefill.hip", "norm.hip", "rope_kv.hip", "paged_attn.hip", "prefill_attn.hip", "moe.hip",
            "sampler.hip", "cp_chain.hip", "bb_chain.hip", "moe_chain.hip", "allreduce.hip", "codec.hip", "conv_unit.hip"]
-DECODER_SOURCES = ["errors.hip", "gemm_prefill.hip", "sampler.hip", "decoder_rows.hip", "gemm_stream.hip", "head_gemm.hip", "latent_attn.hip"]
+DECODER_SOURCES = ["errors.hip", "gemm_prefill.hip", "sampler.hip", "decoder_rows.hip", "gemm_stream.hip", "head_gemm.hip", "latent_attn.hip",
+                   "window_attn.hip", "decay_rec.hip"]
 # debug library only: the probes, and the losing A/B arms of the backbone chain (no product knob reaches them)
 DEBUG_ONLY = ["debug.hip", "bb_engine.hip", "bb_all.hip"]
 # per-file extra flags

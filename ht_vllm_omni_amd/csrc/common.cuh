@@ -159,6 +159,11 @@ __device__ __forceinline__ float xielu(float z, float ap, float an) {
     return fmaf(0.5f, z, z > 0.f ? ap * z * z : an * (expm1f(fminf(z, 0.f)) - z));
 }
 
+// ---- the other activations of the language models' products
+__device__ __forceinline__ float relu2(float z) { z = fmaxf(z, 0.f); return z * z; }
+__device__ __forceinline__ float gelu_tanh(float z) { return 0.5f * z * (1.0f + tanhf(0.79788456080286536f * fmaf(0.044715f * z * z, z, z))); }
+__device__ __forceinline__ float sigmoidf_(float z) { return 1.0f / (1.0f + expf(-z)); }
+
 // ---- OCP e4m3fn <-> f32 (saturating, round-nearest-even: clamp then hardware cvt)
 #define OMNI_FP8_MAX 448.0f
 __device__ __forceinline__ uint32_t pack_fp8x4(float a, float b, float c, float d) {

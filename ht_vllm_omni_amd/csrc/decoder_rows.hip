@@ -68,6 +68,8 @@ __global__ __launch_bounds__(DR_THREADS) void stream_rows_kernel(const omni_stre
     const int wp = a.wp;
     const E* table = reinterpret_cast<const E*>(a.table);
     const E* mu = reinterpret_cast<const E*>(a.mu);
+    const E* yw = reinterpret_cast<const E*>(a.y_w);
+    const E* fw = reinterpret_cast<const E*>(a.final_w);
     E* h_out = reinterpret_cast<E*>(a.h_out);
     auto load_new = [&](int t, float (&v)[MAXC][4]) {      // the stream row of token t behind the sublayer that just ran
         if (a.ids) {
@@ -78,6 +80,10 @@ __global__ __launch_bounds__(DR_THREADS) void stream_rows_kernel(const omni_stre
                 const int k = (c * DR_THREADS + threadIdx.x) * 4;
                 v[c][0] = v[c][1] = v[c][2] = v[c][3] = 0.f;
                 if (ok && k < wp) ld4<E>(table + (size_t)id * wp + k, v[c]);
+                if (a.table_scale != 0.f) {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) v[c][e] *= a.table_scale;
+                }
             }
             return;
         }
@@ -93,14 +99,28 @@ __global__ __launch_bounds__(DR_THREADS) void stream_rows_kernel(const omni_stre
             }
         }
         if (!a.y) return;
+        if (a.post) {                                      // the norm takes the sum, not the sublayer's output
+#pragma unroll
+            for (int c = 0; c < MAXC; ++c)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) { y[c][e] = fmaf(a.alpha, v[c][e], y[c][e]); v[c][e] = 0.f; }
+        }
 #pragma unroll
         for (int c = 0; c < MAXC; ++c) ss += sq4_sum(y[c][0], y[c][1], y[c][2], y[c][3]);
         ss = bsum(ss);
-        const float r = a.gain / sqrtf(ss / (float)a.width + a.eps);
+        const float r = (yw ? 1.0f : a.gain) / sqrtf(ss / (float)a.width + a.eps);
 #pragma unroll
-        for (int c = 0; c < MAXC; ++c)
+        for (int c = 0; c < MAXC; ++c) {
+            if (yw) {
+                const int k = (c * DR_THREADS + threadIdx.x) * 4;
+                float w[4] = {0.f, 0.f, 0.f, 0.f};
+                if (k < wp) ld4<E>(yw + k, w);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) y[c][e] *= w[e];
+            }
 #pragma unroll
             for (int e = 0; e < 4; ++e) v[c][e] = fmaf(y[c][e], r, v[c][e]);
+        }
     };
     const int i0 = blockIdx.x * strip, i1 = min(i0 + strip, a.rows);
     float cur[MAXC][4], prev[MAXC][4];
@@ -133,7 +153,7 @@ __global__ __launch_bounds__(DR_THREADS) void stream_rows_kernel(const omni_stre
             float ss = 0.f;
 #pragma unroll
             for (int c = 0; c < MAXC; ++c) ss += sq4_sum(cur[c][0], cur[c][1], cur[c][2], cur[c][3]);
-            rf = a.final_gain / sqrtf(bsum(ss) / (float)a.width + a.eps);
+            rf = (fw ? 1.0f : a.final_gain) / sqrtf(bsum(ss) / (float)a.width + a.eps);
         }
 #pragma unroll
         for (int c = 0; c < MAXC; ++c) {
@@ -150,6 +170,12 @@ __global__ __launch_bounds__(DR_THREADS) void stream_rows_kernel(const omni_stre
             } else {
 #pragma unroll
                 for (int e = 0; e < 4; ++e) h[e] = a.use_final ? cur[c][e] * rf : cur[c][e];
+                if (a.use_final && fw) {
+                    float w[4];
+                    ld4<E>(fw + k, w);
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) h[e] *= w[e];
+                }
             }
             st4<E>(h_out + (a.frag ? frag_off(i, k, wp) : (size_t)i * wp + k), h);
         }
@@ -183,6 +209,7 @@ extern "C" int omni_stream_rows_run(const omni_stream_rows* p, void* stream) {
     OMNI_CHECK_ARG(!a.frag || a.elem == 0, "omni_stream_rows: fragment-major output is bf16");
     OMNI_CHECK_ARG(!a.mu || (a.state && a.state_slot && a.row_of_tok && a.positions && !a.sel && !a.use_final), "omni_stream_rows: token shift needs state, rows and positions, and no selection");
     OMNI_CHECK_ARG(!a.sel || !a.x_out, "omni_stream_rows: a selection writes h only");
+    OMNI_CHECK_ARG(!a.post || (a.y && !a.ids), "omni_stream_rows: the norm behind the sum needs y");
     // (a strip's first token and the shift read rows of x_in that another workgroup may already have rewritten: never in place)
     OMNI_CHECK_ARG(a.x_out == nullptr || a.x_out != a.x_in, "omni_stream_rows: x_out must not be x_in");
     if (a.rows <= 0) return OMNI_OK;
@@ -266,5 +293,171 @@ extern "C" int omni_latent_write_run(const omni_latent_write* p, void* stream) {
     if (a.elem) hipLaunchKernelGGL(latent_write_kernel<float>, dim3(a.T), dim3(DR_THREADS), lds, (hipStream_t)stream, a);
     else hipLaunchKernelGGL(latent_write_kernel<uint16_t>, dim3(a.T), dim3(DR_THREADS), lds, (hipStream_t)stream, a);
     OMNI_CHECK_LAUNCH("omni_latent_write");
+    return OMNI_OK;
+}
+
+// ---- grouped attention: norms over whole projections, rotation, cache write, gate.  One workgroup per token; q and k stay in LDS between the norm's
+// sum and the rotation (a pair's other half belongs to another thread)
+template <typename E>
+__global__ __launch_bounds__(DR_THREADS) void qkv_write_kernel(const omni_qkv_write a) {
+    extern __shared__ __attribute__((aligned(16))) float sp[];     // [q | k] of the token, partial sums added up
+    __shared__ float red[2][DR_WAVES];
+    const int t = blockIdx.x;
+    const int row = a.row_of_tok[t], pos = a.positions[t];
+    const bool live = !a.num_live || row < *a.num_live;
+    const int nq = a.heads * a.dp, nk = a.kc ? a.kv_heads * a.dp : 0, nv = a.kc ? a.kv_heads * a.vp : 0, ng = a.heads * a.vp;
+    const float* y = a.proj + (size_t)t * a.ld;
+    // cache rows of this token: head g at base + g * block_size
+    const size_t base = a.kc ? (size_t)a.block_table[(size_t)row * a.bt_stride + pos / a.block_size] * a.kv_heads * a.block_size + pos % a.block_size : 0;
+    float sq = 0.f, sk = 0.f;
+    for (int k = threadIdx.x * 4; k < nq + nk; k += DR_THREADS * 4) {
+        float v[4];
+        ld4_slabs(y + k, a.slabs, a.slab_stride, v);
+        st4<float>(sp + k, v);
+        const float ss = sq4_sum(v[0], v[1], v[2], v[3]);
+        if (k < nq) sq += ss;
+        else sk += ss;
+    }
+    if (a.kc && live)
+        for (int k = threadIdx.x * 4; k < nv; k += DR_THREADS * 4) {
+            float v[4];
+            ld4_slabs(y + nq + nk + k, a.slabs, a.slab_stride, v);
+            const int g = k / a.vp, d = k - g * a.vp;
+            st4<E>(reinterpret_cast<E*>(a.vc) + (base + (size_t)g * a.block_size) * a.vp + d, v);
+        }
+    if (a.gate)
+        for (int k = threadIdx.x * 4; k < ng; k += DR_THREADS * 4) {
+            float v[4];
+            ld4_slabs(y + nq + nk + nv + k, a.slabs, a.slab_stride, v);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = 1.0f / (1.0f + expf(-v[e]));
+            st4<E>(reinterpret_cast<E*>(a.gate) + (size_t)t * ng + k, v);
+        }
+    sq = wave_sum(sq);
+    sk = wave_sum(sk);
+    if ((threadIdx.x & 63) == 0) { red[0][threadIdx.x >> 6] = sq; red[1][threadIdx.x >> 6] = sk; }
+    __syncthreads();
+    sq = sk = 0.f;
+#pragma unroll
+    for (int w = 0; w < DR_WAVES; ++w) { sq += red[0][w]; sk += red[1][w]; }
+    const float rq = a.qw ? 1.0f / sqrtf(sq / (float)(a.heads * a.dim) + a.eps) : 1.0f;
+    const float rk = a.kw ? 1.0f / sqrtf(sk / (float)(a.kv_heads * a.dim) + a.eps) : 1.0f;
+    const int half = a.rot_dims >> 1;
+    const float* cs = a.rot + (size_t)min(pos, a.rot_rows - 1) * a.rot_dims;
+    for (int k = threadIdx.x * 4; k < nq + nk; k += DR_THREADS * 4) {
+        const bool key = k >= nq;
+        if (key && !live) break;
+        const int kk = key ? k - nq : k, hd = kk / a.dp, d0 = kk - hd * a.dp;
+        const E* w = reinterpret_cast<const E*>(key ? a.kw : a.qw);
+        const float r = key ? rk : rq;
+        const float* s = sp + (key ? nq : 0) + hd * a.dp;
+        auto normed = [&](int d) {
+            float wd = 1.0f;
+            if (w) {
+                if constexpr (sizeof(E) == 4) wd = w[hd * a.dp + d];
+                else wd = bf2f(w[hd * a.dp + d]);
+            }
+            return s[d] * r * wd;
+        };
+        float v[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int d = d0 + e;
+            v[e] = normed(d);
+            if (d < a.rot_dims) {
+                const bool lo = d < half;
+                const float o = normed(lo ? d + half : d - half);
+                const float2 c = *reinterpret_cast<const float2*>(cs + 2 * (lo ? d : d - half));
+                v[e] = lo ? fmaf(v[e], c.x, -(o * c.y)) : fmaf(v[e], c.x, o * c.y);
+            }
+        }
+        if (key) st4<E>(reinterpret_cast<E*>(a.kc) + (base + (size_t)hd * a.block_size) * a.dp + d0, v);
+        else st4<E>(reinterpret_cast<E*>(a.q) + (size_t)t * nq + k, v);
+    }
+}
+
+template <typename E>
+static int qkv_write_launch(const omni_qkv_write& a, size_t lds, hipStream_t st) {
+    if (lds > 60 * 1024) {
+        static const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(qkv_write_kernel<E>), hipFuncAttributeMaxDynamicSharedMemorySize, 156 * 1024);
+        if (e != hipSuccess) { omni_set_error("omni_qkv_write: LDS attribute: %s", hipGetErrorString(e)); return OMNI_EHIP; }
+    }
+    hipLaunchKernelGGL(qkv_write_kernel<E>, dim3(a.T), dim3(DR_THREADS), lds, st, a);
+    OMNI_CHECK_LAUNCH("omni_qkv_write");
+    return OMNI_OK;
+}
+
+extern "C" int omni_qkv_write_run(const omni_qkv_write* p, void* stream) {
+    OMNI_CHECK_ARG(p && p->proj && p->q && p->row_of_tok && p->positions && (!p->kc == !p->vc), "omni_qkv_write: null pointer");
+    const omni_qkv_write& a = *p;
+    OMNI_CHECK_ARG(a.heads > 0 && a.kv_heads > 0 && a.heads % a.kv_heads == 0 && a.dim > 0 && a.dp >= a.dim && a.dp % 32 == 0 && a.vp > 0 && a.vp % 32 == 0,
+                   "omni_qkv_write: heads %d / %d, dim %d / %d, vp %d", a.heads, a.kv_heads, a.dim, a.dp, a.vp);
+    const int need = a.heads * a.dp + (a.kc ? a.kv_heads * (a.dp + a.vp) : 0) + (a.gate ? a.heads * a.vp : 0);
+    OMNI_CHECK_ARG(a.ld >= need && a.ld % 4 == 0, "omni_qkv_write: ld=%d (>= %d)", a.ld, need);
+    OMNI_CHECK_ARG(a.rot_dims >= 0 && a.rot_dims % 2 == 0 && a.rot_dims <= a.dim && (a.rot_dims == 0 || (a.rot && a.rot_rows > 0)), "omni_qkv_write: rot_dims=%d of %d", a.rot_dims, a.dim);
+    OMNI_CHECK_ARG(!a.kc || (a.block_table && a.block_size > 0 && a.bt_stride > 0), "omni_qkv_write: block_size=%d bt_stride=%d", a.block_size, a.bt_stride);
+    OMNI_CHECK_ARG(a.slabs <= OMNI_STREAM_MAX_SPLITS && (a.elem == 0 || a.elem == 1), "omni_qkv_write: slabs=%d elem=%d", a.slabs, a.elem);
+    const size_t lds = ((size_t)a.heads * a.dp + (a.kc ? (size_t)a.kv_heads * a.dp : 0)) * sizeof(float);
+    OMNI_CHECK_ARG(lds <= 156 * 1024, "omni_qkv_write: %d query and %d key heads of %d (a token's are staged in LDS)", a.heads, a.kv_heads, a.dp);
+    if (a.T <= 0) return OMNI_OK;
+    return a.elem ? qkv_write_launch<float>(a, lds, (hipStream_t)stream) : qkv_write_launch<uint16_t>(a, lds, (hipStream_t)stream);
+}
+
+// ---- a recurrence's output: norm over all heads together, times the gate.  One workgroup per token
+template <typename E, int MAXC>
+__global__ __launch_bounds__(DR_THREADS) void gated_norm_kernel(const omni_gated_norm a) {
+    __shared__ float red[2 * DR_WAVES];
+    BlockSum bsum{red, 0};
+    const int t = blockIdx.x;
+    float v[MAXC][4], g[MAXC][4], ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+        const int k = (c * DR_THREADS + threadIdx.x) * 4;
+        v[c][0] = v[c][1] = v[c][2] = v[c][3] = 0.f;
+        if (k >= a.n) continue;
+        ld4<float>(a.o + (size_t)t * a.n + k, v[c]);
+        if (a.slabs > 0) {
+            ld4_slabs(reinterpret_cast<const float*>(a.gate) + (size_t)t * a.ld + k, a.slabs, a.slab_stride, g[c]);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) g[c][e] = 1.0f / (1.0f + expf(-g[c][e]));
+        } else {
+            ld4<E>(reinterpret_cast<const E*>(a.gate) + (size_t)t * a.ld + k, g[c]);
+        }
+    }
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) ss += sq4_sum(v[c][0], v[c][1], v[c][2], v[c][3]);
+    const float r = 1.0f / sqrtf(bsum(ss) / (float)a.count + a.eps);
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+        const int k = (c * DR_THREADS + threadIdx.x) * 4;
+        if (k >= a.n) continue;
+        float w[4];
+        ld4<E>(reinterpret_cast<const E*>(a.w) + k, w);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[c][e] = v[c][e] * r * w[e] * g[c][e];
+        st4<E>(reinterpret_cast<E*>(a.out) + (a.frag ? frag_off(t, k, a.n) : (size_t)t * a.n + k), v[c]);
+    }
+}
+
+template <typename E>
+static void gated_norm_launch(const omni_gated_norm& a, hipStream_t st) {
+    const int chunks = (a.n / 4 + DR_THREADS - 1) / DR_THREADS;
+    const dim3 grid(a.T), block(DR_THREADS);
+    if (chunks <= 1) hipLaunchKernelGGL((gated_norm_kernel<E, 1>), grid, block, 0, st, a);
+    else if (chunks <= 2) hipLaunchKernelGGL((gated_norm_kernel<E, 2>), grid, block, 0, st, a);
+    else if (chunks <= 4) hipLaunchKernelGGL((gated_norm_kernel<E, 4>), grid, block, 0, st, a);
+    else hipLaunchKernelGGL((gated_norm_kernel<E, 8>), grid, block, 0, st, a);
+}
+
+extern "C" int omni_gated_norm_run(const omni_gated_norm* p, void* stream) {
+    OMNI_CHECK_ARG(p && p->o && p->w && p->gate && p->out, "omni_gated_norm: null pointer");
+    const omni_gated_norm& a = *p;
+    OMNI_CHECK_ARG(a.n > 0 && a.n % 32 == 0 && a.n <= DR_THREADS * 4 * 8 && a.count > 0 && a.count <= a.n, "omni_gated_norm: n=%d (multiple of 32, <= 8192) count=%d", a.n, a.count);
+    OMNI_CHECK_ARG(a.slabs >= 0 && a.slabs <= OMNI_STREAM_MAX_SPLITS && (a.elem == 0 || (a.elem == 1 && !a.frag)), "omni_gated_norm: slabs=%d elem=%d frag=%d", a.slabs, a.elem, a.frag);
+    OMNI_CHECK_ARG(a.ld >= a.n && a.ld % 4 == 0, "omni_gated_norm: ld=%d", a.ld);
+    if (a.T <= 0) return OMNI_OK;
+    if (a.elem) gated_norm_launch<float>(a, (hipStream_t)stream);
+    else gated_norm_launch<uint16_t>(a, (hipStream_t)stream);
+    OMNI_CHECK_LAUNCH("omni_gated_norm");
     return OMNI_OK;
 }

@@ -12,4 +12,4 @@ void omni_set_error(const char* fmt, ...) {
     va_end(ap);
 }
 extern "C" const char* omni_last_error(void) { return g_err; }
-extern "C" int omni_abi_version(void) { return 6; }
+extern "C" int omni_abi_version(void) { return 7; }

@@ -52,6 +52,8 @@ struct TileArgs {
     long long gx_rows, gw_elems, gout_rows;
     const int32_t* group_rows;
     float act_p, act_n;              // OMNI_TILE_ACT_XIELU
+    int act_cols;                    // OMNI_TILE_ACT_SILU_SIGMOID
+    const uint16_t* mul_table; const int32_t* mul_ids; int mul_rows, mul_ld;      // OMNI_TILE_ACT_GELU_MUL
     long long gx_cols, gout_cols;    // grouped launch: column offset of a group in x and in the outputs (per-head products of one token array)
 };
 
@@ -62,7 +64,7 @@ __device__ __forceinline__ f32x4 tg_mfma(u32x4 a, u32x4 b, f32x4 c) {
 __device__ __forceinline__ float tg_gelu(float v) { return 0.5f * v * (1.0f + erff(v * 0.70710678118654752f)); }
 
 __device__ __forceinline__ bool tile_plain(const TileArgs& a) {
-    return !a.bias && !a.scale && a.act != OMNI_TILE_ACT_GELU && a.act != OMNI_TILE_ACT_XIELU && !a.resid && !a.out_f32 && !a.out2 && a.out;
+    return !a.bias && !a.scale && (a.act == OMNI_TILE_ACT_NONE || a.act == OMNI_TILE_ACT_SILU_MUL_GU8) && !a.resid && !a.out_f32 && !a.out2 && a.out;
 }
 
 // Epilogue of a tile kernel: `acc[j][i]` = this wave's WN n-tiles x WM m-tiles (D[n][m] fragments), first row mw0, first column nw0; `lds` is dead.
@@ -92,7 +94,8 @@ __device__ __forceinline__ void tile_epilogue(const TileArgs& a, f32x4 (&acc)[WN
             if (a.scale) sq[j] = *reinterpret_cast<const f32x4*>(a.scale + n);
         }
     }
-    const bool gelu = !PLAIN && a.act == OMNI_TILE_ACT_GELU, xie = !PLAIN && a.act == OMNI_TILE_ACT_XIELU;
+    const bool gelu = !PLAIN && a.act == OMNI_TILE_ACT_GELU, xie = !PLAIN && a.act == OMNI_TILE_ACT_XIELU, mul = !PLAIN && a.act == OMNI_TILE_ACT_GELU_MUL,
+               other = mul || (!PLAIN && (a.act == OMNI_TILE_ACT_RELU2 || a.act == OMNI_TILE_ACT_SILU_SIGMOID));
     auto write_image = [&](const int pass) {
         if (PLAIN) {
 #pragma unroll
@@ -111,6 +114,20 @@ __device__ __forceinline__ void tile_epilogue(const TileArgs& a, f32x4 (&acc)[WN
                 f32x4 v;
 #pragma unroll
                 for (int e = 0; e < 4; ++e) v[e] = xielu(acc[j][pass][e] + bq[j][e], a.act_p, a.act_n) * sq[j][e];
+                *reinterpret_cast<f32x4*>(img + c * IPITCH + (j * 16 + 4 * q) * 4) = v;
+            }
+        } else if (other) {
+#pragma unroll
+            for (int j = 0; j < WN; ++j) {
+                f32x4 v;
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    const float z = acc[j][pass][e] + bq[j][e];
+                    if (a.act == OMNI_TILE_ACT_RELU2) v[e] = relu2(z);
+                    else if (a.act == OMNI_TILE_ACT_GELU_MUL) v[e] = gelu_tanh(z);
+                    else v[e] = (nw0 + j * 16 + 4 * q < a.act_cols ? z : 1.0f) * sigmoidf_(z);
+                    v[e] *= sq[j][e];
+                }
                 *reinterpret_cast<f32x4*>(img + c * IPITCH + (j * 16 + 4 * q) * 4) = v;
             }
         } else {
@@ -178,6 +195,16 @@ __device__ __forceinline__ void tile_epilogue(const TileArgs& a, f32x4 (&acc)[WN
                     o[2] = pack_bf2(y1[0], y1[1]); o[3] = pack_bf2(y1[2], y1[3]);
                     *reinterpret_cast<u32x4*>(a.out + (size_t)m * a.ldo + n) = o;
                     continue;
+                }
+                if (mul) {
+                    const int id = a.mul_ids[m];
+                    u32x4 z = {0, 0, 0, 0};
+                    if (id >= 0 && id < a.mul_rows) z = *reinterpret_cast<const u32x4*>(a.mul_table + (size_t)id * a.mul_ld + n);
+#pragma unroll
+                    for (int e = 0; e < 2; ++e) {
+                        y0[2 * e] *= bf_lo(z[e]); y0[2 * e + 1] *= bf_hi(z[e]);
+                        y1[2 * e] *= bf_lo(z[2 + e]); y1[2 * e + 1] *= bf_hi(z[2 + e]);
+                    }
                 }
                 if (a.resid) {
                     y0 += rv[it][0];
@@ -656,7 +683,10 @@ extern "C" int omni_gemm_tile(const omni_tile_gemm* g, void* stream) {
     OMNI_CHECK_ARG(g->x_rows > 0 && g->x_rows * (int64_t)g->ldx * 2 < (int64_t)TG_OOB, "omni_gemm_tile: x of %lld rows x %d exceeds the 2 GB descriptor", (long long)g->x_rows, g->ldx);
     OMNI_CHECK_ARG((int64_t)g->N * g->K * 2 < (int64_t)TG_OOB, "omni_gemm_tile: W exceeds the 2 GB descriptor");
     const bool gu8 = g->act == OMNI_TILE_ACT_SILU_MUL_GU8;
-    OMNI_CHECK_ARG(g->act == OMNI_TILE_ACT_NONE || g->act == OMNI_TILE_ACT_GELU || g->act == OMNI_TILE_ACT_XIELU || gu8, "omni_gemm_tile: act=%d", g->act);
+    OMNI_CHECK_ARG(g->act >= OMNI_TILE_ACT_NONE && g->act <= OMNI_TILE_ACT_GELU_MUL, "omni_gemm_tile: act=%d", g->act);
+    OMNI_CHECK_ARG(g->act != OMNI_TILE_ACT_SILU_SIGMOID || (g->act_cols >= 0 && g->act_cols % 4 == 0), "omni_gemm_tile: act_cols=%d (%% 4)", g->act_cols);
+    OMNI_CHECK_ARG(g->act != OMNI_TILE_ACT_GELU_MUL || (g->mul_table && g->mul_ids && g->mul_rows > 0 && g->mul_ld >= g->N && g->mul_ld % 8 == 0 && g->out && !g->out2 && !g->resid &&
+                                                        g->groups <= 1), "omni_gemm_tile: the row table takes ids, mul_ld >= N (%% 8), a bf16 output and one group");
     OMNI_CHECK_ARG(g->tile_hint >= 0 && g->tile_hint <= 7, "omni_gemm_tile: tile_hint=%d", g->tile_hint);
     OMNI_CHECK_ARG(g->tile_hint < 3 || g->N % 256 == 0, "omni_gemm_tile: tile_hint=%d needs N %% 256 == 0", g->tile_hint);
     OMNI_CHECK_ARG(!gu8 || (g->out && !g->resid && !g->out2 && !g->out_f32), "omni_gemm_tile: SiLU-mul takes out only");
@@ -681,7 +711,8 @@ extern "C" int omni_gemm_tile(const omni_tile_gemm* g, void* stream) {
     OMNI_CHECK_ARG(groups == 1 || (int64_t)groups * g->w_group_elems * 2 + (int64_t)g->N * g->K * 2 < ((int64_t)1 << 40), "omni_gemm_tile: W groups");
     a.gx_rows = groups > 1 ? g->x_group_rows : 0; a.gw_elems = groups > 1 ? g->w_group_elems : 0; a.gout_rows = groups > 1 ? g->out_group_rows : 0;
     a.group_rows = g->group_rows;
-    a.act_p = g->act_p; a.act_n = g->act_n;
+    a.act_p = g->act_p; a.act_n = g->act_n; a.act_cols = g->act_cols;
+    a.mul_table = (const uint16_t*)g->mul_table; a.mul_ids = g->mul_ids; a.mul_rows = g->mul_rows; a.mul_ld = g->mul_ld;
     // groups as column ranges of one token array: group g reads x columns [g * x_group_cols, + K) and writes columns [g * out_group_cols, + N)
     OMNI_CHECK_ARG(groups == 1 || (g->x_group_cols >= 0 && g->out_group_cols >= 0 && g->x_group_cols % 8 == 0 && g->out_group_cols % 8 == 0 &&
                                    (groups - 1) * g->x_group_cols + seg_len <= g->ldx &&

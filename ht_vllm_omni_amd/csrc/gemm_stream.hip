@@ -5,19 +5,21 @@
 // flight each, and combine through LDS in a fixed order.  What bounds the op at 64 rows is not only W: every workgroup reads all of
 // x for its K range, 64 rows against its 16 NT columns of W, so wide tiles with K split over workgroups move the fewest bytes through L2.  The
 // S partial sums leave as fp32 slabs [S][M][N]; the row kernels that consume them (decoder_rows.hip) add them up in slab order.
-//   out kinds: fp32 slabs (S >= 1) | bf16 row- or fragment-major | the same through xIELU (common.cuh)
+//   out kinds: fp32 slabs (S >= 1) | bf16 row- or fragment-major | the same through an activation (common.cuh), possibly times a row table
 #include "common.cuh"
 #include "gemm_frag.cuh"
 #include "../../include/omni_decoder.h"
 
 #define GS_WAVES 8
 #define GS_THREADS (GS_WAVES * 64)
-enum { GS_F32 = 0, GS_BF16 = 1, GS_XIELU = 2 };
+enum { GS_F32 = 0, GS_BF16 = 1, GS_ACT = 2 };
 
 struct StreamArgs {
     const uint16_t* x; const uint16_t* W; void* out;
     int M, N, nsteps, split_steps, oshuf;
     float ap, an;
+    int act;
+    omni_row_table rt;
 };
 
 template <int MT, int NT, int KIND>
@@ -89,9 +91,20 @@ __global__ __launch_bounds__(GS_THREADS) void gemm_stream_kernel(const StreamArg
         if (KIND == GS_F32) {
             *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(a.out) + ((size_t)blockIdx.y * a.M + m) * a.N + n) = v;
         } else {
-            if (KIND == GS_XIELU) {
+            if (KIND == GS_ACT) {
+                if (a.act == OMNI_ACT_XIELU) {
 #pragma unroll
-                for (int e = 0; e < 4; ++e) v[e] = xielu(v[e], a.ap, a.an);
+                    for (int e = 0; e < 4; ++e) v[e] = xielu(v[e], a.ap, a.an);
+                } else if (a.act == OMNI_ACT_RELU2) {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) v[e] = relu2(v[e]);
+                } else {
+                    const int id = a.rt.ids[m];
+                    uint2 z = make_uint2(0, 0);
+                    if (id >= 0 && id < a.rt.rows) z = *reinterpret_cast<const uint2*>(reinterpret_cast<const uint16_t*>(a.rt.table) + (size_t)id * a.rt.ld + n);
+                    v[0] = gelu_tanh(v[0]) * bf_lo(z.x); v[1] = gelu_tanh(v[1]) * bf_hi(z.x);
+                    v[2] = gelu_tanh(v[2]) * bf_lo(z.y); v[3] = gelu_tanh(v[3]) * bf_hi(z.y);
+                }
             }
             uint16_t* d = reinterpret_cast<uint16_t*>(a.out) + (a.oshuf ? frag_off(m, n, a.N) : (size_t)m * a.N + n);
             *reinterpret_cast<uint2*>(d) = make_uint2(pack_bf2(v[0], v[1]), pack_bf2(v[2], v[3]));
@@ -134,20 +147,34 @@ extern "C" int omni_gemm_stream_splits(int M, int N, int K) {
     return s;
 }
 
-extern "C" int omni_gemm_stream(const void* x, const void* w, void* out, int M, int N, int K, int kind, int one, float act_p, float act_n, int out_frag, void* stream) {
-    OMNI_CHECK_ARG(x && w && out, "omni_gemm_stream: null pointer");
-    OMNI_CHECK_ARG(M >= 1 && M <= 64 && N > 0 && N % 16 == 0 && K > 0 && K % 32 == 0, "omni_gemm_stream: M=%d (<= 64) N=%d (%% 16) K=%d (%% 32)", M, N, K);
-    OMNI_CHECK_ARG(kind >= GS_F32 && kind <= GS_XIELU && (!out_frag || (kind != GS_F32 && N % 32 == 0)), "omni_gemm_stream: kind=%d out_frag=%d", kind, out_frag);
-    StreamArgs a{(const uint16_t*)x, (const uint16_t*)w, out, M, N, K / 32, 0, out_frag, act_p, act_n};
+static int gs_run(StreamArgs a, int kind, bool one, hipStream_t st) {
     int nt, splits;
-    gs_policy(M, N, a.nsteps, kind == GS_F32 && !one, &nt, &splits);
+    gs_policy(a.M, a.N, a.nsteps, kind == GS_F32 && !one, &nt, &splits);
     a.split_steps = (a.nsteps + splits - 1) / splits;
-    const int mt = M > 32 ? 4 : (M > 16 ? 2 : 1);
-    hipStream_t st = (hipStream_t)stream;
+    const int mt = a.M > 32 ? 4 : (a.M > 16 ? 2 : 1);
 #define GS(MT_, NT_, K_) if (mt == MT_ && nt == NT_ && kind == K_) return gs_launch<MT_, NT_, K_>(a, splits, st);
 #define GS_NT(NT_, K_) GS(1, NT_, K_) GS(2, NT_, K_) GS(4, NT_, K_)
 #define GS_ALL(K_) GS_NT(1, K_) GS_NT(2, K_) GS_NT(3, K_) GS_NT(4, K_)
-    GS_ALL(GS_F32) GS_ALL(GS_BF16) GS_ALL(GS_XIELU)
-    omni_set_error("omni_gemm_stream: no tile for M=%d N=%d", M, N);
+    GS_ALL(GS_F32) GS_ALL(GS_BF16) GS_ALL(GS_ACT)
+    omni_set_error("omni_gemm_stream: no tile for M=%d N=%d", a.M, a.N);
     return OMNI_EINVAL;
+}
+
+#define GS_CHECK(name)                                                                                                                              \
+    OMNI_CHECK_ARG(x && w && out, name ": null pointer");                                                                                           \
+    OMNI_CHECK_ARG(M >= 1 && M <= 64 && N > 0 && N % 16 == 0 && K > 0 && K % 32 == 0, name ": M=%d (<= 64) N=%d (%% 16) K=%d (%% 32)", M, N, K);    \
+    OMNI_CHECK_ARG(!out_frag || N % 32 == 0, name ": out_frag needs N %% 32 == 0 (N=%d)", N)
+
+extern "C" int omni_gemm_stream(const void* x, const void* w, void* out, int M, int N, int K, int kind, int one, float act_p, float act_n, int out_frag, void* stream) {
+    GS_CHECK("omni_gemm_stream");
+    OMNI_CHECK_ARG(kind >= 0 && kind <= 3 && (!out_frag || kind != GS_F32), "omni_gemm_stream: kind=%d out_frag=%d", kind, out_frag);
+    StreamArgs a{(const uint16_t*)x, (const uint16_t*)w, out, M, N, K / 32, 0, out_frag, act_p, act_n, kind == 3 ? OMNI_ACT_RELU2 : OMNI_ACT_XIELU, {}};
+    return gs_run(a, kind == 3 ? (int)GS_ACT : kind, one != 0, (hipStream_t)stream);
+}
+
+extern "C" int omni_gemm_stream_rows(const void* x, const void* w, void* out, int M, int N, int K, const omni_row_table* rt, int out_frag, void* stream) {
+    GS_CHECK("omni_gemm_stream_rows");
+    OMNI_CHECK_ARG(rt && rt->table && rt->ids && rt->rows > 0 && rt->ld >= N && rt->ld % 4 == 0, "omni_gemm_stream_rows: table of %d rows, ld %d", rt ? rt->rows : 0, rt ? rt->ld : 0);
+    StreamArgs a{(const uint16_t*)x, (const uint16_t*)w, out, M, N, K / 32, 0, out_frag, 0.f, 0.f, OMNI_ACT_GELU_MUL, *rt};
+    return gs_run(a, GS_ACT, true, (hipStream_t)stream);
 }

@@ -91,7 +91,7 @@ extern "C" int omni_head_gemm(const void* x, const void* w, void* out, int T, in
 #define GF_T 64
 #define GF_K 16
 __global__ __launch_bounds__(256) void gemm_f32_kernel(const float* __restrict__ x, int ldx, int64_t xb, const float* __restrict__ w, int64_t wb,
-                                                       float* __restrict__ out, int ldo, int64_t ob, int M, int N, int K, int act, float ap, float an) {
+                                                       float* __restrict__ out, int ldo, int64_t ob, int M, int N, int K, int act, float ap, float an, const omni_row_table rt) {
     __shared__ float sx[GF_K][GF_T + 4], sw[GF_K][GF_T + 4];
     const int m0 = blockIdx.y * GF_T, n0 = blockIdx.x * GF_T;
     x += blockIdx.z * xb;
@@ -124,10 +124,16 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const float* __restrict__
     for (int i = 0; i < 4; ++i) {
         const int m = m0 + ty * 4 + i;
         if (m >= M) continue;
+        const int id = act == OMNI_ACT_GELU_MUL ? rt.ids[m] : -1;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int n = n0 + tx * 4 + j;
-            if (n < N) out[(size_t)m * ldo + n] = act ? xielu(acc[i][j], ap, an) : acc[i][j];
+            if (n >= N) continue;
+            float v = acc[i][j];
+            if (act == OMNI_ACT_XIELU) v = xielu(v, ap, an);
+            else if (act == OMNI_ACT_RELU2) v = relu2(v);
+            else if (act == OMNI_ACT_GELU_MUL) v = id >= 0 && id < rt.rows ? gelu_tanh(v) * reinterpret_cast<const float*>(rt.table)[(size_t)id * rt.ld + n] : 0.f;
+            out[(size_t)m * ldo + n] = v;
         }
     }
 }
@@ -135,11 +141,22 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const float* __restrict__
 extern "C" int omni_gemm_f32(const float* x, int ldx, int64_t xb, const float* w, int64_t wb, float* out, int ldo, int64_t ob, int M, int N, int K,
                              int batch, int act, float act_p, float act_n, void* stream) {
     OMNI_CHECK_ARG(x && w && out, "omni_gemm_f32: null pointer");
-    OMNI_CHECK_ARG(N > 0 && K > 0 && ldx >= K && ldo >= N && batch >= 1 && batch <= 65535 && (act == 0 || act == 1), "omni_gemm_f32: N=%d K=%d ldx=%d ldo=%d batch=%d act=%d", N, K, ldx, ldo, batch, act);
+    OMNI_CHECK_ARG(N > 0 && K > 0 && ldx >= K && ldo >= N && batch >= 1 && batch <= 65535 && act >= OMNI_ACT_NONE && act <= OMNI_ACT_RELU2, "omni_gemm_f32: N=%d K=%d ldx=%d ldo=%d batch=%d act=%d", N, K, ldx, ldo, batch, act);
     if (M <= 0) return OMNI_OK;
     const dim3 grid((N + GF_T - 1) / GF_T, (M + GF_T - 1) / GF_T, batch);
     OMNI_CHECK_ARG(grid.y <= 65535, "omni_gemm_f32: M=%d", M);
-    hipLaunchKernelGGL(gemm_f32_kernel, grid, dim3(256), 0, (hipStream_t)stream, x, ldx, xb, w, wb, out, ldo, ob, M, N, K, act, act_p, act_n);
+    hipLaunchKernelGGL(gemm_f32_kernel, grid, dim3(256), 0, (hipStream_t)stream, x, ldx, xb, w, wb, out, ldo, ob, M, N, K, act, act_p, act_n, omni_row_table{});
     OMNI_CHECK_LAUNCH("omni_gemm_f32");
+    return OMNI_OK;
+}
+
+extern "C" int omni_gemm_f32_rows(const float* x, int ldx, const float* w, float* out, int ldo, int M, int N, int K, const omni_row_table* rt, void* stream) {
+    OMNI_CHECK_ARG(x && w && out && rt && rt->table && rt->ids, "omni_gemm_f32_rows: null pointer");
+    OMNI_CHECK_ARG(N > 0 && K > 0 && ldx >= K && ldo >= N && rt->rows > 0 && rt->ld >= N, "omni_gemm_f32_rows: N=%d K=%d ldx=%d ldo=%d, table of %d rows, ld %d", N, K, ldx, ldo, rt->rows, rt->ld);
+    if (M <= 0) return OMNI_OK;
+    const dim3 grid((N + GF_T - 1) / GF_T, (M + GF_T - 1) / GF_T, 1);
+    OMNI_CHECK_ARG(grid.y <= 65535, "omni_gemm_f32_rows: M=%d", M);
+    hipLaunchKernelGGL(gemm_f32_kernel, grid, dim3(256), 0, (hipStream_t)stream, x, ldx, (int64_t)0, w, (int64_t)0, out, ldo, (int64_t)0, M, N, K, OMNI_ACT_GELU_MUL, 0.f, 0.f, *rt);
+    OMNI_CHECK_LAUNCH("omni_gemm_f32_rows");
     return OMNI_OK;
 }

@@ -15,18 +15,8 @@
 //   latent_prefill_kernel  tiles of up to la_tile_rows() query rows of one sequence, 16 per wave; the waves share each 32-key tile
 //                          (double-buffered, one barrier per tile)
 //   latent_plain_kernel    any width, bf16 or fp32: one wave per query row on the vector units (the 32-bit mode)
-#include "common.cuh"
-#include "gemm_frag.cuh"
+#include "attn_tile.cuh"
 #include "../../include/omni_decoder.h"
-
-#define LA_KEYS 32
-#define LA_LOG2E 1.4426950408889634f
-#define LA_DEC_WAVES 4
-#define LA_MAX_SPLIT 16
-#define LA_SENT (-1e30f)
-
-typedef short s16x4 __attribute__((ext_vector_type(4)));
-typedef __attribute__((address_space(3))) s16x4 lds_s16x4;
 
 struct LatentArgs {
     const uint16_t* q; const uint16_t* cache; const float* gate; uint16_t* out;
@@ -35,9 +25,6 @@ struct LatentArgs {
     int heads; float qs;            // scale * log2(e)
     float* partial; int nsplit;
 };
-
-// KV splits a row of `ntiles` 16-key tiles uses, of the nsplit the launch offers: two rounds of the four waves each, or more
-__device__ __forceinline__ int la_row_splits(int ntiles, int nsplit) { return min(nsplit, (ntiles + 7) / 8); }
 
 template <int RS>
 struct LatentGeom {
@@ -94,12 +81,9 @@ __device__ __forceinline__ LaWeights la_weights(const float (&sv)[8], int nlive,
     LaWeights w;
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-        const float a = p[2 * e], b = p[2 * e + 1];
-        const float ar = a - bfround(a), br = b - bfround(b);
-        const float am = bfround(ar), bm = bfround(br);
-        w.hi[e] = pack_bf2(a, b);
-        w.mid[e] = pack_bf2(am, bm);
-        w.lo[e] = pack_bf2(ar - am, br - bm);
+        uint32_t hi, mid, lo;
+        split3(p[2 * e], p[2 * e + 1], hi, mid, lo);
+        w.hi[e] = hi; w.mid[e] = mid; w.lo[e] = lo;
     }
     return w;
 }
@@ -107,12 +91,7 @@ __device__ __forceinline__ LaWeights la_weights(const float (&sv)[8], int nlive,
 // C^T fragment of d tile dt: lane (d = c, qk) gets the 8 keys of its contraction slots
 template <int RS>
 __device__ __forceinline__ u32x4 la_transposed(const unsigned char* img, int dt, int c, int qk) {
-    constexpr int PITCH = LatentGeom<RS>::PITCH;
-    const unsigned char* p = img + (4 * qk + (c >> 2)) * PITCH + (16 * dt + (c & 3) * 4) * 2;
-    const s16x4 a = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4*)p);
-    const s16x4 b = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4*)(p + 16 * PITCH));
-    const u32x2 x = __builtin_bit_cast(u32x2, a), y = __builtin_bit_cast(u32x2, b);
-    return (u32x4){x[0], x[1], y[0], y[1]};
+    return la_transposed_at(img, LatentGeom<RS>::PITCH, dt, c, qk);
 }
 
 template <int RS>
@@ -214,12 +193,9 @@ __global__ __launch_bounds__(64 * LA_DEC_WAVES, 2) void latent_decode_kernel(con
         u32x2 w3[3];                                  // three bf16 terms whose sum is the fp32 weight
 #pragma unroll
         for (int e = 0; e < 2; ++e) {
-            const float x = p[2 * e], y = p[2 * e + 1];
-            const float xr = x - bfround(x), yr = y - bfround(y);
-            const float xm = bfround(xr), ym = bfround(yr);
-            w3[0][e] = pack_bf2(x, y);
-            w3[1][e] = pack_bf2(xm, ym);
-            w3[2][e] = pack_bf2(xr - xm, yr - ym);
+            uint32_t hi, mid, lo;
+            split3(p[2 * e], p[2 * e + 1], hi, mid, lo);
+            w3[0][e] = hi; w3[1][e] = mid; w3[2][e] = lo;
         }
 #pragma unroll
         for (int i = 0; i < 3; ++i) reinterpret_cast<u32x2*>(pw + ((wave >> 1) * 3 + i) * 64 + lane)[wave & 1] = w3[i];
@@ -432,14 +408,7 @@ __global__ __launch_bounds__(64) void latent_plain_kernel(const E* __restrict__ 
 static constexpr int la_tile_rows(int rp) { return rp > 256 ? 128 : 64; }
 extern "C" int omni_latent_attn_tile_rows(int rp) { return la_tile_rows(rp); }
 
-static int la_splits(int n_decode, int heads, int max_keys) {
-    const int wgs = n_decode * ((heads + 15) / 16);
-    int ns = 512 / (wgs > 0 ? wgs : 1);                 // two workgroups per CU
-    const int cap = (max_keys + 63) / 64;               // at least one tile per wave and split
-    if (ns > cap) ns = cap;
-    if (ns > LA_MAX_SPLIT) ns = LA_MAX_SPLIT;
-    return ns < 1 ? 1 : ns;
-}
+static int la_splits(int n_decode, int heads, int max_keys) { return la_split_count(n_decode * ((heads + 15) / 16), max_keys); }
 
 extern "C" int64_t omni_latent_attn_workspace_bytes(int n_decode, int heads, int rp) {
     return (int64_t)n_decode * heads * LA_MAX_SPLIT * (rp + 4) * (int64_t)sizeof(float);

@@ -1,112 +1,80 @@
-"""DecoderEngine: device-resident weights, paged latent cache, per-sequence state and the step function of decoder-only language models.
+"""DecoderEngine: device-resident weights, paged cache, per-sequence state and the step function of decoder-only language models.
 
-One forward serves every step: a batch is T tokens, sequence after sequence, the single-token sequences (decoded tokens) first; per layer
+One forward serves every step: a batch is T tokens, sequence after sequence, the single-token sequences (decoded tokens) first.  Per layer
 
-  stream_rows    x += g * y / rms(y) of the sublayer before, token shift against the previous token (state for a batch's first one) -> h
+  stream_rows    the sublayer before joins the residual stream -- x += g * y / rms(y), or x = w * (alpha x + y) / rms(..) -- and h follows from x
+                 (token shift against the previous token, or x itself)
+  mixer          h -> y (decoder_mixers.py): joint projection, cache write / state update, attention or recurrence, output projection
+  stream_rows, GEMM with its activation in the epilogue, GEMM       the feed-forward -> y (fp32)
+  stream_rows, GEMM (gelu * the token's side row), GEMM             the side input, where the model has one -> y (fp32)
+
+Latent attention, as launches:
   GEMM           [W_dq ; W_dkv ; W_g] h -> fp32: the three products of h are one
   latent_write   both latent norms, the new latent into the cache, gates, the shift state of each sequence's last token
   GEMM, head     q = W_uq c_q, then q_h W_uk,h: queries in the latent space, so that the cache row is key AND value of every head
   latent_attn    causal softmax over the cache (fp32 scores and weights), gate applied to the normalised sum
   head, GEMM     W_uv,h per head, W_o -> y (fp32)
-  stream_rows    x += g * y / rms(y) -> bf16 x;  GEMM with xIELU in its epilogue;  GEMM -> y (fp32)
+Windowed attention:
+  GEMM           [W_q ; W_k ; W_v ; W_g] h -> fp32
+  qkv_write      norms over whole projections, rotation, keys and values into the cache, the gate
+  window_attn    softmax over the window (and the sink), gate applied;   GEMM  W_o -> y (fp32)
+Decay recurrence:
+  GEMM           [W_q ; W_k ; W_v ; W_g] h -> fp32 (prompts: SiLU / sigmoid in the epilogue, bf16)
+  decay_rec      state update and outputs (prompts: chunks);  gated_norm  the norm over all heads, the gate;  GEMM  W_o -> y (fp32)
 
-The residual stream, norms, gates, scores and state are fp32; matrix operands are bf16 (``dtype="bfloat16"``) or everything is fp32
+The residual stream, norms, gates of norms, scores and state are fp32; matrix operands are bf16 (``dtype="bfloat16"``) or everything is fp32
 (``dtype="float32"``).  GEMMs of up to 64 tokens stream fragment-major weights (omni_gemm_stream), larger ones run omni_gemm_tile on the
 SAME bytes.  Every width is padded to a multiple of 32 with zero weights at load, so no size is special.
 """
 from __future__ import annotations
 
 import ctypes as C
-from dataclasses import dataclass
+from dataclasses import dataclass, field
 
 import torch
 
 from . import _lib as L
 from . import ops
 from .decoder_config import DecoderDims
-from .engine import frag_shuffle
+from .decoder_mixers import (ELEM, LATENT_WIDTHS, WORK, Elem, Matrix, attention_tiles, cache_traffic, latent_width, make_mixer, pad1, pad2, r32,  # noqa: F401
+                             state_bytes)
 
 SKINNY = 64            # most tokens of the weight-streaming GEMMs
 HEAD_TILE = 512        # from this many tokens on the per-head products run on omni_gemm_tile's column groups
 
-
-@dataclass(frozen=True)
-class Elem:
-    code: int
-    torch: torch.dtype
-    kv_names: tuple[str, ...]
+# a feed-forward's activation in the three products: (omni_gemm_stream kind, omni_gemm_tile act, omni_gemm_f32 act)
+MLP_ACTS = {"xielu": (L.STREAM_XIELU, L.TILE_ACT_XIELU, L.ACT_XIELU), "relu2": (L.STREAM_RELU2, L.TILE_ACT_RELU2, L.ACT_RELU2)}
 
 
-ELEM = {"bfloat16": Elem(0, torch.bfloat16, ("auto", "bf16", "bfloat16")), "float32": Elem(1, torch.float32, ("auto", "float32", "fp32"))}
-
-
-def r32(n: int) -> int:
-    return (n + 31) // 32 * 32
-
-
-# latent widths the matrix-core attention is instantiated for (csrc/latent_attn.hip LA_WIDTHS)
-LATENT_WIDTHS = tuple(32 * n for n in (1, 2, 3, 4, 5, 6, 7, 8, 10, 12, 14, 16))
-
-
-def latent_width(kv_rank: int, elem_code: int) -> int:
-    """Padded width of a cache row."""
-    if elem_code == 0:
-        for w in LATENT_WIDTHS:
-            if w >= kv_rank:
-                return w
-    return r32(kv_rank)
-
-
-def pad2(w: torch.Tensor, rows: int, cols: int) -> torch.Tensor:
-    out = torch.zeros(rows, cols, dtype=w.dtype)
-    out[:w.shape[0], :w.shape[1]] = w
-    return out
-
-
-def pad1(v: torch.Tensor, n: int) -> torch.Tensor:
-    out = torch.zeros(n, dtype=v.dtype)
-    out[:v.shape[0]] = v
-    return out
-
-
-class _Matrix:
-    """One weight [N, K] (or [heads, N, K]) of a layer, padded, on the device: fragment-major in bf16, row-major in fp32."""
-
-    def __init__(self, w: torch.Tensor, elem: Elem, device):
-        w = w.to(device=device, dtype=elem.torch).contiguous()
-        self.t = frag_shuffle(w) if elem.code == 0 else w
-        self.N, self.K = w.shape[-2:]
+@dataclass
+class Act:
+    name: str
+    params: tuple[float, float] = (0.0, 0.0)
 
 
 class _Layer:
     """Device tensors of one weight-owning layer."""
 
-    def __init__(self, d: DecoderDims, i: int, w: dict, elem: Elem, device):
-        s, p = d.layers[i], f"l{i}."
-        m = s.mixer
-        H, W = m.heads, r32(d.hidden)
-        self.qp, self.rp, self.dp, self.vp = r32(m.q_rank), latent_width(m.kv_rank, elem.code), r32(m.dim), r32(m.vdim)
-        up = lambda t: t.to(device=device, dtype=elem.torch).contiguous()  # noqa: E731
-        parts = [pad2(w[p + "mix.dq"], self.qp, W), pad2(w[p + "mix.dkv"], self.rp, W)]
-        if m.out_gate:
-            parts.append(pad2(w[p + "mix.g"], r32(H), W))
-        self.down = _Matrix(torch.cat(parts), elem, device)
-        self.qw, self.kw = up(pad1(w[p + "mix.dq.norm"], self.qp)), up(pad1(w[p + "mix.dkv.norm"], self.rp))
-        uq = torch.stack([pad2(h, self.dp, self.qp) for h in w[p + "mix.uq"].reshape(H, m.dim, m.q_rank)])
-        self.uq = _Matrix(uq.reshape(H * self.dp, self.qp), elem, device)
-        # per head: queries into the latent space (the transpose of W_uk) and latents to values
-        self.uk = _Matrix(torch.stack([pad2(h.T, self.rp, self.dp) for h in w[p + "mix.uk"].reshape(H, m.dim, m.kv_rank)]), elem, device)
-        self.uv = _Matrix(torch.stack([pad2(h, self.vp, self.rp) for h in w[p + "mix.uv"].reshape(H, m.vdim, m.kv_rank)]), elem, device)
-        o = torch.stack([pad2(h, W, self.vp) for h in w[p + "mix.o"].reshape(d.hidden, H, m.vdim).permute(1, 0, 2)], 1)
-        self.o = _Matrix(o.reshape(W, H * self.vp), elem, device)
-        self.mu = up(pad1(w[p + "shift"], W))
-        self.gain1 = float(w[p + "norm1"])
+    def __init__(self, eng: "DecoderEngine", i: int, w: dict):
+        d, elem, dev = eng.d, eng.elem, eng.device
+        s, p, W = d.layers[i], f"l{i}.", eng.width
+        self.mixer = make_mixer(eng, i, w)
+        self.mu = eng.up(pad1(w[p + "shift"], W)) if d.token_shift else None
+        self.norm1 = eng.norm_gain(w[p + "norm1"])
+        self.mats = self.mixer.matrices()
         if s.mlp is not None:
             F = r32(s.mlp.ff)
-            self.gain2 = float(w[p + "norm2"])
-            self.up, self.dn = _Matrix(pad2(w[p + "mlp.up"], F, W), elem, device), _Matrix(pad2(w[p + "mlp.down"], W, F), elem, device)
-            ap, an = torch.nn.functional.softplus(w[p + "mlp.act"].double()).tolist()
-            self.act = (ap, 0.5 + an)
+            self.norm2 = eng.norm_gain(w[p + "norm2"])
+            self.up, self.dn = Matrix(pad2(w[p + "mlp.up"], F, W), elem, dev), Matrix(pad2(w[p + "mlp.down"], W, F), elem, dev)
+            self.mats += [self.up, self.dn]
+            self.act = Act(s.mlp.act)
+            if s.mlp.act == "xielu":
+                ap, an = torch.nn.functional.softplus(w[p + "mlp.act"].double()).tolist()
+                self.act.params = (ap, 0.5 + an)
+        if d.side_dim:
+            self.side_gate, self.side_proj = Matrix(pad2(w[p + "side.gate"], eng.side_width, W), elem, dev), Matrix(pad2(w[p + "side.proj"], W, eng.side_width), elem, dev)
+            self.side_norm = eng.up(pad1(w[p + "side.norm"], W))
+            self.mats += [self.side_gate, self.side_proj]
 
 
 class _Scratch:
@@ -115,47 +83,37 @@ class _Scratch:
     def __init__(self, eng: "DecoderEngine", rows: int):
         self.rows = rows
         r16 = (rows + 15) // 16 * 16                       # fragment-major operands come in whole 16-row tiles
-        dev, E = eng.device, eng.elem.torch
-        ls = [eng.layer_w[eng.d.owner(i)] for i in range(eng.d.num_layers)]
-        hs = [s.mixer.heads for s in eng.d.layers]
-        W = eng.width
-        z = lambda n, dt: torch.zeros(n, dtype=dt, device=dev)  # noqa: E731
-        self.x = (z(rows * W, torch.float32), z(rows * W, torch.float32))
         # products that leave as partial sums (omni_gemm_stream): as many slabs as up to SKINNY rows may take
-        slabs = lambda n: max(rows, min(rows, SKINNY) * L.STREAM_MAX_SPLITS) * n  # noqa: E731
-        self.y, self.h = z(slabs(W), torch.float32), z(r16 * W, E)
-        self.proj = z(slabs(max(l.down.N for l in ls)), torch.float32)
-        self.cq = z(r16 * max(l.qp for l in ls), E)
-        self.q = z(rows * max(h * l.dp for h, l in zip(hs, ls)), E)
-        self.ql = z(rows * max(h * l.rp for h, l in zip(hs, ls)), E)
-        self.ol = torch.zeros_like(self.ql)
-        self.v = z(r16 * max(h * l.vp for h, l in zip(hs, ls)), E)
-        self.gate = z(rows * max(hs), torch.float32)
-        self.act = z(r16 * max([r32(s.mlp.ff) for s in eng.d.layers if s.mlp is not None] or [32]), E)
-        self.hn = z(r16 * W, E)
+        count = {"rows": rows, "tiles": r16, "slabs": max(rows, min(rows, SKINNY) * L.STREAM_MAX_SPLITS)}
+        W = eng.width
+        needs = [{"x0": (W, torch.float32, "rows"), "x1": (W, torch.float32, "rows"), "y": (W, torch.float32, "slabs"), "h": (W, "elem", "tiles"), "hn": (W, "elem", "tiles"),
+                  "act": (max([r32(s.mlp.ff) for s in eng.d.layers if s.mlp is not None] + [eng.side_width, 32]), "elem", "tiles")}]
+        needs += [l.mixer.needs() for l in eng.layer_w.values()]
+        size: dict[str, tuple] = {}
+        for n in needs:
+            for k, (width, dt, per) in n.items():
+                have = size.get(k)
+                assert have is None or have[1:] == (dt, per), k
+                size[k] = (max(width, have[0] if have else 0), dt, per)
+        for k, (width, dt, per) in size.items():
+            setattr(self, k, torch.zeros(count[per] * width, dtype=eng.elem.torch if dt == "elem" else dt, device=eng.device))
+        self.x = (self.x0, self.x1)
 
 
 @dataclass
 class Batch:
-    """One forward's tokens (device tensors).  Tokens [0, n_decode) are single-token sequences; `tiles` covers the rest per (head count, rows of a work item)."""
+    """One forward's tokens (device tensors).  Tokens [0, n_decode) are single-token sequences; `work` holds the others' work items per kind."""
     T: int
     n_decode: int
     ids: torch.Tensor                   # int32 [T]
     row_of_tok: torch.Tensor            # int32 [T]
     positions: torch.Tensor             # int32 [T]
-    tiles: dict[tuple, torch.Tensor]    # (heads, tile rows) -> int32 [2 n]
     max_keys: int                       # most keys a decode token sees
+    work: dict[tuple, tuple[torch.Tensor, int]] = field(default_factory=dict)      # work key -> (int32 items, how many)
     num_live: torch.Tensor | None = None
 
-
-def attention_tiles(seg_starts: list[int], seg_lens: list[int], heads: int, tile_rows: int) -> list[tuple[int, int]]:
-    """Work items of the prompt attention: runs of up to `tile_rows` query rows (token-major, heads inside) of ONE sequence.  Longest first: a later
-    tile of a prompt sees more keys."""
-    out = []
-    for s, n in zip(seg_starts, seg_lens):
-        lo, hi = s * heads, (s + n) * heads
-        out += [(lo - f, f, min(tile_rows, hi - f)) for f in range(lo, hi, tile_rows)]
-    return [(f, n) for _, f, n in sorted(out)]
+    def items(self, key: tuple) -> tuple[torch.Tensor | None, int]:
+        return self.work.get(key, (None, 0))
 
 
 class DecoderEngine:
@@ -177,16 +135,23 @@ class DecoderEngine:
         self.bt_stride = (dims.max_model_len + block_size - 1) // block_size
         dev, E = self.device, self.elem.torch
         # ---- weights
+        self._shared: dict = {}
+        self._chunk_states: torch.Tensor | None = None
         self.embed = pad2(weights["embed"], dims.vocab, self.width).to(device=dev, dtype=E)
-        self.head = _Matrix(pad2(weights["head"], r32(dims.vocab), self.width), self.elem, dev)
-        self.final_gain = float(weights["final.norm"])
-        self.layer_w = {i: _Layer(dims, i, weights, self.elem, dev) for i in range(dims.num_layers) if dims.owner(i) == i}
-        # per layer: heads and query rows per work item of its prompt attention
-        self.tile_kinds = [(s.mixer.heads, self.lib.omni_latent_attn_tile_rows(self.layer_w[dims.owner(i)].rp)) for i, s in enumerate(dims.layers)]
+        self.side_width = r32(dims.side_dim) if dims.side_dim else 0
+        if dims.side_dim:                                   # [vocab, layers, padded]: a layer's slice is a column range
+            t = weights["side.embed"].reshape(dims.vocab * dims.num_layers, dims.side_dim)
+            self.side_embed = pad2(t, t.shape[0], self.side_width).reshape(dims.vocab, dims.num_layers * self.side_width).to(device=dev, dtype=E)
+        self.head = Matrix(pad2(weights["head"], r32(dims.vocab), self.width), self.elem, dev)
+        self.final_norm = self.norm_gain(weights["final.norm"])
+        self.layer_w = {i: _Layer(self, i, weights) for i in range(dims.num_layers) if dims.owner(i) == i}
+        self.mixers = [self.layer_w[dims.owner(i)].mixer for i in range(dims.num_layers)]
+        self.work_keys = sorted({k for m in self.mixers for k in m.work})
         self._alloc_kv(num_blocks)
-        # ---- per-sequence state: what each layer's mixer read at the sequence's last token; slot 0 belongs to no sequence
+        # ---- per-sequence state, slot 0 of no sequence: what each layer's mixer read at the sequence's last token, and the mixers' own
         self.state_slots = max_batch + 1
-        self.state = torch.zeros(dims.num_layers, self.state_slots, self.width, dtype=torch.float32, device=dev)
+        self.shift_state = torch.zeros(dims.num_layers, self.state_slots, self.width, dtype=torch.float32, device=dev) if dims.token_shift else None
+        self.rec_state = [m.state(self.state_slots) for m in self.mixers]
         # ---- persistent per-row buffers (graph-stable addresses)
         Bm = max_batch
         i32 = dict(dtype=torch.int32, device=dev)
@@ -206,20 +171,38 @@ class DecoderEngine:
         # ---- scratch: the decode step's own (its addresses are recorded in graphs), and one that grows with the prompts
         self._dec = _Scratch(self, Bm)
         self._any: _Scratch | None = None
-        heads = max(s.mixer.heads for s in dims.layers)
-        rp = max(l.rp for l in self.layer_w.values())
-        nbytes = self.lib.omni_latent_attn_workspace_bytes(Bm, heads, rp)
-        self.attn_ws = torch.zeros(nbytes // 4, dtype=torch.float32, device=dev)
+        self.attn_ws = torch.zeros(max(m.workspace_bytes(Bm) for m in self.mixers) // 4 + 1, dtype=torch.float32, device=dev)
         self.persistent_chains = False
+
+    # ------------------------------------------------------------------ tensors
+    def up(self, t: torch.Tensor) -> torch.Tensor:
+        """A vector of weights in the model's element type."""
+        return t.to(device=self.device, dtype=self.elem.torch).contiguous()
+
+    def norm_gain(self, t: torch.Tensor):
+        """A norm's weight: one number, or a padded vector."""
+        return float(t) if t.dim() == 0 else self.up(pad1(t, self.width))
+
+    def shared(self, key: tuple, make) -> torch.Tensor:
+        """A table that several layers read."""
+        if key not in self._shared:
+            self._shared[key] = make()
+        return self._shared[key]
+
+    def chunk_states(self, elements: int) -> torch.Tensor:
+        """Scratch of the chunked recurrence, shared by the layers (prompt steps only: it grows)."""
+        if self._chunk_states is None or self._chunk_states.numel() < elements:
+            self._chunk_states = None
+            self._chunk_states = torch.empty(elements, dtype=torch.float32, device=self.device)
+        return self._chunk_states
 
     # ------------------------------------------------------------------ cache
     def _alloc_kv(self, num_blocks: int) -> None:
         self.num_blocks = int(num_blocks)
-        self.kv_caches = [torch.zeros(self.num_blocks, self.block_size, self.layer_w[self.d.owner(i)].rp, dtype=self.elem.torch, device=self.device)
-                          for i in range(self.d.num_layers)]
+        self.kv_caches = [m.cache(self.num_blocks, self.block_size) for m in self.mixers]
 
     def kv_cache_bytes(self) -> int:
-        return sum(c.numel() * c.element_size() for c in self.kv_caches)
+        return sum(c.numel() * c.element_size() for layer in self.kv_caches for c in layer)
 
     def resize_kv_cache(self, num_blocks: int) -> None:
         """Another number of blocks (before any graph capture)."""
@@ -259,25 +242,38 @@ class DecoderEngine:
             getattr(self, "row_" + k)[row] = v
 
     # ------------------------------------------------------------------ products
-    def _mm(self, x: torch.Tensor, w: _Matrix, out: torch.Tensor, T: int, *, f32_out: bool = False, one: bool = False, act=None, out_frag: bool = False) -> int:
-        """out [T, N] = (xIELU of) x . w^T.  x: fragment-major when T <= SKINNY and bf16 (its producer wrote it so), else row-major.  Returns how
+    def _mm(self, x: torch.Tensor, w: Matrix, out: torch.Tensor, T: int, *, f32_out: bool = False, one: bool = False, act: Act | None = None, out_frag: bool = False) -> int:
+        """out [T, N] = act(x . w^T).  x: fragment-major when T <= SKINNY and bf16 (its producer wrote it so), else row-major.  Returns how
         many partial sums [T, N] an fp32 output consists of (its consumer adds them up; one: a single one)."""
         st, lib = L.current_stream(), self.lib
-        a, b = act or (0.0, 0.0)
+        a, b = act.params if act else (0.0, 0.0)
+        stream, tile, plain = MLP_ACTS[act.name] if act else (L.STREAM_BF16, L.TILE_ACT_NONE, L.ACT_NONE)
         if self.elem.code == 1:
-            L.check(lib.omni_gemm_f32(x.data_ptr(), w.K, 0, w.t.data_ptr(), 0, out.data_ptr(), w.N, 0, T, w.N, w.K, 1, int(act is not None), a, b, st),
-                    "omni_gemm_f32", lib)
+            L.check(lib.omni_gemm_f32(x.data_ptr(), w.K, 0, w.t.data_ptr(), 0, out.data_ptr(), w.N, 0, T, w.N, w.K, 1, plain, a, b, st), "omni_gemm_f32", lib)
         elif T <= SKINNY:
-            kind = L.STREAM_F32 if f32_out else (L.STREAM_BF16 if act is None else L.STREAM_XIELU)
+            kind = L.STREAM_F32 if f32_out else stream
             L.check(lib.omni_gemm_stream(x.data_ptr(), w.t.data_ptr(), out.data_ptr(), T, w.N, w.K, kind, int(one), a, b, int(out_frag), st), "omni_gemm_stream", lib)
             return lib.omni_gemm_stream_splits(T, w.N, w.K) if f32_out and not one else 1
         else:
-            o = out[:T * w.N].view(T, w.N)
-            ops.gemm_tile(x[:T * w.K].view(T, w.K), w.t, act=L.TILE_ACT_NONE if act is None else L.TILE_ACT_XIELU, act_params=(a, b),
-                          want="f" if f32_out else "b", lib=lib, **({"out_f32": o} if f32_out else {"out": o}))
+            self._tile(x, w, out, T, f32_out=f32_out, act=tile, act_params=(a, b))
         return 1
 
-    def _heads_mm(self, x: torch.Tensor, w: _Matrix, out: torch.Tensor, T: int, heads: int, out_frag: bool = False) -> None:
+    def _tile(self, x: torch.Tensor, w: Matrix, out: torch.Tensor, T: int, *, f32_out: bool = False, **kw) -> None:
+        """omni_gemm_tile on row-major rows."""
+        o = out[:T * w.N].view(T, w.N)
+        ops.gemm_tile(x[:T * w.K].view(T, w.K), w.t, want="f" if f32_out else "b", lib=self.lib, **({"out_f32": o} if f32_out else {"out": o}), **kw)
+
+    def _mm_rows(self, x: torch.Tensor, w: Matrix, out: torch.Tensor, T: int, table: L.RowTable, out_frag: bool) -> None:
+        """out [T, N] = gelu_tanh(x . w^T) * the tokens' rows of a table."""
+        st, lib = L.current_stream(), self.lib
+        if self.elem.code == 1:
+            L.check(lib.omni_gemm_f32_rows(x.data_ptr(), w.K, w.t.data_ptr(), out.data_ptr(), w.N, T, w.N, w.K, C.byref(table), st), "omni_gemm_f32_rows", lib)
+        elif T <= SKINNY:
+            L.check(lib.omni_gemm_stream_rows(x.data_ptr(), w.t.data_ptr(), out.data_ptr(), T, w.N, w.K, C.byref(table), int(out_frag), st), "omni_gemm_stream_rows", lib)
+        else:
+            self._tile(x, w, out, T, act=L.TILE_ACT_GELU_MUL, mul=table)
+
+    def _heads_mm(self, x: torch.Tensor, w: Matrix, out: torch.Tensor, T: int, heads: int, out_frag: bool = False) -> None:
         """out[t, h] = x[t, h] . w[h]^T."""
         st, lib = L.current_stream(), self.lib
         if self.elem.code == 1:
@@ -298,22 +294,21 @@ class DecoderEngine:
     def make_batch(self, ids: torch.Tensor, row_of_tok, positions, seg_lens: list[int], *, n_decode: int = 0, max_keys: int = 0, ids_device=None) -> Batch:
         """A batch from host arrays: tokens [0, n_decode) single-token sequences, then segments of `seg_lens` tokens.  One upload."""
         T = len(row_of_tok)
-        kinds = sorted(set(self.tile_kinds)) if T > n_decode else []
+        keys = self.work_keys if T > n_decode else []
         starts, o = [], n_decode
         for n in seg_lens:
             starts.append(o)
             o += n
         assert o == T, (o, T)
-        tl = {k: attention_tiles(starts, seg_lens, *k) for k in kinds}
         flat = [torch.as_tensor(ids, dtype=torch.int32), torch.as_tensor(row_of_tok, dtype=torch.int32), torch.as_tensor(positions, dtype=torch.int32)]
-        flat += [torch.tensor(tl[k], dtype=torch.int32).reshape(-1) for k in kinds]
+        made = {k: WORK[k[0]](starts, seg_lens, *k[1:]) for k in keys}
+        flat += [torch.tensor(made[k], dtype=torch.int32).reshape(-1) for k in keys]
         buf = torch.cat(flat).pin_memory().to(self.device, non_blocking=True)
-        tiles, o = {}, 3 * T
-        for k in kinds:
-            n = 2 * len(tl[k])
-            tiles[k] = buf[o:o + n]
-            o += n
-        return Batch(T, n_decode, buf[:T] if ids_device is None else ids_device, buf[T:2 * T], buf[2 * T:3 * T], tiles, max_keys)
+        work, o = {}, 3 * T
+        for k, t in zip(keys, flat[3:]):
+            work[k] = (buf[o:o + t.numel()], len(made[k]))
+            o += t.numel()
+        return Batch(T, n_decode, buf[:T] if ids_device is None else ids_device, buf[T:2 * T], buf[2 * T:3 * T], max_keys, work)
 
     def _scratch(self, T: int) -> _Scratch:
         if self._any is None or self._any.rows < T:
@@ -321,28 +316,12 @@ class DecoderEngine:
             self._any = _Scratch(self, max(T, 256) if T <= 256 else (T + 1023) // 1024 * 1024)
         return self._any
 
-    def _mixer(self, b: Batch, i: int, s: _Scratch, x: torch.Tensor, frag: bool) -> int:
-        """s.h -> s.y (returns its partial sums)"""
-        m, w, lib, st = self.d.layers[i].mixer, self.layer_w[self.d.owner(i)], self.lib, L.current_stream()
-        T, H = b.T, m.heads
-        slabs = self._mm(s.h, w.down, s.proj, T, f32_out=True)
-        gate = s.gate if m.out_gate else None
-        a = L.LatentWrite(proj=s.proj.data_ptr(), slabs=slabs, slab_stride=T * w.down.N, ld=w.down.N, q_rank=m.q_rank, qp=w.qp, kv_rank=m.kv_rank, rp=w.rp, heads=H, qw=w.qw.data_ptr(),
-                          kw=w.kw.data_ptr(), eps=self.d.eps, cq=s.cq.data_ptr(), frag=int(frag), cache=self.kv_caches[i].data_ptr(), gate=L.ptr(gate),
-                          block_table=self.block_table.data_ptr(), bt_stride=self.bt_stride, block_size=self.block_size, row_of_tok=b.row_of_tok.data_ptr(),
-                          positions=b.positions.data_ptr(), num_live=L.ptr(b.num_live), x=x.data_ptr(), wp=self.width, state=self.state[i].data_ptr(),
-                          state_slot=self.state_slot.data_ptr(), T=T, elem=self.elem.code)
-        L.check(lib.omni_latent_write_run(C.byref(a), st), "omni_latent_write", lib)
-        self._mm(s.cq, w.uq, s.q, T)
-        self._heads_mm(s.q, w.uk, s.ql, T, H)
-        tiles = b.tiles.get(self.tile_kinds[i])
-        a = L.LatentAttn(q=s.ql.data_ptr(), cache=self.kv_caches[i].data_ptr(), gate=L.ptr(gate), out=s.ol.data_ptr(), block_table=self.block_table.data_ptr(),
-                         bt_stride=self.bt_stride, block_size=self.block_size, row_of_tok=b.row_of_tok.data_ptr(), positions=b.positions.data_ptr(),
-                         tiles=L.ptr(tiles), n_tiles=0 if tiles is None else tiles.numel() // 2, tile_rows=self.tile_kinds[i][1], T=T, n_decode=b.n_decode, heads=H, rp=w.rp, scale=m.scale,
-                         max_keys=b.max_keys, workspace=self.attn_ws.data_ptr(), workspace_bytes=self.attn_ws.numel() * 4, elem=self.elem.code)
-        L.check(lib.omni_latent_attn_run(C.byref(a), st), "omni_latent_attn", lib)
-        self._heads_mm(s.ol, w.uv, s.v, T, H, out_frag=frag)
-        return self._mm(s.v, w.o, s.y, T, f32_out=True)
+    def _join(self, k: int, s: _Scratch, ny: int, T: int, gain) -> dict:
+        """stream_rows arguments that let the sublayer output s.y (ny partial sums) join the stream s.x[k] through its norm."""
+        add = dict(x_in=s.x[k], y=s.y, y_slabs=ny, y_stride=T * self.width)
+        if self.d.norm == "post":
+            return dict(add, post=1, alpha=self.d.alpha, y_w=gain)
+        return dict(add, gain=gain)
 
     def forward(self, b: Batch, *, sel: torch.Tensor | None = None, logits: torch.Tensor | None = None, scratch: _Scratch | None = None,
                 trail: list | None = None) -> torch.Tensor | None:
@@ -351,32 +330,44 @@ class DecoderEngine:
         d, s = self.d, scratch or self._scratch(b.T)
         T = b.T
         frag = self.elem.code == 0 and T <= SKINNY
-        lw = lambda i: self.layer_w[d.owner(i)]  # noqa: E731
-        where = dict(row_of_tok=b.row_of_tok, positions=b.positions, state_slot=self.state_slot, rows=T)
         k = 0
-        self._rows(ids=b.ids, table=self.embed, vocab=d.vocab, mu=lw(0).mu, state=self.state[0], x_out=s.x[k], h_out=s.h, frag=int(frag), **where)
-        for i in range(d.num_layers):
-            w = lw(i)
-            ny, gain = self._mixer(b, i, s, s.x[k], frag), w.gain1
-            if d.layers[i].mlp is not None:
-                self._rows(x_in=s.x[k], y=s.y, y_slabs=ny, y_stride=T * self.width, gain=gain, x_out=s.x[k ^ 1], h_out=s.h, frag=int(frag), rows=T)
+
+        def operand(i: int | None, **source) -> None:
+            """The stream's new rows from `source`, and h of them: layer i's mixer input, or (None) the rows themselves."""
+            nonlocal k
+            if "x_in" in source:
                 k ^= 1
+            if i is not None and d.token_shift:
+                source.update(mu=self.layer_w[d.owner(i)].mu, state=self.shift_state[i], row_of_tok=b.row_of_tok, positions=b.positions, state_slot=self.state_slot)
+            self._rows(**source, x_out=s.x[k], h_out=s.h, frag=int(frag), rows=T)
+
+        operand(0, ids=b.ids, table=self.embed, vocab=d.vocab, table_scale=d.embed_scale)
+        for i in range(d.num_layers):
+            w = self.layer_w[d.owner(i)]
+            add = self._join(k, s, w.mixer.run(b, i, s, s.x[k], frag), T, w.norm1)
+            if d.layers[i].mlp is not None:
+                operand(None, **add)
                 self._mm(s.h, w.up, s.act, T, act=w.act, out_frag=frag)
-                ny, gain = self._mm(s.act, w.dn, s.y, T, f32_out=True), w.gain2
-            add = dict(x_in=s.x[k], y=s.y, y_slabs=ny, y_stride=T * self.width, gain=gain)
+                add = self._join(k, s, self._mm(s.act, w.dn, s.y, T, f32_out=True), T, w.norm2)
+            if d.side_dim:
+                operand(None, **add)
+                table = L.RowTable(self.side_embed[:, i * self.side_width:].data_ptr(), b.ids.data_ptr(), d.vocab, self.side_embed.shape[1])
+                self._mm_rows(s.h, w.side_gate, s.act, T, table, frag)
+                ny = self._mm(s.act, w.side_proj, s.y, T, f32_out=True)
+                add = dict(x_in=s.x[k], y=s.y, y_slabs=ny, y_stride=T * self.width, y_w=w.side_norm)
             if trail is not None:
                 self._rows(**add, x_out=s.x[k ^ 1], rows=T)
                 trail.append(s.x[k ^ 1][:T * self.width].view(T, self.width)[:, :d.hidden].clone())
             if i + 1 < d.num_layers:
-                self._rows(**add, mu=lw(i + 1).mu, state=self.state[i + 1], x_out=s.x[k ^ 1], h_out=s.h, frag=int(frag), **where)
-                k ^= 1
+                operand(i + 1, **add)
         n = T if sel is None else sel.numel()
         if n == 0:
             return None
         if n > s.rows:
             raise L.OmniError(f"logits of {n} rows from a batch of {T} tokens")
         nfrag = self.elem.code == 0 and n <= SKINNY
-        self._rows(**add, use_final=1, final_gain=self.final_gain, sel=sel, h_out=s.hn, frag=int(nfrag), rows=n)
+        final = dict(final_gain=self.final_norm) if isinstance(self.final_norm, float) else dict(final_w=self.final_norm)
+        self._rows(**add, use_final=1, **final, sel=sel, h_out=s.hn, frag=int(nfrag), rows=n)
         if logits is None:
             logits = torch.empty(n, self.head.N, dtype=torch.float32, device=self.device)
         self._mm(s.hn, self.head, logits.view(-1), n, f32_out=True, one=True)
@@ -391,17 +382,21 @@ class DecoderEngine:
 
     def decode_step(self, B: int, advance: bool = True) -> None:
         """One decode step of rows [0, B) from the persistent buffers (capturable): layers, logits, sampler, counters."""
-        b = Batch(B, B, self.input_ids, self.row_ids, self.positions, {}, self.d.max_model_len, self.num_live)
+        b = Batch(B, B, self.input_ids, self.row_ids, self.positions, self.d.max_model_len, num_live=self.num_live)
         self.forward(b, logits=self.logits[:B], scratch=self._dec)
         if advance and self.d.vocab <= self.MAX_SAMPLED_VOCAB:
             self.sample_rows_in_place(B, self.num_live)
 
     # ------------------------------------------------------------------ roofline accounting
     def step_bytes(self, ctx_lens) -> dict:
-        """Bytes a decode step must move: matrices of every layer run, the head, and the latents read and written."""
+        """Bytes a decode step must move: matrices of every layer run, the head, the cache read and written, the recurrent state read and written."""
         from .weights import decoder_weight_bytes
         es = torch.empty((), dtype=self.elem.torch).element_size()
-        per_tok = sum(s.mixer.kv_rank for s in self.d.layers) * es
         w = decoder_weight_bytes(self.d) * es // 2
-        return {"weights": w, "kv_read": int(sum(int(c) for c in ctx_lens)) * per_tok, "kv_write": len(ctx_lens) * per_tok,
-                "total": w + (int(sum(int(c) for c in ctx_lens)) + len(ctx_lens)) * per_tok}
+        read = wrote = 0
+        for c in ctx_lens:
+            for i in range(self.d.num_layers):
+                r, n = cache_traffic(self.d, i, int(c))
+                read, wrote = read + r * es, wrote + n * es
+        state = 2 * len(ctx_lens) * sum(state_bytes(self.d, i) for i in range(self.d.num_layers))
+        return {"weights": w, "kv_read": read, "kv_write": wrote, "state": state, "total": w + read + wrote + state}

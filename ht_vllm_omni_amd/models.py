@@ -29,8 +29,8 @@ class ModelEntry:
 
 
 @dataclass(frozen=True)
-class LatentCacheSpec:
-    """One layer's share of a cache block: block_size latents of (padded) width `width`."""
+class RowCacheSpec:
+    """One layer's share of a cache block: block_size rows of (padded) width `width` -- latents, or keys and values side by side."""
     block_size: int
     width: int
     dtype: torch.dtype
@@ -78,10 +78,10 @@ def _decoder() -> ModelEntry:
         return make_decoder_weights(dims, seed=seed)
 
     def cache_spec(dims, cfg, tp):
-        from .decoder_engine import ELEM, latent_width
+        from .decoder_mixers import ELEM, cache_row_widths
         e = ELEM[cfg.dtype]
-        return {f"model.layers.{l}.mixer": LatentCacheSpec(int(cfg.block_size), latent_width(s.mixer.kv_rank, e.code), e.torch)
-                for l, s in enumerate(dims.layers)}
+        rows = {l: sum(cache_row_widths(dims, l, e.code)) for l in range(dims.num_layers)}
+        return {f"model.layers.{l}.mixer": RowCacheSpec(int(cfg.block_size), w, e.torch) for l, w in rows.items() if w}
 
     def build_engine(worker, num_blocks):
         from .decoder_engine import DecoderEngine

@@ -294,7 +294,7 @@ def rope_table(max_pos: int, head_dim: int, theta: float) -> torch.Tensor:
 def gemm_tile(x: torch.Tensor, w_frag: torch.Tensor, *, M: int | None = None, bias=None, scale=None, act: int = L.TILE_ACT_NONE,
               resid=None, out=None, out_f32=None, out2=None, snake=None, taps: int = 1, dilation: int = 1,
               row_off: int | None = None, want: str = "b", tile_hint: int = 0, groups: int = 1, group_rows=None,
-              act_params: tuple[float, float] = (0.0, 0.0), group_cols: bool = False, lib=None):
+              act_params: tuple[float, float] = (0.0, 0.0), group_cols: bool = False, act_cols: int = 0, mul=None, lib=None):
     """omni_gemm_tile: y[M, N] = act(A . W^T + bias) * scale (+ resid) on the matrix cores, A = x for taps == 1, else the
     causal conv window A[m] = [x[m + row_off], x[m + row_off + dilation], ...] (taps rows of x.shape[1] channels; row_off
     defaults to -(taps - 1) * dilation; rows outside x read as zero).  x bf16 [rows, C] (row stride = x.stride(0)); w_frag bf16
@@ -305,7 +305,8 @@ def gemm_tile(x: torch.Tensor, w_frag: torch.Tensor, *, M: int | None = None, bi
     groups > 1: the batched form -- x [groups * cap, C] (cap rows per group), w_frag [groups, N, K] (each matrix fragment-major),
     outputs [groups * cap, N]; group_rows int32 [groups] (device) = live rows per group (the rest is neither computed nor written).
     group_cols: the groups are column ranges instead -- x [rows, groups * K], output [rows, groups * N] (one product per head).
-    act_params: the two coefficients of TILE_ACT_XIELU.  lib: the library to launch from (default: the talker's)."""
+    act_params: the two coefficients of TILE_ACT_XIELU; act_cols: where TILE_ACT_SILU_SIGMOID changes over; mul: the omni_row_table of
+    TILE_ACT_GELU_MUL.  lib: the library to launch from (default: the talker's)."""
     assert x.dtype == BF16 and w_frag.dtype == BF16 and x.dim() == 2 and x.stride(1) == 1
     rows, Cin = x.shape
     if group_cols:
@@ -324,6 +325,9 @@ def gemm_tile(x: torch.Tensor, w_frag: torch.Tensor, *, M: int | None = None, bi
     nout = (N // 2 if gu8 else N) * (groups if group_cols else 1)
     g = L.TileGemm()
     g.act_p, g.act_n = act_params
+    g.act_cols = act_cols
+    if mul is not None:
+        g.mul_table, g.mul_ids, g.mul_rows, g.mul_ld = mul.table, mul.ids, mul.rows, mul.ld
     g.x, g.x_rows, g.ldx = x.data_ptr(), rows, x.stride(0)
     g.seg_len, g.seg_rows = Cin, dilation
     g.row_off = (-(taps - 1) * dilation if row_off is None else row_off) if taps > 1 or row_off is not None else 0

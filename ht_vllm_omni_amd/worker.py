@@ -266,7 +266,11 @@ class MI355XARWorker:
                 per.append(int(getattr(tns, "size")) // page)
             nb = min(per)
         if nb is None:
-            nb = max(self.determine_available_memory() // self.kv_bytes_per_block(), 2)
+            page = self.kv_bytes_per_block()
+            if page:
+                nb = max(self.determine_available_memory() // page, 2)
+            else:                            # nothing is paged (recurrent layers only): blocks are a count
+                nb = cfg.max_num_seqs * -(-self.dims.max_model_len // cfg.block_size) + 1
         if self.engine is not None:          # built (and measured) by determine_available_memory on a probe cache: give it the real one
             self.engine.resize_kv_cache(int(nb))
         else:

@@ -54,7 +54,7 @@ extern "C" {
                                  * finished act columns, so any number of tiles per workgroup divides the chip evenly */
 
 const char* omni_last_error(void);
-int omni_abi_version(void);   /* 6: omni_tile_gemm column groups and the xIELU activation (5: omni_ar_peers.tile_flags, omni_talker_set_chains
+int omni_abi_version(void);   /* 7: omni_tile_gemm activations RELU2, SILU_SIGMOID, GELU_MUL (6: column groups, xIELU; 5: omni_ar_peers.tile_flags, omni_talker_set_chains
                                  modes 2 / 3, a zero-filled attention workspace) */
 
 /* ------------------------------------------------------------------ per-op entry points */
@@ -148,7 +148,9 @@ int omni_moe_experts_resid(const void* x, const int32_t* topk_idx, const void* t
  *            K = k * C_in, seg_len = C_in, seg_rows = d, row_off = -(k - 1) * d.
  *   w        bf16 [N, K] fragment-major (OMNI_LAYOUT_W_FRAG); N % 16 == 0, K % 32 == 0, seg_len % 32 == 0.
  *   bias / scale  fp32 [N] or NULL.  y = act(acc + bias) * scale (+ resid), all fp32.
- *   act      OMNI_TILE_ACT_NONE | _GELU (erf) | _XIELU (act_p, act_n) | _SILU_MUL_GU8 (w rows interleaved as OMNI_EPI_SILU_MUL_GU8; out is [M, N / 2],
+ *   act      OMNI_TILE_ACT_NONE | _GELU (erf) | _XIELU (act_p, act_n) | _RELU2 (max(y, 0)^2) | _SILU_SIGMOID (SiLU in columns
+ *            [0, act_cols), sigmoid behind them) | _GELU_MUL (gelu_tanh(y) times a bf16 table row: mul_table[mul_ids[m] * mul_ld + n], 0 for an id
+ *            outside [0, mul_rows); bf16 out only) | _SILU_MUL_GU8 (w rows interleaved as OMNI_EPI_SILU_MUL_GU8; out is [M, N / 2],
  *            = bf16(bf16(SiLU(bf16 gate)) * bf16 up), omni_silu_mul's rounding points; no other output).
  *   resid    fp32 [M, ldr] or NULL (may alias out_f32: the residual stream updated in place).
  *   out_f32  fp32 [M, ldf] or NULL: y.   out  bf16 [M, ldo] or NULL: bf16(y).
@@ -158,6 +160,9 @@ int omni_moe_experts_resid(const void* x, const int32_t* topk_idx, const void* t
 #define OMNI_TILE_ACT_GELU 1
 #define OMNI_TILE_ACT_SILU_MUL_GU8 2
 #define OMNI_TILE_ACT_XIELU 3
+#define OMNI_TILE_ACT_RELU2 4
+#define OMNI_TILE_ACT_SILU_SIGMOID 5
+#define OMNI_TILE_ACT_GELU_MUL 6
 typedef struct omni_tile_gemm {
     const void* x; int64_t x_rows; int ldx;
     int seg_len, seg_rows, row_off;
@@ -180,6 +185,8 @@ typedef struct omni_tile_gemm {
     float act_p, act_n;                          /* OMNI_TILE_ACT_XIELU: coefficients of the two branches */
     int64_t x_group_cols, out_group_cols;        /* groups > 1: column offset of group g in x / out / out_f32 (elements): per-head products of
                                                     one [tokens, heads * K] array with x_group_rows = out_group_rows = 0 */
+    int act_cols;                                /* OMNI_TILE_ACT_SILU_SIGMOID (% 4 == 0) */
+    const void* mul_table; const int32_t* mul_ids; int mul_rows, mul_ld;      /* OMNI_TILE_ACT_GELU_MUL (mul_ld % 8 == 0) */
 } omni_tile_gemm;
 int omni_gemm_tile(const omni_tile_gemm* g, void* stream);
 

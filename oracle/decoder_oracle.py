@@ -96,3 +96,116 @@ def zefedra_forward(weights: dict, config: dict, tokens: list[int], dtype=torch.
             x = x + scalar_rms_norm(xielu_mlp(x, mlp), own["norm2"], eps)
         trail.append(x)
     return scalar_rms_norm(x, weights["final.norm"], eps) @ weights["head"].T, trail
+
+
+# ---------------------------------------------------------------- Koronex
+# A decoder-only language model of two sequence mixers, norms behind the sums and a second token embedding read by every layer:
+#   layer      x = norm(a x + mixer(x), w1);  x = norm(a x + ff(x), w2)  (a layer may have no feed-forward);  x += side input of the token
+#   mixers     lightning: a linear recurrence with one decay per head;  attention: a sliding window, grouped key / value heads, partly rotated,
+#              one extra number per head in the softmax's denominator; a layer may read an earlier layer's keys and values
+#   head       logits = W norm(s, w_f), the stream starts at scale * embedding
+
+
+def gelu_tanh(z: torch.Tensor) -> torch.Tensor:
+    return 0.5 * z * (1 + torch.tanh(math.sqrt(2 / math.pi) * (z + 0.044715 * z ** 3)))
+
+
+def post_norm(x: torch.Tensor, y: torch.Tensor, w: torch.Tensor, alpha: float, eps: float) -> torch.Tensor:
+    return rms_norm(alpha * x + y, w, eps)
+
+
+def side_input(x: torch.Tensor, e: torch.Tensor, w: dict, eps: float) -> torch.Tensor:
+    """What a token's own embedding e adds to its stream row; w: gate, proj, norm."""
+    return rms_norm((gelu_tanh(x @ w["gate"].T) * e) @ w["proj"].T, w["norm"], eps)
+
+
+def relu2_mlp(x: torch.Tensor, w: dict) -> torch.Tensor:
+    return torch.relu(x @ w["up"].T) ** 2 @ w["down"].T
+
+
+def decay_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay) -> torch.Tensor:
+    """q, k [T, H, D], v [T, H, E]: S <- decay S + k v^T, o = S^T q, token by token from a zero state."""
+    T, H, D = q.shape
+    out = torch.empty(T, H, v.shape[-1], dtype=q.dtype)
+    for h in range(H):
+        S = torch.zeros(D, v.shape[-1], dtype=q.dtype)
+        for t in range(T):
+            S = decay[h] * S + k[t, h][:, None] * v[t, h][None, :]
+            out[t, h] = q[t, h] @ S
+    return out
+
+
+def lightning(h: torch.Tensor, w: dict, heads: int, dim: int, vdim: int, decay, eps: float) -> torch.Tensor:
+    """w: q, k, v, g, o, norm."""
+    T = h.shape[0]
+    silu = lambda z: z * torch.sigmoid(z)  # noqa: E731
+    q, k, v = silu(h @ w["q"].T).reshape(T, heads, dim), silu(h @ w["k"].T).reshape(T, heads, dim), silu(h @ w["v"].T).reshape(T, heads, vdim)
+    o = decay_recurrence(q, k, v, decay).reshape(T, heads * vdim)
+    return (rms_norm(o, w["norm"], eps) * torch.sigmoid(h @ w["g"].T)) @ w["o"].T
+
+
+def rotate_half(x: torch.Tensor, dims: int, base: float) -> torch.Tensor:
+    """x [T, H, D]: dimensions i and i + dims / 2 of the first `dims` turn by t * base^(-2 i / dims)."""
+    out, half = x.clone(), dims // 2
+    freq = torch.tensor([base ** (-2.0 * i / dims) for i in range(half)], dtype=torch.float64)
+    for t in range(x.shape[0]):
+        a = (t * freq).to(torch.float64)
+        c, s = a.cos().to(x.dtype), a.sin().to(x.dtype)
+        u, v = x[t, :, :half], x[t, :, half:dims]
+        out[t, :, :half], out[t, :, half:dims] = u * c - v * s, v * c + u * s
+    return out
+
+
+def window_attention(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, scale: float, window: int | None = None, sink: torch.Tensor | None = None) -> torch.Tensor:
+    """q [T, H, D], k [T, G, D], v [T, G, E] -> [T, H, E]: token i sees j <= i with i - j < window; the softmax's denominator counts exp(sink) once."""
+    T, H, _ = q.shape
+    G = k.shape[1]
+    out = torch.empty(T, H, v.shape[-1], dtype=q.dtype)
+    i, j = torch.arange(T)[:, None], torch.arange(T)[None, :]
+    seen = (j <= i) if window is None else (j <= i) & (i - j < window)
+    for h in range(H):
+        g = h // (H // G)
+        s = (q[:, h] @ k[:, g].T * scale).masked_fill(~seen, -math.inf)
+        if sink is not None:
+            s = torch.cat([s, sink[h].to(s.dtype).reshape(1, 1).expand(T, 1)], 1)
+        out[:, h] = torch.softmax(s, -1)[:, :T] @ v[:, g]
+    return out
+
+
+def attention_keys(h: torch.Tensor, w: dict, m: dict, eps: float) -> tuple[torch.Tensor, torch.Tensor]:
+    """(keys behind norm and rotation, values) of a layer with projections of its own."""
+    T = h.shape[0]
+    k = rms_norm(h @ w["k"].T, w["k_norm"], eps).reshape(T, m["kv_heads"], m["dim"])
+    return rotate_half(k, m["rot"]["dims"], m["rot"]["base"]), (h @ w["v"].T).reshape(T, m["kv_heads"], m["vdim"])
+
+
+def grouped_attention(h: torch.Tensor, w: dict, m: dict, k: torch.Tensor, v: torch.Tensor, eps: float) -> torch.Tensor:
+    """w: q, q_norm, sink, g, o; k, v of this layer or of the one it reads."""
+    T = h.shape[0]
+    q = rms_norm(h @ w["q"].T, w["q_norm"], eps).reshape(T, m["heads"], m["dim"])
+    o = window_attention(rotate_half(q, m["rot"]["dims"], m["rot"]["base"]), k, v, m["scale"], m["mask"]["size"], w["sink"])
+    return (o.reshape(T, -1) * torch.sigmoid(h @ w["g"].T)) @ w["o"].T
+
+
+def koronex_forward(weights: dict, config: dict, tokens: list[int], dtype=torch.float32) -> tuple[torch.Tensor, list[torch.Tensor]]:
+    """(logits [T, vocab], residual stream after every layer) of one whole sequence."""
+    weights = {k: t.to(dtype) for k, t in weights.items()}
+    eps, alpha, sd = float(config["norm"]["eps"]), float(config["postln_alpha"]), config["token_side"]["dim"]
+    ids = torch.as_tensor(tokens)
+    x = weights["embed"][ids] * config["embedding"]["scale"]
+    trail, kv = [], {}
+    for i, spec in enumerate(config["layers"]):
+        own, mix, mlp = layer_tensors(weights, config, i)
+        m = spec["mixer"]
+        if spec["type"] == "lightning":
+            y = lightning(x, mix, m["heads"], m["dim"], m["vdim"], m["decay"], eps)
+        else:
+            src = m.get("kv_from")
+            kv[i] = kv[src] if src is not None else attention_keys(x, mix, m, eps)
+            y = grouped_attention(x, mix, m, *kv[i], eps)
+        x = post_norm(x, y, own["norm1"], alpha, eps)
+        if spec["mlp"] is not None:
+            x = post_norm(x, relu2_mlp(x, mlp), own["norm2"], alpha, eps)
+        x = x + side_input(x, weights["side.embed"][ids][:, i * sd:(i + 1) * sd], {n: own["side." + n] for n in ("gate", "proj", "norm")}, eps)
+        trail.append(x)
+    return rms_norm(x, weights["final.norm"], eps) @ weights["head"].T, trail

@@ -9,13 +9,14 @@ from ht_vllm_omni_amd import models
 from ht_vllm_omni_amd.checkpoint import load_decoder_checkpoint
 from ht_vllm_omni_amd.config import TalkerDims
 from ht_vllm_omni_amd.decoder_config import dims_from_config, tensor_shapes
-from ht_vllm_omni_amd.decoder_engine import LATENT_WIDTHS, attention_tiles, latent_width
+from ht_vllm_omni_amd.decoder_mixers import (LATENT_WIDTHS, attention_tiles, cache_row_widths, cache_traffic, latent_width, pad_head_cols, pad_head_rows, pad_heads,
+                                             recurrence_chunks, recurrence_segments, state_bytes)
 from ht_vllm_omni_amd.payloads import OmniModelRunnerOutput, SamplingParams
 from ht_vllm_omni_amd.sched import SlotPool
 from ht_vllm_omni_amd.scheduler import MI355XARScheduler, Request
 from ht_vllm_omni_amd.worker import MI355XARWorker, make_config
 from oracle import decoder_oracle as D
-from tests.decoder_util import CONFIGS, G, config, layer, model
+from tests.decoder_util import CONFIGS, G, attention, config, koronex, layer, lightning, model
 
 
 # ---------------------------------------------------------------- configuration
@@ -192,3 +193,118 @@ def test_oracle_borrowed_layer_is_the_owner_run_again():
     for i, o in ((2, 0), (3, 1)):
         copies.update({k.replace(f"l{o}.", f"l{i}.", 1): t for k, t in w.items() if k.startswith(f"l{o}.")})
     assert torch.equal(D.zefedra_forward(w, cfg, toks)[0], D.zefedra_forward(copies, full, toks)[0])
+
+
+# ---------------------------------------------------------------- Koronex
+def test_koronex_config_gives_every_size_and_constant():
+    cfg = koronex([lightning(3, 11, 13, [0.25, 0.5, 1.0], ff=None), attention(6, 3, 14, 9, 0.77, 5, 6, 321.0, ff=23), attention(2, 3 - 2, 4, 5, 0.1, 7, 0, 2.0),
+                   attention(9, 3, 14, 9, 0.5, 2, 6, 321.0, kv_from=1)], width=29, vocab=31, eps=3e-4, alpha=1.25, scale=0.5, side=7)
+    d = dims_from_config(cfg, 99)
+    a, b = d.layers[0].mixer, d.layers[1].mixer
+    assert (a.heads, a.dim, a.vdim, a.decay) == (3, 11, 13, (0.25, 0.5, 1.0)) and d.layers[0].mlp is None
+    assert (b.heads, b.kv_heads, b.dim, b.vdim, b.scale, b.window, b.rot_dims, b.rot_base, b.kv_from) == (6, 3, 14, 9, 0.77, 5, 6, 321.0, None)
+    assert b.qk_norm and b.sink and b.out_gate and (d.layers[1].mlp.ff, d.layers[1].mlp.act) == (23, "relu2")
+    assert (d.layers[3].mixer.kv_from, d.layers[3].mixer.window, d.kv_owner(3), d.kv_owner(1), d.kv_owner(0)) == (1, 2, 1, 1, None)
+    assert (d.hidden, d.vocab, d.eps, d.alpha, d.embed_scale, d.side_dim, d.norm, d.token_shift, d.max_model_len) == (29, 31, 3e-4, 1.25, 0.5, 7, "post", False, 99)
+    names = tensor_shapes(d)
+    assert names["side.embed"] == (31, 4 * 7) and names["l0.mix.norm"] == (3 * 13,) and names["l1.mix.k.norm"] == (3 * 14,) and names["l3.mix.q.norm"] == (9 * 14,)
+    assert names["l1.mix.g"] == (6 * 9, 29) and names["l1.mix.sink"] == (6,) and names["final.norm"] == (29,) and names["l2.side.proj"] == (29, 7)
+    assert not any(n.startswith("l3.mix.") and n.split(".")[2] in ("k", "v") for n in names) and "l0.norm2" not in names and "l1.shift" not in names
+
+
+@pytest.mark.parametrize("layers", [
+    [attention(kv_from=0)], [attention(), attention(kv_from=1)], [lightning(), attention(kv_from=0)], [attention(), attention(kv_from=0), attention(kv_from=1)],
+    [attention(), attention(kv_from=0, dim=44)], [attention(), attention(kv_from=0, rot=8)], [attention(), attention(3, 1, kv_from=0)], [attention(7, 2)], [attention(rot=41)],
+    [attention(rot=42)], [attention(window=0)], [lightning(2, decay=[0.5])], [lightning(1, decay=[0.0])], [dict(lightning(), type="delta")], [dict(attention(), weights_of=0)],
+    [dict(attention(), mlp={"kind": "experts", "ff": 8})], [dict(attention(), mixer=dict(attention()["mixer"], cap=30.0))],
+    [dict(attention(), mixer={k: v for k, v in attention()["mixer"].items() if k != "rot"})]])
+def test_unknown_or_contradictory_koronex_configs_are_refused(layers):
+    with pytest.raises(ValueError):
+        dims_from_config(koronex(layers))
+
+
+def test_what_a_layer_keeps():
+    """Cache pages for layers with keys of their own, state for recurrences, neither for a layer that reads another's."""
+    d = model("k_mixed")[0]
+    assert models.entry_for_dims(d).name == "decoder" and models.entry_for_config(CONFIGS["k_mixed"]).name == "decoder"
+    assert [sum(cache_row_widths(d, i, 0)) for i in range(6)] == [2 * (64 + 32), 0, 0, 0, 4 * 64, 0]
+    wk = MI355XARWorker(make_config(d, max_num_seqs=3))
+    assert sorted(wk.get_kv_cache_spec()) == ["model.layers.0.mixer", "model.layers.4.mixer"] and wk.kv_bytes_per_block() == 16 * 2 * (192 + 256)
+    assert [state_bytes(d, i) for i in range(6)] == [0, 4 * 3 * 24 * 40, 0, 4 * 2 * 40 * 16, 0, 0]
+    assert cache_traffic(d, 2, 100) == (20 * 2 * 64, 0) and cache_traffic(d, 0, 4) == (4 * 2 * 64, 2 * 64) and cache_traffic(d, 1, 50) == (0, 0)
+    assert MI355XARWorker(make_config(model("k_state")[0])).kv_bytes_per_block() == 0
+
+
+def test_recurrence_chunks_cover_every_token_once():
+    starts, lens = [3, 8, 400], [5, 300, 128]
+    ch, sg = recurrence_chunks(starts, lens), recurrence_segments(starts, lens)
+    assert [t for f, n, _, _ in ch for t in range(f, f + n)] == [t for s, n in zip(starts, lens) for t in range(s, s + n)]
+    assert sg == [(0, 1), (1, 3), (4, 1)] and [c[2] for c in ch] == [0, 0, 1, 2, 0] and max(c[1] for c in ch) == 128
+
+
+def test_heads_are_padded_where_they_lie():
+    w = torch.arange(2 * 3 * 5, dtype=torch.float32).reshape(6, 5) + 1
+    p = pad_head_rows(w, 2, 3, 4, 8)
+    assert p.shape == (8, 8) and torch.equal(p[4:7, :5], w[3:]) and not p[3].any() and not p[:, 5:].any()
+    c = pad_head_cols(w.T.contiguous(), 2, 3, 4, 6)
+    assert torch.equal(c[:5], p[:, :5].T) and not c[5].any()
+    assert pad_heads(torch.ones(6), 2, 3, 4).tolist() == [1, 1, 1, 0, 1, 1, 1, 0]
+
+
+def test_oracle_recurrence_and_lightning():
+    g = torch.Generator().manual_seed(4)
+    rnd = lambda *s: torch.randn(*s, generator=g, dtype=torch.float64)  # noqa: E731
+    T, H, dim, vdim, W = 6, 2, 3, 4, 5
+    decay = [0.5, 0.9]
+    w = dict(q=rnd(H * dim, W), k=rnd(H * dim, W), v=rnd(H * vdim, W), g=rnd(H * vdim, W), o=rnd(W, H * vdim), norm=rnd(H * vdim))
+    h = rnd(T, W)
+    got = D.lightning(h, w, H, dim, vdim, decay, 1e-3)
+    silu = lambda z: z / (1 + math.exp(-z))  # noqa: E731
+    act = lambda m, t: [silu(float(r @ h[t])) for r in m]  # noqa: E731
+    for t in range(T):
+        o = []
+        for n in range(H):
+            q = act(w["q"], t)[n * dim:(n + 1) * dim]
+            for e in range(vdim):                                          # o = sum over earlier tokens of decay^(age) (q . k_j) v_j
+                o.append(sum(decay[n] ** (t - j) * sum(a * b for a, b in zip(q, act(w["k"], j)[n * dim:(n + 1) * dim])) * act(w["v"], j)[n * vdim + e] for j in range(t + 1)))
+        r = math.sqrt(sum(v * v for v in o) / len(o) + 1e-3)
+        y = torch.tensor([v / r * float(w["norm"][i]) / (1 + math.exp(-float(w["g"][i] @ h[t]))) for i, v in enumerate(o)], dtype=torch.float64)
+        assert torch.allclose(got[t], w["o"] @ y, atol=1e-9)
+
+
+def test_oracle_window_attention_rotation_and_sink():
+    g = torch.Generator().manual_seed(5)
+    rnd = lambda *s: torch.randn(*s, generator=g, dtype=torch.float64)  # noqa: E731
+    T, H, G, dim, vdim, rot, base = 7, 4, 2, 6, 3, 4, 50.0
+    q, k, v, sink = rnd(T, H, dim), rnd(T, G, dim), rnd(T, G, vdim), rnd(H)
+    turned = D.rotate_half(q, rot, base)
+    for t in range(T):
+        for n in range(H):
+            for i, f in ((0, 1.0), (1, base ** -0.5)):
+                z = complex(q[t, n, i], q[t, n, i + 2]) * complex(math.cos(t * f), math.sin(t * f))
+                assert float(turned[t, n, i]) == pytest.approx(z.real) and float(turned[t, n, i + 2]) == pytest.approx(z.imag)
+    assert torch.equal(turned[:, :, rot:], q[:, :, rot:])
+    for window in (1, 3, None):
+        got = D.window_attention(q, k, v, 0.4, window, sink)
+        for t in range(T):
+            for n in range(H):
+                js = [j for j in range(t + 1) if window is None or t - j < window]
+                e = [math.exp(0.4 * float(q[t, n] @ k[j, n // 2])) for j in js]
+                want = sum(a * v[j, n // 2] for a, j in zip(e, js)) / (sum(e) + math.exp(float(sink[n])))
+                assert torch.allclose(got[t, n], want, atol=1e-10)
+
+
+def test_oracle_koronex_layer_parts():
+    g = torch.Generator().manual_seed(6)
+    rnd = lambda *s: torch.randn(*s, generator=g, dtype=torch.float64)  # noqa: E731
+    x, y, w = rnd(2, 4), rnd(2, 4), rnd(4)
+    z = 1.5 * x + y
+    assert torch.allclose(D.post_norm(x, y, w, 1.5, 0.1), torch.stack([r / math.sqrt(float((r * r).mean()) + 0.1) * w for r in z]))
+    s = dict(gate=rnd(3, 4), proj=rnd(4, 3), norm=rnd(4))
+    e = rnd(2, 3)
+    gelu = lambda u: 0.5 * u * (1 + math.tanh(math.sqrt(2 / math.pi) * (u + 0.044715 * u ** 3)))  # noqa: E731
+    for t, got in enumerate(D.side_input(x, e, s, 0.1)):
+        r = s["proj"] @ torch.tensor([gelu(float(s["gate"][i] @ x[t])) * float(e[t, i]) for i in range(3)], dtype=torch.float64)
+        assert torch.allclose(got, r / math.sqrt(float((r * r).mean()) + 0.1) * s["norm"])
+    m = dict(up=rnd(3, 4), down=rnd(4, 3))
+    assert torch.allclose(D.relu2_mlp(x, m)[0], m["down"] @ torch.tensor([max(float(r @ x[0]), 0.0) ** 2 for r in m["up"]], dtype=torch.float64))

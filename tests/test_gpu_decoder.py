@@ -14,8 +14,7 @@ from ht_vllm_omni_amd.payloads import SamplingParams
 from ht_vllm_omni_amd.replay import Replayer
 from ht_vllm_omni_amd.scheduler import Request
 from ht_vllm_omni_amd.serving import serve
-from oracle import decoder_oracle as D
-from tests.decoder_util import CONFIGS, TOL, assert_logits, model, oracle_logits, tokens
+from tests.decoder_util import CONFIGS, TOL, assert_logits, model, oracle, oracle_logits, tokens
 
 pytestmark = pytest.mark.gpu
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
@@ -45,7 +44,7 @@ def test_residual_stream_of_every_layer(name, dtype):
     b = eng.make_batch(torch.tensor(toks), np.full(77, 2), np.arange(77), [77])
     trail = []
     logits = eng.forward(b, trail=trail)
-    ref, ref_trail = D.zefedra_forward(w, cfg, toks)
+    ref, ref_trail = oracle(w, cfg, toks)
     for i, (a, r) in enumerate(zip(trail, ref_trail)):
         err = float((a.cpu() - r).pow(2).mean().sqrt() / r.pow(2).mean().sqrt())
         assert err <= TOL[dtype], f"layer {i}: {err:.3g}"
@@ -55,16 +54,18 @@ def test_residual_stream_of_every_layer(name, dtype):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("n", [1, 2, 16, 17, 64, 65, 300, 700])
-def test_whole_prompts(n, dtype):
-    d, w, cfg = model("mixed", seed=2, sharp=3.0)
+@pytest.mark.parametrize("name", ["mixed", "k_mixed"])
+def test_whole_prompts(name, n, dtype):
+    d, w, cfg = model(name, seed=2, sharp=3.0)
     rep = Replayer(d, dtype, 1024, weights=w)
     toks = tokens(n, d.vocab, n)
     assert_logits(feed(rep, "a", toks, [n]), oracle_logits(w, cfg, toks), dtype, f"{n} tokens")
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-def test_wide_model_long_prompt(dtype):
-    d, w, cfg = model("wide", seed=3, sharp=2.0)
+@pytest.mark.parametrize("name", ["wide", "k_wide", "k_plain"])
+def test_wide_model_long_prompt(name, dtype):
+    d, w, cfg = model(name, seed=3, sharp=2.0)
     rep = Replayer(d, dtype, 1024, weights=w)
     toks = tokens(600, d.vocab, 5)
     assert_logits(feed(rep, "a", toks, [590, 1]), oracle_logits(w, cfg, toks), dtype)
@@ -72,7 +73,7 @@ def test_wide_model_long_prompt(dtype):
 
 # ---------------------------------------------------------------- decoding and portions
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("name", ["mixed", "narrow", "behind"])
+@pytest.mark.parametrize("name", ["mixed", "narrow", "behind", "k_mixed", "k_narrow", "k_state"])
 def test_token_by_token_equals_the_whole_prompt(name, dtype):
     d, w, cfg = model(name, seed=4, sharp=4.0)
     rep = Replayer(d, dtype, 128, weights=w)
@@ -84,17 +85,19 @@ def test_token_by_token_equals_the_whole_prompt(name, dtype):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("cuts", [[2], [3, 2], [16], [15, 2, 31, 1, 1, 5], [64, 2], [65, 64], [33, 1]])
-def test_portions(cuts, dtype):
-    d, w, cfg = model("mixed", seed=5, sharp=4.0)
+@pytest.mark.parametrize("name", ["mixed", "k_mixed", "k_wide"])
+def test_portions(name, cuts, dtype):
+    d, w, cfg = model(name, seed=5, sharp=4.0)
     rep = Replayer(d, dtype, 256, weights=w)
     toks = tokens(190, d.vocab, 7)
     assert_logits(feed(rep, "a", toks, cuts), oracle_logits(w, cfg, toks), dtype, str(cuts))
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-def test_long_decoding_with_far_keys(dtype):
+@pytest.mark.parametrize("name,sharp", [("narrow", 8.0), ("k_mixed", 3.0)])
+def test_long_decoding_with_far_keys(name, sharp, dtype):
     """Sharp scores (single keys decide), 400 decoded tokens behind a prompt of 3: keys hundreds of tokens back, over many page borders."""
-    d, w, cfg = model("narrow", seed=6, sharp=8.0)
+    d, w, cfg = model(name, seed=6, sharp=sharp)
     rep = Replayer(d, dtype, 512, weights=w)
     toks = tokens(403, d.vocab, 8)
     assert_logits(feed(rep, "a", toks, [3, 1]), oracle_logits(w, cfg, toks), dtype)
@@ -102,7 +105,7 @@ def test_long_decoding_with_far_keys(dtype):
 
 # ---------------------------------------------------------------- batches, pages, slots
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("name", ["mixed", "wide"])
+@pytest.mark.parametrize("name", ["mixed", "wide", "k_mixed", "k_wide", "k_plain", "k_state"])
 def test_mixed_batches_equal_each_request_alone(name, dtype):
     """Up to four live requests at different places, portions beside single tokens, some left out of a step, ends and re-admissions into a pool
     that only just holds them: pages and slots change owners all the time."""
@@ -145,9 +148,10 @@ def test_mixed_batches_equal_each_request_alone(name, dtype):
         assert_logits(torch.cat(got[k]), refs[k], dtype, k)
 
 
-def test_a_reused_slot_and_page_hold_nothing_of_their_last_owner():
+@pytest.mark.parametrize("name", ["mixed", "k_mixed"])
+def test_a_reused_slot_and_page_hold_nothing_of_their_last_owner(name):
     """The same request before and after the pool was filled by others: identical bits."""
-    d, w, _ = model("mixed", seed=8)
+    d, w, _ = model(name, seed=8)
     rep = Replayer(d, "bfloat16", 128, max_live=1, weights=w)
     toks = tokens(50, d.vocab, 3)
     first = feed(rep, "a", toks, [20, 1])
@@ -187,7 +191,7 @@ def generate(d, w, prompts, n, **kw):
     return [out[str(i)] for i in range(len(prompts))], core
 
 
-@pytest.mark.parametrize("name", ["mixed", "wide"])
+@pytest.mark.parametrize("name", ["mixed", "wide", "k_mixed", "k_narrow"])
 def test_greedy_generation_equals_the_oracles(name):
     """fp32 through the engine-core loop: prompts that chunk over the token budget, decode graphs, requests that finish and make room."""
     d, w, cfg = model(name, seed=10, sharp=2.0)
@@ -199,10 +203,11 @@ def test_greedy_generation_equals_the_oracles(name):
         assert g == want or min(margins) < 1e-4, (g, want, min(margins))
 
 
-def test_generation_does_not_depend_on_how_it_is_run():
+@pytest.mark.parametrize("name", ["mixed", "k_mixed"])
+def test_generation_does_not_depend_on_how_it_is_run(name):
     """bf16: graphs or eager, synchronous or asynchronous, ample or scarce cache (preemption: recomputed requests), seeded sampling -- the same ids
     up to near-ties, and the same ids exactly where the kernels are the same."""
-    d, w, _ = model("mixed", seed=11)
+    d, w, _ = model(name, seed=11)
     prompts = [tokens(n, d.vocab, 80 + n) for n in (7, 30, 18, 25)]
     sp = SamplingParams(temperature=0.8, top_k=20, repetition_penalty=1.1, seed=5, max_tokens=20, stop_token_ids=(), logprobs=2)
     base = dict(num_blocks=40, max_num_seqs=4, max_model_len=128, sampling=sp)
@@ -215,10 +220,11 @@ def test_generation_does_not_depend_on_how_it_is_run():
     assert tight == roomy, "preempted requests must carry on where they were"
 
 
-def test_replays_of_a_captured_step_match_eager_steps():
+@pytest.mark.parametrize("name", ["behind", "k_mixed"])
+def test_replays_of_a_captured_step_match_eager_steps(name):
     """A captured decode step replayed several times, with the runner's own eager prompt steps between the replays, against an engine that never
     captures (same bits: same kernels)."""
-    d, w, _ = model("behind", seed=12)
+    d, w, _ = model(name, seed=12)
     outs = []
     for eager in (False, True):
         sp = SamplingParams(temperature=0.0, repetition_penalty=1.0, max_tokens=9, stop_token_ids=())
@@ -256,8 +262,9 @@ def test_stops_logprobs_and_seeds():
     assert core.scheduler.pool.num_free == 19 and not core.worker.model_runner.slots.owned
 
 
-def test_worker_measures_memory_and_resizes_the_cache():
-    d, w, cfg = model("mixed", seed=14)
+@pytest.mark.parametrize("name", ["mixed", "k_mixed"])
+def test_worker_measures_memory_and_resizes_the_cache(name):
+    d, w, cfg = model(name, seed=14)
     from ht_vllm_omni_amd.worker import MI355XARWorker, make_config
     wk = MI355XARWorker(make_config(d.with_(max_model_len=256), weights=w, max_num_seqs=2))
     wk.init_device()
@@ -269,10 +276,11 @@ def test_worker_measures_memory_and_resizes_the_cache():
 
 
 # ---------------------------------------------------------------- command line
-def test_command_lines(tmp_path):
+@pytest.mark.parametrize("name", ["behind", "k_narrow"])
+def test_command_lines(name, tmp_path):
     """bin/trace_run and `generate` on a checkpoint directory, in processes of their own."""
     from safetensors.torch import save_file
-    d, w, cfg = model("behind", seed=15)
+    d, w, cfg = model(name, seed=15)
     save_file(w, str(tmp_path / "model.safetensors"))
     (tmp_path / "config.json").write_text(json.dumps(cfg))
     toks = tokens(21, d.vocab, 4)
