@@ -14,9 +14,10 @@ the child's code; under torchrun (WORLD_SIZE set) each rank runs the tensor-para
 The timed window is centred on the BASELINE context (mean ctx 352) whatever --steps is: untimed decode steps advance
 the batch there first, over KV the steps themselves wrote.  Prints ONE JSON line on rank 0.
 
-  python bench.py --decoder [2048|1024|all]
-Another measurement, of its own: prefill and decode throughput of the decoder-only design (Zefedra-shaped layers, random weights) beside the
-talker's backbone at equal width, depth and matrix bytes.  The default workload is not run.
+  python bench.py --decoder [2048|1024|all]        (Zefedra-shaped layers beside the talker backbone)
+  python bench.py --koronex [2048|1024|all]        (Koronex-shaped layers beside Zefedra-shaped ones)
+Other measurements, of their own: prefill and decode throughput of a decoder-only design (random weights) beside the closest other model at equal
+width, depth and matrix bytes.  The default workload is not run.
 """
 from __future__ import annotations
 
@@ -280,10 +281,46 @@ def eager_ms(fn, n=5, warm=2):
     return e0.elapsed_time(e1) / n
 
 
-def decoder_bench(args):
+# Koronex-shaped models beside the Zefedra ones of the same width, depth and (within 2 %) matrix bytes per layer: recurrence and windowed attention in turn
+KORONEX_SIZES = {
+    "2048": dict(width=2048, heads=16, kv_heads=4, dim=128, vdim=128, window=1024, rot=64, rec_heads=16, rec_dim=128, ff=7936, side=256),
+    "1024": dict(width=1024, heads=16, kv_heads=4, dim=128, vdim=128, window=1024, rot=64, rec_heads=16, rec_dim=128, ff=2560, side=256),
+}
+
+
+def decoder_dims(kind: str, size: str, layers: int, vocab: int, maxlen: int):
+    from ht_vllm_omni_amd.decoder_config import DecayRecurrenceSpec, DecoderDims, DenseMLPSpec, LatentAttentionSpec, LayerSpec, WindowAttentionSpec
+    if kind == "zefedra":
+        z = DECODER_SIZES[size]
+        mix = [LatentAttentionSpec(heads=z["heads"], dim=z["dim"], vdim=z["vdim"], q_rank=z["q_rank"], kv_rank=z["kv_rank"], scale=z["dim"] ** -0.5, out_gate=bool(i % 2))
+               for i in range(layers)]
+        return DecoderDims("zefedra", z["width"], vocab, tuple(LayerSpec(m, DenseMLPSpec(z["ff"])) for m in mix), 1e-6, maxlen)
+    z = KORONEX_SIZES[size]
+    rec = DecayRecurrenceSpec(z["rec_heads"], z["rec_dim"], z["rec_dim"], tuple(1 - 2.0 ** -(1 + h / 2) for h in range(z["rec_heads"])))
+    att = WindowAttentionSpec(z["heads"], z["kv_heads"], z["dim"], z["vdim"], z["dim"] ** -0.5, z["window"], z["rot"], 1e5, sink=True, out_gate=True)
+    return DecoderDims("koronex", z["width"], vocab, tuple(LayerSpec(att if i % 2 else rec, DenseMLPSpec(z["ff"], "relu2")) for i in range(layers)), 1e-6, maxlen,
+                       norm="post", alpha=2.0, token_shift=False, embed_scale=1.0, side_dim=z["side"])
+
+
+def mixer_flops(d, n: int) -> int:
+    """FLOP of the mixers (scores, values, states; no projections) over one prompt of n tokens."""
+    from ht_vllm_omni_amd.decoder_config import DecayRecurrenceSpec, LatentAttentionSpec
+    fl = 0
+    for s in d.layers:
+        m = s.mixer
+        if isinstance(m, DecayRecurrenceSpec):
+            fl += n * 4 * m.heads * m.dim * m.vdim
+        elif isinstance(m, LatentAttentionSpec):
+            fl += n * (n + 1) // 2 * 4 * m.heads * m.kv_rank
+        else:
+            w = min(m.window or n, n)
+            fl += (w * (w + 1) // 2 + (n - w) * w) * 2 * m.heads * (m.dim + m.vdim)
+    return fl
+
+
+def decoder_bench(sizes, kinds):
     """Decode (a captured step, rows x context) and prefill (one forward over whole prompts) of both models of a size, on one GPU."""
     from ht_vllm_omni_amd.config import get_dims
-    from ht_vllm_omni_amd.decoder_config import DecoderDims, DenseMLPSpec, LatentAttentionSpec, LayerSpec
     from ht_vllm_omni_amd.decoder_engine import DecoderEngine
     from ht_vllm_omni_amd.engine import TalkerEngine
     from ht_vllm_omni_amd.weights import make_decoder_weights, make_weights, weight_bytes
@@ -291,16 +328,16 @@ def decoder_bench(args):
     prefill_points = [(16, 128), (1, 2048), (4, 2048), (1, 8192)]
     maxlen, block = 8448, 16
     res = {}
-    for size in (DECODER_SIZES if args.decoder == "all" else (args.decoder,)):
+    for size in sizes:
         z, td = DECODER_SIZES[size], get_dims(DECODER_SIZES[size]["talker"]).with_(max_model_len=maxlen)
-        mix = [LatentAttentionSpec(heads=z["heads"], dim=z["dim"], vdim=z["vdim"], q_rank=z["q_rank"], kv_rank=z["kv_rank"], scale=z["dim"] ** -0.5, out_gate=bool(i % 2))
-               for i in range(td.layers)]
-        dd = DecoderDims("zefedra", z["width"], td.vocab, tuple(LayerSpec(m, DenseMLPSpec(z["ff"])) for m in mix), 1e-6, maxlen)
         out = {"config": {"zefedra": {k: v for k, v in z.items() if k != "talker"}, "layers": td.layers, "vocab": td.vocab, "talker": z["talker"],
                           "talker_kv": "bf16", "zefedra_cache": "bf16 latents"}}
+        if "koronex" in kinds:
+            out["config"].update(koronex=KORONEX_SIZES[size], koronex_cache="bf16 keys and values, fp32 states")
         nblk = 64 * ((2048 + 32) // block) + 2
-        for kind in ("zefedra", "talker"):
-            if kind == "zefedra":
+        for kind in kinds:
+            if kind != "talker":
+                dd = decoder_dims(kind, size, td.layers, td.vocab, maxlen)
                 eng = DecoderEngine(dd, make_decoder_weights(dd, device="cuda"), num_blocks=nblk, block_size=block, max_batch=64)
             else:
                 eng = TalkerEngine(td, make_weights(td, seed=1, device="cuda"), kv_dtype="bf16", num_blocks=nblk, block_size=block, max_batch=64, allow_eos=False)
@@ -312,10 +349,12 @@ def decoder_bench(args):
                 for i in range(rows):
                     bt[i, :need] = torch.arange(1 + i * need, 1 + (i + 1) * need)
                 eng.block_table.copy_(bt)
+                if kind != "talker":
+                    eng.state_slot.copy_(torch.arange(1, 65))
                 eng.positions.fill_(ctx - 1)
                 eng.seq_lens.fill_(ctx)
                 eng.num_live.fill_(rows)
-                if kind == "zefedra":
+                if kind != "talker":
                     ms = graph_ms(lambda: eng.decode_step(rows, advance=False))
                     by = eng.step_bytes([ctx] * rows)["total"]
                 else:
@@ -331,27 +370,27 @@ def decoder_bench(args):
                 eng.block_table.copy_(bt)
                 T = seqs * n
                 row, pos = torch.arange(seqs).repeat_interleave(n).to(torch.int32), torch.arange(n).repeat(seqs).to(torch.int32)
-                if kind == "zefedra":
+                if kind != "talker":
                     b = eng.make_batch(torch.randint(0, dd.vocab, (T,), dtype=torch.int32), row, pos, [n] * seqs)
                     last = (torch.arange(1, seqs + 1) * n - 1).to(torch.int32).cuda()
                     ms = eager_ms(lambda: eng.forward(b, sel=last))
                     per_tok = sum(2 * m.t.numel() for l in eng.layer_w.values() for m in l.mats)
-                    attn = sum(4 * m.heads * m.kv_rank for m in mix)
+                    attn = mixer_flops(dd, n)
                 else:
                     x = torch.randn(T, td.hidden, device="cuda").to(torch.bfloat16)
                     slots = (bt[row.long(), pos.long() // block] * block + pos % block).to(torch.int64).cuda()
                     pd, rd = pos.cuda(), row.cuda()
                     ms = eager_ms(lambda: eng.prefill_wide(x, pd, rd, slots))
                     per_tok = weight_bytes(td)["backbone"]
-                    attn = td.layers * 4 * td.q_heads * td.head_dim
-                fl = T * per_tok + seqs * n * (n + 1) // 2 * attn
+                    attn = n * (n + 1) // 2 * td.layers * 4 * td.q_heads * td.head_dim
+                fl = T * per_tok + seqs * attn
                 r["prefill"][f"{seqs}x{n}"] = {"ms": round(ms, 3), "tokens_per_s": round(T / ms * 1e3, 1), "tflop": round(fl / 1e12, 3), "tflops": round(fl / ms / 1e9, 1)}
                 log(size, kind, "prefill", seqs, n, r["prefill"][f"{seqs}x{n}"])
             out[kind] = r
             del eng
             torch.cuda.empty_cache()
         res[size] = out
-    return {"metric": "decoder-only design beside the talker backbone", "unit": "ms / tokens per s", "n_gpus": 1, "dtype": "bf16", "data": "synthetic", "sizes": res}
+    return {"metric": f"{kinds[0]}-shaped language model beside {'the talker backbone' if kinds[1] == 'talker' else kinds[1] + '-shaped'}", "unit": "ms / tokens per s", "n_gpus": 1, "dtype": "bf16", "data": "synthetic", "sizes": res}
 
 
 def main():
@@ -398,11 +437,14 @@ def main():
                     "steps advance the batch until the window is centred there (0: time from wherever warm-up ends)")
     ap.add_argument("--decoder", nargs="?", const="all", choices=("all", *DECODER_SIZES), default=None, help="measure the decoder-only design beside the talker "
                     "backbone instead (prefill and decode throughput at widths 2048 / 1024)")
+    ap.add_argument("--koronex", nargs="?", const="all", choices=("all", *KORONEX_SIZES), default=None, help="likewise Koronex-shaped layers (recurrence and windowed "
+                    "attention in turn) beside Zefedra-shaped ones of equal matrix bytes")
     ap.add_argument("--master-port", type=int, default=0, help="N > 1 self-launch: rendezvous port (0: pick a free one)")
     args = ap.parse_args()
 
-    if args.decoder:
-        out = decoder_bench(args)
+    if args.decoder or args.koronex:
+        which = args.koronex or args.decoder
+        out = decoder_bench(list(DECODER_SIZES) if which == "all" else [which], ("koronex", "zefedra") if args.koronex else ("zefedra", "talker"))
         sys.stdout.flush()
         os.write(json_fd, (json.dumps(out) + "\n").encode())
         return

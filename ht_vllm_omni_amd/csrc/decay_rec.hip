@@ -1,32 +1,32 @@
 // Linear recurrence with one decay per head (include/omni_decoder.h omni_decay_rec): S <- decay S + k v^T, out = S^T q, fp32 state per sequence.
 //
-//   rec_run_kernel          token by token: a workgroup keeps 64 columns of one head's S in registers while it walks its tokens.  A decoded token is a
-//                           run of one: S is read and written once, in 256-byte pieces -- that traffic is the op's bound
+//   rec_run_kernel          token by token: a workgroup keeps 64 or 128 columns of one head's S in registers while it walks its tokens.  A decoded token
+//                           is a run of one: S is read and written once -- that traffic is the op's bound
 //   chunks of 128 tokens, for prompts (matrix cores; a decay's powers enter as fp32 factors, fp32 operands as three bf16 terms whose sum is the value):
 //   rec_chunk_state_kernel  what a chunk adds to S:  sum_j decay^(n-1-j) k_j v_j^T, every chunk on its own
 //   rec_scan_kernel         S at every chunk's start, in place of its contribution, and the sequence's new state
 //   rec_chunk_out_kernel    out_i = decay^(i+1) S_start^T q_i + sum_(j <= i) decay^(i-j) (q_i . k_j) v_j
 #include "attn_tile.cuh"
-#include "../../include/omni_decoder.h"
+#include "row_io.cuh"
 
 #define RC_T OMNI_REC_CHUNK
-#define RC_COLS 64               // state columns of a run's workgroup
 #define RC_VB 128                // value columns of an output workgroup
 #define RC_VPITCH (RC_VB * 2 + 32)
 
 __device__ __forceinline__ float rc_silu(float z) { return z * sigmoidf_(z); }
 
-// ---- token by token.  Threads: 16 column quads x 16 row groups; row group g owns rows g, g + 16, ...
+// ---- token by token.  Threads: CQ column quads x 256 / CQ row groups; row group g owns rows g, g + 256 / CQ, ...
 // RAW: projections fp32 (partial sums), SiLU here; else bf16 behind it
-template <int MAXR, bool RAW>
+template <int CQ, int MAXR, bool RAW>
 __global__ __launch_bounds__(256) void rec_run_kernel(const omni_decay_rec a, const int32_t* items) {
+    constexpr int RG = 256 / CQ;
     extern __shared__ __attribute__((aligned(16))) float qk_lds[];     // q | k of the token
-    __shared__ f32x4 red[4][16];
+    __shared__ f32x4 red[4][CQ];
     const int tid = threadIdx.x, h = blockIdx.y, item = blockIdx.z;
     const int t0 = items ? items[2 * item] : item, n = items ? items[2 * item + 1] : 1;
     const int row = a.row_of_tok[t0];
     if (a.num_live && row >= *a.num_live) return;
-    const int cq = tid & 15, g = tid >> 4, col = blockIdx.x * RC_COLS + cq * 4;
+    const int cq = tid % CQ, g = tid / CQ, col = (blockIdx.x * CQ + cq) * 4;
     const bool mine = col < a.vp;
     float* sq = qk_lds;
     float* sk = qk_lds + a.dp;
@@ -36,33 +36,33 @@ __global__ __launch_bounds__(256) void rec_run_kernel(const omni_decay_rec a, co
 #pragma unroll
     for (int i = 0; i < MAXR; ++i) {
         S[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
-        const int d = g + 16 * i;
+        const int d = g + RG * i;
         if (mine && !zero && d < a.dp) S[i] = *reinterpret_cast<const f32x4*>(st + (size_t)d * a.vp);
     }
     const float decay = a.decay[h];
-    auto value = [&](int t, int c) {
+    auto value = [&](int t, int c, float (&v)[4]) {
         if constexpr (RAW) {
-            const float* p = reinterpret_cast<const float*>(a.proj) + (size_t)t * a.ld + c;
-            float v = p[0];
-            for (int s = 1; s < a.slabs; ++s) v += p[s * a.slab_stride];
-            return rc_silu(v);
+            ld4_slabs(reinterpret_cast<const float*>(a.proj) + (size_t)t * a.ld + c, a.slabs, a.slab_stride, v);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = rc_silu(v[e]);
         } else {
-            return bf2f(reinterpret_cast<const uint16_t*>(a.proj)[(size_t)t * a.ld + c]);
+            ld4<uint16_t>(reinterpret_cast<const uint16_t*>(a.proj) + (size_t)t * a.ld + c, v);
         }
     };
     const int kcol = a.heads * a.dp, vcol = 2 * a.heads * a.dp;
     for (int t = t0; t < t0 + n; ++t) {
-        for (int c = tid; c < 2 * a.dp; c += 256) qk_lds[c] = c < a.dp ? value(t, h * a.dp + c) : value(t, kcol + h * a.dp + c - a.dp);
-        f32x4 v = {0.f, 0.f, 0.f, 0.f};
-        if (mine) {
-#pragma unroll
-            for (int e = 0; e < 4; ++e) v[e] = value(t, vcol + h * a.vp + col + e);
+        for (int c = tid * 4; c < 2 * a.dp; c += 1024) {
+            float z[4];
+            value(t, c < a.dp ? h * a.dp + c : kcol + h * a.dp + c - a.dp, z);
+            st4<float>(qk_lds + c, z);
         }
+        float v[4] = {0.f, 0.f, 0.f, 0.f};
+        if (mine) value(t, vcol + h * a.vp + col, v);
         __syncthreads();                              // q and k of this token
         f32x4 o = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int i = 0; i < MAXR; ++i) {
-            const int d = g + 16 * i;
+            const int d = g + RG * i;
             if (d >= a.dp) continue;
             const float qd = sq[d], kd = sk[d];
 #pragma unroll
@@ -72,10 +72,10 @@ __global__ __launch_bounds__(256) void rec_run_kernel(const omni_decay_rec a, co
             }
         }
 #pragma unroll
-        for (int e = 0; e < 4; ++e) o[e] = xor32_sum(xor16_sum(o[e]));
-        if ((tid & 63) < 16) red[tid >> 6][cq] = o;
+        for (int e = 0; e < 4; ++e) o[e] = xor32_sum(CQ == 16 ? xor16_sum(o[e]) : o[e]);
+        if ((tid & 63) < CQ) red[tid >> 6][cq] = o;
         __syncthreads();                              // the waves' sums (and: nobody reads this token's q, k any more)
-        if (tid < 16 && mine) {
+        if (tid < CQ && mine) {
             const f32x4 s = (red[0][cq] + red[1][cq]) + (red[2][cq] + red[3][cq]);
             *reinterpret_cast<f32x4*>(a.out + ((size_t)t * a.heads + h) * a.vp + col) = s;
         }
@@ -83,7 +83,7 @@ __global__ __launch_bounds__(256) void rec_run_kernel(const omni_decay_rec a, co
     if (!mine) return;
 #pragma unroll
     for (int i = 0; i < MAXR; ++i) {
-        const int d = g + 16 * i;
+        const int d = g + RG * i;
         if (d < a.dp) *reinterpret_cast<f32x4*>(st + (size_t)d * a.vp) = S[i];
     }
 }
@@ -294,15 +294,22 @@ __global__ __launch_bounds__(512, 2) void rec_chunk_out_kernel(const omni_decay_
 }
 
 // ---- host side
+template <int CQ, bool RAW>
+static void rec_runs_launch(const omni_decay_rec& a, const int32_t* items, int n, hipStream_t st) {
+    constexpr int RG = 256 / CQ;
+    const dim3 grid((a.vp + 4 * CQ - 1) / (4 * CQ), a.heads, n), block(256);
+    const size_t lds = 2 * (size_t)a.dp * sizeof(float);
+    if (a.dp <= 4 * RG) hipLaunchKernelGGL((rec_run_kernel<CQ, 4, RAW>), grid, block, lds, st, a, items);
+    else if (a.dp <= 8 * RG) hipLaunchKernelGGL((rec_run_kernel<CQ, 8, RAW>), grid, block, lds, st, a, items);
+    else if (a.dp <= 16 * RG) hipLaunchKernelGGL((rec_run_kernel<CQ, 16, RAW>), grid, block, lds, st, a, items);
+    else hipLaunchKernelGGL((rec_run_kernel<CQ, 32, RAW>), grid, block, lds, st, a, items);
+}
+
 template <bool RAW>
 static int rec_runs(const omni_decay_rec& a, const int32_t* items, int n, hipStream_t st) {
     if (n <= 0) return OMNI_OK;
-    const dim3 grid((a.vp + RC_COLS - 1) / RC_COLS, a.heads, n), block(256);
-    const size_t lds = 2 * (size_t)a.dp * sizeof(float);
-    if (a.dp <= 64) hipLaunchKernelGGL((rec_run_kernel<4, RAW>), grid, block, lds, st, a, items);
-    else if (a.dp <= 128) hipLaunchKernelGGL((rec_run_kernel<8, RAW>), grid, block, lds, st, a, items);
-    else if (a.dp <= 256) hipLaunchKernelGGL((rec_run_kernel<16, RAW>), grid, block, lds, st, a, items);
-    else hipLaunchKernelGGL((rec_run_kernel<32, RAW>), grid, block, lds, st, a, items);
+    if (a.vp > 64 && a.dp <= 256) rec_runs_launch<32, RAW>(a, items, n, st);
+    else rec_runs_launch<16, RAW>(a, items, n, st);
     OMNI_CHECK_LAUNCH("omni_decay_rec(runs)");
     return OMNI_OK;
 }

@@ -1,46 +1,9 @@
 // Row-wise kernels of the decoder-only language models (include/omni_decoder.h): everything between two matrix products of a layer.
 // The residual stream is fp32; norms, gates and the token-shift state are fp32; only matrix operands are rounded (once) to bf16.
-#include "common.cuh"
-#include "../../include/omni_decoder.h"
+#include "row_io.cuh"
 
 #define DR_THREADS 256
 #define DR_WAVES (DR_THREADS / 64)
-
-// ---- element type of matrix operands: 4 consecutive values
-template <typename E>
-__device__ __forceinline__ void ld4(const E* p, float (&v)[4]);
-template <>
-__device__ __forceinline__ void ld4<float>(const float* p, float (&v)[4]) {
-    const float4 a = *reinterpret_cast<const float4*>(p);
-    v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
-}
-template <>
-__device__ __forceinline__ void ld4<uint16_t>(const uint16_t* p, float (&v)[4]) {
-    const uint2 a = *reinterpret_cast<const uint2*>(p);
-    v[0] = bf_lo(a.x); v[1] = bf_hi(a.x); v[2] = bf_lo(a.y); v[3] = bf_hi(a.y);
-}
-template <typename E>
-__device__ __forceinline__ void st4(E* p, const float (&v)[4]);
-template <>
-__device__ __forceinline__ void st4<float>(float* p, const float (&v)[4]) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
-template <>
-__device__ __forceinline__ void st4<uint16_t>(uint16_t* p, const float (&v)[4]) {
-    *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf2(v[0], v[1]), pack_bf2(v[2], v[3]));
-}
-
-// 4 consecutive values of an array that arrives as `slabs` partial sums `stride` elements apart, added in slab order.  More than one: all
-// OMNI_STREAM_MAX_SPLITS loads leave at once (past the last slab: a repeated address, not added)
-__device__ __forceinline__ void ld4_slabs(const float* p, int slabs, int64_t stride, float (&v)[4]) {
-    ld4<float>(p, v);
-    if (slabs <= 1) return;
-    float z[OMNI_STREAM_MAX_SPLITS][4];
-#pragma unroll
-    for (int s = 1; s < OMNI_STREAM_MAX_SPLITS; ++s) ld4<float>(p + min(s, slabs - 1) * stride, z[s]);
-#pragma unroll
-    for (int s = 1; s < OMNI_STREAM_MAX_SPLITS; ++s)
-#pragma unroll
-        for (int e = 0; e < 4; ++e) v[e] += s < slabs ? z[s][e] : 0.f;
-}
 
 // sum over the workgroup, result in every thread; `buf` alternates between calls so that one barrier per sum is enough
 struct BlockSum {
@@ -296,93 +259,115 @@ extern "C" int omni_latent_write_run(const omni_latent_write* p, void* stream) {
     return OMNI_OK;
 }
 
-// ---- grouped attention: norms over whole projections, rotation, cache write, gate.  One workgroup per token; q and k stay in LDS between the norm's
-// sum and the rotation (a pair's other half belongs to another thread)
-template <typename E>
+// ---- grouped attention: norms over whole projections, rotation, cache write, gate.  Three workgroups per token, by what they read: queries | keys and
+// values | gate.  Queries and keys stay in LDS between the norm's sum and the rotation (a pair's other half belongs to another thread)
+template <typename E, bool WIDE>                       // WIDE: half a rotation is a multiple of 4, so 4 consecutive dimensions have 4 consecutive partners
 __global__ __launch_bounds__(DR_THREADS) void qkv_write_kernel(const omni_qkv_write a) {
-    extern __shared__ __attribute__((aligned(16))) float sp[];     // [q | k] of the token, partial sums added up
-    __shared__ float red[2][DR_WAVES];
-    const int t = blockIdx.x;
-    const int row = a.row_of_tok[t], pos = a.positions[t];
-    const bool live = !a.num_live || row < *a.num_live;
+    extern __shared__ __attribute__((aligned(16))) float sp[];     // q or k of the token, partial sums added up
+    __shared__ float red[DR_WAVES];
+    const int t = blockIdx.x, part = blockIdx.y;
     const int nq = a.heads * a.dp, nk = a.kc ? a.kv_heads * a.dp : 0, nv = a.kc ? a.kv_heads * a.vp : 0, ng = a.heads * a.vp;
     const float* y = a.proj + (size_t)t * a.ld;
-    // cache rows of this token: head g at base + g * block_size
-    const size_t base = a.kc ? (size_t)a.block_table[(size_t)row * a.bt_stride + pos / a.block_size] * a.kv_heads * a.block_size + pos % a.block_size : 0;
-    float sq = 0.f, sk = 0.f;
-    for (int k = threadIdx.x * 4; k < nq + nk; k += DR_THREADS * 4) {
-        float v[4];
-        ld4_slabs(y + k, a.slabs, a.slab_stride, v);
-        st4<float>(sp + k, v);
-        const float ss = sq4_sum(v[0], v[1], v[2], v[3]);
-        if (k < nq) sq += ss;
-        else sk += ss;
-    }
-    if (a.kc && live)
-        for (int k = threadIdx.x * 4; k < nv; k += DR_THREADS * 4) {
-            float v[4];
-            ld4_slabs(y + nq + nk + k, a.slabs, a.slab_stride, v);
-            const int g = k / a.vp, d = k - g * a.vp;
-            st4<E>(reinterpret_cast<E*>(a.vc) + (base + (size_t)g * a.block_size) * a.vp + d, v);
-        }
-    if (a.gate)
+    if (part == 2) {
         for (int k = threadIdx.x * 4; k < ng; k += DR_THREADS * 4) {
             float v[4];
             ld4_slabs(y + nq + nk + nv + k, a.slabs, a.slab_stride, v);
 #pragma unroll
-            for (int e = 0; e < 4; ++e) v[e] = 1.0f / (1.0f + expf(-v[e]));
+            for (int e = 0; e < 4; ++e) v[e] = sigmoidf_(v[e]);
             st4<E>(reinterpret_cast<E*>(a.gate) + (size_t)t * ng + k, v);
         }
-    sq = wave_sum(sq);
-    sk = wave_sum(sk);
-    if ((threadIdx.x & 63) == 0) { red[0][threadIdx.x >> 6] = sq; red[1][threadIdx.x >> 6] = sk; }
+        return;
+    }
+    const int row = a.row_of_tok[t], pos = a.positions[t];
+    if (part == 1 && (!a.kc || (a.num_live && row >= *a.num_live))) return;
+    // cache rows of this token: head g at base + g * block_size
+    const size_t base = part ? (size_t)a.block_table[(size_t)row * a.bt_stride + pos / a.block_size] * a.kv_heads * a.block_size + pos % a.block_size : 0;
+    const int n = part ? nk : nq, heads = part ? a.kv_heads : a.heads;
+    const E* w = reinterpret_cast<const E*>(part ? a.kw : a.qw);
+    if (part) y += nq;
+    float ss = 0.f;
+    for (int k = threadIdx.x * 4; k < n; k += DR_THREADS * 4) {
+        float v[4];
+        ld4_slabs(y + k, a.slabs, a.slab_stride, v);
+        st4<float>(sp + k, v);
+        ss += sq4_sum(v[0], v[1], v[2], v[3]);
+    }
+    if (part)
+        for (int k = threadIdx.x * 4; k < nv; k += DR_THREADS * 4) {
+            float v[4];
+            ld4_slabs(y + nk + k, a.slabs, a.slab_stride, v);
+            const int g = k / a.vp, d = k - g * a.vp;
+            st4<E>(reinterpret_cast<E*>(a.vc) + (base + (size_t)g * a.block_size) * a.vp + d, v);
+        }
+    ss = wave_sum(ss);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
     __syncthreads();
-    sq = sk = 0.f;
+    ss = 0.f;
 #pragma unroll
-    for (int w = 0; w < DR_WAVES; ++w) { sq += red[0][w]; sk += red[1][w]; }
-    const float rq = a.qw ? 1.0f / sqrtf(sq / (float)(a.heads * a.dim) + a.eps) : 1.0f;
-    const float rk = a.kw ? 1.0f / sqrtf(sk / (float)(a.kv_heads * a.dim) + a.eps) : 1.0f;
+    for (int i = 0; i < DR_WAVES; ++i) ss += red[i];
+    const float r = w ? 1.0f / sqrtf(ss / (float)(heads * a.dim) + a.eps) : 1.0f;
     const int half = a.rot_dims >> 1;
     const float* cs = a.rot + (size_t)min(pos, a.rot_rows - 1) * a.rot_dims;
-    for (int k = threadIdx.x * 4; k < nq + nk; k += DR_THREADS * 4) {
-        const bool key = k >= nq;
-        if (key && !live) break;
-        const int kk = key ? k - nq : k, hd = kk / a.dp, d0 = kk - hd * a.dp;
-        const E* w = reinterpret_cast<const E*>(key ? a.kw : a.qw);
-        const float r = key ? rk : rq;
-        const float* s = sp + (key ? nq : 0) + hd * a.dp;
-        auto normed = [&](int d) {
-            float wd = 1.0f;
-            if (w) {
-                if constexpr (sizeof(E) == 4) wd = w[hd * a.dp + d];
-                else wd = bf2f(w[hd * a.dp + d]);
-            }
-            return s[d] * r * wd;
-        };
-        float v[4];
+    for (int k = threadIdx.x * 4; k < n; k += DR_THREADS * 4) {
+        const int hd = k / a.dp, d0 = k - hd * a.dp;
+        float v[4], o[4] = {0.f, 0.f, 0.f, 0.f}, wv[4] = {1.f, 1.f, 1.f, 1.f};
+        ld4<float>(sp + k, v);
+        if (w) ld4<E>(w + k, wv);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const int d = d0 + e;
-            v[e] = normed(d);
-            if (d < a.rot_dims) {
-                const bool lo = d < half;
-                const float o = normed(lo ? d + half : d - half);
-                const float2 c = *reinterpret_cast<const float2*>(cs + 2 * (lo ? d : d - half));
-                v[e] = lo ? fmaf(v[e], c.x, -(o * c.y)) : fmaf(v[e], c.x, o * c.y);
+        for (int e = 0; e < 4; ++e) v[e] = v[e] * r * wv[e];
+        if (d0 < a.rot_dims) {                         // (the vector may end past the rotated dimensions)
+            float c[4] = {1.f, 1.f, 1.f, 1.f}, sn[4] = {0.f, 0.f, 0.f, 0.f};
+            if constexpr (WIDE) {
+                const bool lo = d0 < half;
+                const int q = lo ? k + half : k - half;
+                const float* p = cs + 2 * (lo ? d0 : d0 - half);
+                ld4<float>(sp + q, o);
+                float wo[4] = {1.f, 1.f, 1.f, 1.f}, z[4];
+                if (w) ld4<E>(w + q, wo);
+                ld4<float>(p, z);
+                c[0] = z[0]; sn[0] = z[1]; c[1] = z[2]; sn[1] = z[3];
+                ld4<float>(p + 4, z);
+                c[2] = z[0]; sn[2] = z[1]; c[3] = z[2]; sn[3] = z[3];
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    o[e] = o[e] * r * wo[e];
+                    if (lo) o[e] = -o[e];
+                }
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    const int d = d0 + e;
+                    if (d >= a.rot_dims) continue;
+                    const bool lo = d < half;
+                    const int q = k + e + (lo ? half : -half);
+                    float wo = 1.0f;
+                    if (w) {
+                        if constexpr (sizeof(E) == 4) wo = w[q];
+                        else wo = bf2f(w[q]);
+                    }
+                    o[e] = sp[q] * r * wo;
+                    if (lo) o[e] = -o[e];
+                    const float2 f = *reinterpret_cast<const float2*>(cs + 2 * (lo ? d : d - half));
+                    c[e] = f.x; sn[e] = f.y;
+                }
             }
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = fmaf(v[e], c[e], o[e] * sn[e]);
         }
-        if (key) st4<E>(reinterpret_cast<E*>(a.kc) + (base + (size_t)hd * a.block_size) * a.dp + d0, v);
+        if (part) st4<E>(reinterpret_cast<E*>(a.kc) + (base + (size_t)hd * a.block_size) * a.dp + d0, v);
         else st4<E>(reinterpret_cast<E*>(a.q) + (size_t)t * nq + k, v);
     }
 }
 
-template <typename E>
+template <typename E, bool WIDE>
 static int qkv_write_launch(const omni_qkv_write& a, size_t lds, hipStream_t st) {
     if (lds > 60 * 1024) {
-        static const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(qkv_write_kernel<E>), hipFuncAttributeMaxDynamicSharedMemorySize, 156 * 1024);
+        static const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(qkv_write_kernel<E, WIDE>), hipFuncAttributeMaxDynamicSharedMemorySize, 156 * 1024);
         if (e != hipSuccess) { omni_set_error("omni_qkv_write: LDS attribute: %s", hipGetErrorString(e)); return OMNI_EHIP; }
     }
-    hipLaunchKernelGGL(qkv_write_kernel<E>, dim3(a.T), dim3(DR_THREADS), lds, st, a);
+    // parts in launch order: queries, (keys and values, of a layer with its own), (gate): a missing part in the middle starts and leaves
+    const int parts = a.gate ? 3 : (a.kc ? 2 : 1);
+    hipLaunchKernelGGL((qkv_write_kernel<E, WIDE>), dim3(a.T, parts), dim3(DR_THREADS), lds, st, a);
     OMNI_CHECK_LAUNCH("omni_qkv_write");
     return OMNI_OK;
 }
@@ -397,10 +382,12 @@ extern "C" int omni_qkv_write_run(const omni_qkv_write* p, void* stream) {
     OMNI_CHECK_ARG(a.rot_dims >= 0 && a.rot_dims % 2 == 0 && a.rot_dims <= a.dim && (a.rot_dims == 0 || (a.rot && a.rot_rows > 0)), "omni_qkv_write: rot_dims=%d of %d", a.rot_dims, a.dim);
     OMNI_CHECK_ARG(!a.kc || (a.block_table && a.block_size > 0 && a.bt_stride > 0), "omni_qkv_write: block_size=%d bt_stride=%d", a.block_size, a.bt_stride);
     OMNI_CHECK_ARG(a.slabs <= OMNI_STREAM_MAX_SPLITS && (a.elem == 0 || a.elem == 1), "omni_qkv_write: slabs=%d elem=%d", a.slabs, a.elem);
-    const size_t lds = ((size_t)a.heads * a.dp + (a.kc ? (size_t)a.kv_heads * a.dp : 0)) * sizeof(float);
-    OMNI_CHECK_ARG(lds <= 156 * 1024, "omni_qkv_write: %d query and %d key heads of %d (a token's are staged in LDS)", a.heads, a.kv_heads, a.dp);
+    const size_t lds = (size_t)a.heads * a.dp * sizeof(float);      // (there are no more key heads than query heads)
+    OMNI_CHECK_ARG(lds <= 156 * 1024, "omni_qkv_write: %d query heads of %d (a token's are staged in LDS)", a.heads, a.dp);
     if (a.T <= 0) return OMNI_OK;
-    return a.elem ? qkv_write_launch<float>(a, lds, (hipStream_t)stream) : qkv_write_launch<uint16_t>(a, lds, (hipStream_t)stream);
+    hipStream_t st = (hipStream_t)stream;
+    if (a.rot_dims % 8 == 0) return a.elem ? qkv_write_launch<float, true>(a, lds, st) : qkv_write_launch<uint16_t, true>(a, lds, st);
+    return a.elem ? qkv_write_launch<float, false>(a, lds, st) : qkv_write_launch<uint16_t, false>(a, lds, st);
 }
 
 // ---- a recurrence's output: norm over all heads together, times the gate.  One workgroup per token
