@@ -18,12 +18,14 @@ __device__ __forceinline__ int la_row_splits(int ntiles, int nsplit) { return mi
 
 // a pair of fp32 values as three bf16 terms each
 __device__ __forceinline__ void split3(float a, float b, uint32_t& hi, uint32_t& mid, uint32_t& lo) {
-    const float ar = a - bfround(a), br = b - bfround(b);
-    const float am = bfround(ar), bm = bfround(br);
     hi = pack_bf2(a, b);
-    mid = pack_bf2(am, bm);
-    lo = pack_bf2(ar - am, br - bm);
+    const float ar = a - bf_lo(hi), br = b - bf_hi(hi);
+    mid = pack_bf2(ar, br);
+    lo = pack_bf2(ar - bf_lo(mid), br - bf_hi(mid));
 }
+
+// 2^x of weights and decays (one instruction; below 2^-126: zero)
+__device__ __forceinline__ float exp2_w(float x) { return __builtin_amdgcn_exp2f(x); }
 
 // key of contraction slot (qk, j) inside a 32-key tile
 __device__ __forceinline__ int la_slot(int qk, int j) { return j < 4 ? 4 * qk + j : 16 + 4 * qk + (j - 4); }

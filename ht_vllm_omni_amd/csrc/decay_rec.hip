@@ -89,22 +89,32 @@ __global__ __launch_bounds__(256) void rec_run_kernel(const omni_decay_rec a, co
 }
 
 // ---- chunks
-// tokens [t0, t0 + n) of a [tokens, ld] bf16 array, `pieces` 32-wide pieces from column c0 -> row-major LDS image of RC_T rows; rows past n are zero
-template <int THREADS>
-__device__ __forceinline__ void rc_stage(const uint16_t* src, int ld, int t0, int n, int c0, int pieces, unsigned char* img, int pitch) {
-    const int quarter = threadIdx.x & 3;
+// tokens [t0, t0 + n) of a [tokens, ld] bf16 array, up to P 32-wide pieces from column c0, through registers -> row-major LDS image of RC_T rows; rows
+// past n are zero
+template <int THREADS, int P>
+struct RcTile {
+    static constexpr int R = RC_T * 4 / THREADS;
+    u32x4 v[R][P];
+    __device__ __forceinline__ void load(const uint16_t* src, int ld, int t0, int n, int c0, int pieces) {
 #pragma unroll
-    for (int r = 0; r < RC_T * 4 / THREADS; ++r) {
-        const int tok = (threadIdx.x >> 2) + r * (THREADS / 4);
-        const uint16_t* p = src + (size_t)(t0 + min(tok, n - 1)) * ld + c0 + 8 * quarter;
-#pragma unroll 4
-        for (int s = 0; s < pieces; ++s) {
-            u32x4 v = ld16(p + 32 * s);
-            if (tok >= n) v = (u32x4){0, 0, 0, 0};
-            *reinterpret_cast<u32x4*>(img + tok * pitch + (32 * s + 8 * quarter) * 2) = v;
+        for (int r = 0; r < R; ++r) {
+            const int tok = (threadIdx.x >> 2) + r * (THREADS / 4);
+            const uint16_t* p = src + (size_t)(t0 + min(tok, n - 1)) * ld + c0 + 8 * (threadIdx.x & 3);
+#pragma unroll
+            for (int s = 0; s < P; ++s)
+                if (s < pieces) v[r][s] = ld16(p + 32 * s);
         }
     }
-}
+    __device__ __forceinline__ void store(unsigned char* img, int pitch, int n, int pieces) const {
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+            const int tok = (threadIdx.x >> 2) + r * (THREADS / 4);
+#pragma unroll
+            for (int s = 0; s < P; ++s)
+                if (s < pieces) *reinterpret_cast<u32x4*>(img + tok * pitch + (32 * s + 8 * (threadIdx.x & 3)) * 2) = tok < n ? v[r][s] : (u32x4){0, 0, 0, 0};
+        }
+    }
+};
 
 // D[v][d] = V^T . K': A = V^T (lane: v, 8 tokens), B = K' (lane: d, the same tokens) = decay^(n-1-j) k_j in three terms
 __global__ __launch_bounds__(256, 2) void rec_chunk_state_kernel(const omni_decay_rec a) {
@@ -116,8 +126,14 @@ __global__ __launch_bounds__(256, 2) void rec_chunk_state_kernel(const omni_deca
     unsigned char* kimg = img;
     unsigned char* vimg = img + RC_T * kp;
     const uint16_t* src = reinterpret_cast<const uint16_t*>(a.proj);
-    rc_stage<256>(src, a.ld, t0, n, (a.heads + h) * a.dp, a.dp / 32, kimg, kp);
-    rc_stage<256>(src, a.ld, t0, n, 2 * a.heads * a.dp + h * a.vp, a.vp / 32, vimg, vpitch);
+    constexpr int P = 4;                              // pieces in flight
+    for (int s = 0; s < a.dp / 32 || s < a.vp / 32; s += P) {
+        RcTile<256, P> k, v;
+        k.load(src, a.ld, t0, n, (a.heads + h) * a.dp + 32 * s, a.dp / 32 - s);
+        v.load(src, a.ld, t0, n, 2 * a.heads * a.dp + h * a.vp + 32 * s, a.vp / 32 - s);
+        k.store(kimg + 64 * s, kp, n, a.dp / 32 - s);
+        v.store(vimg + 64 * s, vpitch, n, a.vp / 32 - s);
+    }
     const float l2 = a.log2_decay[h];
     float f[RC_T / 32][8];
 #pragma unroll
@@ -125,7 +141,7 @@ __global__ __launch_bounds__(256, 2) void rec_chunk_state_kernel(const omni_deca
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
             const int back = n - 1 - (32 * ks + la_slot(qk, j));
-            f[ks][j] = back >= 0 ? exp2f(l2 * (float)back) : 0.f;
+            f[ks][j] = back >= 0 ? exp2_w(l2 * (float)back) : 0.f;
         }
     __syncthreads();
     float* out = a.chunk_states + ((size_t)chunk * a.heads + h) * a.dp * a.vp;
@@ -183,7 +199,7 @@ __global__ __launch_bounds__(256) void rec_scan_kernel(const omni_decay_rec a) {
 #pragma unroll
         for (int p = 0; p < P; ++p) {
             if (i + p >= nc) continue;
-            const float f = exp2f(l2 * (float)a.chunks[4 * (c0 + i + p) + 1]);
+            const float f = exp2_w(l2 * (float)a.chunks[4 * (c0 + i + p) + 1]);
             *reinterpret_cast<f32x4*>(cs + (i + p) * stride) = S;
 #pragma unroll
             for (int k = 0; k < 4; ++k) S[k] = fmaf(f, S[k], x[p][k]);
@@ -208,21 +224,25 @@ __global__ __launch_bounds__(512, 2) void rec_chunk_out_kernel(const omni_decay_
     const uint16_t* qrow = src + (size_t)(t0 + min(i, n - 1)) * a.ld + h * dp;
     const float l2 = a.log2_decay[h];
     const bool carry = a.chunks[4 * chunk + 2] != 0 || a.positions[t0] != 0;      // S_start is not zero
-    rc_stage<512>(src, a.ld, t0, n, 2 * a.heads * dp + h * a.vp + vb0, vcols / 32, vimg, RC_VPITCH);
     f32x4 O[RC_VB / 16];
 #pragma unroll
     for (int v = 0; v < RC_VB / 16; ++v) O[v] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    const float* cs = a.chunk_states + ((size_t)chunk * a.heads + h) * dp * a.vp + vb0;
+    const int sr = tid >> 4, sc = (tid & 15) * 8;     // this thread's piece of a 32-row slab of states: 8 columns
+    f32x4 x[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+    auto slab = [&](int s) {
+        if (sc >= vcols) return;
+        const float* p = cs + (size_t)(32 * s + sr) * a.vp + sc;
+        x[0] = *reinterpret_cast<const f32x4*>(p);
+        x[1] = *reinterpret_cast<const f32x4*>(p + 4);
+    };
+    // everything the chunk reads is on its way before the first wait, in the order it is needed
+    if (carry) slab(0);
+    RcTile<512, RC_VB / 32> vt;
+    RcTile<512, DS> kt_;
+    vt.load(src, a.ld, t0, n, 2 * a.heads * dp + h * a.vp + vb0, vcols / 32);
+    kt_.load(src, a.ld, t0, n, (a.heads + h) * dp, DS);
     if (carry) {                                      // (uniform)
-        const float* cs = a.chunk_states + ((size_t)chunk * a.heads + h) * dp * a.vp + vb0;
-        const int sr = tid >> 4, sc = (tid & 15) * 8; // this thread's piece of a 32-row slab: 8 columns
-        f32x4 x[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
-        auto slab = [&](int s) {
-            if (sc >= vcols) return;
-            const float* p = cs + (size_t)(32 * s + sr) * a.vp + sc;
-            x[0] = *reinterpret_cast<const f32x4*>(p);
-            x[1] = *reinterpret_cast<const f32x4*>(p + 4);
-        };
-        slab(0);
 #pragma unroll 1
         for (int s = 0; s < DS; ++s) {
             u32x4 w[3];
@@ -247,12 +267,13 @@ __global__ __launch_bounds__(512, 2) void rec_chunk_out_kernel(const omni_decay_
                 for (int p = 2; p >= 0; --p) O[v] = mfma16(la_transposed_at(kimg + p * PLANE, RC_VPITCH, v, c, qk), B, O[v]);
             }
         }
-        const float f = exp2f(l2 * (float)(i + 1));
+        const float f = exp2_w(l2 * (float)(i + 1));
 #pragma unroll
         for (int v = 0; v < RC_VB / 16; ++v) O[v] *= f;
         __syncthreads();                              // the planes have been read
     }
-    rc_stage<512>(src, a.ld, t0, n, (a.heads + h) * dp, DS, kimg, KP);
+    vt.store(vimg, RC_VPITCH, n, vcols / 32);
+    kt_.store(kimg, KP, n, DS);
     u32x4 Q[DS];
 #pragma unroll
     for (int s = 0; s < DS; ++s) Q[s] = ld16(qrow + 32 * s + 8 * qk);
@@ -272,7 +293,7 @@ __global__ __launch_bounds__(512, 2) void rec_chunk_out_kernel(const omni_decay_
 #pragma unroll
             for (int u = 0; u < 2; ++u) {
                 const int j = 2 * e + u, back = i - (j0 + la_slot(qk, j));
-                p[u] = back >= 0 ? S[j >> 2][j & 3] * exp2f(l2 * (float)back) : 0.f;
+                p[u] = back >= 0 ? S[j >> 2][j & 3] * exp2_w(l2 * (float)back) : 0.f;
             }
             uint32_t hi, mid, lo;
             split3(p[0], p[1], hi, mid, lo);

@@ -151,7 +151,7 @@ class DecoderEngine:
         # ---- per-sequence state, slot 0 of no sequence: what each layer's mixer read at the sequence's last token, and the mixers' own
         self.state_slots = max_batch + 1
         self.shift_state = torch.zeros(dims.num_layers, self.state_slots, self.width, dtype=torch.float32, device=dev) if dims.token_shift else None
-        self.rec_state = [m.state(self.state_slots) for m in self.mixers]
+        self.rec_state = [m.state(self, self.state_slots) for m in self.mixers]
         # ---- persistent per-row buffers (graph-stable addresses)
         Bm = max_batch
         i32 = dict(dtype=torch.int32, device=dev)
@@ -171,7 +171,7 @@ class DecoderEngine:
         # ---- scratch: the decode step's own (its addresses are recorded in graphs), and one that grows with the prompts
         self._dec = _Scratch(self, Bm)
         self._any: _Scratch | None = None
-        self.attn_ws = torch.zeros(max(m.workspace_bytes(Bm) for m in self.mixers) // 4 + 1, dtype=torch.float32, device=dev)
+        self.attn_ws = torch.zeros(max(m.workspace_bytes(self, Bm) for m in self.mixers) // 4 + 1, dtype=torch.float32, device=dev)
         self.persistent_chains = False
 
     # ------------------------------------------------------------------ tensors
@@ -199,7 +199,7 @@ class DecoderEngine:
     # ------------------------------------------------------------------ cache
     def _alloc_kv(self, num_blocks: int) -> None:
         self.num_blocks = int(num_blocks)
-        self.kv_caches = [m.cache(self.num_blocks, self.block_size) for m in self.mixers]
+        self.kv_caches = [m.cache(self, self.num_blocks, self.block_size) for m in self.mixers]
 
     def kv_cache_bytes(self) -> int:
         return sum(c.numel() * c.element_size() for layer in self.kv_caches for c in layer)
@@ -344,7 +344,7 @@ class DecoderEngine:
         operand(0, ids=b.ids, table=self.embed, vocab=d.vocab, table_scale=d.embed_scale)
         for i in range(d.num_layers):
             w = self.layer_w[d.owner(i)]
-            add = self._join(k, s, w.mixer.run(b, i, s, s.x[k], frag), T, w.norm1)
+            add = self._join(k, s, w.mixer.run(self, b, i, s, s.x[k], frag), T, w.norm1)
             if d.layers[i].mlp is not None:
                 operand(None, **add)
                 self._mm(s.h, w.up, s.act, T, act=w.act, out_frag=frag)

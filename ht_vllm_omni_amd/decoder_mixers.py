@@ -1,6 +1,6 @@
 """Sequence mixers of the decoder-only language models: weights on the device, cache and state of a layer, launches.
 
-A mixer object belongs to the layer that owns the weights; ``run(b, i, s, x, frag)`` runs it as layer ``i`` (a borrowing layer has its own place in the
+A mixer object belongs to the layer that owns the weights; ``run(engine, b, i, s, x, frag)`` runs it as layer ``i`` (a borrowing layer has its own place in the
 cache and the state) on the operand ``s.h`` and returns how many partial sums its output ``s.y`` consists of.  ``needs`` names the
 activations it wants per token; every layer of a model shares them (``decoder_engine._Scratch``).  ``work`` names the lists of work items its
 kernels walk, one builder per kind (``WORK``), made once per batch.
@@ -121,21 +121,22 @@ WORK = {"tiles": attention_tiles, "chunks": recurrence_chunks, "segs": recurrenc
 
 
 class Mixer:
-    """What the engine asks of a mixer; `eng` is the DecoderEngine (products, cache, state, block table)."""
+    """What the engine asks of a mixer; `eng` / `e` is the DecoderEngine (products, cache, state, block table) -- handed in, never kept: an engine that
+    goes out of use gives its memory back at once."""
     work: tuple = ()
 
-    def __init__(self, eng, spec):
-        self.eng, self.spec = eng, spec
+    def __init__(self, spec):
+        self.spec = spec
 
-    def cache(self, num_blocks: int, block_size: int) -> tuple[torch.Tensor, ...]:
+    def cache(self, eng, num_blocks: int, block_size: int) -> tuple[torch.Tensor, ...]:
         """Cache tensors of one layer (none: nothing is paged)."""
         return ()
 
-    def state(self, slots: int) -> torch.Tensor | None:
+    def state(self, eng, slots: int) -> torch.Tensor | None:
         """State of one layer, one entry per slot."""
         return None
 
-    def workspace_bytes(self, rows: int) -> int:
+    def workspace_bytes(self, eng, rows: int) -> int:
         """Of the decode attention's KV splits."""
         return 0
 
@@ -143,18 +144,19 @@ class Mixer:
         """Activations: name -> (elements per token, dtype or "elem", "rows" | "tiles" of 16 rows | "slabs" of partial sums)."""
         return {}
 
-    def _where(self, b) -> dict:
-        e = self.eng
+    @staticmethod
+    def _where(e, b) -> dict:
         return dict(block_table=e.block_table.data_ptr(), bt_stride=e.bt_stride, block_size=e.block_size, row_of_tok=b.row_of_tok.data_ptr(),
                     positions=b.positions.data_ptr())
 
-    def _launch(self, name: str, s) -> None:
-        L.check(getattr(self.eng.lib, name + "_run")(C.byref(s), L.current_stream()), name, self.eng.lib)
+    @staticmethod
+    def _launch(e, name: str, s) -> None:
+        L.check(getattr(e.lib, name + "_run")(C.byref(s), L.current_stream()), name, e.lib)
 
 
 class LatentMixer(Mixer):
     def __init__(self, eng, i: int, m: LatentAttentionSpec, w: dict):
-        super().__init__(eng, m)
+        super().__init__(m)
         elem, dev, W, H = eng.elem, eng.device, eng.width, m.heads
         self.qp, self.rp, self.dp, self.vp = r32(m.q_rank), latent_width(m.kv_rank, elem.code), r32(m.dim), r32(m.vdim)
         parts = [pad2(w["dq"], self.qp, W), pad2(w["dkv"], self.rp, W)]
@@ -173,35 +175,35 @@ class LatentMixer(Mixer):
     def matrices(self):
         return [self.down, self.uq, self.uk, self.uv, self.o]
 
-    def cache(self, num_blocks, block_size):
-        return (torch.zeros(num_blocks, block_size, self.rp, dtype=self.eng.elem.torch, device=self.eng.device),)
+    def cache(self, eng, num_blocks, block_size):
+        return (torch.zeros(num_blocks, block_size, self.rp, dtype=eng.elem.torch, device=eng.device),)
 
-    def workspace_bytes(self, rows):
-        return self.eng.lib.omni_latent_attn_workspace_bytes(rows, self.spec.heads, self.rp)
+    def workspace_bytes(self, eng, rows):
+        return eng.lib.omni_latent_attn_workspace_bytes(rows, self.spec.heads, self.rp)
 
     def needs(self):
         H = self.spec.heads
         return {"proj": (self.down.N, torch.float32, "slabs"), "cq": (self.qp, "elem", "tiles"), "q": (H * self.dp, "elem", "rows"), "ql": (H * self.rp, "elem", "rows"),
                 "ol": (H * self.rp, "elem", "rows"), "v": (H * self.vp, "elem", "tiles"), "head_gate": (H, torch.float32, "rows")}
 
-    def run(self, b, i, s, x, frag):
-        e, m = self.eng, self.spec
+    def run(self, e, b, i, s, x, frag):
+        m = self.spec
         T, H, (cache,) = b.T, m.heads, e.kv_caches[i]
         slabs = e._mm(s.h, self.down, s.proj, T, f32_out=True)
         gate = s.head_gate if m.out_gate else None
         shift = e.shift_state
-        self._launch("omni_latent_write", L.LatentWrite(
+        self._launch(e, "omni_latent_write", L.LatentWrite(
             proj=s.proj.data_ptr(), slabs=slabs, slab_stride=T * self.down.N, ld=self.down.N, q_rank=m.q_rank, qp=self.qp, kv_rank=m.kv_rank, rp=self.rp, heads=H,
             qw=self.qw.data_ptr(), kw=self.kw.data_ptr(), eps=e.d.eps, cq=s.cq.data_ptr(), frag=int(frag), cache=cache.data_ptr(), gate=L.ptr(gate),
             num_live=L.ptr(b.num_live), x=x.data_ptr(), wp=e.width, state=None if shift is None else shift[i].data_ptr(), state_slot=e.state_slot.data_ptr(), T=T,
-            elem=e.elem.code, **self._where(b)))
+            elem=e.elem.code, **self._where(e, b)))
         e._mm(s.cq, self.uq, s.q, T)
         e._heads_mm(s.q, self.uk, s.ql, T, H)
         tiles, n_tiles = b.items(self.tiles)
-        self._launch("omni_latent_attn", L.LatentAttn(
+        self._launch(e, "omni_latent_attn", L.LatentAttn(
             q=s.ql.data_ptr(), cache=cache.data_ptr(), gate=L.ptr(gate), out=s.ol.data_ptr(), tiles=L.ptr(tiles), n_tiles=n_tiles, tile_rows=self.tiles[2], T=T,
             n_decode=b.n_decode, heads=H, rp=self.rp, scale=m.scale, max_keys=b.max_keys, workspace=e.attn_ws.data_ptr(), workspace_bytes=e.attn_ws.numel() * 4,
-            elem=e.elem.code, **self._where(b)))
+            elem=e.elem.code, **self._where(e, b)))
         e._heads_mm(s.ol, self.uv, s.v, T, H, out_frag=frag)
         return e._mm(s.v, self.o, s.y, T, f32_out=True)
 
@@ -215,7 +217,7 @@ def rotation_table(rows: int, dims: int, base: float) -> torch.Tensor:
 
 class WindowMixer(Mixer):
     def __init__(self, eng, i: int, m: WindowAttentionSpec, w: dict):
-        super().__init__(eng, m)
+        super().__init__(m)
         elem, dev, W, H, G = eng.elem, eng.device, eng.width, m.heads, m.kv_heads
         self.dp, self.vp, self.own = r32(m.dim), r32(m.vdim), m.kv_from is None
         parts = [pad_head_rows(w["q"], H, m.dim, self.dp, W)]
@@ -235,41 +237,41 @@ class WindowMixer(Mixer):
     def matrices(self):
         return [self.down, self.o]
 
-    def cache(self, num_blocks, block_size):
+    def cache(self, eng, num_blocks, block_size):
         if not self.own:
             return ()
-        z = lambda n: torch.zeros(num_blocks, self.spec.kv_heads, block_size, n, dtype=self.eng.elem.torch, device=self.eng.device)  # noqa: E731
+        z = lambda n: torch.zeros(num_blocks, self.spec.kv_heads, block_size, n, dtype=eng.elem.torch, device=eng.device)  # noqa: E731
         return z(self.dp), z(self.vp)
 
-    def workspace_bytes(self, rows):
-        return self.eng.lib.omni_window_attn_workspace_bytes(rows, self.spec.heads, self.vp)
+    def workspace_bytes(self, eng, rows):
+        return eng.lib.omni_window_attn_workspace_bytes(rows, self.spec.heads, self.vp)
 
     def needs(self):
         H = self.spec.heads
         return {"proj": (self.down.N, torch.float32, "slabs"), "q": (H * self.dp, "elem", "rows"), "gate": (H * self.vp, "elem", "rows"), "v": (H * self.vp, "elem", "tiles")}
 
-    def run(self, b, i, s, x, frag):
-        e, m = self.eng, self.spec
+    def run(self, e, b, i, s, x, frag):
+        m = self.spec
         T, H = b.T, m.heads
         kc, vc = e.kv_caches[e.d.kv_owner(i)]
         slabs = e._mm(s.h, self.down, s.proj, T, f32_out=True)
         gate = s.gate if m.out_gate else None
-        self._launch("omni_qkv_write", L.QkvWrite(
+        self._launch(e, "omni_qkv_write", L.QkvWrite(
             proj=s.proj.data_ptr(), slabs=slabs, slab_stride=T * self.down.N, ld=self.down.N, heads=H, kv_heads=m.kv_heads, dim=m.dim, dp=self.dp, vp=self.vp,
             qw=L.ptr(self.qw), kw=L.ptr(self.kw), eps=e.d.eps, rot=L.ptr(self.rot), rot_dims=m.rot_dims, rot_rows=0 if self.rot is None else self.rot.shape[0],
             q=s.q.data_ptr(), kc=kc.data_ptr() if self.own else None, vc=vc.data_ptr() if self.own else None, gate=L.ptr(gate), num_live=L.ptr(b.num_live), T=T,
-            elem=e.elem.code, **self._where(b)))
+            elem=e.elem.code, **self._where(e, b)))
         tiles, n_tiles = b.items(self.tiles)
-        self._launch("omni_window_attn", L.WindowAttn(
+        self._launch(e, "omni_window_attn", L.WindowAttn(
             q=s.q.data_ptr(), kc=kc.data_ptr(), vc=vc.data_ptr(), gate=L.ptr(gate), sink=L.ptr(self.sink), out=s.v.data_ptr(), frag=int(frag), tiles=L.ptr(tiles),
             n_tiles=n_tiles, tile_rows=self.tiles[2], T=T, n_decode=b.n_decode, heads=H, kv_heads=m.kv_heads, dp=self.dp, vp=self.vp, scale=m.scale, window=m.window or 0,
-            max_keys=b.max_keys, workspace=e.attn_ws.data_ptr(), workspace_bytes=e.attn_ws.numel() * 4, elem=e.elem.code, **self._where(b)))
+            max_keys=b.max_keys, workspace=e.attn_ws.data_ptr(), workspace_bytes=e.attn_ws.numel() * 4, elem=e.elem.code, **self._where(e, b)))
         return e._mm(s.v, self.o, s.y, T, f32_out=True)
 
 
 class DecayMixer(Mixer):
     def __init__(self, eng, i: int, m: DecayRecurrenceSpec, w: dict):
-        super().__init__(eng, m)
+        super().__init__(m)
         elem, dev, W, H = eng.elem, eng.device, eng.width, m.heads
         self.dp, self.vp = r32(m.dim), r32(m.vdim)
         self.down = Matrix(torch.cat([pad_head_rows(w["q"], H, m.dim, self.dp, W), pad_head_rows(w["k"], H, m.dim, self.dp, W),
@@ -284,15 +286,15 @@ class DecayMixer(Mixer):
     def matrices(self):
         return [self.down, self.o]
 
-    def state(self, slots):
-        return torch.zeros(slots, self.spec.heads, self.dp, self.vp, dtype=torch.float32, device=self.eng.device)
+    def state(self, eng, slots):
+        return torch.zeros(slots, self.spec.heads, self.dp, self.vp, dtype=torch.float32, device=eng.device)
 
     def needs(self):
         n = self.spec.heads * self.vp
         return {"proj": (self.down.N, torch.float32, "slabs"), "rec": (n, torch.float32, "rows"), "v": (n, "elem", "tiles")}
 
-    def run(self, b, i, s, x, frag):
-        e, m = self.eng, self.spec
+    def run(self, e, b, i, s, x, frag):
+        m = self.spec
         T, H, ld, n = b.T, m.heads, self.down.N, m.heads * self.vp
         gcol = H * (2 * self.dp + self.vp)
         wide = e.elem.code == 0 and not frag              # prompts: activations in the product's epilogue, bf16 rows
@@ -313,8 +315,8 @@ class DecayMixer(Mixer):
         else:
             runs, a.n_runs = b.items(("runs",))
             a.runs = L.ptr(runs)
-        self._launch("omni_decay_rec", a)
-        self._launch("omni_gated_norm", L.GatedNorm(o=s.rec.data_ptr(), w=self.norm.data_ptr(), gate=gate, slabs=slabs, slab_stride=T * ld, ld=ld, n=n, count=H * m.vdim,
+        self._launch(e, "omni_decay_rec", a)
+        self._launch(e, "omni_gated_norm", L.GatedNorm(o=s.rec.data_ptr(), w=self.norm.data_ptr(), gate=gate, slabs=slabs, slab_stride=T * ld, ld=ld, n=n, count=H * m.vdim,
                                                     eps=e.d.eps, out=s.v.data_ptr(), frag=int(frag), T=T, elem=e.elem.code))
         return e._mm(s.v, self.o, s.y, T, f32_out=True)
 

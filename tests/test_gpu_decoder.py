@@ -301,3 +301,21 @@ def test_command_lines(name, tmp_path):
     assert r.returncode == 0, r.stderr[-2000:]
     want, margins = greedy_oracle(w, cfg, toks, 5)
     assert min(margins) > 1e-4 and json.loads(r.stdout.strip().split("\n")[-1])["token_ids"] == want
+
+
+@pytest.mark.parametrize("name", ["mixed", "k_mixed"])
+def test_an_engine_out_of_use_gives_its_memory_back_at_once(name):
+    """No reference circle keeps it for the collector: the next engine's memory accounting would count it."""
+    import gc
+    import weakref
+    d, w, _ = model(name, seed=16)
+    gc.collect()
+    gc.disable()
+    try:
+        eng = DecoderEngine(d, w, num_blocks=8, max_batch=2)
+        gone = weakref.ref(eng)
+        eng.forward(eng.make_batch(torch.tensor([1, 2, 3]), [0] * 3, [0, 1, 2], [3]))
+        del eng
+        assert gone() is None
+    finally:
+        gc.enable()

@@ -65,11 +65,9 @@ def test_weight_vectors_of_added_and_final_norms_and_scaled_embedding(elem):
     close(out[:, :width], D.rms_norm(new, fw.double(), 1e-6)[sel.long()], RTOL[elem])
 
 
-@pytest.mark.parametrize("elem", [0, 1])
-@pytest.mark.parametrize("heads,dim,form", [(1, 8, "sums"), (3, 40, "sums"), (16, 128, "sums"), (3, 40, "rows"), (20, 200, "rows")])
+@pytest.mark.parametrize("elem,form", [(0, "sums"), (1, "sums"), (0, "rows")])
+@pytest.mark.parametrize("heads,dim", [(1, 8), (3, 40), (16, 128), (20, 200)])
 def test_gated_norm(elem, heads, dim, form):
-    if form == "rows" and elem:
-        pytest.skip("rows behind the sigmoid are bf16")
     g, T, dp = gen(dim), 9, r32(dim)
     n = heads * dp
     o, z, w = torch.randn(T, heads * dim, generator=g), torch.randn(T, heads * dim, generator=g), torch.randn(heads * dim, generator=g).to(ELEMS[elem])
