@@ -22,18 +22,20 @@ struct StreamArgs {
     omni_row_table rt;
 };
 
-template <int MT, int NT, int KIND>
+// P: k-steps in flight per wave: 2 on a grid that fills the chip (4 measured the same or slower at 1 .. 64 rows).
+// grid.z: groups of MT row tiles (more than one on narrow products only)
+template <int MT, int NT, int KIND, int P>
 __global__ __launch_bounds__(GS_THREADS) void gemm_stream_kernel(const StreamArgs a) {
-    constexpr int P = 2;                               // (4 measured the same or slower at 1 .. 64 rows)
     extern __shared__ __attribute__((aligned(16))) f32x4 part[];      // [wave][NT * MT][lane]
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int k0 = blockIdx.y * a.split_steps, nk = min(a.split_steps, a.nsteps - k0);
+    const int m0 = blockIdx.z * MT;
     const uint16_t* wp[NT];
     const uint16_t* xp[MT];
 #pragma unroll
     for (int j = 0; j < NT; ++j) wp[j] = a.W + ((size_t)(blockIdx.x * NT + j) * a.nsteps + k0 + wave) * 512 + lane * 8;
 #pragma unroll
-    for (int i = 0; i < MT; ++i) xp[i] = a.x + ((size_t)min(i, ((a.M + 15) >> 4) - 1) * a.nsteps + k0 + wave) * 512 + lane * 8;      // row tiles past M: re-read, discarded
+    for (int i = 0; i < MT; ++i) xp[i] = a.x + ((size_t)min(m0 + i, ((a.M + 15) >> 4) - 1) * a.nsteps + k0 + wave) * 512 + lane * 8;      // row tiles past M: re-read, discarded
     f32x4 acc[NT][MT];
 #pragma unroll
     for (int j = 0; j < NT; ++j)
@@ -83,7 +85,7 @@ __global__ __launch_bounds__(GS_THREADS) void gemm_stream_kernel(const StreamArg
     __syncthreads();
     for (int it = threadIdx.x; it < NT * MT * 64; it += GS_THREADS) {
         const int l = it & 63, f = it >> 6, j = f / MT, i = f - j * MT;
-        const int m = i * 16 + (l & 15), n = (blockIdx.x * NT + j) * 16 + 4 * (l >> 4);
+        const int m = (m0 + i) * 16 + (l & 15), n = (blockIdx.x * NT + j) * 16 + 4 * (l >> 4);
         if (m >= a.M) continue;
         f32x4 v = part[f * 64 + l];
 #pragma unroll
@@ -129,14 +131,14 @@ static void gs_policy(int M, int N, int nsteps, bool slabs, int* nt, int* splits
     }
 }
 
-template <int MT, int NT, int KIND>
+template <int MT, int NT, int KIND, int P>
 static int gs_launch(const StreamArgs& a, int splits, hipStream_t st) {
     constexpr int LDS = GS_WAVES * NT * MT * 1024;
     if (LDS > 64 * 1024) {
-        static const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(gemm_stream_kernel<MT, NT, KIND>), hipFuncAttributeMaxDynamicSharedMemorySize, LDS);
+        static const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(gemm_stream_kernel<MT, NT, KIND, P>), hipFuncAttributeMaxDynamicSharedMemorySize, LDS);
         if (e != hipSuccess) { omni_set_error("omni_gemm_stream: LDS attribute: %s", hipGetErrorString(e)); return OMNI_EHIP; }
     }
-    hipLaunchKernelGGL((gemm_stream_kernel<MT, NT, KIND>), dim3(a.N / (16 * NT), splits), dim3(GS_THREADS), LDS, st, a);
+    hipLaunchKernelGGL((gemm_stream_kernel<MT, NT, KIND, P>), dim3(a.N / (16 * NT), splits, ((a.M + 15) / 16 + MT - 1) / MT), dim3(GS_THREADS), LDS, st, a);
     OMNI_CHECK_LAUNCH("omni_gemm_stream");
     return OMNI_OK;
 }
@@ -152,7 +154,12 @@ static int gs_run(StreamArgs a, int kind, bool one, hipStream_t st) {
     gs_policy(a.M, a.N, a.nsteps, kind == GS_F32 && !one, &nt, &splits);
     a.split_steps = (a.nsteps + splits - 1) / splits;
     const int mt = a.M > 32 ? 4 : (a.M > 16 ? 2 : 1);
-#define GS(MT_, NT_, K_) if (mt == MT_ && nt == NT_ && kind == K_) return gs_launch<MT_, NT_, K_>(a, splits, st);
+    // a narrow product (a side input's gate): its few workgroups would each pull all of x through one CU, so the rows are dealt out as well
+    if (a.N / 16 * splits <= 32) {
+        if (kind == GS_F32) return gs_launch<1, 1, GS_F32, 4>(a, splits, st);
+        return kind == GS_BF16 ? gs_launch<1, 1, GS_BF16, 4>(a, splits, st) : gs_launch<1, 1, GS_ACT, 4>(a, splits, st);
+    }
+#define GS(MT_, NT_, K_) if (mt == MT_ && nt == NT_ && kind == K_) return gs_launch<MT_, NT_, K_, 2>(a, splits, st);
 #define GS_NT(NT_, K_) GS(1, NT_, K_) GS(2, NT_, K_) GS(4, NT_, K_)
 #define GS_ALL(K_) GS_NT(1, K_) GS_NT(2, K_) GS_NT(3, K_) GS_NT(4, K_)
     GS_ALL(GS_F32) GS_ALL(GS_BF16) GS_ALL(GS_ACT)
