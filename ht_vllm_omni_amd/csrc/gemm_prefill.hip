@@ -63,15 +63,22 @@ __device__ __forceinline__ f32x4 tg_mfma(u32x4 a, u32x4 b, f32x4 c) {
 
 __device__ __forceinline__ float tg_gelu(float v) { return 0.5f * v * (1.0f + erff(v * 0.70710678118654752f)); }
 
-__device__ __forceinline__ bool tile_plain(const TileArgs& a) {
-    return !a.bias && !a.scale && (a.act == OMNI_TILE_ACT_NONE || a.act == OMNI_TILE_ACT_SILU_MUL_GU8) && !a.resid && !a.out_f32 && !a.out2 && a.out;
+// Epilogues, each a body of its own: one that held every activation outgrew the compiler's unrolling of its passes at 256 rows, and accumulators
+// indexed by a run-time pass live in scratch memory (+ 25 us per launch).
+//   EPI_PLAIN  bf16 out        EPI_ACT  XIELU, RELU2, SILU_SIGMOID, GELU_MUL or none -> bf16 and / or fp32 out
+//   EPI_FULL   bias, scale, GELU or none, residual, any outputs
+enum { EPI_PLAIN = 0, EPI_ACT = 1, EPI_FULL = 2 };
+__device__ __forceinline__ int tile_epi(const TileArgs& a) {
+    if (a.bias || a.scale || a.act == OMNI_TILE_ACT_GELU || a.resid || a.out2) return EPI_FULL;
+    return a.out_f32 || a.act >= OMNI_TILE_ACT_XIELU ? EPI_ACT : EPI_PLAIN;
 }
 
 // Epilogue of a tile kernel: `acc[j][i]` = this wave's WN n-tiles x WM m-tiles (D[n][m] fragments), first row mw0, first column nw0; `lds` is dead.
-// PLAIN = no bias, scale, GELU, residual, fp32 or snake output (the talker prefill's four GEMMs): the same values (acc + 0 and * 1 change
-// nothing) without ~20 wave-uniform branches per pass -- they, not the stores, were most of an 11 k-cycle epilogue (profiles/r05_gemm_pp_stamps.txt).
-template <int WN, int WM, bool GU8, bool PLAIN>
+// EPI_PLAIN (the talker prefill's four GEMMs): the same values as EPI_FULL (acc + 0 and * 1 change nothing) without ~20 wave-uniform branches per
+// pass -- they, not the stores, were most of an 11 k-cycle epilogue (profiles/r05_gemm_pp_stamps.txt).
+template <int WN, int WM, bool GU8, int EPI>
 __device__ __forceinline__ void tile_epilogue(const TileArgs& a, f32x4 (&acc)[WN][WM], uint8_t* lds, int wave, int lane, int mw0, int nw0) {
+    asm volatile("" : "+v"(lane));                        // addresses are this body's own: shared ones would be computed, and held, before the branch
     const int c = lane & 15, q = lane >> 4;
     // ---- epilogue.  Register side: y = act(acc + bias) * scale in fp32, transposed through this wave's LDS image in fp32, ONE m-tile
     // (16 rows x the wave's WN * 16 columns) per pass.  Row side: 8 columns per lane, a row's lanes cover WN * 64 contiguous bytes
@@ -83,68 +90,47 @@ __device__ __forceinline__ void tile_epilogue(const TileArgs& a, f32x4 (&acc)[WN
     constexpr int PER_ROW = GU8 ? WN : WN * 2;            // lane items per image row: a [8 gate | 8 up] tile, or 8 columns
     constexpr int RIT = (16 * PER_ROW + 63) / 64;         // row-side iterations per pass
     uint8_t* img = lds + wave * (16 * IPITCH);
-    f32x4 bq[WN], sq[WN];
-#pragma unroll
-    for (int j = 0; j < WN; ++j) {
+    auto bias_scale = [&](int j, f32x4& b, f32x4& s) {
         const int n = nw0 + j * 16 + 4 * q;
-        bq[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-        sq[j] = f32x4{1.f, 1.f, 1.f, 1.f};
-        if (!PLAIN && n < a.N) {
-            if (a.bias) bq[j] = *reinterpret_cast<const f32x4*>(a.bias + n);
-            if (a.scale) sq[j] = *reinterpret_cast<const f32x4*>(a.scale + n);
+        b = f32x4{0.f, 0.f, 0.f, 0.f};
+        s = f32x4{1.f, 1.f, 1.f, 1.f};
+        if (EPI == EPI_FULL && n < a.N) {
+            if (a.bias) b = *reinterpret_cast<const f32x4*>(a.bias + n);
+            if (a.scale) s = *reinterpret_cast<const f32x4*>(a.scale + n);
         }
+    };
+    constexpr bool HELD = WN < 8;                         // wider waves read them once per pass: their registers are full
+    f32x4 bq[WN], sq[WN];
+    if (HELD) {
+#pragma unroll
+        for (int j = 0; j < WN; ++j) bias_scale(j, bq[j], sq[j]);
     }
-    const bool gelu = !PLAIN && a.act == OMNI_TILE_ACT_GELU, xie = !PLAIN && a.act == OMNI_TILE_ACT_XIELU, mul = !PLAIN && a.act == OMNI_TILE_ACT_GELU_MUL,
-               other = mul || (!PLAIN && (a.act == OMNI_TILE_ACT_RELU2 || a.act == OMNI_TILE_ACT_SILU_SIGMOID));
-    auto write_image = [&](const int pass) {
-        if (PLAIN) {
+    const bool gelu = EPI == EPI_FULL && a.act == OMNI_TILE_ACT_GELU, mul = EPI == EPI_ACT && a.act == OMNI_TILE_ACT_GELU_MUL;
+    auto write_as = [&](const int pass, auto f) {         // f(value, n-tile, bias, scale)
 #pragma unroll
-            for (int j = 0; j < WN; ++j) *reinterpret_cast<f32x4*>(img + c * IPITCH + (j * 16 + 4 * q) * 4) = acc[j][pass];
-        } else if (gelu) {
+        for (int j = 0; j < WN; ++j) {
+            f32x4 v, b = bq[j], s = sq[j];
+            if (!HELD) bias_scale(j, b, s);
 #pragma unroll
-            for (int j = 0; j < WN; ++j) {
-                f32x4 v;
-#pragma unroll
-                for (int e = 0; e < 4; ++e) v[e] = tg_gelu(acc[j][pass][e] + bq[j][e]) * sq[j][e];
-                *reinterpret_cast<f32x4*>(img + c * IPITCH + (j * 16 + 4 * q) * 4) = v;
-            }
-        } else if (xie) {
-#pragma unroll
-            for (int j = 0; j < WN; ++j) {
-                f32x4 v;
-#pragma unroll
-                for (int e = 0; e < 4; ++e) v[e] = xielu(acc[j][pass][e] + bq[j][e], a.act_p, a.act_n) * sq[j][e];
-                *reinterpret_cast<f32x4*>(img + c * IPITCH + (j * 16 + 4 * q) * 4) = v;
-            }
-        } else if (other) {
-#pragma unroll
-            for (int j = 0; j < WN; ++j) {
-                f32x4 v;
-#pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    const float z = acc[j][pass][e] + bq[j][e];
-                    if (a.act == OMNI_TILE_ACT_RELU2) v[e] = relu2(z);
-                    else if (a.act == OMNI_TILE_ACT_GELU_MUL) v[e] = gelu_tanh(z);
-                    else v[e] = (nw0 + j * 16 + 4 * q < a.act_cols ? z : 1.0f) * sigmoidf_(z);
-                    v[e] *= sq[j][e];
-                }
-                *reinterpret_cast<f32x4*>(img + c * IPITCH + (j * 16 + 4 * q) * 4) = v;
-            }
-        } else {
-#pragma unroll
-            for (int j = 0; j < WN; ++j) {
-                f32x4 v;
-#pragma unroll
-                for (int e = 0; e < 4; ++e) v[e] = (acc[j][pass][e] + bq[j][e]) * sq[j][e];
-                *reinterpret_cast<f32x4*>(img + c * IPITCH + (j * 16 + 4 * q) * 4) = v;
-            }
+            for (int e = 0; e < 4; ++e) v[e] = f(acc[j][pass][e], j, b[e], s[e]);
+            *reinterpret_cast<f32x4*>(img + c * IPITCH + (j * 16 + 4 * q) * 4) = v;
         }
+    };
+    auto write_image = [&](const int pass) {
+        if (EPI == EPI_ACT && a.act == OMNI_TILE_ACT_XIELU) write_as(pass, [&](float z, int, float, float) { return xielu(z, a.act_p, a.act_n); });
+        else if (EPI == EPI_ACT && a.act == OMNI_TILE_ACT_RELU2) write_as(pass, [&](float z, int, float, float) { return relu2(z); });
+        else if (EPI == EPI_ACT && a.act == OMNI_TILE_ACT_SILU_SIGMOID)
+            write_as(pass, [&](float z, int j, float, float) { return (nw0 + j * 16 + 4 * q < a.act_cols ? z : 1.0f) * sigmoidf_(z); });
+        else if (mul) write_as(pass, [&](float z, int, float, float) { return gelu_tanh(z); });
+        else if (gelu) write_as(pass, [&](float z, int, float b, float s) { return tg_gelu(z + b) * s; });
+        else if (EPI == EPI_FULL) write_as(pass, [&](float z, int, float b, float s) { return (z + b) * s; });
+        else write_as(pass, [&](float z, int, float, float) { return z; });
     };
     f32x4 rv[RIT][2];
 #pragma unroll
     for (int pass = 0; pass < WM; ++pass) {
         const int mp0 = mw0 + pass * 16;
-        if (!PLAIN && !GU8 && a.resid) {
+        if (EPI == EPI_FULL && !GU8 && a.resid) {
 #pragma unroll
             for (int it = 0; it < RIT; ++it) {
                 const int idx = lane + 64 * it;
@@ -189,7 +175,7 @@ __device__ __forceinline__ void tile_epilogue(const TileArgs& a, f32x4 (&acc)[WN
                 if (idx >= 16 * PER_ROW || m >= a.M || n >= a.N) continue;
                 f32x4 y0 = *reinterpret_cast<const f32x4*>(img + row * IPITCH + ch * 32);
                 f32x4 y1 = *reinterpret_cast<const f32x4*>(img + row * IPITCH + ch * 32 + 16);
-                if (PLAIN) {
+                if (EPI == EPI_PLAIN) {
                     u32x4 o;
                     o[0] = pack_bf2(y0[0], y0[1]); o[1] = pack_bf2(y0[2], y0[3]);
                     o[2] = pack_bf2(y1[0], y1[1]); o[3] = pack_bf2(y1[2], y1[3]);
@@ -206,7 +192,7 @@ __device__ __forceinline__ void tile_epilogue(const TileArgs& a, f32x4 (&acc)[WN
                         y1[2 * e] *= bf_lo(z[2 + e]); y1[2 * e + 1] *= bf_hi(z[2 + e]);
                     }
                 }
-                if (a.resid) {
+                if (EPI == EPI_FULL && a.resid) {
                     y0 += rv[it][0];
                     y1 += rv[it][1];
                 }
@@ -221,7 +207,7 @@ __device__ __forceinline__ void tile_epilogue(const TileArgs& a, f32x4 (&acc)[WN
                     o[2] = pack_bf2(y1[0], y1[1]); o[3] = pack_bf2(y1[2], y1[3]);
                     *reinterpret_cast<u32x4*>(a.out + (size_t)m * a.ldo + n) = o;
                 }
-                if (a.out2) {
+                if (EPI == EPI_FULL && a.out2) {
                     const f32x4 al0 = *reinterpret_cast<const f32x4*>(a.snake_alpha + n), al1 = *reinterpret_cast<const f32x4*>(a.snake_alpha + n + 4);
                     const f32x4 ib0 = *reinterpret_cast<const f32x4*>(a.snake_inv_beta + n), ib1 = *reinterpret_cast<const f32x4*>(a.snake_inv_beta + n + 4);
                     f32x4 z0, z1;
@@ -240,6 +226,14 @@ __device__ __forceinline__ void tile_epilogue(const TileArgs& a, f32x4 (&acc)[WN
         }
         __builtin_amdgcn_wave_barrier();
     }
+}
+
+template <int WN, int WM, bool GU8>
+__device__ __forceinline__ void tile_epilogue_of(const TileArgs& a, f32x4 (&acc)[WN][WM], uint8_t* lds, int wave, int lane, int mw0, int nw0) {
+    const int epi = tile_epi(a);
+    if (epi == EPI_PLAIN) tile_epilogue<WN, WM, GU8, EPI_PLAIN>(a, acc, lds, wave, lane, mw0, nw0);
+    else if (!GU8 && epi == EPI_ACT) tile_epilogue<WN, WM, GU8, EPI_ACT>(a, acc, lds, wave, lane, mw0, nw0);
+    else tile_epilogue<WN, WM, GU8, EPI_FULL>(a, acc, lds, wave, lane, mw0, nw0);
 }
 
 // Geometry of one instantiation: 8 waves (two per SIMD: while one issues its LDS-DMA pieces -- 60 - 180 cycles each -- or waits
@@ -411,8 +405,7 @@ __global__ __launch_bounds__(TG_THREADS) void gemm_tile_kernel(const TileArgs a_
 #undef TG_SLICE
     asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");   // the ring is dead: its tail loads (zeros) landed
 
-    if (tile_plain(a)) tile_epilogue<WN, WM, GU8, true>(a, acc, lds, wave, lane, m0 + wm * WM * 16, n0 + wn * WN * 16);
-    else tile_epilogue<WN, WM, GU8, false>(a, acc, lds, wave, lane, m0 + wm * WM * 16, n0 + wn * WN * 16);
+    tile_epilogue_of<WN, WM, GU8>(a, acc, lds, wave, lane, m0 + wm * WM * 16, n0 + wn * WN * 16);
 }
 
 // ---- the two-group ("ping-pong") form of the 256-column tile.  Same images, same MFMA, same accumulation order as gemm_tile_kernel
@@ -609,8 +602,7 @@ __global__ __launch_bounds__(TG_THREADS) void gemm_tile_pp_kernel(const TileArgs
         for (int i = 0; i < st_n && i < 1023; ++i) g_pp_stamps[grp][1 + i] = st_buf[i];
     if (st_wave) g_pp_stamps[grp][0] = st_n;
 #endif
-    if (tile_plain(a)) tile_epilogue<4, MW, GU8, true>(a, acc, lds, wave, lane, m0 + grp * MW * 16, n0 + wc * 64);
-    else tile_epilogue<4, MW, GU8, false>(a, acc, lds, wave, lane, m0 + grp * MW * 16, n0 + wc * 64);
+    tile_epilogue_of<4, MW, GU8>(a, acc, lds, wave, lane, m0 + grp * MW * 16, n0 + wc * 64);
 #if defined(PP_STAMPS) && PP_STAMPS == 3
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     PP_C(3);
@@ -684,6 +676,7 @@ extern "C" int omni_gemm_tile(const omni_tile_gemm* g, void* stream) {
     OMNI_CHECK_ARG((int64_t)g->N * g->K * 2 < (int64_t)TG_OOB, "omni_gemm_tile: W exceeds the 2 GB descriptor");
     const bool gu8 = g->act == OMNI_TILE_ACT_SILU_MUL_GU8;
     OMNI_CHECK_ARG(g->act >= OMNI_TILE_ACT_NONE && g->act <= OMNI_TILE_ACT_GELU_MUL, "omni_gemm_tile: act=%d", g->act);
+    OMNI_CHECK_ARG(g->act < OMNI_TILE_ACT_XIELU || (!g->bias && !g->scale && !g->resid && !g->out2), "omni_gemm_tile: act=%d takes no bias, scale, residual or second output", g->act);
     OMNI_CHECK_ARG(g->act != OMNI_TILE_ACT_SILU_SIGMOID || (g->act_cols >= 0 && g->act_cols % 4 == 0), "omni_gemm_tile: act_cols=%d (%% 4)", g->act_cols);
     OMNI_CHECK_ARG(g->act != OMNI_TILE_ACT_GELU_MUL || (g->mul_table && g->mul_ids && g->mul_rows > 0 && g->mul_ld >= g->N && g->mul_ld % 8 == 0 && g->out && !g->out2 && !g->resid &&
                                                         g->groups <= 1), "omni_gemm_tile: the row table takes ids, mul_ld >= N (%% 8), a bf16 output and one group");
