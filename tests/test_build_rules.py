@@ -3,7 +3,10 @@
 Rule 1: no packed fp32 operation (v_pk_fma_f32 / v_pk_mul_f32 / v_pk_add_f32) in any kernel.  hipcc -O3 forms them by itself from ordinary
 float code, and the forms that read the high dword of a VGPR src1 pair in the low lane return wrong results while another wave of the same
 SIMD issues MFMAs (profiles/r04_pkfma_probe.txt) -- parity-green and bit-stable alone, wrong beside a neighbour.  The libraries are built
-with the feature off (build.FLAGS); this test compiles with the same flags and looks at what came out."""
+with the feature off (build.FLAGS); this test compiles with the same flags and looks at what came out.
+
+Rule 2: no scratch memory in the kernels of the language models' library.  A tile kernel whose epilogue outgrew the compiler's unrolling kept its
+accumulators there -- right results, 25 us more per launch."""
 import os
 import re
 import shutil
@@ -30,6 +33,10 @@ def packed_fp32(lines):
     return [l.strip() for l in lines if PACKED.match(l)]
 
 
+def scratch_bytes(lines):
+    return [int(m.group(1)) for m in (re.match(r"^; ScratchSize: (\d+)", l) for l in lines) if m]
+
+
 def test_the_scanner_sees_the_form():
     got = packed_fp32(["_Zk:", "\tv_pk_fma_f32 v[0:1], v[2:3], v[4:5], v[0:1] op_sel:[0,1,0]", "\tv_pk_mul_f32 v[0:1], v[2:3], v[4:5]",
                        "\tv_pk_add_f32 v[0:1], v[2:3], s[4:5]", "\tv_pk_fma_f16 v0, v1, v2, v3", "\tv_fma_f32 v0, v1, v2, v3"])
@@ -52,3 +59,7 @@ def test_no_kernel_holds_a_packed_fp32_op(tmp_path, defines):
     bad = [(n, x) for n, lines in zip(names, asms) for x in packed_fp32(lines)]
     assert sum(len(a) for a in asms) > 10000
     assert not bad, f"{len(bad)} packed fp32 ops, e.g. {bad[:4]}"
+    if not defines:
+        scratch = {n: scratch_bytes(lines) for n, lines in zip(names, asms) if n in B.DECODER_SOURCES}
+        assert sum(map(len, scratch.values())) > 50
+        assert not any(map(any, scratch.values())), {n: v for n, v in scratch.items() if any(v)}
